@@ -6,5 +6,6 @@ from .nenotar import NenotarConfig
 from .bonerax import BoneraxConfig
 from .givozen import GivozenConfig
 from .salipel import SalipelConfig
+from .neruzen import NeruzenConfig
 
-__all__ = ["ConfigError", "KeyReader", "read_json", "MiniMaxM3Config", "NenotarConfig", "BoneraxConfig", "GivozenConfig", "SalipelConfig"]
+__all__ = ["ConfigError", "KeyReader", "read_json", "MiniMaxM3Config", "NenotarConfig", "BoneraxConfig", "GivozenConfig", "SalipelConfig", "NeruzenConfig"]

@@ -1,5 +1,8 @@
 // Latent attention on the matrix cores (bfloat16): the attention of latent.hip for steps whose sizes the 16x16x32
-// instruction takes (latent C a multiple of 16 up to 512, C + R a multiple of 32, pages of a multiple of 8 tokens).
+// instruction takes (latent C a multiple of 16 up to 512, R a multiple of 8, cache rows of ldc values, a multiple of 32, with
+// zeros behind the C + R, pages of a multiple of 8 tokens).
+// Under a window of `window` keys (0: none) a row at position p sees keys p - window + 1 .. p: an item starts at the segment
+// of its first row's lowest key, keys below a column's own lowest weigh 0, and no page below the item's lowest key is read.
 //
 // Decoded rows (one row of a request in the step) share out their context: blocks of 128 keys each go to an item of their
 // own, which stores partial sums, and a second kernel joins them (so a decoded row's bits depend on its own context
@@ -24,7 +27,7 @@ typedef float f32x4_t __attribute__((ext_vector_type(4)));
 struct LatentMfmaArgs {
     const bf16_t* q_lat;    // [H, T, C]
     const bf16_t* q_rot;    // [H, T, R]
-    const bf16_t* cache;    // [pages, page_tokens, C + R]
+    const bf16_t* cache;    // [pages, page_tokens, ldc]
     const bf16_t* cache_t;  // [pages, C, page_tokens]
     const int* pos;
     const int* row_entry;
@@ -34,8 +37,35 @@ struct LatentMfmaArgs {
     float* part_o;          // [slots, 16, C]: a split item's sums, not yet divided
     float* part_ml;         // [slots, 16, 2]: its maximum and its sum of weights
     float scale;
-    int T, H, C, R, page_tokens, max_blocks;
+    int T, H, C, R, ldc, page_tokens, max_blocks, window, row_major;
 };
+
+// Where a (head, row)'s queries and result lie, in rows of C (or R) values.
+__device__ __forceinline__ size_t latent_row(const LatentMfmaArgs& a, int h, int r) {
+    return a.row_major ? (size_t)r * a.H + h : (size_t)h * a.T + r;
+}
+
+// The keys an item walks: from the segment of the lowest key its first row sees to its last row's position, or, for a split
+// item, a block of them (item[4] .. item[5] - 1; under a window item[4] counts blocks of item[5] keys from the block of
+// the row's lowest key on, so that a list of items fits every position).
+struct LatentKeys {
+    int lo_min, begin, last;
+};
+__device__ __forceinline__ LatentKeys latent_keys(const LatentMfmaArgs& a, const int* item, int p_first, int p_max) {
+    LatentKeys k;
+    k.lo_min = a.window > 0 ? max(0, p_first - a.window + 1) : 0;
+    if (item[6] < 0) {
+        k.begin = (k.lo_min / 64) * 64;
+        k.last = p_max;
+    } else if (a.window > 0) {
+        k.begin = (k.lo_min / item[5] + item[4]) * item[5];
+        k.last = min(k.begin + item[5] - 1, p_max);
+    } else {
+        k.begin = item[4];
+        k.last = min(item[5] - 1, p_max);
+    }
+    return k;
+}
 
 #define LM_SEG 64
 #define LM_ITEM_INTS 8
@@ -47,11 +77,11 @@ struct LatentMfmaArgs {
 // of weights in its slot; the merge kernel joins a column's slots in key order.
 template <int CT>
 __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArgs a) {
-    extern __shared__ __align__(16) bf16_t qs[];   // [16][C + R + 8]
+    extern __shared__ __align__(16) bf16_t qs[];   // [16][ldc + 8]
     const int lane = threadIdx.x, col = lane & 15, g = lane >> 4;
     const int* item = a.items + LM_ITEM_INTS * (size_t)blockIdx.x;
     const int row0 = item[0], rows = item[1], head0 = item[2], heads = item[3], slot = item[6];
-    const int C = a.C, R = a.R, CR = C + R, ldq = CR + 8, pt = a.page_tokens;
+    const int C = a.C, R = a.R, CR = a.ldc, ldq = CR + 8, pt = a.page_tokens;
     const int n_cols = rows * heads;
 
     // the columns' queries into LDS, 16 bytes a lane and turn, eight turns' loads in flight together; columns without a
@@ -67,8 +97,8 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
                 v[u] = uint4{0, 0, 0, 0};
                 if (i < chunks && c < n_cols) {
                     const int r = row0 + c / heads, h = head0 + c % heads;
-                    v[u] = d < C ? *reinterpret_cast<const uint4*>(a.q_lat + ((size_t)h * a.T + r) * C + d)
-                                 : *reinterpret_cast<const uint4*>(a.q_rot + ((size_t)h * a.T + r) * R + (d - C));
+                    if (d < C) v[u] = *reinterpret_cast<const uint4*>(a.q_lat + latent_row(a, h, r) * C + d);
+                    else if (d < C + R) v[u] = *reinterpret_cast<const uint4*>(a.q_rot + latent_row(a, h, r) * R + (d - C));
                 }
             }
 #pragma unroll
@@ -82,13 +112,14 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
 
     const bool live = col < n_cols;
     const int c_row = row0 + (live ? col / heads : 0), c_head = head0 + (live ? col % heads : 0);
-    const int p_col = a.pos[c_row];
+    const int p_col = a.pos[c_row], lo_col = a.window > 0 ? p_col - a.window + 1 : 0;
     const int p_max = a.pos[row0 + rows - 1];
     const int* table = a.tables + (size_t)a.row_entry[row0] * a.max_blocks;
     const int steps = CR / 32;
     const int last_group = (p_max / 8) * 8;
-    const int key_begin = slot < 0 ? 0 : item[4];
-    const int key_last = slot < 0 ? p_max : min(item[5] - 1, p_max);
+    const LatentKeys range = latent_keys(a, item, a.pos[row0], p_max);
+    const int key_begin = range.begin, key_last = range.last;
+    const int first_group = (range.lo_min / 8) * 8;
 
     f32x4_t o[CT];
 #pragma unroll
@@ -101,7 +132,7 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
 #pragma unroll
         for (int v = 0; v < 4; ++v) {
             int key = seg0 + 32 * (v >> 1) + 8 * (col >> 2) + 4 * (v & 1) + (col & 3);
-            key = key < p_max ? key : p_max;     // keys beyond the last row's position weigh nothing; read a key that exists
+            key = min(max(key, range.lo_min), p_max);     // keys outside the rows' range weigh nothing; read a key that exists
             kp[v] = a.cache + ((size_t)table[key / pt] * pt + key % pt) * CR + 8 * g;
         }
         f32x4_t s[4];
@@ -136,12 +167,12 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
                 const int key = seg0 + 32 * (v >> 1) + 8 * g + 4 * (v & 1) + i;
-                s[v][i] = key <= p_col ? s[v][i] * a.scale : -INFINITY;
+                s[v][i] = key <= p_col && key >= lo_col ? s[v][i] * a.scale : -INFINITY;
                 top = fmaxf(top, s[v][i]);
             }
         top = rows_max4(top);
-        const float m_new = fmaxf(m, top);           // finite from the first segment on: its first key counts for every column
-        const float correction = __expf(m - m_new);  // 0 in the first segment, 1 where the segment holds no key of the column
+        const float m_new = fmaxf(m, top);           // -inf as long as no segment held a key of the column (under a window)
+        const float correction = m_new == -INFINITY ? 1.0f : __expf(m - m_new);  // 0 at its first segment, 1 where a segment holds none
         float sum = 0.0f;
         bf16x8_t pf[2];
 #pragma unroll
@@ -159,7 +190,7 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
 #pragma unroll
         for (int c = 0; c < 2; ++c) {
             int key0 = seg0 + 32 * c + 8 * g;
-            key0 = key0 < last_group ? key0 : last_group;   // a group wholly beyond the last key weighs nothing; read one that exists
+            key0 = min(max(key0, first_group), last_group);   // a group wholly outside the range weighs nothing; read one that exists
             const bf16_t* vp = a.cache_t + ((size_t)table[key0 / pt] * C + col) * pt + key0 % pt;
 #pragma unroll
             for (int d0 = 0; d0 < CT; d0 += LM_VTILES) {
@@ -187,7 +218,7 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
         return;
     }
     if (!live) return;
-    bf16_t* out = a.out + ((size_t)c_head * a.T + c_row) * C;
+    bf16_t* out = a.out + latent_row(a, c_head, c_row) * C;
     const float inv = 1.0f / l;
 #pragma unroll
     for (int dt = 0; dt < CT; ++dt) {
@@ -204,7 +235,7 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
 // the slots in order, eight slots' loads in flight.
 #define LM_MERGE_MAX 1024    // slots of one column whose weights fit the workgroup's LDS; longer columns take rounds
 __global__ void __launch_bounds__(256) latent_attention_merge_kernel(const int* __restrict__ merges, const float* __restrict__ part_o,
-                                                                   const float* __restrict__ part_ml, bf16_t* __restrict__ out, int T, int C) {
+                                                                   const float* __restrict__ part_ml, bf16_t* __restrict__ out, int T, int C, int H, int row_major) {
     __shared__ float weight[LM_MERGE_MAX];
     __shared__ float scratch[4];
     const int* mg = merges + LM_ITEM_INTS * (size_t)blockIdx.x;
@@ -246,7 +277,7 @@ __global__ void __launch_bounds__(256) latent_attention_merge_kernel(const int* 
     const float inv = 1.0f / L;
 #pragma unroll
     for (int e = 0; e < 2; ++e)
-        if (threadIdx.x + 256 * e < C) out[((size_t)(head0 + c) * T + row) * C + threadIdx.x + 256 * e] = f32_to_bf16(acc[e] * inv);
+        if (threadIdx.x + 256 * e < C) out[(row_major ? (size_t)row * H + head0 + c : (size_t)(head0 + c) * T + row) * C + threadIdx.x + 256 * e] = f32_to_bf16(acc[e] * inv);
 }
 
 // ---------------------------------------------------------------------------
@@ -265,11 +296,11 @@ template <int DPW, int LW_TILES, int KS>    // dim tiles of 16 a wave owns; colu
 __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaArgs a) {
     constexpr int COLS = 16 * LW_TILES;
     constexpr bool EARLY_VALUES = LW_TILES == 1;
-    extern __shared__ __align__(16) bf16_t qs[];   // [64][C + R + 8], then the weights and the waves' maxima
+    extern __shared__ __align__(16) bf16_t qs[];   // [64][ldc + 8], then the weights and the waves' maxima
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int* item = a.items + LM_ITEM_INTS * (size_t)blockIdx.x;
     const int row0 = item[0], rows = item[1], head0 = item[2], heads = item[3], slot = item[6];
-    const int C = a.C, R = a.R, CR = C + R, ldq = CR + 8, pt = a.page_tokens;
+    const int C = a.C, R = a.R, CR = a.ldc, ldq = CR + 8, pt = a.page_tokens;
     const int per = heads >= 16 ? 1 : 16 / heads;      // rows a column tile holds
     float* ws = reinterpret_cast<float*>(qs + COLS * ldq);        // [2][COLS][LW_LDW]
     float* pmax = ws + 2 * COLS * LW_LDW;                           // [2][4][COLS]
@@ -286,8 +317,8 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
                 v[u] = uint4{0, 0, 0, 0};
                 if (i < chunks && c < per * heads && r < rows) {
                     const int h = head0 + c % heads;
-                    v[u] = d < C ? *reinterpret_cast<const uint4*>(a.q_lat + ((size_t)h * a.T + row0 + r) * C + d)
-                                 : *reinterpret_cast<const uint4*>(a.q_rot + ((size_t)h * a.T + row0 + r) * R + (d - C));
+                    if (d < C) v[u] = *reinterpret_cast<const uint4*>(a.q_lat + latent_row(a, h, row0 + r) * C + d);
+                    else if (d < C + R) v[u] = *reinterpret_cast<const uint4*>(a.q_rot + latent_row(a, h, row0 + r) * R + (d - C));
                 }
             }
 #pragma unroll
@@ -300,21 +331,23 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
     __syncthreads();
 
     bool live[LW_TILES];
-    int p_col[LW_TILES], c_row[LW_TILES];
+    int p_col[LW_TILES], lo_col[LW_TILES], c_row[LW_TILES];
 #pragma unroll
     for (int ct = 0; ct < LW_TILES; ++ct) {
         const int r = ct * per + col / heads;
         live[ct] = col < per * heads && r < rows;
         c_row[ct] = row0 + (live[ct] ? r : 0);
         p_col[ct] = a.pos[c_row[ct]];
+        lo_col[ct] = a.window > 0 ? p_col[ct] - a.window + 1 : 0;
     }
     const int c_head = head0 + col % heads;
     const int p_max = a.pos[row0 + rows - 1];
     const int* table = a.tables + (size_t)a.row_entry[row0] * a.max_blocks;
     const int steps = CR / 32;
     const int last_group = (p_max / 8) * 8;
-    const int key_begin = slot < 0 ? 0 : item[4];
-    const int key_last = slot < 0 ? p_max : min(item[5] - 1, p_max);
+    const LatentKeys range = latent_keys(a, item, a.pos[row0], p_max);
+    const int key_begin = range.begin, key_last = range.last;
+    const int first_group = (range.lo_min / 8) * 8;
 
     f32x4_t o[LW_TILES][DPW];
     float m[LW_TILES], l[LW_TILES];
@@ -332,7 +365,7 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
         float* mbuf = pmax + buf * 4 * COLS;
         // scores of this wave's 16 keys (key 16 wave + lane % 16 in the tile's row lane % 16) against the four tiles
         int key = seg0 + 16 * wave + col;
-        key = key < p_max ? key : p_max;
+        key = min(max(key, range.lo_min), p_max);
         const bf16_t* kp = a.cache + ((size_t)table[key / pt] * pt + key % pt) * CR + 8 * g;
         f32x4_t s[LW_TILES];
 #pragma unroll
@@ -342,7 +375,7 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
         bf16x8_t vf[2][DPW];
         auto value_loads = [&](int c) {
             int key0 = seg0 + 32 * c + 8 * g;
-            key0 = key0 < last_group ? key0 : last_group;
+            key0 = min(max(key0, first_group), last_group);
             const bf16_t* vp = a.cache_t + ((size_t)table[key0 / pt] * C + col) * pt + key0 % pt;
 #pragma unroll
             for (int dt = 0; dt < DPW; ++dt) {
@@ -375,7 +408,8 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
             float top = -INFINITY;
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
-                s[ct][i] = seg0 + 16 * wave + 4 * g + i <= p_col[ct] ? s[ct][i] * a.scale : -INFINITY;
+                const int k = seg0 + 16 * wave + 4 * g + i;
+                s[ct][i] = k <= p_col[ct] && k >= lo_col[ct] ? s[ct][i] * a.scale : -INFINITY;
                 top = fmaxf(top, s[ct][i]);
             }
             top = rows_max4(top);
@@ -388,7 +422,7 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
             const int cc = 16 * ct + col;
             const float top = fmaxf(fmaxf(mbuf[cc], mbuf[COLS + cc]), fmaxf(mbuf[2 * COLS + cc], mbuf[3 * COLS + cc]));
             const float m_new = fmaxf(m[ct], top);
-            correction[ct] = __expf(m[ct] - m_new);
+            correction[ct] = m_new == -INFINITY ? 1.0f : __expf(m[ct] - m_new);
             m[ct] = m_new;
             f32x4_t w;
 #pragma unroll
@@ -443,7 +477,7 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
 #pragma unroll
     for (int ct = 0; ct < LW_TILES; ++ct) {
         if (!live[ct]) continue;
-        bf16_t* out = a.out + ((size_t)c_head * a.T + c_row[ct]) * C;
+        bf16_t* out = a.out + latent_row(a, c_head, c_row[ct]) * C;
         const float inv = 1.0f / l[ct];
 #pragma unroll
         for (int dt = 0; dt < DPW; ++dt) {
@@ -457,19 +491,19 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
 }
 
 extern "C" int llmx_latent_attention_mfma_ok(int C, int R, int page_tokens) {
-    return C >= 16 && C <= 512 && C % 16 == 0 && R >= 0 && R % 8 == 0 && (C + R) % 32 == 0 && page_tokens > 0 && page_tokens % 8 == 0 ? 1 : 0;
+    return C >= 16 && C <= 512 && C % 16 == 0 && R >= 0 && R % 8 == 0 && R <= 448 && page_tokens > 0 && page_tokens % 8 == 0 ? 1 : 0;
 }
 
 extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, const void* cache, const void* cache_t, const int* pos,
                                           const int* row_entry, const int* tables, const int* items, int n_items, int n_tile_items, int n_row_items,
                                           const int* merges, int n_merges,
-                                          void* out, float* part_o, float* part_ml, float scale, int T, int H, int C, int R, int page_tokens,
-                                          int max_blocks, hipStream_t stream) {
+                                          void* out, float* part_o, float* part_ml, float scale, int T, int H, int C, int R, int ldc, int page_tokens,
+                                          int max_blocks, int window, int row_major, hipStream_t stream) {
     if (n_items <= 0 && n_tile_items <= 0 && n_row_items <= 0) return 0;
-    if (!llmx_latent_attention_mfma_ok(C, R, page_tokens)) return -2;
+    if (!llmx_latent_attention_mfma_ok(C, R, page_tokens) || ldc < C + R || ldc % 32 || window < 0) return -2;
     if (n_merges > 0 && (!merges || !part_o || !part_ml)) return -2;
     LatentMfmaArgs a{(const bf16_t*)q_lat, (const bf16_t*)q_rot, (const bf16_t*)cache, (const bf16_t*)cache_t, pos, row_entry, tables, items,
-                     (bf16_t*)out, part_o, part_ml, scale, T, H, C, R, page_tokens, max_blocks};
+                     (bf16_t*)out, part_o, part_ml, scale, T, H, C, R, ldc, page_tokens, max_blocks, window, row_major};
 #define LLMX_LT(DPW, TILES, KS, count, first)                                                                                        \
     {                                                                                                                                 \
         static bool raised = false;                                                                                                   \
@@ -478,7 +512,7 @@ extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, 
             raised = true;                                                                                                            \
         }                                                                                                                             \
         a.items = items + LM_ITEM_INTS * (size_t)(first);                                                                             \
-        const size_t lds = sizeof(bf16_t) * 16 * TILES * (size_t)(C + R + 8) + sizeof(float) * (2 * 16 * TILES * LW_LDW + 2 * 4 * 16 * TILES); \
+        const size_t lds = sizeof(bf16_t) * 16 * TILES * (size_t)(ldc + 8) + sizeof(float) * (2 * 16 * TILES * LW_LDW + 2 * 4 * 16 * TILES); \
         hipLaunchKernelGGL((latent_attention_tiles_kernel<DPW, TILES, KS>), dim3(count), dim3(256), lds, stream, a);                 \
     }
     if (n_tile_items > 0) {      // the list's first items: four column tiles each, a workgroup of four waves
@@ -499,7 +533,7 @@ extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, 
     if (n_items > 0) {
         llmx_note_launch(LK_LATENT_ATTENTION_MFMA);
         a.items = items + LM_ITEM_INTS * (size_t)(n_tile_items + n_row_items);
-        const size_t lds = sizeof(bf16_t) * 16 * (size_t)(C + R + 8);
+        const size_t lds = sizeof(bf16_t) * 16 * (size_t)(ldc + 8);
         const dim3 grid(n_items), block(64);
         if (C <= 64) hipLaunchKernelGGL(latent_attention_mfma_kernel<4>, grid, block, lds, stream, a);
         else if (C <= 128) hipLaunchKernelGGL(latent_attention_mfma_kernel<8>, grid, block, lds, stream, a);
@@ -508,7 +542,7 @@ extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, 
     }
     if (n_merges > 0) {
         llmx_note_launch(LK_LATENT_ATTENTION_MERGE);
-        hipLaunchKernelGGL(latent_attention_merge_kernel, dim3(n_merges, 16), dim3(256), 0, stream, merges, part_o, part_ml, (bf16_t*)out, T, C);
+        hipLaunchKernelGGL(latent_attention_merge_kernel, dim3(n_merges, 16), dim3(256), 0, stream, merges, part_o, part_ml, (bf16_t*)out, T, C, H, row_major);
     }
     return LLMX_CHECK_LAUNCH();
 }

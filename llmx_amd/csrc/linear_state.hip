@@ -10,6 +10,7 @@
 // Around it: the preparation of a delta-rule row (short causal convolutions with silu, unit-norm q and k, the decay and
 // beta), the decay of gated linear attention, and the gated RMS norm of the read-out.
 #include "common.h"
+#include "state_operands.h"
 
 __device__ __forceinline__ float sigmoid_ls(float v) { return 1.0f / (1.0f + expf(-v)); }
 
@@ -149,6 +150,8 @@ struct StateScanArgs {
     int H, share, D, V;
     const float* tail_src;
     int tail_ld, tail_C, taps, tail_off;
+    int max_rows_here;   // > 0: entries of more rows are left to another kernel
+    StateOperands operands;
 };
 
 // Rows are worked on in chunks of CH: the block brings a chunk's q, k and decay values (its head's D of each, padded to
@@ -161,7 +164,7 @@ __device__ __forceinline__ float column_sum(float v) { return wave_sum(v); }    
 #define SCAN_COLS 8     // value channels a block of four waves owns
 #define SCAN_LANES 64   // lanes that share a column: a wave
 #define SCAN_THREADS (SCAN_COLS * SCAN_LANES)
-template <int R, int CH>
+template <int R, int CH, int KIND>
 __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs a) {
     constexpr int DP = SCAN_LANES * R;              // a head's key channels, padded
     constexpr int PER_TOKEN = 3 * DP;               // k | q | decay
@@ -175,6 +178,7 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
     const int h = blockIdx.x / tiles, tile = blockIdx.x % tiles;
     const int e = blockIdx.y;
     const int row0 = a.entry_rows[2 * e], n = a.entry_rows[2 * e + 1];
+    if (a.max_rows_here > 0 && n > a.max_rows_here) return;
     const int j = tile * SCAN_COLS + c;
     const bool col = j < a.V;
     const int d0 = s * R;           // where the lane's operands lie in a staged row; its i-th key channel is 32 i + s
@@ -207,12 +211,12 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
             const size_t row = (size_t)(row0 + min(t0 + tt, n - 1));
             const int dd = d < a.D ? d : 0;
             const float* src = which == 0 ? kp + row * a.ldk : which == 1 ? qp + row * a.ldq : gp + row * a.ldg;
-            const float x = src[dd];
+            const float x = KIND == STATE_OPERANDS_PLAIN || which == 2 ? src[dd] : state_key<KIND>(a.operands, src, row, dd);
             stage[u] = d < a.D ? x : 0.0f;
         }
         if (tid < CH * SCAN_COLS) {
             const int tt = min(tid / SCAN_COLS, CH - 1), cc = tid % SCAN_COLS;
-            vstage = vp[(size_t)(row0 + min(t0 + tt, n - 1)) * a.ldv + min(cc, a.V - 1 - tile * SCAN_COLS)];
+            vstage = state_value<KIND>(vp[(size_t)(row0 + min(t0 + tt, n - 1)) * a.ldv + min(cc, a.V - 1 - tile * SCAN_COLS)]);
         }
         if (a.beta) bstage = a.beta[(size_t)(row0 + min(t0 + min(tid, CH - 1), n - 1)) * a.H + h];
     };
@@ -328,20 +332,28 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
 extern "C" int llmx_state_scan(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* decay, int ldg,
                                const float* beta, float* state, long state_stride, const int* slot_read, const int* slot_write,
                                const int* entry_rows, float* out, float out_scale, int n_entries, int H, int share, int D, int V,
-                               const float* tail_src, int tail_ld, int tail_C, int taps, int tail_off, int max_rows, hipStream_t stream) {
+                               const float* tail_src, int tail_ld, int tail_C, int taps, int tail_off, int max_rows, int max_rows_here, int operands,
+                               const float* cos_sin, const int* pos, int rot_dims, hipStream_t stream) {
     if (n_entries <= 0) return 0;
+    if (operands < 0 || operands > 2 || (operands == STATE_OPERANDS_ROTATED && (!cos_sin || !pos || rot_dims < 2 || rot_dims % 2 || rot_dims > D))) return -2;
     if (H < 1 || share < 1 || H % share || D < 1 || D > 256 || V < 1 || (taps > 1 && !tail_src)) return -2;
     StateScanArgs a{q, k, v, decay, beta, ldq, ldk, ldv, ldg, state, state_stride, slot_read, slot_write, entry_rows, out, out_scale,
-                    H, share, D, V, tail_src, tail_ld, tail_C, taps, tail_off};
+                    H, share, D, V, tail_src, tail_ld, tail_C, taps, tail_off, max_rows_here, StateOperands{cos_sin, pos, rot_dims}};
     const dim3 grid((unsigned)(H * ((V + SCAN_COLS - 1) / SCAN_COLS)), (unsigned)n_entries);
     llmx_note_launch(LK_STATE_SCAN);
     const int per_lane = (D + SCAN_LANES - 1) / SCAN_LANES;
     // steps of single decoded tokens stage chunks of two rows (a quarter of the LDS, so more blocks a compute unit); a
     // row's arithmetic does not depend on the chunk it came in
+#define LLMX_SCAN_KIND(R_, CH_, KIND_) \
+    do { \
+        if (max_rows > 0 && max_rows <= 2) hipLaunchKernelGGL((state_scan_kernel<R_, 2, KIND_>), grid, dim3(SCAN_THREADS), 0, stream, a); \
+        else hipLaunchKernelGGL((state_scan_kernel<R_, CH_, KIND_>), grid, dim3(SCAN_THREADS), 0, stream, a); \
+    } while (0)
 #define LLMX_SCAN(R_, CH_) \
     do { \
-        if (max_rows > 0 && max_rows <= 2) hipLaunchKernelGGL((state_scan_kernel<R_, 2>), grid, dim3(SCAN_THREADS), 0, stream, a); \
-        else hipLaunchKernelGGL((state_scan_kernel<R_, CH_>), grid, dim3(SCAN_THREADS), 0, stream, a); \
+        if (operands == STATE_OPERANDS_SILU) LLMX_SCAN_KIND(R_, CH_, STATE_OPERANDS_SILU); \
+        else if (operands == STATE_OPERANDS_ROTATED) LLMX_SCAN_KIND(R_, CH_, STATE_OPERANDS_ROTATED); \
+        else LLMX_SCAN_KIND(R_, CH_, STATE_OPERANDS_PLAIN); \
     } while (0)
     // chunks of 16 rows where LDS holds two of them (heads of at most 128 key channels): a chunk's work then outlasts the
     // next chunk's way from memory
@@ -349,6 +361,7 @@ extern "C" int llmx_state_scan(const float* q, int ldq, const float* k, int ldk,
     else if (per_lane <= 2) LLMX_SCAN(2, 16);
     else LLMX_SCAN(4, 8);
 #undef LLMX_SCAN
+#undef LLMX_SCAN_KIND
     return LLMX_CHECK_LAUNCH();
 }
 
@@ -376,8 +389,12 @@ struct HeadNormArgs {
     const float* den_floor;
 };
 
-template <typename TO>
-__global__ void __launch_bounds__(64) head_norm_gate_kernel(HeadNormArgs a, TO* __restrict__ out) {
+// WAVES 1: a wave a head, as above.  More: a workgroup of that many waves a head, for norms over long rows (all heads of a row
+// normed together); the waves' sums are added in wave order.
+template <typename TO, int WAVES>
+__global__ void __launch_bounds__(64 * WAVES) head_norm_gate_kernel(HeadNormArgs a, TO* __restrict__ out) {
+    __shared__ float scratch[WAVES];
+    constexpr int NT = 64 * WAVES;
     const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
     const int H = a.H, V = a.V;
     const float* row = a.o + ((size_t)t * H + h) * a.o_head;
@@ -390,15 +407,15 @@ __global__ void __launch_bounds__(64) head_norm_gate_kernel(HeadNormArgs a, TO* 
         return x;
     };
     float ss = 0.0f;
-    for (int j = lane; j < V; j += 64) {
+    for (int j = lane; j < V; j += NT) {
         const float x = value(j);
         ss = fmaf(x, x, ss);
     }
-    const float r = 1.0f / sqrtf(wave_sum(ss) / (float)V + a.eps);
+    const float r = 1.0f / sqrtf((WAVES == 1 ? wave_sum(ss) : block_sum<WAVES>(ss, scratch)) / (float)V + a.eps);
     const float* zr = a.z ? a.z + (size_t)t * a.ldz + (size_t)h * V : nullptr;
     const float* w = a.w ? (a.w_wide ? a.w + (size_t)h * V : a.w) : nullptr;
     TO* dst = out + ((size_t)t * H + h) * V;
-    for (int j = lane; j < V; j += 64) {
+    for (int j = lane; j < V; j += NT) {
         float y = value(j) * r;
         if (w) y = y * w[j];
         if (zr) {
@@ -418,8 +435,13 @@ extern "C" int llmx_head_norm_gate(const float* o, const float* w, const float* 
     if (o_head < V || sub < 0 || (sub > 0 && (den_floor || o_head < sub + V)) || (den_floor && o_head < V + 1)) return -2;
     HeadNormArgs a{o, o_head, w, w_wide, z, ldz, eps, H, V, gate, sub, lambda, post, den_floor};
     llmx_note_launch(LK_HEAD_NORM_GATE);
-    if (out_dtype == LLMX_F32) hipLaunchKernelGGL(head_norm_gate_kernel<float>, dim3(rows, H), dim3(64), 0, stream, a, (float*)out);
-    else hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, dim3(rows, H), dim3(64), 0, stream, a, (bf16_t*)out);
+    if (V > 512) {
+        if (out_dtype == LLMX_F32) hipLaunchKernelGGL((head_norm_gate_kernel<float, 8>), dim3(rows, H), dim3(512), 0, stream, a, (float*)out);
+        else hipLaunchKernelGGL((head_norm_gate_kernel<bf16_t, 8>), dim3(rows, H), dim3(512), 0, stream, a, (bf16_t*)out);
+        return LLMX_CHECK_LAUNCH();
+    }
+    if (out_dtype == LLMX_F32) hipLaunchKernelGGL((head_norm_gate_kernel<float, 1>), dim3(rows, H), dim3(64), 0, stream, a, (float*)out);
+    else hipLaunchKernelGGL((head_norm_gate_kernel<bf16_t, 1>), dim3(rows, H), dim3(64), 0, stream, a, (bf16_t*)out);
     return LLMX_CHECK_LAUNCH();
 }
 

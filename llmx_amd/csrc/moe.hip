@@ -48,20 +48,42 @@ __device__ __forceinline__ void load_row_256(float* __restrict__ row, const floa
     }
 }
 
-// Sigmoid scores and the k <= 64 picks of such a row: lane j < k ends with pick j's id and weight (-1 and 0 for a row with
+// The experts a row can pick from when they form equal groups of neighbours: those of the `keep` groups with the largest
+// best key.  The largest key outside the groups kept so far names the next group (the lowest number among equals).
+struct RouteGroups {
+    int per, keep;     // experts a group; groups kept (per 0: no groups)
+};
+
+// The scores and the k <= 64 picks of such a row: lane j < k ends with pick j's id and weight (-1 and 0 for a row with
 // a non-finite key).  A pick is the largest key not yet taken, the lowest id among equal keys: the wave's maximum of
 // the keys (exact, so its order does not matter), then the first slot and in it the first lane that holds it.  The
 // formulas and the order of the picks' sum are those of route_topk_kernel's general path.
 __device__ __forceinline__ void route_row_256(const float (&x)[4], const float (&bias_v)[4], bool has_bias, int n_experts, int k, int normalize,
-                                              float scale, int lane, int& pick_id, float& pick_weight) {
+                                              float scale, int score, RouteGroups groups, int lane, int& pick_id, float& pick_weight) {
     float s[4], b[4];
     int finite = 1;
+    if (score == SCORE_SOFTMAX) {
+        float top = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (lane + 64 * i < n_experts) top = fmaxf(top, x[i]);
+        top = wave_max(top);
+        float sum = 0.0f;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            s[i] = lane + 64 * i < n_experts ? expf(x[i] - top) : 0.0f;
+            sum += s[i];
+        }
+        sum = wave_sum(sum);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) s[i] = s[i] / sum;
+    }
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-        s[i] = 0.0f;
+        if (score == SCORE_SIGMOID) s[i] = 0.0f;
         b[i] = -INFINITY;   // no expert, or taken: below every finite key
         if (lane + 64 * i < n_experts) {
-            s[i] = 1.0f / (1.0f + expf(-x[i]));
+            if (score == SCORE_SIGMOID) s[i] = 1.0f / (1.0f + expf(-x[i]));
             b[i] = has_bias ? s[i] + bias_v[i] : s[i];
             if (!isfinite(b[i])) finite = 0;
         }
@@ -69,6 +91,32 @@ __device__ __forceinline__ void route_row_256(const float (&x)[4], const float (
     pick_id = -1;
     pick_weight = 0.0f;
     if (!__all(finite)) return;
+    if (groups.per > 0) {
+        bool kept[4] = {false, false, false, false};
+        for (int r = 0; r < groups.keep; ++r) {
+            float mx = -INFINITY;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) mx = fmaxf(mx, kept[i] ? -INFINITY : b[i]);
+            mx = wave_max(mx);
+            unsigned long long m = 0;
+            int slot = 0;
+#pragma unroll
+            for (int i = 3; i >= 0; --i) {
+                const unsigned long long mi = __ballot(!kept[i] && b[i] == mx);
+                if (mi) {
+                    m = mi;
+                    slot = i;
+                }
+            }
+            const int g = (__ffsll((long long)m) - 1 + 64 * slot) / groups.per;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if ((lane + 64 * i) / groups.per == g) kept[i] = true;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (!kept[i]) b[i] = -INFINITY;
+    }
     float mine = 0.0f;
     for (int j = 0; j < k; ++j) {
         const float best = wave_max(fmaxf(fmaxf(b[0], b[1]), fmaxf(b[2], b[3])));
@@ -91,7 +139,8 @@ __device__ __forceinline__ void route_row_256(const float (&x)[4], const float (
     }
     float total = 0.0f;
     for (int j = 0; j < k; ++j) total += __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(mine), j));
-    pick_weight = (normalize ? mine / total : mine) * scale;
+    const bool divide = normalize == 2 || (normalize && (score == SCORE_SIGMOID || k > 1));   // 2: also a single softmax pick (its weight is 1)
+    pick_weight = (divide ? mine / total : mine) * scale;
 }
 
 // One wave per row.  score s_e = sigmoid(z_e) (or softmax over the row); the pick key is b_e = s_e + bias_e; k times
@@ -99,6 +148,7 @@ __device__ __forceinline__ void route_row_256(const float (&x)[4], const float (
 // picks' sum (added in pick order) when `normalize` (1: a single softmax pick keeps its score; 2: it too is divided, so its
 // weight is 1: the softmax over the picked logits alone), then times `scale`.  A row with a non-finite key gets ids -1 and
 // weights 0.  Ids and weights come out in pick order, best first.
+// `groups`: the picks come from some of the experts only (see RouteGroups).
 // `logit_bias` (optional): added to the logits (and kept in z) before anything else: a router whose bias is part of its
 // logits, so that scores and weights see it too.
 // `parts` (optional): the logits arrive as `slices` partial sums [slices][rows][experts]; the row adds them in slice order
@@ -106,17 +156,17 @@ __device__ __forceinline__ void route_row_256(const float (&x)[4], const float (
 __global__ void __launch_bounds__(64) route_topk_kernel(float* __restrict__ z, const float* __restrict__ parts, int slices, long slice_stride,
                                                        const float* __restrict__ bias, int* __restrict__ ids,
                                                        float* __restrict__ weights, int n_experts, int k, int score, int normalize,
-                                                       float scale, const float* __restrict__ logit_bias) {
+                                                       float scale, const float* __restrict__ logit_bias, RouteGroups groups) {
     __shared__ float s[ROUTE_MAX_EXPERTS];
     __shared__ float b[ROUTE_MAX_EXPERTS];
     __shared__ float chosen[ROUTE_MAX_K];
     const int r = blockIdx.x, lane = threadIdx.x;
     float* row = z + (size_t)r * n_experts;
-    if (score == SCORE_SIGMOID && n_experts <= 256 && k <= 64 && !logit_bias) {   // the row fits the wave's registers
+    if (n_experts <= 256 && k <= 64 && !logit_bias) {   // the row fits the wave's registers
         float x[4], bias_v[4], weight;
         int id;
         load_row_256(row, parts ? parts + (size_t)r * n_experts : nullptr, slices, slice_stride, bias, n_experts, lane, x, bias_v);
-        route_row_256(x, bias_v, bias != nullptr, n_experts, k, normalize, scale, lane, id, weight);
+        route_row_256(x, bias_v, bias != nullptr, n_experts, k, normalize, scale, score, groups, lane, id, weight);
         if (lane < k) {
             ids[(size_t)r * k + lane] = id;
             weights[(size_t)r * k + lane] = weight;
@@ -165,6 +215,29 @@ __global__ void __launch_bounds__(64) route_topk_kernel(float* __restrict__ z, c
         }
         return;
     }
+    if (groups.per > 0) {
+        __shared__ unsigned char kept[ROUTE_MAX_EXPERTS];
+        for (int e = lane; e < n_experts; e += 64) kept[e] = 0;
+        __syncthreads();
+        for (int g = 0; g < groups.keep; ++g) {
+            float best = -INFINITY;
+            int at = 0x7fffffff;
+            for (int e = lane; e < n_experts; e += 64) {
+                if (!kept[e] && b[e] > best) {
+                    best = b[e];
+                    at = e;
+                }
+            }
+            wave_best(best, at);
+            __syncthreads();
+            for (int e = lane; e < n_experts; e += 64)
+                if (e / groups.per == at / groups.per) kept[e] = 1;
+            __syncthreads();
+        }
+        for (int e = lane; e < n_experts; e += 64)
+            if (!kept[e]) b[e] = -INFINITY;
+        __syncthreads();
+    }
     for (int j = 0; j < k; ++j) {
         // lane's best: first larger key in its ids in increasing order, so a lane's tie keeps its lowest id
         float best = -INFINITY;
@@ -192,14 +265,25 @@ __global__ void __launch_bounds__(64) route_topk_kernel(float* __restrict__ z, c
     }
 }
 
+// False when the groups do not divide the experts or the kept ones do not offer k picks.
+static bool route_groups(int count, int keep, int n_experts, int k, RouteGroups& out) {
+    out = RouteGroups{0, 0};
+    if (count <= 0) return true;
+    if (n_experts % count || keep < 1 || keep > count || k > keep * (n_experts / count)) return false;
+    if (keep < count) out = RouteGroups{n_experts / count, keep};
+    return true;
+}
+
 extern "C" int llmx_route_topk(float* z, const float* parts, int slices, long slice_stride, const float* bias, int* ids, float* weights,
                                int rows, int n_experts, int k, int score, int normalize, float scale, const float* logit_bias,
-                               hipStream_t stream) {
+                               int group_count, int group_keep, hipStream_t stream) {
     if (rows <= 0) return 0;
+    RouteGroups groups;
+    if (!route_groups(group_count, group_keep, n_experts, k, groups)) return -2;
     if (n_experts > ROUTE_MAX_EXPERTS || k > ROUTE_MAX_K || k > n_experts || k <= 0 || (parts && (slices < 1 || slices > ROUTE_MAX_SLICES))) return -2;
     llmx_note_launch(LK_ROUTE_TOPK);
     hipLaunchKernelGGL(route_topk_kernel, dim3(rows), dim3(64), 0, stream, z, parts, slices, slice_stride, bias, ids, weights, n_experts, k, score,
-                       normalize, scale, logit_bias);
+                       normalize, scale, logit_bias, groups);
     return LLMX_CHECK_LAUNCH();
 }
 
@@ -448,9 +532,9 @@ extern "C" int llmx_moe_align(const int* ids, int n_pairs, int n_experts, int* c
 __global__ void __launch_bounds__(1024) route_topk_align_kernel(float* __restrict__ z, const float* __restrict__ parts, int slices,
                                                                long slice_stride, const float* __restrict__ bias,
                                                                int* __restrict__ ids, float* __restrict__ weights, int rows, int n_experts,
-                                                               int k, int normalize, float scale, int* __restrict__ counts,
-                                                               int* __restrict__ offsets, int* __restrict__ list, int* __restrict__ active,
-                                                               int* __restrict__ n_active) {
+                                                               int k, int score, int normalize, float scale, RouteGroups groups,
+                                                               int* __restrict__ counts, int* __restrict__ offsets, int* __restrict__ list,
+                                                               int* __restrict__ active, int* __restrict__ n_active) {
     __shared__ int pair_expert[ALIGN_SMALL_PAIRS];
     __shared__ int cnt[1024];
     __shared__ int offs[1024];
@@ -460,7 +544,7 @@ __global__ void __launch_bounds__(1024) route_topk_align_kernel(float* __restric
         int id;
         load_row_256(z + (size_t)r * n_experts, parts ? parts + (size_t)r * n_experts : nullptr, slices, slice_stride, bias, n_experts, lane, x,
                      bias_v);
-        route_row_256(x, bias_v, bias != nullptr, n_experts, k, normalize, scale, lane, id, weight);
+        route_row_256(x, bias_v, bias != nullptr, n_experts, k, normalize, scale, score, groups, lane, id, weight);
         if (lane < k) {
             ids[(size_t)r * k + lane] = id;
             weights[(size_t)r * k + lane] = weight;
@@ -471,16 +555,17 @@ __global__ void __launch_bounds__(1024) route_topk_align_kernel(float* __restric
     align_in_block(pair_expert, rows * k, n_experts, cnt, offs, counts, offsets, list, active, n_active);
 }
 
-// Sigmoid scores only; at most 16 rows (a wave each), rows * k <= 1024, at most 256 experts and 64 picks.  Returns -2 otherwise.
+// At most 16 rows (a wave each), rows * k <= 1024, at most 256 experts and 64 picks.  Returns -2 otherwise.
 extern "C" int llmx_route_topk_align(float* z, const float* parts, int slices, long slice_stride, const float* bias, int* ids, float* weights,
-                                     int rows, int n_experts, int k, int normalize, float scale, int* counts, int* offsets, int* list,
-                                     int* active, int* n_active, hipStream_t stream) {
+                                     int rows, int n_experts, int k, int score, int normalize, float scale, int group_count, int group_keep,
+                                     int* counts, int* offsets, int* list, int* active, int* n_active, hipStream_t stream) {
     if (rows <= 0) return 0;
+    RouteGroups groups;
+    if (!route_groups(group_count, group_keep, n_experts, k, groups)) return -2;
     if (rows > 16 || rows * k > ALIGN_SMALL_PAIRS || n_experts > 256 || k > 64 || k > n_experts || k <= 0) return -2;
     if (parts && (slices < 1 || slices > ROUTE_MAX_SLICES)) return -2;
     llmx_note_launch(LK_ROUTE_TOPK_ALIGN);
     hipLaunchKernelGGL(route_topk_align_kernel, dim3(1), dim3(1024), 0, stream, z, parts, slices, slice_stride, bias, ids, weights, rows, n_experts, k,
-                       normalize, scale,
-                       counts, offsets, list, active, n_active);
+                       score, normalize, scale, groups, counts, offsets, list, active, n_active);
     return LLMX_CHECK_LAUNCH();
 }

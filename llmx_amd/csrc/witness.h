@@ -82,7 +82,11 @@
     X(MEMORY_PREP, "memory_prep")                                                                                         \
     X(ATTENTION_RULES, "attention.rules")                                                                                 \
     X(ATTENTION_RULES_MERGE, "attention.rules_merge")                                                                     \
-    X(ATTENTION_RULES_SHARED, "attention.rules_shared")
+    X(ATTENTION_RULES_SHARED, "attention.rules_shared")                                                                   \
+    X(EMBED_BIGRAM, "embed_bigram")                                                                                       \
+    X(TOKEN_SHIFT, "token_shift")                                                                                         \
+    X(RMSNORM_SHIFT, "rmsnorm_shift")                                                                                     \
+    X(DECAYED_STATE_CHUNKS, "decayed_state.chunks")
 
 enum LlmxLaunchKind : int {
 #define LLMX_X(id, name) LK_##id,

@@ -151,6 +151,11 @@ class Engine:
         n_pages = self.kv_tokens // self.page_tokens
         # the needs' leaves in run-order numbering: (cache number, path of member indices, need)
         leaves = []
+        needs = list(needs)
+        embedding_number = None
+        if self.model.embedding.cache_need() is not None:       # an embedding that keeps something: numbered after the run order's
+            embedding_number = len(needs)
+            needs.append(self.model.embedding.cache_need())
 
         def walk(number, path, need):
             if isinstance(need, CompositeNeed):
@@ -187,6 +192,8 @@ class Engine:
                                 for t in need.tensors})
         # which states a step must copy into its slot beforehand: those of mixers that step in place
         writers = {e.cache: self.model.blocks[e.layer].mixer for e in self.spec.run_order if e.writes}
+        if embedding_number is not None:
+            writers[embedding_number] = self.model.embedding
 
         def member_of(mixer, path):
             for i in path:
@@ -214,6 +221,7 @@ class Engine:
             return LayerCache(writes=writes)
 
         self._layer_caches: List[LayerCache] = [cache_of(e.cache, (), needs[e.cache], e.writes) for e in self.spec.run_order]
+        self._embedding_cache = None if embedding_number is None else cache_of(embedding_number, (), needs[embedding_number], True)
 
     # -- requests ---------------------------------------------------------------
     def add_request(self, request: Hashable) -> int:
@@ -407,14 +415,20 @@ class Engine:
             self._graph_seen[key] = self._graph_seen.get(key, 0) + 1
         return logits
 
+    def _embed(self, step: StepState, out: torch.Tensor) -> None:
+        if self._embedding_cache is None:
+            self.model.embedding.forward(step, out)
+        else:
+            self.model.embedding.forward(step, out, self._embedding_cache)
+
     def _forward(self, step: StepState) -> torch.Tensor:
         T, E = step.rows, self.spec.hidden_size
         x = step.buf("residual", (T, E), torch.float32)
-        self.model.embedding.forward(step, x)
+        self._embed(step, x)
         kept = None
         if any(p.wants_embedding for p in self.model.inputs):     # a residual input adds the embedding's rows again later
             kept = step.buf("embedding.rows", (T, E), torch.float32)
-            self.model.embedding.forward(step, kept)
+            self._embed(step, kept)
         for i, (entry, cache) in enumerate(zip(self.spec.run_order, self._layer_caches)):
             step.run_index = i
             if entry.before is not None:

@@ -7,6 +7,7 @@ from . import nenotar  # noqa: F401  (registers Nenotar)
 from . import bonerax  # noqa: F401  (registers Bonerax)
 from . import givozen  # noqa: F401  (registers Givozen)
 from . import salipel  # noqa: F401  (registers Salipel)
+from . import neruzen  # noqa: F401  (registers Neruzen)
 
 __all__ = ["ArchitectureEntry", "architecture_of", "architectures", "assemble", "read_config", "read_model_dir",
            "register_architecture", "unregister_architecture"]

@@ -61,11 +61,15 @@ def _declare(h) -> None:
         "llmx_act_gelu_gather": [P, P, I, P, P, I, I, I, I, I, P],
         "llmx_mingru_scan": [P, P, P, P, P, P, P, P, I, I, I, P],
         "llmx_mingru_scan_chunks": [P, P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, P],
-        "llmx_latent_prep": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, P],
-        "llmx_latent_attention_mfma": [P, P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, P],
+        "llmx_latent_prep": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, I, I, I, P],
+        "llmx_latent_down": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, I, P],
+        "llmx_latent_queries": [P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
+        "llmx_latent_attention_mfma": [P, P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, I, I, P],
         "llmx_latent_attention_mfma_ok": [I, I, I],
-        "llmx_latent_attention_generic": [P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, P],
+        "llmx_latent_attention_generic": [P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, P],
         "llmx_head_gate": [P, P, I, P, I, I, I, I, P],
+        "llmx_embed_bigram": [P, P, I, P, P, P, P, P, P, P, I, I, F, I, L, L, P],
+        "llmx_token_shift": [P, P, F, P, P, L, P, P, P, P, P, P, P, I, I, I, P],
         "llmx_rmsnorm": [P, P, P, F, P, I, P, I, I, P],
         "llmx_moe_combine": [P, P, P, P, I, I, I, I, P],
         "llmx_fill_i32": [P, I, L, P],
@@ -89,7 +93,9 @@ def _declare(h) -> None:
         "llmx_delta_prep": [P, I, P, P, I, P, P, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
         "llmx_cast_cols": [P, I, P, I, I, I, P],
         "llmx_sigmoid_root": [P, P, F, P, I, I, P],
-        "llmx_state_scan": [P, I, P, I, P, I, P, I, P, P, L, P, P, P, P, F, I, I, I, I, I, P, I, I, I, I, I, P],
+        "llmx_state_scan": [P, I, P, I, P, I, P, I, P, P, L, P, P, P, P, F, I, I, I, I, I, P, I, I, I, I, I, I, I, P, P, I, P],
+        "llmx_decayed_state_chunks": [P, I, P, I, P, I, P, P, L, P, P, P, I, P, I, P, P, F, I, I, I, I, P, P, I, P],
+        "llmx_decayed_state_rows": [],
         "llmx_head_norm_gate": [P, P, P, I, P, I, F, I, I, I, I, I, I, I, F, F, P, P],
         "llmx_attention_rules": [P, P, P, P, P, P, P, I, P, I, P, I, P, I, P, P, F, F, I, I, I, I, I, I, I, I, I, I, P, P, P, I, I, I, P],
         "llmx_attention_rules_shared_ok": [I, I],
@@ -97,9 +103,9 @@ def _declare(h) -> None:
         "llmx_attention_rules_segment": [],
         "llmx_memory_prep": [P, I, I, I, I, I, P, P, F, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
         "llmx_paged_attention_mfma": [P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, P, I, P],
-        "llmx_route_topk": [P, P, I, L, P, P, P, I, I, I, I, I, F, P, P],
+        "llmx_route_topk": [P, P, I, L, P, P, P, I, I, I, I, I, F, P, I, I, P],
         "llmx_moe_align": [P, I, I, P, P, P, P, P, P, P, P],
-        "llmx_route_topk_align": [P, P, I, L, P, P, P, I, I, I, I, F, P, P, P, P, P, P],
+        "llmx_route_topk_align": [P, P, I, L, P, P, P, I, I, I, I, I, F, I, I, P, P, P, P, P, P],
         "llmx_gemm_skinny": [P, P, P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, I, L, I, P, P, F, I, I, P, I, F, P, P, I, P],
         "llmx_gemm_skinny_normed_ok": [I, I],
         "llmx_gemm_skinny_f32_normed_ok": [I, I],
@@ -197,6 +203,46 @@ def embed_gather(table: torch.Tensor, ids: torch.Tensor, out: torch.Tensor, scal
     _check(lib().llmx_embed_gather(_dev(table, "table", shape=(table.shape[0], width)), _code(table.dtype),
                                    _dev(ids, "ids", torch.int32, (rows,)), _dev(out, "out", torch.float32),
                                    rows, width, float(scale), _stream()), "embed_gather")
+
+
+def embed_bigram(table: torch.Tensor, bigram: torch.Tensor, ids: torch.Tensor, state: torch.Tensor, slot_read: torch.Tensor,
+                 slot_write: torch.Tensor, row_entry: torch.Tensor, entry_rows: torch.Tensor, out: torch.Tensor, buckets: int, mul_prev: int,
+                 mul_cur: int, scale: float = 1.0) -> None:
+    """out[t] = table[ids[t]] * scale + bigram[row], row = (previous id * mul_prev + ids[t] * mul_cur) mod buckets, row `buckets`
+    for a request's first token.  The previous id of an entry's first row comes from state [slots, 1] int32 at slot_read[e]
+    (the id + 1; 0: none); an entry's last id is left at slot_write[e], another slot for entries of several rows."""
+    rows, width = out.shape
+    n_e = entry_rows.shape[0]
+    if bigram.dtype != table.dtype or buckets < 1 or tuple(bigram.shape) != (buckets + 1, width) or buckets > (1 << 31) - 1:
+        raise KernelError(f"embed_bigram: a table {tuple(bigram.shape)} for {buckets} buckets of width {width}")
+    # ids and reduced multipliers are below 2^31 each: their products' sum fits 64 bits
+    _check(lib().llmx_embed_bigram(_dev(table, "table", shape=(table.shape[0], width)), _dev(bigram, "bigram"), _code(table.dtype),
+                                   _dev(ids, "ids", torch.int32, (rows,)), _dev(state, "state", torch.int32, (state.shape[0], 1)),
+                                   _dev(slot_read, "slot_read", torch.int32, (n_e,)), _dev(slot_write, "slot_write", torch.int32, (n_e,)),
+                                   _dev(row_entry, "row_entry", torch.int32, (rows,)), _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)),
+                                   _dev(out, "out", torch.float32), rows, width, float(scale), int(buckets), int(mul_prev) % int(buckets),
+                                   int(mul_cur) % int(buckets), _stream()), "embed_bigram")
+
+
+def token_shift(x: torch.Tensor, shift: torch.Tensor, state: torch.Tensor, slot_read: torch.Tensor, slot_write: torch.Tensor,
+                row_entry: torch.Tensor, entry_rows: torch.Tensor, shifted: torch.Tensor, norm=None, out: Optional[torch.Tensor] = None,
+                out32: Optional[torch.Tensor] = None) -> None:
+    """shifted[t] = h[t] + (h[t-1] - h[t]) * shift over float32 rows h = x, or with `norm` = (weight, eps) h = RMSNorm(x), which
+    `out` (in shifted's type) and `out32` then receive.  h[-1] of an entry is the state's row at slot_read[e] (state [slots, >= n]
+    float32); its last h is left at slot_write[e], another slot for entries of several rows."""
+    rows, n = x.shape
+    n_e = entry_rows.shape[0]
+    if state.dim() != 2 or state.shape[1] < n or (norm is None and (out is not None or out32 is not None)):
+        raise KernelError("token_shift: the state does not hold a row, or the rows themselves are asked for without a norm")
+    if out is not None and out.dtype != shifted.dtype:
+        raise KernelError("token_shift: both results have one type")
+    weight, eps = norm if norm is not None else (None, 0.0)
+    _check(lib().llmx_token_shift(_dev(x, "x", torch.float32), _dev(weight, "norm weight", torch.float32, (n,)), float(eps),
+                                  _dev(shift, "shift", torch.float32, (n,)), _dev(state, "state", torch.float32), state.shape[1],
+                                  _dev(slot_read, "slot_read", torch.int32, (n_e,)), _dev(slot_write, "slot_write", torch.int32, (n_e,)),
+                                  _dev(row_entry, "row_entry", torch.int32, (rows,)), _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)),
+                                  _dev(shifted, "shifted", shape=(rows, n)), _dev(out, "out", shape=(rows, n)),
+                                  _dev(out32, "out32", torch.float32, (rows, n)), _code(shifted.dtype), rows, n, _stream()), "token_shift")
 
 
 def rmsnorm_pair(x: torch.Tensor, w1: torch.Tensor, w2: Optional[torch.Tensor], eps: float, out1: torch.Tensor,
@@ -382,43 +428,95 @@ def mingru_scan(zxg: torch.Tensor, bz: Optional[torch.Tensor], bx: Optional[torc
                                   _dev(out, "out"), _code(out.dtype), n_e, W, _stream()), "mingru_scan")
 
 
+def _latent_layout(q: torch.Tensor, heads: int, rows: int, row_major: bool):
+    """The leading axes of a tensor that holds a row of values for every (head, row)."""
+    return (rows, heads) if row_major else (heads, rows)
+
+
+def _latent_cache(cache: torch.Tensor, cache_t: Optional[torch.Tensor], rank: int, rot_dim: int, what: str):
+    n_pages, page_tokens, width = cache.shape
+    if cache_t is not None and (tuple(cache_t.shape) != (n_pages, rank, page_tokens) or cache_t.dtype != cache.dtype):
+        raise KernelError(f"{what}: the transposed copy does not fit the cache")
+    if width < rank + rot_dim:
+        raise KernelError(f"{what}: the cache does not fit the latent and the key part")
+    return page_tokens, width
+
+
 def latent_prep(proj: torch.Tensor, norm_w: torch.Tensor, cos_sin: torch.Tensor, pos: torch.Tensor, row_entry: torch.Tensor,
                 tables: torch.Tensor, q_plain: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor, eps: float, heads: int, dim: int,
-                rot_dim: int, rank: int, write_cache: bool = True, cache_t: Optional[torch.Tensor] = None) -> None:
+                rot_dim: int, rank: int, write_cache: bool = True, cache_t: Optional[torch.Tensor] = None,
+                pairing: int = ROPE_INTERLEAVED, row_major: bool = False) -> None:
     """From the float32 rows proj = [q of `heads` x (dim | rot_dim) | latent of `rank` | key part of rot_dim | ...]: the
-    queries head by head (q_plain [H, T, dim], q_rot [H, T, rot_dim] rotated), and into the row's cache place the
-    RMS-normed latent and the rotated key part.  cos_sin [positions, dims]: the first `dims` of a rotated part turn as
-    interleaved pairs.  `cache_t` [pages, rank, page_tokens]: a second copy of the latent, transposed within the page."""
+    queries head by head (q_plain [H, T, dim], q_rot [H, T, rot_dim] rotated; with `row_major` [T, H, ...]), and into the row's
+    cache place the RMS-normed latent and the rotated key part.  cos_sin [positions, dims]: the first `dims` of a rotated part
+    turn as pairs of the given `pairing`.  `cache_t` [pages, rank, page_tokens]: a second copy of the latent, transposed
+    within the page.  The cache's rows may be wider than rank + rot_dim; what lies behind is not written."""
     T, ldp = proj.shape
-    n_pages, page_tokens, width = cache.shape
     dims = cos_sin.shape[1]
-    if cache_t is not None and (tuple(cache_t.shape) != (n_pages, rank, page_tokens) or cache_t.dtype != cache.dtype):
-        raise KernelError("latent_prep: the transposed copy does not fit the cache")
-    if width != rank + rot_dim or q_plain.dtype != cache.dtype or q_rot.dtype != cache.dtype:
-        raise KernelError("latent_prep: the cache does not fit the latent and the key part")
+    page_tokens, width = _latent_cache(cache, cache_t, rank, rot_dim, "latent_prep")
+    if q_plain.dtype != cache.dtype or q_rot.dtype != cache.dtype:
+        raise KernelError("latent_prep: the queries do not have the cache's type")
+    lead = _latent_layout(q_plain, heads, T, row_major)
     _check(lib().llmx_latent_prep(_dev(proj, "proj", torch.float32), _dev(norm_w, "norm_w", torch.float32, (rank,)),
                                   _dev(cos_sin, "cos_sin", torch.float32), _dev(pos, "pos", torch.int32, (T,)),
                                   _dev(row_entry, "row_entry", torch.int32, (T,)), _dev(tables, "tables", torch.int32),
-                                  _dev(q_plain, "q_plain", shape=(heads, T, dim)), _dev(q_rot, "q_rot", shape=(heads, T, rot_dim)),
-                                  _dev(cache, "cache"), _dev(cache_t, "cache_t"), _code(cache.dtype), float(eps), T, ldp, heads, dim, rot_dim, rank, dims, page_tokens,
-                                  tables.shape[1], 1 if write_cache else 0, _stream()), "latent_prep")
+                                  _dev(q_plain, "q_plain", shape=(*lead, dim)), _dev(q_rot, "q_rot", shape=(*lead, rot_dim)),
+                                  _dev(cache, "cache"), _dev(cache_t, "cache_t"), _code(cache.dtype), float(eps), T, ldp, heads, dim, rot_dim, rank,
+                                  width, dims, page_tokens, tables.shape[1], 1 if write_cache else 0, 1 if pairing == ROPE_HALVES else 0,
+                                  1 if row_major else 0, _stream()), "latent_prep")
+
+
+def latent_down(proj: torch.Tensor, q_norm_w: torch.Tensor, q_normed: torch.Tensor, norm_w: torch.Tensor, cos_sin: torch.Tensor,
+                pos: torch.Tensor, row_entry: torch.Tensor, tables: torch.Tensor, cache: torch.Tensor, eps: float, q_rank: int, rot_dim: int,
+                rank: int, write_cache: bool = True, cache_t: Optional[torch.Tensor] = None, pairing: int = ROPE_INTERLEAVED) -> None:
+    """For queries that come through a latent of their own: from the float32 rows proj = [query latent of q_rank | latent of
+    `rank` | key part of rot_dim | ...] the RMS-normed query latent (q_normed [T, q_rank], what the second query product reads)
+    and, into the row's cache place, what latent_prep writes there."""
+    T, ldp = proj.shape
+    page_tokens, width = _latent_cache(cache, cache_t, rank, rot_dim, "latent_down")
+    if q_normed.dtype != cache.dtype:
+        raise KernelError("latent_down: the query latent does not have the cache's type")
+    _check(lib().llmx_latent_down(_dev(proj, "proj", torch.float32), _dev(q_norm_w, "q_norm_w", torch.float32, (q_rank,)),
+                                  _dev(q_normed, "q_normed", shape=(T, q_rank)), _dev(norm_w, "norm_w", torch.float32, (rank,)),
+                                  _dev(cos_sin, "cos_sin", torch.float32), _dev(pos, "pos", torch.int32, (T,)),
+                                  _dev(row_entry, "row_entry", torch.int32, (T,)), _dev(tables, "tables", torch.int32), _dev(cache, "cache"),
+                                  _dev(cache_t, "cache_t"), _code(cache.dtype), float(eps), T, ldp, q_rank, rot_dim, rank, width, cos_sin.shape[1],
+                                  page_tokens, tables.shape[1], 1 if write_cache else 0, 1 if pairing == ROPE_HALVES else 0, _stream()), "latent_down")
+
+
+def latent_queries(q: torch.Tensor, cos_sin: torch.Tensor, pos: torch.Tensor, q_plain: torch.Tensor, q_rot: torch.Tensor, heads: int, dim: int,
+                   rot_dim: int, pairing: int = ROPE_INTERLEAVED, row_major: bool = False) -> None:
+    """The float32 rows q [T, >= heads (dim + rot_dim)], head by head [dim | rot_dim], as latent_prep lays queries out."""
+    T, ldq = q.shape
+    lead = _latent_layout(q_plain, heads, T, row_major)
+    if q_plain.dtype != q_rot.dtype:
+        raise KernelError("latent_queries: both parts have one type")
+    _check(lib().llmx_latent_queries(_dev(q, "q", torch.float32), _dev(cos_sin, "cos_sin", torch.float32), _dev(pos, "pos", torch.int32, (T,)),
+                                     _dev(q_plain, "q_plain", shape=(*lead, dim)), _dev(q_rot, "q_rot", shape=(*lead, rot_dim)), _code(q_plain.dtype),
+                                     T, ldq, heads, dim, rot_dim, cos_sin.shape[1], 1 if pairing == ROPE_HALVES else 0, 1 if row_major else 0,
+                                     _stream()), "latent_queries")
 
 
 def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor, pos: torch.Tensor, row_entry: torch.Tensor,
                      tables: torch.Tensor, out: torch.Tensor, scale: float, window: int = 0, scratch=None,
-                     cache_t: Optional[torch.Tensor] = None, plan: Optional["LatentPlan"] = None) -> None:
-    """Causal softmax attention of every (head, row) over its request's paged latents: score = (q_lat . c + q_rot . k_rot)
-    * scale, result = sum of weights * c.  q_lat and out [H, T, C], q_rot [H, T, R], cache [pages, page_tokens, C + R].
-    `scratch(name, shape, dtype)`: storage that lives as long as the caller's step.  With `cache_t` (the latents once
-    more, [pages, C, page_tokens]) and a `plan` (latent_plan) the matrix-core kernel runs, where latent_attention_mfma_ok
-    says it can; otherwise the universal kernel."""
-    H, T, C = q_lat.shape
+                     cache_t: Optional[torch.Tensor] = None, plan: Optional["LatentPlan"] = None, row_major: bool = False) -> None:
+    """Causal softmax attention of every (head, row) over its request's paged latents, the last `window` keys (0: all): score =
+    (q_lat . c + q_rot . k_rot) * scale, result = sum of weights * c.  q_lat and out [H, T, C], q_rot [H, T, R] (with
+    `row_major` [T, H, ...]), cache [pages, page_tokens, at least C + R].  `scratch(name, shape, dtype)`: storage that lives as
+    long as the caller's step.  With `cache_t` (the latents once more, [pages, C, page_tokens]) and a `plan` (latent_plan, made
+    for the same window) the matrix-core kernel runs, where latent_attention_mfma_ok says it can and the cache's rows are
+    latent_cache_width wide with zeros behind the key part; otherwise the universal kernel."""
+    if row_major:
+        T, H, C = q_lat.shape
+    else:
+        H, T, C = q_lat.shape
     R = q_rot.shape[2]
     n_pages, page_tokens, width = cache.shape
-    if width != C + R or tuple(q_rot.shape[:2]) != (H, T) or out.shape != q_lat.shape or len({q_lat.dtype, q_rot.dtype, cache.dtype, out.dtype}) != 1:
+    if width < C + R or q_rot.shape[:2] != q_lat.shape[:2] or out.shape != q_lat.shape or len({q_lat.dtype, q_rot.dtype, cache.dtype, out.dtype}) != 1:
         raise KernelError("latent_attention: shapes or dtypes do not agree")
-    if cache_t is not None and plan is not None and window == 0 and latent_attention_mfma_ok(q_lat.dtype, C, R, page_tokens):
-        if plan.heads != H or plan.rows != T or tuple(cache_t.shape) != (n_pages, C, page_tokens) or cache_t.dtype != cache.dtype:
+    if cache_t is not None and plan is not None and width % 32 == 0 and latent_attention_mfma_ok(q_lat.dtype, C, R, page_tokens):
+        if plan.heads != H or plan.rows != T or plan.window != int(window) or tuple(cache_t.shape) != (n_pages, C, page_tokens) \
+                or cache_t.dtype != cache.dtype:
             raise KernelError("latent_attention: the plan or the transposed copy does not fit the step")
         part_o = part_ml = None
         if plan.n_slots:
@@ -430,14 +528,19 @@ def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tens
                                                 _dev(pos, "pos", torch.int32, (T,)), _dev(row_entry, "row_entry", torch.int32, (T,)),
                                                 _dev(tables, "tables", torch.int32), _dev(plan.items, "items", torch.int32), plan.n_items,
                                                 plan.n_tile_items, plan.n_row_items, _dev(plan.merges, "merges", torch.int32), plan.n_merges, _dev(out, "out"),
-                                                _dev(part_o, "part_o"), _dev(part_ml, "part_ml"), float(scale), T, H, C, R, page_tokens,
-                                                tables.shape[1], _stream()),
+                                                _dev(part_o, "part_o"), _dev(part_ml, "part_ml"), float(scale), T, H, C, R, width, page_tokens,
+                                                tables.shape[1], int(window), 1 if row_major else 0, _stream()),
                "latent_attention_mfma")
         return
     _check(lib().llmx_latent_attention_generic(_dev(q_lat, "q_lat"), _dev(q_rot, "q_rot"), _dev(cache, "cache"), _dev(pos, "pos", torch.int32, (T,)),
                                                _dev(row_entry, "row_entry", torch.int32, (T,)), _dev(tables, "tables", torch.int32),
-                                               _dev(out, "out"), _code(q_lat.dtype), float(scale), T, H, C, R, page_tokens, tables.shape[1],
-                                               int(window), _stream()), "latent_attention")
+                                               _dev(out, "out"), _code(q_lat.dtype), float(scale), T, H, C, R, width, page_tokens, tables.shape[1],
+                                               int(window), 1 if row_major else 0, _stream()), "latent_attention")
+
+
+def latent_cache_width(rank: int, rot_dim: int) -> int:
+    """Values of a token's cache row for the matrix-core kernel: the latent and the key part, padded with zeros to whole k-steps."""
+    return -(-(rank + rot_dim) // 32) * 32
 
 
 def latent_attention_mfma_ok(dtype: torch.dtype, rank: int, rot_dim: int, page_tokens: int) -> bool:
@@ -445,14 +548,16 @@ def latent_attention_mfma_ok(dtype: torch.dtype, rank: int, rot_dim: int, page_t
 
 
 LATENT_SPLIT_KEYS = 128    # keys a split item of a decoded row takes (two segments of the kernel)
+LATENT_SPLIT_WINDOW_KEYS = 64   # ... under a window, which leaves few items
 
 
 class LatentPlan:
     """Work items of the matrix-core latent attention for one step's rows: each up to 16 (row, head) columns of one request,
     whole or, for decoded rows, one block of the context; and the list of joins of the split ones.  It holds no positions."""
 
-    def __init__(self, tiles, row_items, items, merges, n_slots, heads, rows, device):
+    def __init__(self, tiles, row_items, items, merges, n_slots, heads, rows, device, window=0):
         import numpy as np
+        self.window = window
         self.heads, self.rows, self.n_items, self.n_merges, self.n_slots = heads, rows, len(items), len(merges), n_slots
         self.n_tile_items = len(tiles)       # the list's first items: four column tiles each, for a workgroup of four waves
         self.n_row_items = len(row_items)    # then the decoded rows' items: one column tile, a workgroup of four waves
@@ -467,15 +572,19 @@ _LATENT_PLANS: dict = {}
 LATENT_TILES = 4           # column tiles of 16 that a workgroup of the prompt form takes (the kernel's LW_TILES)
 
 
-def latent_plan(row_counts, heads: int, device, contexts=None, tiles: bool = True) -> LatentPlan:
+def latent_plan(row_counts, heads: int, device, contexts=None, tiles: bool = True, window: int = 0) -> LatentPlan:
     """row_counts[i]: rows of entry i (entries' rows are consecutive, in order); contexts[i]: the tokens it holds after the
     step (None: nothing is split).  With 16 heads or more an item is one row and up to 16 of its heads; with fewer,
     16 // heads consecutive rows of one entry with all their heads; later rows (longer key ranges) come first.  An entry of
     one row (a decoded token) whose context is longer than LATENT_SPLIT_KEYS gets an item for every block of that many
     keys, a function of its own context only.  An entry of several rows (a prompt's portion) goes, `tiles` allowing, to
-    workgroups of four waves that take four column tiles each and read the keys once for all of them; the same bits."""
-    blocks = tuple(-(-c // LATENT_SPLIT_KEYS) if n == 1 else 1 for n, c in zip(row_counts, contexts)) if contexts is not None else None
-    key = (tuple(row_counts), heads, blocks, bool(tiles), str(device))
+    workgroups of four waves that take four column tiles each and read the keys once for all of them; the same bits.
+    Under a `window` a decoded row's items count LATENT_SPLIT_WINDOW_KEYS-blocks from the block of its lowest key on, as many
+    as a window can touch (the last may hold no key), so that the plan stays the same while the row moves on."""
+    split = LATENT_SPLIT_WINDOW_KEYS if window else LATENT_SPLIT_KEYS
+    most = (window + split - 2) // split + 1 if window else 1 << 30       # blocks that `window` neighbouring keys can touch
+    blocks = tuple(min(-(-c // split), most) if n == 1 else 1 for n, c in zip(row_counts, contexts)) if contexts is not None else None
+    key = (tuple(row_counts), heads, blocks, bool(tiles), str(device), int(window))
     plan = _LATENT_PLANS.get(key)
     if plan is None:
         wide, single, items, merges, row0, slot = [], [], [], [], 0, 0
@@ -500,12 +609,12 @@ def latent_plan(row_counts, heads: int, device, contexts=None, tiles: bool = Tru
                         continue
                     merges.append([row0, h0, nh, slot, nb, 0, 0, 0])
                     for b in range(nb):
-                        to.append([row0, 1, h0, nh, b * LATENT_SPLIT_KEYS, (b + 1) * LATENT_SPLIT_KEYS, slot + b, 0])
+                        to.append([row0, 1, h0, nh, b if window else b * split, split if window else (b + 1) * split, slot + b, 0])
                     slot += nb
             row0 += n
         if len(_LATENT_PLANS) > 256:
             _LATENT_PLANS.clear()
-        plan = _LATENT_PLANS[key] = LatentPlan(wide, single, items, merges, slot, heads, row0, device)
+        plan = _LATENT_PLANS[key] = LatentPlan(wide, single, items, merges, slot, heads, row0, device, int(window))
     return plan
 
 
@@ -526,16 +635,19 @@ def head_gate(values: torch.Tensor, gate: Optional[torch.Tensor], out: torch.Ten
 _HEAD_GROUPS: dict = {}
 
 
-def head_groups(heads: int, rows: int, device):
-    """What grouped_gemm wants for `heads` groups of `rows` rows each, laid out group by group: (offsets, pairs, active,
-    n_active) on the device.  Cached: a step's launches may be recorded into a graph that reads them later."""
-    key = (heads, rows, str(device))
+def head_groups(heads: int, rows: int, device, row_major: bool = False):
+    """What grouped_gemm wants for `heads` groups of `rows` rows each, laid out group by group (with `row_major`: row by row,
+    a row's groups together): (offsets, pairs, active, n_active) on the device.  Cached: a step's launches may be recorded
+    into a graph that reads them later."""
+    key = (heads, rows, str(device), bool(row_major))
     got = _HEAD_GROUPS.get(key)
     if got is None:
         if len(_HEAD_GROUPS) > 512:
             _HEAD_GROUPS.clear()
-        got = _HEAD_GROUPS[key] = (torch.arange(0, (heads + 1) * rows, rows, dtype=torch.int32, device=device),
-                                   torch.arange(heads * rows, dtype=torch.int32, device=device),
+        pairs = torch.arange(heads * rows, dtype=torch.int32, device=device)
+        if row_major:
+            pairs = pairs.view(rows, heads).t().contiguous().view(-1)
+        got = _HEAD_GROUPS[key] = (torch.arange(0, (heads + 1) * rows, rows, dtype=torch.int32, device=device), pairs,
                                    torch.arange(heads, dtype=torch.int32, device=device),
                                    torch.full((1,), heads, dtype=torch.int32, device=device))
     return got
@@ -667,14 +779,17 @@ def state_matrix_plain(flat: torch.Tensor, H: int, D: int, V: int) -> torch.Tens
 
 def state_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, beta: Optional[torch.Tensor], state: torch.Tensor,
                slot_read: torch.Tensor, slot_write: torch.Tensor, entry_rows: torch.Tensor, out: torch.Tensor, out_scale: float,
-               H: int, qk_heads: int, D: int, V: int, tail=None, max_rows: int = 0) -> None:
+               H: int, qk_heads: int, D: int, V: int, tail=None, max_rows: int = 0, operands: Optional["StateOperands"] = None,
+               max_rows_here: int = 0) -> None:
     """The matrix-state recurrence over each entry's rows (csrc/linear_state.hip): per head S <- diag(decay) S;
     u = beta (v - S^T k) (u = v without beta); S <- S + k u^T; out = out_scale * S^T q.  q, k [T, qk_heads*D], v [T, H*V],
     decay [T, H*D] are float32 views whose rows may be columns of wider tensors; state [slots, width] float32 holds S at
     its start in tiles of 8 value channels ([H, ceil(V / 8), D, 8]: `state_matrix_size`, `state_matrix_tiled`), read at
     slot_read[e], written at slot_write[e].  `max_rows`: the most rows an entry has, when the caller knows it (steps of
     single tokens stage smaller chunks; the results are the same).  `tail` = (source [T, C] view, taps, offset):
-    the convolution tail [taps - 1, C] at `offset` of the state is handed on from the step's rows of `source`."""
+    the convolution tail [taps - 1, C] at `offset` of the state is handed on from the step's rows of `source`.  `operands`: what
+    is made of q, k and v as they are read (None: nothing).  `max_rows_here` > 0: entries of more rows are left alone (another
+    kernel takes them: decayed_state_chunks)."""
     T = out.shape[0]
     n_e = entry_rows.shape[0]
     if H % qk_heads or state.dim() != 2 or state.shape[1] < state_matrix_size(H, D, V) or D > 256:
@@ -693,7 +808,100 @@ def state_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     _check(lib().llmx_state_scan(qa, ldq, ka, ldk, va, ldv, ga, ldg, _dev(beta, "beta", torch.float32, (T, H)), _dev(state, "state", torch.float32),
                                  state.shape[1], _dev(slot_read, "slot_read", torch.int32, (n_e,)), _dev(slot_write, "slot_write", torch.int32, (n_e,)),
                                  _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)), _dev(out, "out", torch.float32, (T, H * V)), float(out_scale),
-                                 n_e, H, H // qk_heads, D, V, ta, tld, tC, int(taps), int(toff), int(max_rows), _stream()), "state_scan")
+                                 n_e, H, H // qk_heads, D, V, ta, tld, tC, int(taps), int(toff), int(max_rows), int(max_rows_here),
+                                 *_operand_args(operands, T, D), _stream()), "state_scan")
+
+
+OPERANDS_PLAIN, OPERANDS_SILU, OPERANDS_ROTATED = 0, 1, 2
+
+
+class StateOperands:
+    """What a matrix-state recurrence makes of its projected rows as it reads them: OPERANDS_SILU: silu of q, k and v;
+    OPERANDS_ROTATED: the first dims of every q and k head turn as pairs (i, i + dims/2) by the row's position, cos_sin
+    [positions, dims] float32 (cos of the pairs, then sin), pos int32 [T]."""
+
+    def __init__(self, kind: int, cos_sin: Optional[torch.Tensor] = None, pos: Optional[torch.Tensor] = None):
+        if kind not in (OPERANDS_PLAIN, OPERANDS_SILU, OPERANDS_ROTATED) or (kind == OPERANDS_ROTATED) != (cos_sin is not None and pos is not None):
+            raise KernelError("state operands: plain, silu, or rotated with a table and positions")
+        self.kind, self.cos_sin, self.pos = kind, cos_sin, pos
+
+
+def _operand_args(operands: Optional[StateOperands], T: int, D: int):
+    if operands is None or operands.kind != OPERANDS_ROTATED:
+        return (operands.kind if operands is not None else OPERANDS_PLAIN), 0, 0, 0
+    dims = operands.cos_sin.shape[1]
+    if dims == 0:                # a rotation of no dims leaves q and k as they are
+        return OPERANDS_PLAIN, 0, 0, 0
+    if dims % 2 or dims > D:
+        raise KernelError(f"state operands: {dims} rotated dims in a head of {D}")
+    return OPERANDS_ROTATED, _dev(operands.cos_sin, "cos_sin", torch.float32), _dev(operands.pos, "pos", torch.int32, (T,)), dims
+
+
+DECAYED_CHUNKS_MIN_ROWS = 128   # an entry of at least this many rows in the step goes chunk by chunk over the matrix cores
+
+
+class DecayedPlan:
+    """The chunks of a step's long entries for decayed_state_chunks, and the most rows an entry may have that is not one."""
+
+    def __init__(self, row_counts, rows_a_chunk, device):
+        import numpy as np
+        chunks, entries, row0 = [], [], 0
+        for e, n in enumerate(row_counts):
+            if n >= DECAYED_CHUNKS_MIN_ROWS:
+                entries.append([e, len(chunks), -(-n // rows_a_chunk), 0])
+                chunks += [[e, row0 + r, min(rows_a_chunk, n - r), 0] for r in range(0, n, rows_a_chunk)]
+            row0 += n
+        self.n_chunks, self.n_long = len(chunks), len(entries)
+        self.short_entries = len(row_counts) - len(entries)
+        self.rows = row0
+        self.chunks = torch.tensor(np.asarray(chunks, dtype=np.int32), device=device)
+        self.entry_chunks = torch.tensor(np.asarray(entries, dtype=np.int32), device=device)
+
+
+_DECAYED_PLANS: dict = {}
+
+
+def decayed_plan(row_counts, device) -> Optional[DecayedPlan]:
+    """The chunk lists for a step with these rows an entry, or None when no entry is long enough."""
+    if max(row_counts) < DECAYED_CHUNKS_MIN_ROWS:
+        return None
+    key = (tuple(row_counts), str(device))
+    plan = _DECAYED_PLANS.get(key)
+    if plan is None:
+        if len(_DECAYED_PLANS) > 64:
+            _DECAYED_PLANS.clear()
+        plan = _DECAYED_PLANS[key] = DecayedPlan(row_counts, lib().llmx_decayed_state_rows(), device)
+    return plan
+
+
+def decay_powers(decay, device) -> torch.Tensor:
+    """float32 [H, rows a chunk + 1]: g^0, g^1, ... of every head's decay g (rounded to float32, as the scan applies it)."""
+    import numpy as np
+    g = np.asarray(decay, dtype=np.float32).astype(np.float64)
+    return torch.from_numpy((g[:, None] ** np.arange(lib().llmx_decayed_state_rows() + 1)[None, :]).astype(np.float32)).to(device)
+
+
+def decayed_state_chunks(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, powers: torch.Tensor, state: torch.Tensor, slot_read: torch.Tensor,
+                         slot_write: torch.Tensor, out: torch.Tensor, out_scale: float, H: int, D: int, V: int, plan: DecayedPlan,
+                         operands: Optional[StateOperands] = None, scratch=None) -> None:
+    """state_scan's recurrence for one constant decay a head (`powers`: decay_powers), over the rows of the plan's long entries
+    only: q, k [T, H*D], v [T, H*V] float32 views, out [T, H*V], the state as state_scan keeps it (csrc/decayed_state.hip).
+    `scratch(name, shape, dtype)`: storage that lives as long as the caller's step."""
+    T = out.shape[0]
+    if state.dim() != 2 or state.shape[1] < state_matrix_size(H, D, V) or D > 256 or plan.rows != T:
+        raise KernelError("decayed_state_chunks: heads, widths, plan or state do not fit")
+    qa, ldq = _rows_view(q, "q", T, H * D)
+    ka, ldk = _rows_view(k, "k", T, H * D)
+    va, ldv = _rows_view(v, "v", T, H * V)
+    n_e = slot_read.shape[0]
+    starts = (scratch or _scratch_now(out.device))("decayed.starts", (plan.n_chunks, H, -(-V // 16) * 16, -(-D // 16) * 16), torch.float32)
+    _check(lib().llmx_decayed_state_chunks(qa, ldq, ka, ldk, va, ldv,
+                                           _dev(powers, "powers", torch.float32, (H, lib().llmx_decayed_state_rows() + 1)),
+                                           _dev(state, "state", torch.float32), state.shape[1], _dev(slot_read, "slot_read", torch.int32, (n_e,)),
+                                           _dev(slot_write, "slot_write", torch.int32, (n_e,)), _dev(plan.chunks, "chunks", torch.int32), plan.n_chunks,
+                                           _dev(plan.entry_chunks, "entry_chunks", torch.int32), plan.n_long, _dev(starts, "starts"),
+                                           _dev(out, "out", torch.float32, (T, H * V)), float(out_scale), H, D, V, *_operand_args(operands, T, D),
+                                           _stream()), "decayed_state_chunks")
 
 
 GATE_SIGMOID, GATE_SILU = 0, 1
@@ -1315,18 +1523,21 @@ def _parts_args(z: torch.Tensor, parts: Optional[torch.Tensor]):
 
 
 def route_topk(z: torch.Tensor, bias: Optional[torch.Tensor], ids: torch.Tensor, weights: torch.Tensor, k: int, score: int,
-               normalize: bool, scale: float, parts: Optional[torch.Tensor] = None, logit_bias: Optional[torch.Tensor] = None) -> None:
+               normalize: bool, scale: float, parts: Optional[torch.Tensor] = None, logit_bias: Optional[torch.Tensor] = None,
+               groups=None) -> None:
     """`parts` [slices, rows, experts]: the logits arrive as partial sums (gemm_f32's `parts`); they are added in slice
     order into z first.  `logit_bias` [experts]: added to the logits (z keeps the sum) before scores are formed.
     `normalize`: False, True (the picks' weights are divided by their sum; a single softmax pick keeps its score), or
-    "always" (a single softmax pick is divided too: the softmax over the picked logits alone)."""
+    "always" (a single softmax pick is divided too: the softmax over the picked logits alone).  `groups` = (count, keep): the
+    experts form `count` equal groups of neighbours, and only those of the `keep` groups with the largest best pick key (score
+    plus bias) can be picked."""
     rows, n_experts = z.shape
     if n_experts > MAX_EXPERTS or k > MAX_TOP_K or k > n_experts:
         raise KernelError(f"route_topk takes at most {MAX_EXPERTS} experts and {MAX_TOP_K} picks, not {n_experts} and {k}")
     _check(lib().llmx_route_topk(_dev(z, "z", torch.float32), *_parts_args(z, parts), _dev(bias, "bias", torch.float32, (n_experts,)),
                                  _dev(ids, "ids", torch.int32, (rows, k)), _dev(weights, "weights", torch.float32, (rows, k)),
                                  rows, n_experts, k, score, 2 if normalize == "always" else 1 if normalize else 0, float(scale),
-                                 _dev(logit_bias, "logit_bias", torch.float32, (n_experts,)), _stream()), "route_topk")
+                                 _dev(logit_bias, "logit_bias", torch.float32, (n_experts,)), *(groups or (0, 0)), _stream()), "route_topk")
 
 
 def moe_align_scratch(n_pairs: int, n_experts: int) -> int:
@@ -1362,20 +1573,20 @@ def route_topk_align(z: torch.Tensor, bias: Optional[torch.Tensor], ids: torch.T
                      normalize: bool, scale: float, counts: torch.Tensor, offsets: torch.Tensor, pairs: torch.Tensor,
                      active: torch.Tensor, n_active: torch.Tensor, parts: Optional[torch.Tensor] = None,
                      scratch: Optional[torch.Tensor] = None, tile_stats: Optional[torch.Tensor] = None,
-                     logit_bias: Optional[torch.Tensor] = None) -> None:
-    """route_topk followed by moe_align; a step of at most 16 rows (sigmoid scores, at most 256 experts and 64 picks) does
+                     logit_bias: Optional[torch.Tensor] = None, groups=None) -> None:
+    """route_topk followed by moe_align; a step of at most 16 rows (at most 256 experts and 64 picks, no logit bias) does
     both in one launch, with the same bits."""
     rows, n_experts = z.shape
-    if score == SCORE_SIGMOID and rows <= 16 and rows * k <= 1024 and n_experts <= 256 and k <= 64 and logit_bias is None and normalize != "always":
+    if rows <= 16 and rows * k <= 1024 and n_experts <= 256 and k <= 64 and logit_bias is None:
         _check(lib().llmx_route_topk_align(
             _dev(z, "z", torch.float32), *_parts_args(z, parts), _dev(bias, "bias", torch.float32, (n_experts,)),
             _dev(ids, "ids", torch.int32, (rows, k)),
-            _dev(weights, "weights", torch.float32, (rows, k)), rows, n_experts, k, 1 if normalize else 0, float(scale),
-            _dev(counts, "counts", torch.int32, (n_experts,)), _dev(offsets, "offsets", torch.int32, (n_experts + 1,)),
+            _dev(weights, "weights", torch.float32, (rows, k)), rows, n_experts, k, score, 2 if normalize == "always" else 1 if normalize else 0,
+            float(scale), *(groups or (0, 0)), _dev(counts, "counts", torch.int32, (n_experts,)), _dev(offsets, "offsets", torch.int32, (n_experts + 1,)),
             _dev(pairs, "pairs", torch.int32, (rows * k,)), _dev(active, "active", torch.int32, (n_experts,)),
             _dev(n_active, "n_active", torch.int32, (1,)), _stream()), "route_topk_align")
         return
-    route_topk(z, bias, ids, weights, k, score, normalize, scale, parts, logit_bias)
+    route_topk(z, bias, ids, weights, k, score, normalize, scale, parts, logit_bias, groups)
     moe_align(ids, n_experts, counts, offsets, pairs, active, n_active, scratch, tile_stats)
 
 

@@ -154,6 +154,13 @@ class FeedForward(Part):
 
 
 class Embedding(Part):
+    #: as Mixer.steps_between_slots, for an embedding with state
+    steps_between_slots = False
+
+    def cache_need(self) -> Optional[StateNeed]:
+        """What the embedding keeps a request from token to token, or None; with a state `forward` gets it as `cache`."""
+        return None
+
     def forward(self, step, out: torch.Tensor) -> None:
         """out (float32 [T, hidden]) = rows of the table for step.token_ids."""
         raise NotImplementedError

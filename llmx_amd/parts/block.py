@@ -4,7 +4,7 @@
 /root/reference/src/model/arch/minimax_m3.hpp:247-287 (norm, mixer joined into the residual, norm, feed-forward joined).
 "parallel": x += s1 * mixer(norm1(x)) + s2 * ffn(norm2(x)) with both norms of the same x, learned factors s1, s2 a
 coordinate (or constants), and an optional per-layer token input after the sum; without a second norm both sublayers read
-norm1's rows.
+norm1's rows.  Without factors each result is added to x where it is formed: (x + mixer(h)) + ffn(h).
 "outnorm": x += norm1(mixer(x)); x += norm2(ffn(x)): the sublayers read the residual itself and only their results are
 normed.
 "sandwich": x += norm1b(mixer(norm1(x))); x += norm2b(ffn(norm2(x))): a norm on both sides of each sublayer.
@@ -88,7 +88,8 @@ class ParallelBlock:
     new x.  The slots: mixer_norm, mixer, ffn_norm, ffn (a feed-forward without a norm of its own reads the mixer's normed
     rows: one norm for both sublayers); in `extra`: "mixer_scale" and "ffn_scale" (family "scale": a factor a coordinate, or
     a constant, on each result before the sum, optional) and "token_input" (family "token_input", optional).  Two RMS norms
-    with one eps are one pass over x with two gains."""
+    with one eps are one pass over x with two gains; an RMS norm before a mixer of token-shifted rows is one launch with the
+    shift where the feed-forward reads the same norm."""
     graph_safe = True
 
     def __init__(self, spec: BlockSpec, ctx: BuildContext):
@@ -124,6 +125,12 @@ class ParallelBlock:
             raise ValueError("parallel block: a token input goes with factors a coordinate")
         if self.ffn is not None and self.ffn.wants_f32_input:
             self._one_pass = False
+        # the norm and the mixer's token shift in one launch: where one norm serves both sublayers, or the mixer is alone
+        self._norm_and_shift = (self._shared_norm or self.ffn is None) and getattr(self.mixer, "fuses", None) is not None and self.mixer.fuses(a)
+        if self.mixer.wants_f32_input:
+            self._one_pass = False
+        # no factor on either result and nothing after the sum: both sublayers add into x
+        self._adds_into = not scales and self.token_input is None
 
     def parts(self):
         return [p for p in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn, self.mixer_scale, self.ffn_scale, self.token_input)
@@ -136,17 +143,30 @@ class ParallelBlock:
         h2 = step.buf("block.h2", (T, E), act) if self.ffn is not None and not self._shared_norm else None
         # a feed-forward whose router reads unrounded rows gets them from its norm
         h32 = step.buf("block.h32", (T, E), torch.float32) if self.ffn is not None and self.ffn.wants_f32_input else None
-        if self._shared_norm:
-            self.mixer_norm.forward(step, x, h1, h32)
+        mixer, mixer_rows, mixer_cache, mixer32 = self.mixer, h1, cache, None
+        if self._norm_and_shift:
+            mixer_rows = self.mixer.normed_and_shifted(step, self.mixer_norm, x, cache, h1 if self.ffn is not None else None, h32)
+            mixer, mixer_cache, h2 = self.mixer.inner, cache.members[0], h1
+        elif self._shared_norm:
+            if self.mixer.wants_f32_input:
+                mixer32 = h32 if h32 is not None else step.buf("block.mixer_h32", (T, E), torch.float32)
+            self.mixer_norm.forward(step, x, h1, h32 if h32 is not None else mixer32)
             h2 = h1
         elif self._one_pass:
             ops.rmsnorm_pair(x, self.mixer_norm.weight, self.ffn_norm.weight if h2 is not None else None, self.mixer_norm.eps, h1, h2)
         else:
-            self.mixer_norm.forward(step, x, h1)
+            if self.mixer.wants_f32_input:
+                mixer32 = step.buf("block.mixer_h32", (T, E), torch.float32)
+            self.mixer_norm.forward(step, x, h1, mixer32)
             if h2 is not None:
                 self.ffn_norm.forward(step, x, h2, h32)
+        if self._adds_into:
+            mixer.forward(step, mixer_rows, x, True, mixer_cache, mixer32)
+            if self.ffn is not None:
+                self.ffn.forward(step, h2, x, True, h32)
+            return
         y1 = step.buf("block.y1", (T, E), torch.float32)
-        self.mixer.forward(step, h1, y1, False, cache)
+        mixer.forward(step, mixer_rows, y1, False, mixer_cache, mixer32)
         y2 = None
         if self.ffn is not None:
             y2 = step.buf("block.y2", (T, E), torch.float32)

@@ -1,7 +1,8 @@
 """Token embedding and the language-model head.
 
 x[t] = table[id[t]] widened to float32, times the embedding's scale where the model has one (/root/reference/src/model/arch/blocks.hpp:95-97); logits = rows . W^T in
-float32 for the wanted rows only (:267-272).  A tied head reads the embedding's table.
+float32 for the wanted rows only (:267-272).  A tied head reads the embedding's table.  A bigram embedding adds a second
+table's row, chosen by the token and the one before it.
 """
 
 from __future__ import annotations
@@ -9,8 +10,8 @@ from __future__ import annotations
 import torch
 
 from .. import ops
-from .base import Embedding, Head, register
-from .spec import TensorSpec
+from .base import Embedding, Head, LayerCache, register
+from .spec import StateNeed, TensorSpec
 
 
 class TokenEmbedding(Embedding):
@@ -41,6 +42,36 @@ class TokenEmbedding(Embedding):
 
     def forward(self, step, out):
         ops.embed_gather(self.weight, step.token_ids, out, self.scale)
+
+
+class BigramEmbedding(TokenEmbedding):
+    """A token embedding with a second table's row added: row (previous token * mul_prev + token * mul_cur) mod buckets, and the
+    table's last row for a request's first token.  params: those of TokenEmbedding, and bigram {tensor (its full name), buckets,
+    mul_prev, mul_cur}.  Tensors: the embedding's, and <bigram tensor> (buckets + 1, hidden).  State: the last token."""
+    steps_between_slots = True      # reads the state at step.entry_held_slots, writes it at step.entry_slots
+
+    def __init__(self, params, prefix, ctx):
+        super().__init__(params, prefix, ctx)
+        b = params["bigram"]
+        self.bigram_name = str(b["tensor"])
+        self.buckets, self.mul_prev, self.mul_cur = int(b["buckets"]), int(b["mul_prev"]), int(b["mul_cur"])
+        if self.buckets < 1:
+            raise ValueError("bigram embedding: at least one bucket")
+        self.bigram = None
+
+    def cache_need(self):
+        return StateNeed((1,), "int32")
+
+    def tensor_specs(self, available):
+        return super().tensor_specs(available) + [TensorSpec(self.bigram_name, (self.buckets + 1, self.hidden), "table")]
+
+    def load(self, tensors):
+        super().load(tensors)
+        self.bigram = tensors[self.bigram_name]
+
+    def forward(self, step, out, cache: LayerCache):
+        ops.embed_bigram(self.weight, self.bigram, step.token_ids, cache.state, step.entry_held_slots, step.entry_slots, step.row_entry,
+                         step.entry_rows, out, self.buckets, self.mul_prev, self.mul_cur, self.scale)
 
 
 class LinearHead(Head):
@@ -78,4 +109,5 @@ class LinearHead(Head):
 
 
 register("embedding", "token_embedding", TokenEmbedding)
+register("embedding", "bigram_embedding", BigramEmbedding)
 register("head", "linear", LinearHead)

@@ -3,6 +3,7 @@
 All decay S's rows (channel by channel, or a head's all alike) and add an outer product a token; they differ in what is added:
     S_t = diag(g_t) S_(t-1) + k_t u_t^T,   o_t = S_t^T q_t
     gated linear attention:  u_t = v_t,                               g_t = sigmoid(z_t)^(1/tau)
+    constant decay a head:   u_t = v_t,                               g_t = a number of the model
     gated delta rule:        u_t = beta_t (v_t - (diag(g_t) S_(t-1))^T k_t),   g_t = exp(-exp(A) softplus(step_t + dt_bias))
 with z_t and step_t low-rank projections of the input.  The delta rule's q, k and v first pass a short causal convolution
 over time and silu, and q and k are made unit vectors a head.  The read-out is RMS-normed a head, gated, and projected.
@@ -16,8 +17,8 @@ from __future__ import annotations
 import torch
 
 from .. import ops
-from .base import LayerCache, Mixer, register
-from .spec import StateNeed, TensorSpec
+from .base import LayerCache, Mixer, build_part, register
+from .spec import PartSpec, StateNeed, TensorSpec
 
 
 class GatedLinearAttention(Mixer):
@@ -222,6 +223,91 @@ class GatedMatrixMemory(Mixer):
         ops.gemm(gated, self.w_o, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)
 
 
+class DecayedLinearAttention(Mixer):
+    """Linear attention with one constant decay a head: S_t = g_h S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.
+    params: hidden, heads, dim, vdim, decay (a number a head), eps; operands ("silu": silu of q, k and v | "rotated": q and k
+    turned by `position` (PartSpec of a rotary encoding with halved pairs) | "plain"), key_scale (a factor on k, 1);
+    norm ("joint": an RMS norm over all heads' values with a weight [heads * vdim] | "head": every head's values divided by
+    their root mean square), gate ("sigmoid" | "silu": of W_g h).  result = W_o (norm(o) * gate).
+    Tensors <prefix>q, k, v, g, o, and norm for the joint norm.  Runs of many rows go chunk by chunk over the matrix cores, short
+    ones row by row; everything from the projections' results to the gated rows is float32."""
+    graph_safe = True
+    steps_between_slots = True
+    _GATES = {"sigmoid": ops.GATE_SIGMOID, "silu": ops.GATE_SILU}
+
+    def __init__(self, params, prefix, ctx):
+        super().__init__(params, prefix, ctx)
+        p = params
+        self.hidden, self.heads, self.dim, self.vdim = int(p["hidden"]), int(p["heads"]), int(p["dim"]), int(p["vdim"])
+        self.eps = float(p["eps"])
+        self.decay = [float(g) for g in p["decay"]]
+        if min(self.heads, self.dim, self.vdim) < 1 or self.dim > 256:
+            raise ValueError("decayed linear attention: heads, dim (at most 256) and vdim are at least 1")
+        if len(self.decay) != self.heads or not all(0.0 <= g <= 1.0 for g in self.decay):
+            raise ValueError(f"decayed linear attention: {self.heads} decays between 0 and 1, not {self.decay}")
+        self.operands = str(p.get("operands", "plain"))
+        self.norm_kind, self.gate = str(p.get("norm", "head")), str(p.get("gate", "silu"))
+        if self.operands not in ("plain", "silu", "rotated") or self.norm_kind not in ("joint", "head") or self.gate not in self._GATES:
+            raise ValueError(f"decayed linear attention: operands {self.operands!r}, norm {self.norm_kind!r} or gate {self.gate!r} is not one this part has")
+        self.position = build_part("position", p.get("position") or PartSpec("none"), ctx)
+        if self.operands == "rotated":
+            if self.position.pairing != "halves" or self.position.rotation()[1] > self.dim:
+                raise ValueError("decayed linear attention: the rotated dims turn as halved pairs and fit a head")
+        # a factor on every key is a factor on the read-out
+        self.out_scale = float(p.get("key_scale", 1.0))
+        H, HD, HV = self.heads, self.heads * self.dim, self.heads * self.vdim
+        self.cols = {"q": (0, HD), "k": (HD, HD), "v": (2 * HD, HV), "g": (2 * HD + HV, HV)}
+        self.in_width = 2 * HD + 2 * HV
+        self.w_in = self.w_o = self.norm = self.powers = self.decay_row = None
+
+    def cache_need(self):
+        return StateNeed((ops.state_matrix_size(self.heads, self.dim, self.vdim),), "float32")
+
+    def tensor_specs(self, available):
+        E = self.hidden
+        fused, shape = self.name("in"), (self.in_width, E)
+        specs = [TensorSpec(self.name(n), (w, E), into=(fused, shape, (slice(at, at + w),))) for n, (at, w) in self.cols.items()]
+        if self.norm_kind == "joint":
+            specs.append(TensorSpec(self.name("norm"), (self.heads * self.vdim,), "norm"))
+        return specs + [TensorSpec(self.name("o"), (E, self.heads * self.vdim))]
+
+    def load(self, tensors):
+        self.w_in, self.w_o = tensors[self.name("in")], tensors[self.name("o")]
+        self.norm = tensors[self.name("norm")] if self.norm_kind == "joint" else None
+        # the decays as the two forms of the recurrence read them: one row of a decay a key channel; powers of it
+        self.decay_row = torch.tensor(self.decay, dtype=torch.float32, device=self.w_o.device).repeat_interleave(self.dim).view(1, -1)
+        self.powers = ops.decay_powers(self.decay, self.w_o.device)
+
+    def _operands(self, step):
+        if self.operands == "silu":
+            return ops.StateOperands(ops.OPERANDS_SILU)
+        if self.operands == "rotated":
+            return ops.StateOperands(ops.OPERANDS_ROTATED, self.position.rotation()[0], step.positions)
+        return None
+
+    def forward(self, step, h, out, accumulate, cache: LayerCache, h32=None):
+        T, H, D, V = step.rows, self.heads, self.dim, self.vdim
+        pre = step.buf("decayed.pre", (T, self.in_width), torch.float32)
+        ops.gemm(h, self.w_in, pre, scratch=step.buf)
+        view = lambda n: pre[:, self.cols[n][0]:self.cols[n][0] + self.cols[n][1]]
+        o = step.buf("decayed.o", (T, H * V), torch.float32)
+        operands = self._operands(step)
+        # a decode step's entries are never long (nothing for a graph to hold)
+        plan = step.shared("decayed.plan", lambda: ops.decayed_plan([e.n for e in step.entries], step.device))
+        if plan is not None:
+            ops.decayed_state_chunks(view("q"), view("k"), view("v"), self.powers, cache.state, step.entry_held_slots, step.entry_slots, o,
+                                     self.out_scale, H, D, V, plan, operands, step.buf)
+        if plan is None or plan.short_entries:
+            ops.state_scan(view("q"), view("k"), view("v"), self.decay_row.expand(T, H * D), None, cache.state, step.entry_held_slots,
+                           step.entry_slots, step.entry_rows, o, self.out_scale, H, H, D, V, max_rows=step.max_rows_per_entry, operands=operands,
+                           max_rows_here=ops.DECAYED_CHUNKS_MIN_ROWS - 1 if plan is not None else 0)
+        gated = step.buf("decayed.gated", (T, H * V), step.act_dtype)
+        heads, width = (1, H * V) if self.norm_kind == "joint" else (H, V)
+        ops.head_norm_gate(o, self.norm, view("g"), gated, self.eps, heads, width, self._GATES[self.gate])
+        ops.gemm(gated, self.w_o, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)
+
+
+register("mixer", "decayed_linear_attention", DecayedLinearAttention)
 register("mixer", "gated_matrix_memory", GatedMatrixMemory)
 register("mixer", "gated_linear_attention", GatedLinearAttention)
 register("mixer", "channel_delta_rule", ChannelDeltaRule)

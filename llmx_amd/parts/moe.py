@@ -47,7 +47,8 @@ def _names(defaults: dict, given, what: str) -> dict:
 
 class RoutedExperts(FeedForward):
     """params: hidden, experts, top_k, intermediate, score ("sigmoid" | "softmax"), correction_bias (bool: a bias on the pick
-    keys only), logit_bias (bool: a bias that is part of the router's logits), normalize (bool), scale, names ({role: name
+    keys only), logit_bias (bool: a bias that is part of the router's logits), normalize (bool), scale, groups ({count, keep}: the experts form
+    `count` equal groups of neighbours and only those of the `keep` groups with the largest best pick key can be picked; None), names ({role: name
     below the prefix}), files ("fused" | "per_expert": how a model folder of the design holds the experts, for when no file says).  score "softmax" with normalize "always" is the softmax over the picked logits alone, for any top_k.
     unit ("swiglu", the default: silu(gate) * up | "clamped_glu": g = min(gate, limit), u = clamp(up, -limit, limit),
     g sigmoid(1.702 g) (u + 1)) with limit; weight_on ("output", the default: the row's result is sum_j w_j expert_j(h) |
@@ -84,6 +85,12 @@ class RoutedExperts(FeedForward):
         if self.experts > MAX_EXPERTS or self.top_k > MAX_TOP_K:
             raise ValueError(f"routed experts: {self.experts} experts with {self.top_k} picks a token; the routing kernels take at most "
                              f"{MAX_EXPERTS} experts and {MAX_TOP_K} picks")
+        groups = p.get("groups")
+        self.groups = (int(groups["count"]), int(groups["keep"])) if groups else None
+        if self.groups is not None:
+            count, keep = self.groups
+            if count < 1 or self.experts % count or not 0 < keep <= count or self.top_k > keep * (self.experts // count):
+                raise ValueError(f"routed experts: {self.experts} experts in {count} equal groups of which {keep} are kept do not offer {self.top_k} picks")
         if p.get("unit", "swiglu") not in _UNITS and p.get("unit") not in _PLAIN_UNITS:
             raise ValueError(f"routed experts: unit {p.get('unit')!r} is not one of {sorted(list(_UNITS) + list(_PLAIN_UNITS))}")
         self.plain_unit = _PLAIN_UNITS.get(p.get("unit"))         # None: a gated unit
@@ -193,7 +200,7 @@ class RoutedExperts(FeedForward):
         # for steps of many pairs the grouping also counts the experts' tiles of 128 rows, by which the products choose their tiles
         tile_stats = step.buf("experts.tile_stats", (1,), torch.int32) if T * k >= ops.TILE_STATS_MIN_PAIRS else None
         ops.route_topk_align(z, self.bias, ids, weights, k, self.score, self.normalize, self.scale, counts, offsets, pairs, active, n_active,
-                             parts=parts, scratch=scratch, tile_stats=tile_stats, logit_bias=self.logit_bias)
+                             parts=parts, scratch=scratch, tile_stats=tile_stats, logit_bias=self.logit_bias, groups=self.groups)
         step.observe("routing", logits=z, ids=ids, weights=weights)
         act = step.buf("experts.act", (T * k, self.intermediate), step.act_dtype)
         on_input = self.weight_on == "input"

@@ -99,10 +99,12 @@ def wavelength_scaled_frequencies(dims: int, base: float, scaling) -> np.ndarray
     return np.where(wavelength < original / high, f, np.where(wavelength > original / low, f / factor, blended))
 
 
-def scaled_table(positions: int, dims: int, base: float, scaling) -> np.ndarray:
+def scaled_table(positions: int, dims: int, base: float, scaling, exact_angles: bool = False) -> np.ndarray:
     """[positions, dims] float32: magnitude * cos of the dims/2 pairs' angles, then magnitude * sin.  The angle is the
     float32 product of the position and the float32 frequency; cos and sin are evaluated in float64 on it and rounded
-    once, as `neox_table` does."""
+    once, as `neox_table` does.  `exact_angles`: the angle too is a float64 product (unscaled frequencies only)."""
+    if exact_angles and scaling:
+        raise ValueError("rotary table: exact angles go with unscaled frequencies")
     if dims == 0:
         return np.zeros((positions, 0), dtype=np.float32)
     if scaling and "low" in scaling:           # {factor, low, high, original}: rescaled by wavelength
@@ -111,6 +113,9 @@ def scaled_table(positions: int, dims: int, base: float, scaling) -> np.ndarray:
         angle = np.arange(positions, dtype=np.float64)[:, None] * f[None, :]
         return np.concatenate([np.cos(angle), np.sin(angle)], axis=1).astype(np.float32)
     f, magnitude = blended_frequencies(dims, base, scaling)      # None, or {factor, original, fast, slow}
+    if exact_angles:
+        angle = np.arange(positions, dtype=np.float64)[:, None] * f[None, :]
+        return np.concatenate([np.cos(angle), np.sin(angle)], axis=1).astype(np.float32)
     pos = np.arange(positions, dtype=np.float32)[:, None]
     angle = (pos * f.astype(np.float32)[None, :]).astype(np.float32).astype(np.float64)
     return (np.concatenate([np.cos(angle), np.sin(angle)], axis=1) * magnitude).astype(np.float32)
@@ -119,7 +124,7 @@ def scaled_table(positions: int, dims: int, base: float, scaling) -> np.ndarray:
 class ScaledRotary(PositionEncoding):
     """Rotary pairs with optionally rescaled frequencies.  params: dims (even; the rotated dims), base, scaling (None;
     {factor, original, fast, slow}: the YaRN blend over the pair index with its factor on cos and sin; {factor, low, high,
-    original}: frequencies rescaled by wavelength, see `wavelength_scaled_frequencies`), pairing ("interleaved", the default here: dims 2i and 2i + 1; "halves")."""
+    original}: frequencies rescaled by wavelength, see `wavelength_scaled_frequencies`), pairing ("interleaved", the default here: dims 2i and 2i + 1; "halves"), exact_angles (see `scaled_table`)."""
     graph_safe = True
 
     def __init__(self, params, prefix, ctx):
@@ -132,7 +137,8 @@ class ScaledRotary(PositionEncoding):
             raise ValueError(f"rotary width {self.rotary_dim} must be even")
         self.base = float(params["base"])
         self.scaling = dict(params["scaling"]) if params.get("scaling") else None
-        self.cos_sin = torch.from_numpy(scaled_table(ctx.max_positions, self.rotary_dim, self.base, self.scaling)).to(ctx.device)
+        self.cos_sin = torch.from_numpy(scaled_table(ctx.max_positions, self.rotary_dim, self.base, self.scaling,
+                                                     bool(params.get("exact_angles", False)))).to(ctx.device)
 
     def rotation(self):
         return self.cos_sin, self.rotary_dim
