@@ -490,8 +490,10 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
     }
 }
 
-extern "C" int llmx_latent_attention_mfma_ok(int C, int R, int page_tokens) {
-    return C >= 16 && C <= 512 && C % 16 == 0 && R >= 0 && R % 8 == 0 && R <= 448 && page_tokens > 0 && page_tokens % 8 == 0 ? 1 : 0;
+// 960: four column tiles of queries and their weights in a workgroup's LDS
+extern "C" int llmx_latent_attention_mfma_ok(int C, int R, int ldc, int page_tokens) {
+    return C >= 16 && C <= 512 && C % 16 == 0 && R >= 0 && R % 8 == 0 && ldc >= C + R && ldc % 32 == 0 && ldc <= 960 && page_tokens > 0
+                   && page_tokens % 8 == 0 ? 1 : 0;
 }
 
 extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, const void* cache, const void* cache_t, const int* pos,
@@ -500,7 +502,7 @@ extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, 
                                           void* out, float* part_o, float* part_ml, float scale, int T, int H, int C, int R, int ldc, int page_tokens,
                                           int max_blocks, int window, int row_major, hipStream_t stream) {
     if (n_items <= 0 && n_tile_items <= 0 && n_row_items <= 0) return 0;
-    if (!llmx_latent_attention_mfma_ok(C, R, page_tokens) || ldc < C + R || ldc % 32 || window < 0) return -2;
+    if (!llmx_latent_attention_mfma_ok(C, R, ldc, page_tokens) || window < 0) return -2;
     if (n_merges > 0 && (!merges || !part_o || !part_ml)) return -2;
     LatentMfmaArgs a{(const bf16_t*)q_lat, (const bf16_t*)q_rot, (const bf16_t*)cache, (const bf16_t*)cache_t, pos, row_entry, tables, items,
                      (bf16_t*)out, part_o, part_ml, scale, T, H, C, R, ldc, page_tokens, max_blocks, window, row_major};

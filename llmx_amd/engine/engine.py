@@ -8,6 +8,7 @@ before anything is reserved, :633-653 reserve pages, :771-830 run, :1007-1032 co
 
 from __future__ import annotations
 
+import gc
 from dataclasses import replace
 from pathlib import Path
 from typing import Dict, Hashable, List, Optional, Sequence, Union
@@ -446,9 +447,15 @@ class Engine:
         return logits
 
     def _capture(self, step: StepState, key: tuple) -> Optional["_StepGraph"]:
-        """Records the step's launches (a step of this shape ran before, so every scratch tensor exists) into a graph."""
+        """Records the step's launches (a step of this shape ran before, so every scratch tensor exists) into a graph.
+
+        Python's cyclic collector rests meanwhile: what it frees may be another engine's graphs, whose destructor
+        synchronises the device; while a stream is being recorded that is an error, and an error in a destructor ends
+        the process."""
         before = (self._workspace.generation, self._uploader.generation)
         graph = torch.cuda.CUDAGraph()
+        collecting = gc.isenabled()
+        gc.disable()
         try:
             with torch.cuda.graph(graph):
                 logits = self._forward(step)
@@ -457,6 +464,9 @@ class Engine:
             warnings.warn(f"llmx_amd: recording a decode step as a HIP graph failed ({err}); steps run without graphs")
             self.graphs = False
             return None
+        finally:
+            if collecting:
+                gc.enable()
         if (self._workspace.generation, self._uploader.generation) != before:
             return None            # storage moved while recording: the graph holds stale addresses
         if len(self._graphs) >= 32:

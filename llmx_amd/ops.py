@@ -65,7 +65,7 @@ def _declare(h) -> None:
         "llmx_latent_down": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, I, P],
         "llmx_latent_queries": [P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
         "llmx_latent_attention_mfma": [P, P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, I, I, P],
-        "llmx_latent_attention_mfma_ok": [I, I, I],
+        "llmx_latent_attention_mfma_ok": [I, I, I, I],
         "llmx_latent_attention_generic": [P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, P],
         "llmx_head_gate": [P, P, I, P, I, I, I, I, P],
         "llmx_embed_bigram": [P, P, I, P, P, P, P, P, P, P, I, I, F, I, L, L, P],
@@ -514,7 +514,7 @@ def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tens
     n_pages, page_tokens, width = cache.shape
     if width < C + R or q_rot.shape[:2] != q_lat.shape[:2] or out.shape != q_lat.shape or len({q_lat.dtype, q_rot.dtype, cache.dtype, out.dtype}) != 1:
         raise KernelError("latent_attention: shapes or dtypes do not agree")
-    if cache_t is not None and plan is not None and width % 32 == 0 and latent_attention_mfma_ok(q_lat.dtype, C, R, page_tokens):
+    if cache_t is not None and plan is not None and latent_attention_mfma_ok(q_lat.dtype, C, R, page_tokens, width):
         if plan.heads != H or plan.rows != T or plan.window != int(window) or tuple(cache_t.shape) != (n_pages, C, page_tokens) \
                 or cache_t.dtype != cache.dtype:
             raise KernelError("latent_attention: the plan or the transposed copy does not fit the step")
@@ -543,8 +543,10 @@ def latent_cache_width(rank: int, rot_dim: int) -> int:
     return -(-(rank + rot_dim) // 32) * 32
 
 
-def latent_attention_mfma_ok(dtype: torch.dtype, rank: int, rot_dim: int, page_tokens: int) -> bool:
-    return dtype == torch.bfloat16 and bool(lib().llmx_latent_attention_mfma_ok(int(rank), int(rot_dim), int(page_tokens)))
+def latent_attention_mfma_ok(dtype: torch.dtype, rank: int, rot_dim: int, page_tokens: int, width: Optional[int] = None) -> bool:
+    """Whether the matrix-core kernel takes these sizes with cache rows of `width` values (None: nothing behind the key part)."""
+    width = rank + rot_dim if width is None else width
+    return dtype == torch.bfloat16 and bool(lib().llmx_latent_attention_mfma_ok(int(rank), int(rot_dim), int(width), int(page_tokens)))
 
 
 LATENT_SPLIT_KEYS = 128    # keys a split item of a decoded row takes (two segments of the kernel)

@@ -72,7 +72,7 @@ class LatentAttention(Mixer):
         """Whether this engine's steps run the attention on the matrix cores, which read the latents once more, transposed."""
         page = self.ctx.page_tokens
         return bool(page) and self.ctx.device.type == "cuda" \
-            and ops.latent_attention_mfma_ok(self.ctx.act_dtype, self.rank, self.rot_dim, page)
+            and ops.latent_attention_mfma_ok(self.ctx.act_dtype, self.rank, self.rot_dim, page, ops.latent_cache_width(self.rank, self.rot_dim))
 
     def cache_need(self):
         cores = self._matrix_cores()

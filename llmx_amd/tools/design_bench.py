@@ -13,6 +13,12 @@ picks and expert width.  A repeated layer's weights count each time they run.
 unit, the same with routed squared-relu experts, windowed attention that keeps the first tokens beside a gated matrix memory,
 attention in chunks with routed experts) and a MiniMax-M3 of the same width, layers, heads, experts, picks and expert width.
 
+`python bench.py --design neruzen` does the same for a Neruzen (layers in turn: latent attention over a window, linear attention
+with constant decays over silu projections, latent attention, the same linear attention over rotated queries and keys; all
+with routed SwiGLU experts beside a shared one) and the two models nearest to it: a Bonerax of the same width, layers, heads,
+experts, picks and expert width (matrix states of the same size a head, windowed attention, routed experts), and a Nenotar
+of the same width, layers, heads and latent (no window) with the same active feed-forward weights.
+
 `python bench.py --design nenotar` measures, at sizes that resemble a real model's layers, a Nenotar (latent attention
 and minGRU layers in turn, each with a dense xIELU feed-forward and a per-layer token input) and a MiniMax-M3 of the
 same width, layers, heads and vocabulary whose routed experts hold the same active weights a token: one 2,048-token
@@ -220,6 +226,71 @@ def salipel_mixing_flops(cfg, T: int) -> float:
     return total
 
 
+# name -> (width, layers, heads, query latent, window, experts, groups, kept groups, picks, expert ff, shared ff, bigram buckets, vocab);
+# latent heads are 128 unrotated + 64 rotated dims over a latent of 512 (values 128), states 128 x 128 a head
+NERUZEN_SIZES = {
+    "w2048": (2048, 8, 16, 1024, 1024, 8, 4, 2, 2, 2048, 2048, 65536, 32768),
+    "w4096": (4096, 4, 32, 1536, 1024, 8, 4, 2, 2, 4096, 4096, 65536, 32768),
+    "w256": (256, 4, 2, 96, 64, 8, 4, 2, 2, 128, 64, 512, 1024),
+}
+
+
+def neruzen_config(width, layers, heads, q_rank, window, experts, groups, keep, top, ff, shared_ff, buckets, vocab):
+    from llmx_amd.config.neruzen import (BigramConfig, ExpertsConfig, LatentAttentionConfig, LayerConfig, LightningConfig, NeruzenConfig,
+                                         RetentionConfig, Rotation)
+    decay = tuple(1.0 - 2.0 ** -(5.0 + 4.0 * i / heads) for i in range(heads))
+    latent = LatentAttentionConfig(heads=heads, dim=128, rot_dim=64, vdim=128, q_rank=q_rank, kv_rank=512, scale=192 ** -0.5, window=window,
+                                   rot=Rotation(10000.0, 64))
+    kinds = [("latent_attention", latent), ("lightning", LightningConfig(heads, 128, 128, decay)), ("latent_attention", latent),
+             ("retention", RetentionConfig(heads, 128, 128, decay, Rotation(10000.0, 128)))]
+    mlp = ExpertsConfig(ff, experts, top, groups, keep, shared_ff)
+    return NeruzenConfig(vocab=vocab, width=width, norm_eps=1e-6, bigram=BigramConfig(buckets, 40503, 9176),
+                         layers=tuple(LayerConfig(*kinds[i % 4], mlp) for i in range(layers)))
+
+
+def neruzen_bonerax(width, layers, heads, q_rank, window, experts, groups, keep, top, ff, shared_ff, buckets, vocab):
+    return bonerax_config(width, layers, heads, max(1, heads // 4), window, heads, experts, top, ff, vocab)
+
+
+def neruzen_nenotar(width, layers, heads, q_rank, window, experts, groups, keep, top, ff, shared_ff, buckets, vocab):
+    return nenotar_config(width, layers, heads, 3 * (top * ff + shared_ff) // 2, 3 * width // 2, 128, vocab)
+
+
+def neruzen_work(cfg, rows: int):
+    """(weights a step of `rows` rows multiplies a row by, weights it must read), both in elements; of routed experts a row
+    uses `top` and a step reads at most rows x top."""
+    used = read = 0.0
+    E = cfg.width
+    for layer in cfg.layers:
+        m = layer.mixer
+        if layer.type == "latent_attention":
+            mix = E * (m.q_rank + m.kv_rank + m.rot_dim) + m.q_rank * m.heads * (m.dim + m.rot_dim)
+            mix += m.heads * m.kv_rank * (m.dim + m.vdim) + m.heads * m.vdim * E
+        else:
+            mix = E * m.heads * (2 * m.dim + 3 * m.vdim)
+        used += mix
+        read += mix
+        f = layer.mlp
+        if f is not None:
+            fixed = E * f.experts + 3 * E * (f.shared_ff or 0)
+            used += fixed + f.top * 3 * E * f.ff
+            read += fixed + min(f.experts, rows * f.top) * 3 * E * f.ff
+    return used, read
+
+
+def neruzen_mixing_flops(cfg, T: int) -> float:
+    """Multiply-adds x 2 of the mixers' own work over a T-token prompt: scores and value products over the latents of the keys
+    a row sees; the states' decay, outer product and read-out a token."""
+    total = 0.0
+    for layer in cfg.layers:
+        m = layer.mixer
+        if layer.type == "latent_attention":
+            total += 2.0 * m.heads * (2 * m.kv_rank + m.rot_dim) * sum(min(t + 1, m.window) for t in range(T))
+        else:
+            total += T * m.heads * m.dim * m.vdim * 5.0
+    return total
+
+
 def _layer_mixers(layer):
     """(windowed attention or None, [recurrences as (heads, dim, vdim, delta?)]) of a Bonerax layer."""
     m = layer.mixer
@@ -272,6 +343,9 @@ def prompt_flops(engine, T) -> float:
     elif cfg.architecture == "Salipel":
         dense = 2.0 * T * salipel_work(cfg, T)[0] + 2.0 * vocab * engine.spec.hidden_size
         attn = salipel_mixing_flops(cfg, T)
+    elif cfg.architecture == "Neruzen":
+        dense = 2.0 * T * neruzen_work(cfg, T)[0] + 2.0 * vocab * engine.spec.hidden_size
+        attn = neruzen_mixing_flops(cfg, T)
     elif cfg.architecture == "Bonerax":
         attn = 0.0
         for layer in cfg.layers:
@@ -358,6 +432,8 @@ def measure(engine, torch, steps, warmup):
         need -= 2 * vocab * engine.spec.hidden_size                     # and of the embedding
         if cfg.architecture == "Salipel":
             need = 2 * (salipel_work(cfg, batch)[1] + vocab * engine.spec.hidden_size) + batch * cache_bytes_read(engine, CONTEXT - steps / 2)
+        if cfg.architecture == "Neruzen":
+            need = 2 * (neruzen_work(cfg, batch)[1] + vocab * engine.spec.hidden_size) + batch * cache_bytes_read(engine, CONTEXT - steps / 2)
         if cfg.architecture == "Givozen":       # weights by layer run; the head is the embedding's table, read whole
             need = 2 * (givozen_work(cfg, batch)[1] + vocab * engine.spec.hidden_size) + batch * cache_bytes_read(engine, CONTEXT - steps / 2)
         rec.update({f"decode_b{batch}_tok_s": round(batch / dt, 2), f"decode_b{batch}_ms": round(dt * 1e3, 4),
@@ -370,6 +446,8 @@ DESIGNS = {
     "bonerax": ("Bonerax", "MiniMax-M3 (GQA attention, routed SwiGLU experts)", BONERAX_SIZES, bonerax_config, bonerax_closest),
     "givozen": ("Givozen", "MiniMax-M3 (GQA attention, routed SwiGLU experts)", GIVOZEN_SIZES, givozen_config, givozen_closest),
     "salipel": ("Salipel", "MiniMax-M3 (GQA attention, routed SwiGLU experts)", SALIPEL_SIZES, salipel_config, salipel_closest),
+    "neruzen": ("Neruzen", "Bonerax (gated matrix states, windowed attention, routed SwiGLU experts)", NERUZEN_SIZES, neruzen_config, neruzen_bonerax,
+                ("closest_latent", "Nenotar (latent attention, minGRU, dense xIELU)", neruzen_nenotar)),
 }
 
 
@@ -378,15 +456,16 @@ def run(design: str, steps: int, warmup: int, sizes=None) -> dict:
     from llmx_amd import Engine, RandomInit
     if design not in DESIGNS:
         raise SystemExit(f"bench: no design named {design!r} (known: {sorted(DESIGNS)})")
-    title, closest, table, make_design, make_closest = DESIGNS[design]
+    title, closest, table, make_design, make_closest, *more = DESIGNS[design]
     result = {"design": title, "closest": closest, "dtype": "bf16", "prompt": PROMPT,
               "context": CONTEXT, "data": "synthetic: LCG token ids, N(0,0.02) weights generated on the device", "sizes": {}}
+    result.update({name: what for name, what, _ in more})
     for name in (sizes or DEFAULT_SIZES):
         if name not in table:
             raise SystemExit(f"bench: no size named {name!r} (known: {sorted(table)})")
         shape = table[name]
         per = {}
-        for which, make in ((design, make_design), ("closest", make_closest)):
+        for which, make in ((design, make_design), ("closest", make_closest), *((name, make) for name, _, make in more)):
             engine = Engine.from_random(make(*shape), RandomInit(seed=0, std=0.02), dtype="bfloat16", kv_tokens=8 * CONTEXT + 4 * PROMPT,
                                         page_tokens=16, max_requests=8)
             per[which] = measure(engine, torch, steps, max(2, warmup))

@@ -482,3 +482,25 @@ def test_a_long_portion_takes_the_wide_tiles_and_gives_the_bits_of_short_ones(wi
         rows.append(out.clone())
     engine.end_request("p")
     assert torch.equal(torch.cat(rows), whole)
+
+
+def test_the_collector_rests_while_a_step_is_recorded():
+    """A collection during a recording may free another engine's graphs, whose destructor synchronises the device; it is
+    switched off for the recording and back on afterwards."""
+    import gc
+    from llmx_amd.engine import StepEntry
+    engine = make_engine("A", "bfloat16")
+    seen = []
+    inner = engine._forward
+
+    def forward(step):
+        seen.append((torch.cuda.is_current_stream_capturing(), gc.isenabled()))
+        return inner(step)
+
+    engine._forward = forward
+    engine.add_request("r")
+    engine.step([StepEntry("r", tokens_for("A", 5, 1), [4])])
+    for t in tokens_for("A", 4, 2):
+        engine.step([StepEntry("r", [t], [0])])
+    assert (True, False) in seen and (True, True) not in seen and (False, True) in seen and gc.isenabled()
+    assert engine.graph_replays >= 2
