@@ -39,8 +39,73 @@ struct DecayedArgs {
 
 __device__ __forceinline__ f32x4_t mfma4(float a, float b, f32x4_t c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
+// A chunk's keys into LDS rows of LDK floats (channels from D on and rows from n on hold zeros).  VEC: 16-byte loads, as many in
+// flight as a thread has to bring (see state_keys4_load for what they ask for); otherwise value by value.
+template <int NU, int KIND, bool VEC, int LDK>
+__device__ __forceinline__ void stage_keys(const DecayedArgs& a, int row0, int n, int h, float* ks) {
+    constexpr int DP = 16 * NU;
+    const int tid = threadIdx.x;
+    if (VEC) {
+        constexpr int PER_ROW = DP / 4, PER_THREAD = DS_ROWS * PER_ROW / 256, TURN = PER_THREAD < 8 ? PER_THREAD : 8;
+#pragma unroll
+        for (int b = 0; b < PER_THREAD; b += TURN) {
+            StateKeys4 raw[TURN];
+#pragma unroll
+            for (int u = 0; u < TURN; ++u) {
+                const int i = tid + 256 * (b + u), j = i / PER_ROW, d = 4 * (i % PER_ROW);
+                const size_t row = (size_t)(row0 + min(j, n - 1));
+                raw[u] = state_keys4_load<KIND>(a.operands, a.k + row * a.ldk + (size_t)h * a.D, row, d < a.D ? d : 0);
+            }
+#pragma unroll
+            for (int u = 0; u < TURN; ++u) {
+                const int i = tid + 256 * (b + u), j = i / PER_ROW, d = 4 * (i % PER_ROW);
+                const state4_t x = state_keys4<KIND>(raw[u]);
+                *reinterpret_cast<state4_t*>(ks + j * LDK + d) = d < a.D && j < n ? x : state4_t{0.0f, 0.0f, 0.0f, 0.0f};
+            }
+        }
+        return;
+    }
+    for (int i = tid; i < DS_ROWS * DP; i += 256) {
+        const int j = i / DP, d = i % DP;
+        const size_t row = (size_t)(row0 + min(j, n - 1));
+        const float x = state_key<KIND>(a.operands, a.k + row * a.ldk + (size_t)h * a.D, row, min(d, a.D - 1));
+        ks[j * LDK + d] = d < a.D && j < n ? x : 0.0f;
+    }
+}
+
+// 64 value channels from v0 on of a chunk's rows, row j times weight(j).
+template <int KIND, bool VEC, int LDV, typename Weight>
+__device__ __forceinline__ void stage_values(const DecayedArgs& a, int row0, int n, int h, int v0, float* vs, Weight weight) {
+    const int tid = threadIdx.x;
+    if (VEC) {
+        state4_t raw[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int i = tid + 256 * u, j = i / 16, v = v0 + 4 * (i % 16);
+            const size_t row = (size_t)(row0 + min(j, n - 1));
+            raw[u] = *reinterpret_cast<const state4_t*>(a.v + row * a.ldv + (size_t)h * a.V + (v < a.V ? v : 0));
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int i = tid + 256 * u, j = i / 16, v = v0 + 4 * (i % 16);
+            const float w = j < n ? weight(j) : 0.0f;
+            state4_t x;
+#pragma unroll
+            for (int e = 0; e < 4; ++e) x[e] = v < a.V && j < n ? state_value<KIND>(raw[u][e]) * w : 0.0f;
+            *reinterpret_cast<state4_t*>(vs + j * LDV + 4 * (i % 16)) = x;
+        }
+        return;
+    }
+    for (int i = tid; i < DS_ROWS * 64; i += 256) {
+        const int j = i / 64, v = v0 + i % 64;
+        const size_t row = (size_t)(row0 + min(j, n - 1));
+        const float x = state_value<KIND>(a.v[row * a.ldv + (size_t)h * a.V + min(v, a.V - 1)]);
+        vs[j * LDV + i % 64] = v < a.V && j < n ? x * weight(j) : 0.0f;
+    }
+}
+
 // NU: a head's key channels in tiles of 16, padded
-template <int NU, int KIND>
+template <int NU, int KIND, bool VEC>
 __global__ void __launch_bounds__(256) decayed_sums_kernel(DecayedArgs a) {
     constexpr int DP = 16 * NU, LDK = DP + 16, LDV = 64 + 16;     // rows 16 banks apart: four rows' 16 neighbours meet no bank twice
     extern __shared__ __align__(16) float lds[];
@@ -51,18 +116,8 @@ __global__ void __launch_bounds__(256) decayed_sums_kernel(DecayedArgs a) {
     const int row0 = chunk[1], n = chunk[2], h = blockIdx.y, v0 = 64 * blockIdx.z;
     const float* pw = a.powers + (size_t)h * (DS_ROWS + 1);
     const int steps = (n + 3) / 4;
-    for (int i = tid; i < 4 * steps * DP; i += 256) {
-        const int j = i / DP, d = i % DP;
-        const size_t row = (size_t)(row0 + min(j, n - 1));
-        const float x = state_key<KIND>(a.operands, a.k + row * a.ldk + (size_t)h * a.D, row, min(d, a.D - 1));
-        ks[j * LDK + d] = d < a.D && j < n ? x : 0.0f;
-    }
-    for (int i = tid; i < 4 * steps * 64; i += 256) {
-        const int j = i / 64, v = v0 + i % 64;
-        const size_t row = (size_t)(row0 + min(j, n - 1));
-        const float x = state_value<KIND>(a.v[row * a.ldv + (size_t)h * a.V + min(v, a.V - 1)]);
-        vs[j * LDV + i % 64] = v < a.V && j < n ? x * pw[n - 1 - j] : 0.0f;
-    }
+    stage_values<KIND, VEC, LDV>(a, row0, n, h, v0, vs, [&](int j) { return pw[n - 1 - j]; });
+    stage_keys<NU, KIND, VEC, LDK>(a, row0, n, h, ks);
     __syncthreads();
     if (v0 + 16 * wave >= a.VR) return;
     f32x4_t acc[NU];
@@ -121,7 +176,7 @@ __global__ void __launch_bounds__(256) decayed_starts_kernel(DecayedArgs a) {
         if (v < a.V && d + i < a.D) to[8 * i] = S[i];
 }
 
-template <int NU, int KIND>
+template <int NU, int KIND, bool VEC>
 __global__ void __launch_bounds__(256) decayed_rows_kernel(DecayedArgs a) {
     constexpr int DP = 16 * NU, LDK = DP + 4, LDV = 64 + 4;
     extern __shared__ __align__(16) float lds[];
@@ -138,21 +193,34 @@ __global__ void __launch_bounds__(256) decayed_rows_kernel(DecayedArgs a) {
     {
         const size_t row = (size_t)(row0 + min(16 * wave + c, n - 1));
         const float* head = a.q + row * a.ldq + (size_t)h * a.D;
+        if (VEC) {
+            constexpr int TURN = NU < 8 ? NU : 8;
 #pragma unroll
-        for (int u = 0; u < NU; ++u)
+            for (int b = 0; b < NU; b += TURN) {
+                StateKeys4 raw[TURN];
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int d = 16 * u + 4 * g + e;
-                const float x = state_key<KIND>(a.operands, head, row, min(d, a.D - 1));
-                q[u][e] = d < a.D ? x : 0.0f;
+                for (int u = 0; u < TURN; ++u) {
+                    const int d = 16 * (b + u) + 4 * g;
+                    raw[u] = state_keys4_load<KIND>(a.operands, head, row, d < a.D ? d : 0);
+                }
+#pragma unroll
+                for (int u = 0; u < TURN; ++u) {
+                    const state4_t x = state_keys4<KIND>(raw[u]);
+                    q[b + u] = 16 * (b + u) + 4 * g < a.D ? x : state4_t{0.0f, 0.0f, 0.0f, 0.0f};
+                }
             }
+        } else {
+#pragma unroll
+            for (int u = 0; u < NU; ++u)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int d = 16 * u + 4 * g + e;
+                    const float x = state_key<KIND>(a.operands, head, row, min(d, a.D - 1));
+                    q[u][e] = d < a.D ? x : 0.0f;
+                }
+        }
     }
-    for (int i = tid; i < DS_ROWS * DP; i += 256) {
-        const int j = i / DP, d = i % DP;
-        const size_t row = (size_t)(row0 + min(j, n - 1));
-        const float x = state_key<KIND>(a.operands, a.k + row * a.ldk + (size_t)h * a.D, row, min(d, a.D - 1));
-        ks[j * LDK + d] = d < a.D && j < n ? x : 0.0f;
-    }
+    stage_keys<NU, KIND, VEC, LDK>(a, row0, n, h, ks);
     __syncthreads();
     // scores transposed: s[t][e] of key row 16 t + 4 g + e against query row 16 wave + c, t up to the wave's own tile
     f32x4_t s[4];
@@ -180,18 +248,26 @@ __global__ void __launch_bounds__(256) decayed_rows_kernel(DecayedArgs a) {
     const float* start = a.starts + ((size_t)blockIdx.x * a.H + h) * a.VR * a.DR;
     for (int v0 = 0; v0 < a.VR; v0 += 64) {
         __syncthreads();       // the keys, or the slice before, have been read by every wave
-        for (int i = tid; i < 64 * (DP / 4); i += 256) {
-            const int v = i / (DP / 4), d = 4 * (i % (DP / 4));
-            const bool in = v0 + v < a.VR && d < a.DR;
-            const f32x4_t x = *reinterpret_cast<const f32x4_t*>(start + (size_t)(in ? v0 + v : 0) * a.DR + (in ? d : 0));
-            *reinterpret_cast<f32x4_t*>(ks + v * LDK + d) = in ? x : f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+        {
+            constexpr int PER_ROW = DP / 4, PER_THREAD = 64 * PER_ROW / 256, TURN = PER_THREAD < 8 ? PER_THREAD : 8;
+#pragma unroll
+            for (int b = 0; b < PER_THREAD; b += TURN) {
+                f32x4_t x[TURN];
+#pragma unroll
+                for (int u = 0; u < TURN; ++u) {
+                    const int i = tid + 256 * (b + u), v = i / PER_ROW, d = 4 * (i % PER_ROW);
+                    const bool in = v0 + v < a.VR && d < a.DR;
+                    x[u] = *reinterpret_cast<const f32x4_t*>(start + (size_t)(in ? v0 + v : 0) * a.DR + (in ? d : 0));
+                    if (!in) x[u] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
+                }
+#pragma unroll
+                for (int u = 0; u < TURN; ++u) {
+                    const int i = tid + 256 * (b + u);
+                    *reinterpret_cast<f32x4_t*>(ks + (i / PER_ROW) * LDK + 4 * (i % PER_ROW)) = x[u];
+                }
+            }
         }
-        for (int i = tid; i < DS_ROWS * 64; i += 256) {
-            const int j = i / 64, v = v0 + i % 64;
-            const size_t row = (size_t)(row0 + min(j, n - 1));
-            const float x = state_value<KIND>(a.v[row * a.ldv + (size_t)h * a.V + min(v, a.V - 1)]);
-            vs[j * LDV + i % 64] = v < a.V && j < n ? x : 0.0f;
-        }
+        stage_values<KIND, VEC, LDV>(a, row0, n, h, v0, vs, [](int) { return 1.0f; });
         __syncthreads();
         f32x4_t o[4];
 #pragma unroll
@@ -235,20 +311,29 @@ __global__ void __launch_bounds__(256) decayed_rows_kernel(DecayedArgs a) {
     }
 }
 
-template <int NU, int KIND>
+template <int NU, int KIND, bool VEC>
 static int launch_decayed(const DecayedArgs& a, int n_chunks, int n_long, hipStream_t stream) {
     constexpr size_t lds_sums = sizeof(float) * DS_ROWS * (16 * NU + 16 + 64 + 16);
     constexpr size_t lds_rows = sizeof(float) * (DS_ROWS * (16 * NU + 4 + 64 + 4) + DS_ROWS + 1);
     static bool raised = false;
     if (!raised) {
-        if (hipFuncSetAttribute((const void*)decayed_sums_kernel<NU, KIND>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) return -1;
-        if (hipFuncSetAttribute((const void*)decayed_rows_kernel<NU, KIND>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) return -1;
+        if (hipFuncSetAttribute((const void*)decayed_sums_kernel<NU, KIND, VEC>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) return -1;
+        if (hipFuncSetAttribute((const void*)decayed_rows_kernel<NU, KIND, VEC>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) return -1;
         raised = true;
     }
-    hipLaunchKernelGGL((decayed_sums_kernel<NU, KIND>), dim3(n_chunks, a.H, (a.VR + 63) / 64), dim3(256), lds_sums, stream, a);
+    hipLaunchKernelGGL((decayed_sums_kernel<NU, KIND, VEC>), dim3(n_chunks, a.H, (a.VR + 63) / 64), dim3(256), lds_sums, stream, a);
     hipLaunchKernelGGL(decayed_starts_kernel, dim3((unsigned)(((size_t)a.H * a.VR * a.DR / 4 + 255) / 256), n_long), dim3(256), 0, stream, a);
-    hipLaunchKernelGGL((decayed_rows_kernel<NU, KIND>), dim3(n_chunks, a.H), dim3(256), lds_rows, stream, a);
+    hipLaunchKernelGGL((decayed_rows_kernel<NU, KIND, VEC>), dim3(n_chunks, a.H), dim3(256), lds_rows, stream, a);
     return LLMX_CHECK_LAUNCH();
+}
+
+template <int NU>
+static int launch_decayed_kind(const DecayedArgs& a, int kind, bool vec, int n_chunks, int n_long, hipStream_t stream) {
+    if (kind == STATE_OPERANDS_SILU)
+        return vec ? launch_decayed<NU, STATE_OPERANDS_SILU, true>(a, n_chunks, n_long, stream) : launch_decayed<NU, STATE_OPERANDS_SILU, false>(a, n_chunks, n_long, stream);
+    if (kind == STATE_OPERANDS_ROTATED)
+        return vec ? launch_decayed<NU, STATE_OPERANDS_ROTATED, true>(a, n_chunks, n_long, stream) : launch_decayed<NU, STATE_OPERANDS_ROTATED, false>(a, n_chunks, n_long, stream);
+    return vec ? launch_decayed<NU, STATE_OPERANDS_PLAIN, true>(a, n_chunks, n_long, stream) : launch_decayed<NU, STATE_OPERANDS_PLAIN, false>(a, n_chunks, n_long, stream);
 }
 
 extern "C" int llmx_decayed_state_rows(void) { return DS_ROWS; }
@@ -265,12 +350,10 @@ extern "C" int llmx_decayed_state_chunks(const float* q, int ldq, const float* k
     DecayedArgs a{q, k, v, ldq, ldk, ldv, powers, state, state_stride, slot_read, slot_write, chunks, entry_chunks, starts, out, out_scale,
                   H, D, V, DR, VR, StateOperands{cos_sin, pos, rot_dims}};
     llmx_note_launch(LK_DECAYED_STATE_CHUNKS);
-#define LLMX_DS(NU) \
-    (operands == STATE_OPERANDS_SILU ? launch_decayed<NU, STATE_OPERANDS_SILU>(a, n_chunks, n_long, stream) \
-     : operands == STATE_OPERANDS_ROTATED ? launch_decayed<NU, STATE_OPERANDS_ROTATED>(a, n_chunks, n_long, stream) \
-                                          : launch_decayed<NU, STATE_OPERANDS_PLAIN>(a, n_chunks, n_long, stream))
-    if (D <= 64) return LLMX_DS(4);
-    if (D <= 128) return LLMX_DS(8);
-    return LLMX_DS(16);
-#undef LLMX_DS
+    auto at16 = [](const void* p) { return ((uintptr_t)p & 15) == 0; };
+    bool vec = at16(q) && at16(k) && at16(v) && ldq % 4 == 0 && ldk % 4 == 0 && ldv % 4 == 0 && D % 4 == 0 && V % 4 == 0;
+    if (operands == STATE_OPERANDS_ROTATED) vec = vec && at16(cos_sin) && rot_dims % 8 == 0;
+    if (D <= 64) return launch_decayed_kind<4>(a, operands, vec, n_chunks, n_long, stream);
+    if (D <= 128) return launch_decayed_kind<8>(a, operands, vec, n_chunks, n_long, stream);
+    return launch_decayed_kind<16>(a, operands, vec, n_chunks, n_long, stream);
 }

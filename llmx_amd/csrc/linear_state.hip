@@ -232,7 +232,7 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
         if (tid < CH) betas[b][tid] = bstage;
     };
 
-    fetch(0);
+    // the state is asked for before the first chunk, whose values may wait for arithmetic of their own
     float S[R];
     const size_t tile_at = ((size_t)h * tiles + tile) * a.D * SCAN_COLS + c;
     {
@@ -244,6 +244,7 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
             S[i] = (col && d < a.D) ? x : 0.0f;
         }
     }
+    fetch(0);
     put(0);
     __syncthreads();
     const bool delta = a.beta != nullptr;
@@ -329,6 +330,99 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
     }
 }
 
+// Steps of single tokens without a delta correction: the same update and read-out, laid out for the way to memory.  A block
+// of CN waves takes STEP_TILES tiles of a head's state ([D][8] floats each, one run of memory): thread (chunk, lane) holds 4
+// columns of key channel 32 chunk + lane / 2 of every tile, 16-byte loads, all asked for before anything is computed; the
+// channels' products are then added in the scan's order (channels 64 apart, then 32, 16, .. 1 apart), so a row gets the
+// scan's bits.  Grid (H * ceil(tiles / STEP_TILES), entries); every entry has one row.
+#define STEP_TILES 4
+template <int CN, int KIND>
+__global__ void __launch_bounds__(64 * CN) state_step_kernel(StateScanArgs a) {
+    typedef float f32x4_t __attribute__((ext_vector_type(4)));
+    __shared__ __attribute__((aligned(16))) f32x4_t part[STEP_TILES][CN][64];
+    const int tid = threadIdx.x, chunk = tid >> 6, lane = tid & 63;
+    const int tiles = (a.V + SCAN_COLS - 1) / SCAN_COLS, blocks = (tiles + STEP_TILES - 1) / STEP_TILES;
+    const int h = blockIdx.x / blocks, tile0 = (blockIdx.x % blocks) * STEP_TILES, e = blockIdx.y;
+    const int d = 32 * chunk + (lane >> 1), half = lane & 1;
+    const bool live = d < a.D;
+    const int dd = live ? d : 0;
+    const size_t slot_r = (size_t)a.slot_read[e] * a.state_stride, slot_w = (size_t)a.slot_write[e] * a.state_stride;
+    const size_t at = ((size_t)h * tiles + tile0) * a.D * SCAN_COLS + (size_t)dd * SCAN_COLS + 4 * half;
+    const size_t tile_floats = (size_t)a.D * SCAN_COLS;
+    f32x4_t S[STEP_TILES];
+#pragma unroll
+    for (int u = 0; u < STEP_TILES; ++u)
+        S[u] = *reinterpret_cast<const f32x4_t*>(a.state + slot_r + at + (tile0 + u < tiles ? u : 0) * tile_floats);
+    const size_t row = (size_t)a.entry_rows[2 * e];
+    const int hq = h / a.share;
+    const float k = state_key<KIND>(a.operands, a.k + row * a.ldk + (size_t)hq * a.D, row, dd);
+    const float q = state_key<KIND>(a.operands, a.q + row * a.ldq + (size_t)hq * a.D, row, dd);
+    const float g = a.decay[row * a.ldg + (size_t)h * a.D + dd];
+    const float* vp = a.v + row * a.ldv + (size_t)h * a.V;
+    float v[STEP_TILES][4];
+#pragma unroll
+    for (int u = 0; u < STEP_TILES; ++u)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[u][i] = vp[min((tile0 + u) * SCAN_COLS + 4 * half + i, a.V - 1)];
+#pragma unroll
+    for (int u = 0; u < STEP_TILES; ++u) {
+        f32x4_t o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            S[u][i] = fmaf(k, state_value<KIND>(v[u][i]), S[u][i] * g);
+            o[i] = live ? q * S[u][i] : 0.0f;
+        }
+        part[u][chunk][lane] = o;
+        if (tile0 + u < tiles && live) {
+            // columns past V keep what they held
+            float* to = a.state + slot_w + at + u * tile_floats;
+            const int left = a.V - ((tile0 + u) * SCAN_COLS + 4 * half);
+            if (left >= 4) *reinterpret_cast<f32x4_t*>(to) = S[u];
+            else
+                for (int i = 0; i < left; ++i) to[i] = S[u][i];
+        }
+    }
+    __syncthreads();
+    for (int u = chunk; u < STEP_TILES; u += CN) {
+        const int tile = tile0 + u;
+        if (tile >= tiles) break;
+        f32x4_t o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            float x;
+            if (CN == 2) x = part[u][0][lane][i] + part[u][1 % CN][lane][i];
+            else if (CN == 4) x = (part[u][0][lane][i] + part[u][2 % CN][lane][i]) + (part[u][1 % CN][lane][i] + part[u][3 % CN][lane][i]);
+            else
+                x = ((part[u][0][lane][i] + part[u][2 % CN][lane][i]) + (part[u][4 % CN][lane][i] + part[u][6 % CN][lane][i])) +
+                    ((part[u][1 % CN][lane][i] + part[u][3 % CN][lane][i]) + (part[u][5 % CN][lane][i] + part[u][7 % CN][lane][i]));
+            uint32_t p0, p1;
+            halves_pair32(__float_as_uint(x), p0, p1);       // channels 16 apart
+            x = __uint_as_float(p0) + __uint_as_float(p1);
+            rows_pair16(__float_as_uint(x), p0, p1);         // 8 apart
+            x = __uint_as_float(p0) + __uint_as_float(p1);
+            x += row_rotate<8>(x);
+            x += row_rotate<4>(x);
+            x += row_rotate<2>(x);
+            o[i] = x * a.out_scale;
+        }
+        if (lane < 2) {
+            float* to = a.out + row * (size_t)a.H * a.V + (size_t)h * a.V + tile * SCAN_COLS + 4 * lane;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (tile * SCAN_COLS + 4 * lane + i < a.V) to[i] = o[i];
+        }
+    }
+}
+
+template <int CN>
+static void launch_state_step(const StateScanArgs& a, int operands, int n_entries, hipStream_t stream) {
+    const int tiles = (a.V + SCAN_COLS - 1) / SCAN_COLS;
+    const dim3 grid((unsigned)(a.H * ((tiles + STEP_TILES - 1) / STEP_TILES)), (unsigned)n_entries), block(64 * CN);
+    if (operands == STATE_OPERANDS_SILU) hipLaunchKernelGGL((state_step_kernel<CN, STATE_OPERANDS_SILU>), grid, block, 0, stream, a);
+    else if (operands == STATE_OPERANDS_ROTATED) hipLaunchKernelGGL((state_step_kernel<CN, STATE_OPERANDS_ROTATED>), grid, block, 0, stream, a);
+    else hipLaunchKernelGGL((state_step_kernel<CN, STATE_OPERANDS_PLAIN>), grid, block, 0, stream, a);
+}
+
 extern "C" int llmx_state_scan(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* decay, int ldg,
                                const float* beta, float* state, long state_stride, const int* slot_read, const int* slot_write,
                                const int* entry_rows, float* out, float out_scale, int n_entries, int H, int share, int D, int V,
@@ -340,6 +434,13 @@ extern "C" int llmx_state_scan(const float* q, int ldq, const float* k, int ldk,
     StateScanArgs a{q, k, v, decay, beta, ldq, ldk, ldv, ldg, state, state_stride, slot_read, slot_write, entry_rows, out, out_scale,
                     H, share, D, V, tail_src, tail_ld, tail_C, taps, tail_off, max_rows_here, StateOperands{cos_sin, pos, rot_dims}};
     const dim3 grid((unsigned)(H * ((V + SCAN_COLS - 1) / SCAN_COLS)), (unsigned)n_entries);
+    if (max_rows == 1 && !beta && taps <= 1 && state_stride % 4 == 0 && ((uintptr_t)state & 15) == 0) {
+        llmx_note_launch(LK_STATE_STEP);
+        if (D <= 64) launch_state_step<2>(a, operands, n_entries, stream);
+        else if (D <= 128) launch_state_step<4>(a, operands, n_entries, stream);
+        else launch_state_step<8>(a, operands, n_entries, stream);
+        return LLMX_CHECK_LAUNCH();
+    }
     llmx_note_launch(LK_STATE_SCAN);
     const int per_lane = (D + SCAN_LANES - 1) / SCAN_LANES;
     // steps of single decoded tokens stage chunks of two rows (a quarter of the LDS, so more blocks a compute unit); a
@@ -407,6 +508,36 @@ __global__ void __launch_bounds__(64 * WAVES) head_norm_gate_kernel(HeadNormArgs
         return x;
     };
     float ss = 0.0f;
+    // a workgroup's row of at most KEPT values a thread stays in registers, everything asked for before the sum is formed
+    constexpr int KEPT = 8;
+    if (WAVES > 1 && V <= NT * KEPT) {
+        const float* zr = a.z ? a.z + (size_t)t * a.ldz + (size_t)h * V : nullptr;
+        const float* w = a.w ? (a.w_wide ? a.w + (size_t)h * V : a.w) : nullptr;
+        float x[KEPT], z[KEPT], wk[KEPT];
+#pragma unroll
+        for (int u = 0; u < KEPT; ++u) {
+            const int j = lane + NT * u;
+            x[u] = j < V ? value(j) : 0.0f;
+            z[u] = j < V && zr ? zr[j] : 0.0f;
+            wk[u] = j < V && w ? w[j] : 1.0f;
+        }
+#pragma unroll
+        for (int u = 0; u < KEPT; ++u) ss = fmaf(x[u], x[u], ss);
+        const float r = 1.0f / sqrtf(block_sum<WAVES>(ss, scratch) / (float)V + a.eps);
+        TO* dst = out + ((size_t)t * H + h) * V;
+#pragma unroll
+        for (int u = 0; u < KEPT; ++u) {
+            const int j = lane + NT * u;
+            if (j < V) {
+                float y = x[u] * r;
+                if (w) y = y * wk[u];
+                if (zr) y = y * (a.gate == GATE_SIGMOID ? sigmoid_ls(z[u]) : z[u] * sigmoid_ls(z[u]));
+                if (a.post != 1.0f) y = y * a.post;
+                st(dst + j, y);
+            }
+        }
+        return;
+    }
     for (int j = lane; j < V; j += NT) {
         const float x = value(j);
         ss = fmaf(x, x, ss);

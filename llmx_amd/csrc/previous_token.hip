@@ -57,7 +57,7 @@ struct ShiftArgs {
     void* shifted;           // [T, n] in the activation type
     void* out;               // [T, n] in the activation type, or null: h itself
     float* out32;            // [T, n] or null: h unrounded
-    int n;
+    int rows, n;
 };
 
 __device__ __forceinline__ float shifted_value(float h, float before, float s) { return fmaf(before - h, s, h); }
@@ -77,72 +77,93 @@ __global__ void __launch_bounds__(256) token_shift_kernel(ShiftArgs a) {
 }
 
 // The norm and the shift in one launch: h = x * (r * w) with the bits of the norm kernel (1,024 threads a row, the sum in its
-// order); the row above is normed again by the same workgroup, from its own sum, with the bits its own workgroup gives it.
-// Rows of at most 1,024 * SHIFT_KEPT values stay in registers, both asked for before the first sum.
+// order).  A workgroup takes ROWS consecutive rows; the row above its first is normed again, from its own sum, with the bits
+// its own workgroup gives it (or comes from the state, normed already).  KEPT > 0: rows of at most 1,024 * KEPT values stay in
+// registers, all asked for before the first sum.
 #define SHIFT_THREADS 1024
-#define SHIFT_KEPT 8
-template <typename TO, bool KEPT>
+template <typename TO, int KEPT, int ROWS>
 __global__ void __launch_bounds__(SHIFT_THREADS) rmsnorm_shift_kernel(ShiftArgs a) {
-    __shared__ float scratch[2][SHIFT_THREADS / 64];
-    const int t = blockIdx.x, n = a.n;
-    const int e = a.row_entry[t], row0 = a.entry_rows[2 * e], rows = a.entry_rows[2 * e + 1];
-    const bool inside = t > row0;
-    const float* row = a.x + (size_t)t * n;
-    const float* above = inside ? row - n : a.state + (size_t)a.slot_read[e] * a.state_stride;
-    float v[SHIFT_KEPT], u[SHIFT_KEPT], w[SHIFT_KEPT], s[SHIFT_KEPT];
-    float sq = 0.0f, sq_above = 0.0f;
-    if (KEPT) {
+    constexpr int WAVES = SHIFT_THREADS / 64;
+    __shared__ float scratch[ROWS + 1][WAVES];
+    const int n = a.n, t0 = blockIdx.x * ROWS, last = min(t0 + ROWS, a.rows) - 1;
+    const int wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    // row u of the workgroup is the step's row t0 - 1 + u: u 0 is the row above the first
+    auto source = [&](int u) -> const float* {
+        const int t = min(t0 - 1 + u, last);
+        if (u == 0) {
+            const int e = a.row_entry[t0];
+            if (t0 == a.entry_rows[2 * e]) return a.state + (size_t)a.slot_read[e] * a.state_stride;
+        }
+        return a.x + (size_t)t * n;
+    };
+    constexpr int K = KEPT > 0 ? KEPT : 1;
+    float v[ROWS + 1][K], w[K], s[K];
+    if (KEPT > 0) {
 #pragma unroll
-        for (int k = 0; k < SHIFT_KEPT; ++k) {
+        for (int u = 0; u <= ROWS; ++u) {
+            const float* row = source(u);
+#pragma unroll
+            for (int k = 0; k < K; ++k) {
+                const int i = threadIdx.x + k * SHIFT_THREADS;
+                v[u][k] = i < n ? row[i] : 0.0f;
+            }
+        }
+#pragma unroll
+        for (int k = 0; k < K; ++k) {
             const int i = threadIdx.x + k * SHIFT_THREADS;
-            v[k] = i < n ? row[i] : 0.0f;
-            u[k] = i < n ? above[i] : 0.0f;
             w[k] = i < n ? a.norm_w[i] : 0.0f;
             s[k] = i < n ? a.shift[i] : 0.0f;
         }
-#pragma unroll
-        for (int k = 0; k < SHIFT_KEPT; ++k) {
-            sq = fmaf(v[k], v[k], sq);
-            sq_above = fmaf(u[k], u[k], sq_above);
-        }
-    } else {
-        sq = strided_squares<SHIFT_THREADS>(row, n);
-        if (inside) sq_above = strided_squares<SHIFT_THREADS>(above, n);
     }
-    // both sums with one barrier: a butterfly a wave, the waves in order
-    sq = wave_sum(sq);
-    sq_above = wave_sum(sq_above);
-    if ((threadIdx.x & 63) == 0) {
-        scratch[0][threadIdx.x >> 6] = sq;
-        scratch[1][threadIdx.x >> 6] = sq_above;
+#pragma unroll
+    for (int u = 0; u <= ROWS; ++u) {
+        float sq = 0.0f;
+        if (KEPT > 0) {
+#pragma unroll
+            for (int k = 0; k < K; ++k) sq = fmaf(v[u][k], v[u][k], sq);
+        } else {
+            sq = strided_squares<SHIFT_THREADS>(source(u), n);
+        }
+        sq = wave_sum(sq);
+        if (lane == 0) scratch[u][wave] = sq;
     }
     __syncthreads();
-    float sum = scratch[0][0], sum_above = scratch[1][0];
+    float r[ROWS + 1];
 #pragma unroll
-    for (int k = 1; k < SHIFT_THREADS / 64; ++k) {
-        sum += scratch[0][k];
-        sum_above += scratch[1][k];
+    for (int u = 0; u <= ROWS; ++u) {
+        float sum = scratch[u][0];
+#pragma unroll
+        for (int k = 1; k < WAVES; ++k) sum += scratch[u][k];
+        r[u] = 1.0f / sqrtf(sum / (float)n + a.eps);
     }
-    const float r = 1.0f / sqrtf(sum / (float)n + a.eps);
-    const float r_above = 1.0f / sqrtf(sum_above / (float)n + a.eps);
-    float* keep = t == row0 + rows - 1 ? a.state + (size_t)a.slot_write[e] * a.state_stride : nullptr;
-    auto finish = [&](int i, float x, float y, float wi, float si) {
-        const float h = x * (r * wi);
-        const float before = inside ? y * (r_above * wi) : y;        // a state's row is normed already
-        const size_t at = (size_t)t * n + i;
-        st((TO*)a.shifted + at, shifted_value(h, before, si));
-        if (a.out) st((TO*)a.out + at, h);
-        if (a.out32) a.out32[at] = h;
-        if (keep) keep[i] = h;
-    };
-    if (KEPT) {
 #pragma unroll
-        for (int k = 0; k < SHIFT_KEPT; ++k) {
-            const int i = threadIdx.x + k * SHIFT_THREADS;
-            if (i < n) finish(i, v[k], u[k], w[k], s[k]);
+    for (int u = 1; u <= ROWS; ++u) {
+        const int t = t0 - 1 + u;
+        if (t > last) break;
+        const int e = a.row_entry[t], row0 = a.entry_rows[2 * e], rows = a.entry_rows[2 * e + 1];
+        const bool inside = t > row0;
+        const float* opened = a.state + (size_t)a.slot_read[e] * a.state_stride;     // read where an entry begins
+        float* keep = t == row0 + rows - 1 ? a.state + (size_t)a.slot_write[e] * a.state_stride : nullptr;
+        auto finish = [&](int i, float x, float y, float wi, float si) {
+            const float h = x * (r[u] * wi);
+            const float before = inside ? y * (r[u - 1] * wi) : y;
+            const size_t at = (size_t)t * n + i;
+            st((TO*)a.shifted + at, shifted_value(h, before, si));
+            if (a.out) st((TO*)a.out + at, h);
+            if (a.out32) a.out32[at] = h;
+            if (keep) keep[i] = h;
+        };
+        if (KEPT > 0) {
+#pragma unroll
+            for (int k = 0; k < K; ++k) {
+                const int i = threadIdx.x + k * SHIFT_THREADS;
+                if (i < n) finish(i, v[u][k], inside || u == 1 ? v[u - 1][k] : opened[i], w[k], s[k]);
+            }
+        } else {
+            const float* row = a.x + (size_t)t * n;
+            const float* above = inside ? row - n : opened;
+            for (int i = threadIdx.x; i < n; i += SHIFT_THREADS) finish(i, row[i], above[i], a.norm_w[i], a.shift[i]);
         }
-    } else {
-        for (int i = threadIdx.x; i < n; i += SHIFT_THREADS) finish(i, row[i], above[i], a.norm_w[i], a.shift[i]);
     }
 }
 
@@ -152,7 +173,7 @@ extern "C" int llmx_token_shift(const float* x, const float* norm_w, float eps, 
                                 float* out32, int out_dtype, int rows, int n, hipStream_t stream) {
     if (rows <= 0 || n <= 0) return 0;
     if (state_stride < n || !shift || !state || !shifted) return -2;
-    ShiftArgs a{x, norm_w, eps, shift, state, state_stride, slot_read, slot_write, row_entry, entry_rows, shifted, out, out32, n};
+    ShiftArgs a{x, norm_w, eps, shift, state, state_stride, slot_read, slot_write, row_entry, entry_rows, shifted, out, out32, rows, n};
     if (!norm_w) {
         llmx_note_launch(LK_TOKEN_SHIFT);
         if (out_dtype == LLMX_F32) hipLaunchKernelGGL(token_shift_kernel<float>, dim3(rows), dim3(256), 0, stream, a);
@@ -160,14 +181,23 @@ extern "C" int llmx_token_shift(const float* x, const float* norm_w, float eps, 
         return LLMX_CHECK_LAUNCH();
     }
     llmx_note_launch(LK_RMSNORM_SHIFT);
-    const bool kept = n <= SHIFT_THREADS * SHIFT_KEPT;
-#define LLMX_RS(TO, KEPT) hipLaunchKernelGGL((rmsnorm_shift_kernel<TO, KEPT>), dim3(rows), dim3(SHIFT_THREADS), 0, stream, a)
-    if (out_dtype == LLMX_F32) {
-        if (kept) LLMX_RS(float, true);
-        else LLMX_RS(float, false);
+#define LLMX_RS(KEPT, ROWS) \
+    do { \
+        const dim3 grid((unsigned)((rows + ROWS - 1) / ROWS)); \
+        if (out_dtype == LLMX_F32) hipLaunchKernelGGL((rmsnorm_shift_kernel<float, KEPT, ROWS>), grid, dim3(SHIFT_THREADS), 0, stream, a); \
+        else hipLaunchKernelGGL((rmsnorm_shift_kernel<bf16_t, KEPT, ROWS>), grid, dim3(SHIFT_THREADS), 0, stream, a); \
+    } while (0)
+    // steps of many rows: a workgroup takes four rows where their values fit its registers
+    if (n <= SHIFT_THREADS * 2) {
+        if (rows >= 1024) LLMX_RS(2, 4);
+        else LLMX_RS(2, 1);
+    } else if (n <= SHIFT_THREADS * 4) {
+        if (rows >= 1024) LLMX_RS(4, 4);
+        else LLMX_RS(4, 1);
+    } else if (n <= SHIFT_THREADS * 8) {
+        LLMX_RS(8, 1);
     } else {
-        if (kept) LLMX_RS(bf16_t, true);
-        else LLMX_RS(bf16_t, false);
+        LLMX_RS(0, 1);
     }
 #undef LLMX_RS
     return LLMX_CHECK_LAUNCH();

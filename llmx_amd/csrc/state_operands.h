@@ -31,5 +31,44 @@ __device__ __forceinline__ float state_key(const StateOperands& o, const float* 
     }
     return x;
 }
+// Channels d .. d + 3 of such a head, d a multiple of 4 below D, with 16-byte loads: the head's start, its row stride and D are
+// multiples of 4 floats, and so is dims / 2.  The same operations as state_key.
+typedef float state4_t __attribute__((ext_vector_type(4)));
+struct StateKeys4 {
+    state4_t x, y, c, s;      // the channels, their partners, cos and sin of their pairs: asked for together, used later
+    bool turns, first;
+};
+template <int KIND>
+__device__ __forceinline__ StateKeys4 state_keys4_load(const StateOperands& o, const float* __restrict__ head, size_t row, int d) {
+    StateKeys4 k;
+    k.x = *reinterpret_cast<const state4_t*>(head + d);
+    if (KIND == STATE_OPERANDS_ROTATED) {
+        const int half = o.dims / 2;
+        k.turns = d < o.dims;
+        k.first = d < half;
+        const int i = k.turns ? (k.first ? d : d - half) : 0;
+        const float* cs = o.cos_sin + (size_t)o.pos[row] * o.dims;
+        k.y = *reinterpret_cast<const state4_t*>(head + (k.turns ? (k.first ? d + half : i) : d));
+        k.c = *reinterpret_cast<const state4_t*>(cs + i);
+        k.s = *reinterpret_cast<const state4_t*>(cs + half + i);
+    }
+    return k;
+}
+template <int KIND>
+__device__ __forceinline__ state4_t state_keys4(const StateKeys4& k) {
+    state4_t r = k.x;
+    if (KIND == STATE_OPERANDS_SILU) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) r[e] = silu_state(k.x[e]);
+    }
+    if (KIND == STATE_OPERANDS_ROTATED) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float turned = k.first ? fmaf(-k.y[e], k.s[e], k.x[e] * k.c[e]) : fmaf(k.y[e], k.s[e], k.x[e] * k.c[e]);
+            r[e] = k.turns ? turned : k.x[e];
+        }
+    }
+    return r;
+}
 template <int KIND>
 __device__ __forceinline__ float state_value(float v) { return KIND == STATE_OPERANDS_SILU ? silu_state(v) : v; }

@@ -83,6 +83,7 @@
     X(ATTENTION_RULES, "attention.rules")                                                                                 \
     X(ATTENTION_RULES_MERGE, "attention.rules_merge")                                                                     \
     X(ATTENTION_RULES_SHARED, "attention.rules_shared")                                                                   \
+    X(STATE_STEP, "state_step")                                                                                           \
     X(EMBED_BIGRAM, "embed_bigram")                                                                                       \
     X(TOKEN_SHIFT, "token_shift")                                                                                         \
     X(RMSNORM_SHIFT, "rmsnorm_shift")                                                                                     \

@@ -496,7 +496,7 @@ def test_which_kernels_a_serving_step_takes():
             assert seen["attention.rules_shared"] == 4 and seen["attention.rules"] == 4
         else:
             assert seen["attention.generic"] == 2 * 4
-        assert seen["memory_prep"] == 2 and seen["state_scan"] == 2
+        assert seen["memory_prep"] == 2 and seen["state_scan"] + seen.get("state_step", 0) == 2
         assert seen["head_norm_gate"] == 2 * 3                  # two layers of two maps and the memory's read-out
         assert seen["combine_rows"] == 2 * (4 + 1)              # every layer's join, and the side-by-side mixer's
         assert seen["rmsnorm"] >= 2 * 4                         # one norm a layer (and the model's, where a step wants rows)
