@@ -114,7 +114,8 @@ class NeruzenConfig:
         norm.finish((), ARCHITECTURE)
         embedding = r.child("embedding")
         b = embedding.child("bigram")
-        bigram = BigramConfig(buckets=b.integer("buckets"), mul_prev=b.integer("mul_prev", lo=0), mul_cur=b.integer("mul_cur", lo=0))
+        bigram = BigramConfig(buckets=b.integer("buckets"), mul_prev=b.integer("mul_prev", lo=0, hi=1 << 62),
+                              mul_cur=b.integer("mul_cur", lo=0, hi=1 << 62))
         b.finish((), ARCHITECTURE)
         embedding.finish((), ARCHITECTURE)
         raw_layers = r.raw("layers")
