@@ -148,6 +148,8 @@ __device__ __forceinline__ void route_row_256(const float (&x)[4], const float (
 // picks' sum (added in pick order) when `normalize` (1: a single softmax pick keeps its score; 2: it too is divided, so its
 // weight is 1: the softmax over the picked logits alone), then times `scale`.  A row with a non-finite key gets ids -1 and
 // weights 0.  Ids and weights come out in pick order, best first.
+// ldk: slots a row has in ids and weights, k or k + 1; the last of k + 1 holds expert number n_experts with weight 1: one that
+// every row runs.
 // `groups`: the picks come from some of the experts only (see RouteGroups).
 // `logit_bias` (optional): added to the logits (and kept in z) before anything else: a router whose bias is part of its
 // logits, so that scores and weights see it too.
@@ -156,20 +158,24 @@ __device__ __forceinline__ void route_row_256(const float (&x)[4], const float (
 __global__ void __launch_bounds__(64) route_topk_kernel(float* __restrict__ z, const float* __restrict__ parts, int slices, long slice_stride,
                                                        const float* __restrict__ bias, int* __restrict__ ids,
                                                        float* __restrict__ weights, int n_experts, int k, int score, int normalize,
-                                                       float scale, const float* __restrict__ logit_bias, RouteGroups groups) {
+                                                       float scale, const float* __restrict__ logit_bias, RouteGroups groups, int ldk) {
     __shared__ float s[ROUTE_MAX_EXPERTS];
     __shared__ float b[ROUTE_MAX_EXPERTS];
     __shared__ float chosen[ROUTE_MAX_K];
     const int r = blockIdx.x, lane = threadIdx.x;
     float* row = z + (size_t)r * n_experts;
+    if (ldk > k && lane == 0) {
+        ids[(size_t)r * ldk + k] = n_experts;
+        weights[(size_t)r * ldk + k] = 1.0f;
+    }
     if (n_experts <= 256 && k <= 64 && !logit_bias) {   // the row fits the wave's registers
         float x[4], bias_v[4], weight;
         int id;
         load_row_256(row, parts ? parts + (size_t)r * n_experts : nullptr, slices, slice_stride, bias, n_experts, lane, x, bias_v);
         route_row_256(x, bias_v, bias != nullptr, n_experts, k, normalize, scale, score, groups, lane, id, weight);
         if (lane < k) {
-            ids[(size_t)r * k + lane] = id;
-            weights[(size_t)r * k + lane] = weight;
+            ids[(size_t)r * ldk + lane] = id;
+            weights[(size_t)r * ldk + lane] = weight;
         }
         return;
     }
@@ -210,8 +216,8 @@ __global__ void __launch_bounds__(64) route_topk_kernel(float* __restrict__ z, c
     __syncthreads();
     if (!finite) {
         for (int j = lane; j < k; j += 64) {
-            ids[(size_t)r * k + j] = -1;
-            weights[(size_t)r * k + j] = 0.0f;
+            ids[(size_t)r * ldk + j] = -1;
+            weights[(size_t)r * ldk + j] = 0.0f;
         }
         return;
     }
@@ -251,7 +257,7 @@ __global__ void __launch_bounds__(64) route_topk_kernel(float* __restrict__ z, c
         }
         wave_best(best, at);
         if (lane == 0) {
-            ids[(size_t)r * k + j] = at;
+            ids[(size_t)r * ldk + j] = at;
             chosen[j] = s[at];
             b[at] = -INFINITY;  // taken: below every finite key, so never picked again while an untaken id is left (k <= experts)
         }
@@ -261,7 +267,7 @@ __global__ void __launch_bounds__(64) route_topk_kernel(float* __restrict__ z, c
         float total = 0.0f;
         for (int j = 0; j < k; ++j) total += chosen[j];
         const bool divide = normalize == 2 || (normalize && (score == SCORE_SIGMOID || k > 1));   // 2: also a single softmax pick (its weight is 1)
-        for (int j = 0; j < k; ++j) weights[(size_t)r * k + j] = (divide ? chosen[j] / total : chosen[j]) * scale;
+        for (int j = 0; j < k; ++j) weights[(size_t)r * ldk + j] = (divide ? chosen[j] / total : chosen[j]) * scale;
     }
 }
 
@@ -276,14 +282,14 @@ static bool route_groups(int count, int keep, int n_experts, int k, RouteGroups&
 
 extern "C" int llmx_route_topk(float* z, const float* parts, int slices, long slice_stride, const float* bias, int* ids, float* weights,
                                int rows, int n_experts, int k, int score, int normalize, float scale, const float* logit_bias,
-                               int group_count, int group_keep, hipStream_t stream) {
+                               int group_count, int group_keep, int slots, hipStream_t stream) {
     if (rows <= 0) return 0;
     RouteGroups groups;
-    if (!route_groups(group_count, group_keep, n_experts, k, groups)) return -2;
+    if (!route_groups(group_count, group_keep, n_experts, k, groups) || (slots != k && slots != k + 1)) return -2;
     if (n_experts > ROUTE_MAX_EXPERTS || k > ROUTE_MAX_K || k > n_experts || k <= 0 || (parts && (slices < 1 || slices > ROUTE_MAX_SLICES))) return -2;
     llmx_note_launch(LK_ROUTE_TOPK);
     hipLaunchKernelGGL(route_topk_kernel, dim3(rows), dim3(64), 0, stream, z, parts, slices, slice_stride, bias, ids, weights, n_experts, k, score,
-                       normalize, scale, logit_bias, groups);
+                       normalize, scale, logit_bias, groups, slots);
     return LLMX_CHECK_LAUNCH();
 }
 
@@ -532,7 +538,7 @@ extern "C" int llmx_moe_align(const int* ids, int n_pairs, int n_experts, int* c
 __global__ void __launch_bounds__(1024) route_topk_align_kernel(float* __restrict__ z, const float* __restrict__ parts, int slices,
                                                                long slice_stride, const float* __restrict__ bias,
                                                                int* __restrict__ ids, float* __restrict__ weights, int rows, int n_experts,
-                                                               int k, int score, int normalize, float scale, RouteGroups groups,
+                                                               int k, int score, int normalize, float scale, RouteGroups groups, int ldk,
                                                                int* __restrict__ counts, int* __restrict__ offsets, int* __restrict__ list,
                                                                int* __restrict__ active, int* __restrict__ n_active) {
     __shared__ int pair_expert[ALIGN_SMALL_PAIRS];
@@ -546,26 +552,31 @@ __global__ void __launch_bounds__(1024) route_topk_align_kernel(float* __restric
                      bias_v);
         route_row_256(x, bias_v, bias != nullptr, n_experts, k, normalize, scale, score, groups, lane, id, weight);
         if (lane < k) {
-            ids[(size_t)r * k + lane] = id;
-            weights[(size_t)r * k + lane] = weight;
-            pair_expert[r * k + lane] = id;
+            ids[(size_t)r * ldk + lane] = id;
+            weights[(size_t)r * ldk + lane] = weight;
+            pair_expert[r * ldk + lane] = id;
+        }
+        if (ldk > k && lane == 0) {
+            ids[(size_t)r * ldk + k] = n_experts;
+            weights[(size_t)r * ldk + k] = 1.0f;
+            pair_expert[r * ldk + k] = n_experts;
         }
     }
     __syncthreads();
-    align_in_block(pair_expert, rows * k, n_experts, cnt, offs, counts, offsets, list, active, n_active);
+    align_in_block(pair_expert, rows * ldk, n_experts + (ldk - k), cnt, offs, counts, offsets, list, active, n_active);
 }
 
 // At most 16 rows (a wave each), rows * k <= 1024, at most 256 experts and 64 picks.  Returns -2 otherwise.
 extern "C" int llmx_route_topk_align(float* z, const float* parts, int slices, long slice_stride, const float* bias, int* ids, float* weights,
-                                     int rows, int n_experts, int k, int score, int normalize, float scale, int group_count, int group_keep,
+                                     int rows, int n_experts, int k, int score, int normalize, float scale, int group_count, int group_keep, int slots,
                                      int* counts, int* offsets, int* list, int* active, int* n_active, hipStream_t stream) {
     if (rows <= 0) return 0;
     RouteGroups groups;
-    if (!route_groups(group_count, group_keep, n_experts, k, groups)) return -2;
-    if (rows > 16 || rows * k > ALIGN_SMALL_PAIRS || n_experts > 256 || k > 64 || k > n_experts || k <= 0) return -2;
+    if (!route_groups(group_count, group_keep, n_experts, k, groups) || (slots != k && slots != k + 1)) return -2;
+    if (rows > 16 || rows * slots > ALIGN_SMALL_PAIRS || n_experts > 256 || k > 64 || k > n_experts || k <= 0) return -2;
     if (parts && (slices < 1 || slices > ROUTE_MAX_SLICES)) return -2;
     llmx_note_launch(LK_ROUTE_TOPK_ALIGN);
     hipLaunchKernelGGL(route_topk_align_kernel, dim3(1), dim3(1024), 0, stream, z, parts, slices, slice_stride, bias, ids, weights, rows, n_experts, k,
-                       score, normalize, scale, groups, counts, offsets, list, active, n_active);
+                       score, normalize, scale, groups, slots, counts, offsets, list, active, n_active);
     return LLMX_CHECK_LAUNCH();
 }

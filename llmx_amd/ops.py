@@ -103,9 +103,9 @@ def _declare(h) -> None:
         "llmx_attention_rules_segment": [],
         "llmx_memory_prep": [P, I, I, I, I, I, P, P, F, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
         "llmx_paged_attention_mfma": [P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, P, I, P],
-        "llmx_route_topk": [P, P, I, L, P, P, P, I, I, I, I, I, F, P, I, I, P],
+        "llmx_route_topk": [P, P, I, L, P, P, P, I, I, I, I, I, F, P, I, I, I, P],
         "llmx_moe_align": [P, I, I, P, P, P, P, P, P, P, P],
-        "llmx_route_topk_align": [P, P, I, L, P, P, P, I, I, I, I, I, F, I, I, P, P, P, P, P, P],
+        "llmx_route_topk_align": [P, P, I, L, P, P, P, I, I, I, I, I, F, I, I, I, P, P, P, P, P, P],
         "llmx_gemm_skinny": [P, P, P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, I, L, I, P, P, F, I, I, P, I, F, P, P, I, P],
         "llmx_gemm_skinny_normed_ok": [I, I],
         "llmx_gemm_skinny_f32_normed_ok": [I, I],
@@ -1532,14 +1532,23 @@ def route_topk(z: torch.Tensor, bias: Optional[torch.Tensor], ids: torch.Tensor,
     `normalize`: False, True (the picks' weights are divided by their sum; a single softmax pick keeps its score), or
     "always" (a single softmax pick is divided too: the softmax over the picked logits alone).  `groups` = (count, keep): the
     experts form `count` equal groups of neighbours, and only those of the `keep` groups with the largest best pick key (score
-    plus bias) can be picked."""
+    plus bias) can be picked.  ids and weights may have k + 1 slots a row: the last then holds expert number `experts` with weight
+    1, one that every row runs."""
     rows, n_experts = z.shape
+    slots = _route_slots(ids, k)
     if n_experts > MAX_EXPERTS or k > MAX_TOP_K or k > n_experts:
         raise KernelError(f"route_topk takes at most {MAX_EXPERTS} experts and {MAX_TOP_K} picks, not {n_experts} and {k}")
     _check(lib().llmx_route_topk(_dev(z, "z", torch.float32), *_parts_args(z, parts), _dev(bias, "bias", torch.float32, (n_experts,)),
-                                 _dev(ids, "ids", torch.int32, (rows, k)), _dev(weights, "weights", torch.float32, (rows, k)),
+                                 _dev(ids, "ids", torch.int32, (rows, slots)), _dev(weights, "weights", torch.float32, (rows, slots)),
                                  rows, n_experts, k, score, 2 if normalize == "always" else 1 if normalize else 0, float(scale),
-                                 _dev(logit_bias, "logit_bias", torch.float32, (n_experts,)), *(groups or (0, 0)), _stream()), "route_topk")
+                                 _dev(logit_bias, "logit_bias", torch.float32, (n_experts,)), *(groups or (0, 0)), slots, _stream()), "route_topk")
+
+
+def _route_slots(ids: torch.Tensor, k: int) -> int:
+    """Slots a row has in ids and weights: its k picks, or one more for an expert that every row runs."""
+    if ids.dim() != 2 or ids.shape[1] not in (k, k + 1):
+        raise KernelError(f"routing: ids {tuple(ids.shape)} do not hold {k} picks, or {k + 1} slots, a row")
+    return ids.shape[1]
 
 
 def moe_align_scratch(n_pairs: int, n_experts: int) -> int:
@@ -1577,19 +1586,23 @@ def route_topk_align(z: torch.Tensor, bias: Optional[torch.Tensor], ids: torch.T
                      scratch: Optional[torch.Tensor] = None, tile_stats: Optional[torch.Tensor] = None,
                      logit_bias: Optional[torch.Tensor] = None, groups=None) -> None:
     """route_topk followed by moe_align; a step of at most 16 rows (at most 256 experts and 64 picks, no logit bias) does
-    both in one launch, with the same bits."""
+    both in one launch, with the same bits.  With k + 1 slots a row in ids and weights (see route_topk) the pairs of the expert that
+    every row runs are grouped with the others': counts [experts + 1] and so on."""
     rows, n_experts = z.shape
-    if rows <= 16 and rows * k <= 1024 and n_experts <= 256 and k <= 64 and logit_bias is None:
+    slots = _route_slots(ids, k)
+    groups_out = n_experts + slots - k
+    if rows <= 16 and rows * slots <= 1024 and n_experts <= 256 and k <= 64 and logit_bias is None:
         _check(lib().llmx_route_topk_align(
             _dev(z, "z", torch.float32), *_parts_args(z, parts), _dev(bias, "bias", torch.float32, (n_experts,)),
-            _dev(ids, "ids", torch.int32, (rows, k)),
-            _dev(weights, "weights", torch.float32, (rows, k)), rows, n_experts, k, score, 2 if normalize == "always" else 1 if normalize else 0,
-            float(scale), *(groups or (0, 0)), _dev(counts, "counts", torch.int32, (n_experts,)), _dev(offsets, "offsets", torch.int32, (n_experts + 1,)),
-            _dev(pairs, "pairs", torch.int32, (rows * k,)), _dev(active, "active", torch.int32, (n_experts,)),
+            _dev(ids, "ids", torch.int32, (rows, slots)),
+            _dev(weights, "weights", torch.float32, (rows, slots)), rows, n_experts, k, score, 2 if normalize == "always" else 1 if normalize else 0,
+            float(scale), *(groups or (0, 0)), slots, _dev(counts, "counts", torch.int32, (groups_out,)),
+            _dev(offsets, "offsets", torch.int32, (groups_out + 1,)), _dev(pairs, "pairs", torch.int32, (rows * slots,)),
+            _dev(active, "active", torch.int32, (groups_out,)),
             _dev(n_active, "n_active", torch.int32, (1,)), _stream()), "route_topk_align")
         return
     route_topk(z, bias, ids, weights, k, score, normalize, scale, parts, logit_bias, groups)
-    moe_align(ids, n_experts, counts, offsets, pairs, active, n_active, scratch, tile_stats)
+    moe_align(ids, groups_out, counts, offsets, pairs, active, n_active, scratch, tile_stats)
 
 
 def moe_combine(x: torch.Tensor, y: torch.Tensor, ids: torch.Tensor, weights: Optional[torch.Tensor], accumulate: bool = True) -> None:

@@ -55,7 +55,8 @@ class RoutedExperts(FeedForward):
     "input": sum_j expert_j(w_j h), the weight multiplying what the expert reads; the first product being linear, it is
     applied to both pre-activations before the unit); shared ({intermediate, limit (for clamped_glu), switch (bool)}: an
     expert of the same unit that every row runs, added to the routed sum, times sigmoid(W_switch h) (one number a row)
-    where it has a switch).  unit "relu2": an expert is W_down max(W_up h, 0)^2, with no gate tensor (no shared expert
+    where it has a switch; a shared expert of the routed ones' inner width, without a switch, is kept behind them in the same
+    tensors and goes through their launches as one more that every row runs).  unit "relu2": an expert is W_down max(W_up h, 0)^2, with no gate tensor (no shared expert
     or weight on the input is built for it); "geglu_tanh": the tanh form of gelu(gate) * up."""
     graph_safe = True
 
@@ -109,6 +110,10 @@ class RoutedExperts(FeedForward):
             raise ValueError("routed experts: a unit without a gate goes without a shared expert and with the weight on the output")
         if shared and (self.shared_width < 1 or (self.unit == ops.GLU_CLAMPED and not self.shared_limit > 0.0)):
             raise ValueError("routed experts: a shared expert has an inner width of at least 1 and, for the clamped unit, a positive limit")
+        # a shared expert that can go with the routed ones: as wide, no switch, one unit and limit (and its tensors listed one by one)
+        self._shared_alike = bool(shared) and self.shared_width == self.intermediate and not self.shared_switch and self.weight_on == "output" \
+            and self.shared_limit == self.limit and self.experts < MAX_EXPERTS and self.top_k < MAX_TOP_K
+        self.shared_joins = False
         self.per_expert = False
         self.w_router = self.bias = self.logit_bias = self.w_gate_up = self.w_down = None
         self.w_shared_gate_up = self.w_shared_down = self.w_switch = None
@@ -142,16 +147,18 @@ class RoutedExperts(FeedForward):
             raise ValueError(f"{self.prefix}experts holds both fused and per-expert tensors")
         # a design whose files hold a tensor an expert is listed so also where no file is at hand (random weights)
         self.per_expert = has_single or (self.files == "per_expert" and fused not in available)
+        self.shared_joins = self.per_expert and self._shared_alike
         if self.per_expert:
-            # each expert's tensors go from the host straight into their places in the fused tensors
-            down = nm("fused_down")
-            for e in range(X):
-                specs += [TensorSpec(nm("expert_gate", e=e), (F, E), into=(fused, (X, 2 * F, E), (e, slice(0, F)))),
-                          TensorSpec(nm("expert_up", e=e), (F, E), into=(fused, (X, 2 * F, E), (e, slice(F, 2 * F)))),
-                          TensorSpec(nm("expert_down", e=e), (E, F), into=(down, (X, E, F), (e,)))]
+            # each expert's tensors go from the host straight into their places in the fused tensors, a shared one's behind them
+            down, XS = nm("fused_down"), X + int(self.shared_joins)
+            for e in range(XS):
+                names = ("expert_gate", "expert_up", "expert_down") if e < X else ("shared_gate", "shared_up", "shared_down")
+                specs += [TensorSpec(nm(names[0], e=e), (F, E), into=(fused, (XS, 2 * F, E), (e, slice(0, F)))),
+                          TensorSpec(nm(names[1], e=e), (F, E), into=(fused, (XS, 2 * F, E), (e, slice(F, 2 * F)))),
+                          TensorSpec(nm(names[2], e=e), (E, F), into=(down, (XS, E, F), (e,)))]
         else:
             specs += [TensorSpec(fused, (X, 2 * F, E)), TensorSpec(nm("fused_down"), (X, E, F))]
-        if self.shared_width:
+        if self.shared_width and not self.shared_joins:
             S = self.shared_width
             shared = self.name("shared_gate_up")     # gate rows, then up rows, filled from the file's two tensors
             specs += [TensorSpec(nm("shared_gate"), (S, E), into=(shared, (2 * S, E), (slice(0, S),))),
@@ -170,7 +177,7 @@ class RoutedExperts(FeedForward):
         # per-expert files arrive fused too (see tensor_specs)
         self.w_gate_up = tensors[self.name(self.names["fused_gate_up"])]
         self.w_down = tensors[self.name(self.names["fused_down"])]
-        if self.shared_width:
+        if self.shared_width and not self.shared_joins:
             self.w_shared_gate_up = tensors[self.name("shared_gate_up")]
             self.w_shared_down = tensors[self.name(self.names["shared_down"])]
             if self.shared_switch:
@@ -184,37 +191,38 @@ class RoutedExperts(FeedForward):
 
     def forward(self, step, h, out, accumulate, h32=None):
         T, X, k = step.rows, self.experts, self.top_k
+        slots, groups = (k + 1, X + 1) if self.shared_joins else (k, X)      # a row's pairs, and the experts they are grouped by
         z = step.buf("experts.router_logits", (T, X), torch.float32)
         slices = ops.gemm_f32_slices(X, h32.shape[1])
         parts = step.buf("experts.router_parts", (slices, T, X), torch.float32) if slices > 1 else None
         ops.gemm_f32(h32, self.w_router, z, parts=parts)
-        ids = step.buf("experts.ids", (T, k), torch.int32)
-        weights = step.buf("experts.weights", (T, k), torch.float32)
-        counts = step.buf("experts.counts", (X,), torch.int32)
-        offsets = step.buf("experts.offsets", (X + 1,), torch.int32)
-        pairs = step.buf("experts.pairs", (T * k,), torch.int32)
-        active = step.buf("experts.active", (X,), torch.int32)
+        ids = step.buf("experts.ids", (T, slots), torch.int32)
+        weights = step.buf("experts.weights", (T, slots), torch.float32)
+        counts = step.buf("experts.counts", (groups,), torch.int32)
+        offsets = step.buf("experts.offsets", (groups + 1,), torch.int32)
+        pairs = step.buf("experts.pairs", (T * slots,), torch.int32)
+        active = step.buf("experts.active", (groups,), torch.int32)
         n_active = step.buf("experts.n_active", (1,), torch.int32)
-        need = ops.moe_align_scratch(T * k, X)
+        need = ops.moe_align_scratch(T * slots, groups)
         scratch = step.buf("experts.align_scratch", (need,), torch.int32) if need else None
         # for steps of many pairs the grouping also counts the experts' tiles of 128 rows, by which the products choose their tiles
-        tile_stats = step.buf("experts.tile_stats", (1,), torch.int32) if T * k >= ops.TILE_STATS_MIN_PAIRS else None
+        tile_stats = step.buf("experts.tile_stats", (1,), torch.int32) if T * slots >= ops.TILE_STATS_MIN_PAIRS else None
         ops.route_topk_align(z, self.bias, ids, weights, k, self.score, self.normalize, self.scale, counts, offsets, pairs, active, n_active,
                              parts=parts, scratch=scratch, tile_stats=tile_stats, logit_bias=self.logit_bias, groups=self.groups)
-        step.observe("routing", logits=z, ids=ids, weights=weights)
-        act = step.buf("experts.act", (T * k, self.intermediate), step.act_dtype)
+        step.observe("routing", logits=z, ids=ids[:, :k], weights=weights[:, :k])
+        act = step.buf("experts.act", (T * slots, self.intermediate), step.act_dtype)
         on_input = self.weight_on == "input"
         if self.plain_unit is not None:
-            ops.grouped_gemm(h, self.w_gate_up, act, offsets, pairs, k, ops.EPI_STORE, active, n_active, token_rows=T, tile_stats=tile_stats,
+            ops.grouped_gemm(h, self.w_gate_up, act, offsets, pairs, slots, ops.EPI_STORE, active, n_active, token_rows=T, tile_stats=tile_stats,
                              act=(self.plain_unit, None))
         else:
-            glu = ops.Glu(self.unit, self.limit, weights.view(T * k) if on_input else None)
-            ops.grouped_gemm(h, self.w_gate_up, act, offsets, pairs, k, ops.EPI_SWIGLU, active, n_active, token_rows=T, tile_stats=tile_stats,
+            glu = ops.Glu(self.unit, self.limit, weights.view(T * slots) if on_input else None)
+            ops.grouped_gemm(h, self.w_gate_up, act, offsets, pairs, slots, ops.EPI_SWIGLU, active, n_active, token_rows=T, tile_stats=tile_stats,
                              glu=glu, scratch=step.buf)
-        y = step.buf("experts.y", (T * k, self.hidden), torch.float32)
+        y = step.buf("experts.y", (T * slots, self.hidden), torch.float32)
         ops.grouped_gemm(act, self.w_down, y, offsets, pairs, 1, ops.EPI_STORE, active, n_active, token_rows=T, tile_stats=tile_stats)
         ops.moe_combine(out, y, ids, None if on_input else weights, accumulate)
-        if self.shared_width:
+        if self.shared_width and not self.shared_joins:
             # the shared expert: its switch is a factor on the rows its second product reads (that product is linear), so the
             # product can add straight into the routed sum
             switch = None

@@ -209,9 +209,9 @@ def _window_case(dtype, H, C, R, page, length, window, runs, sharp=None, row_maj
     cache = torch.zeros(n_pages + 4, page, width, device="cuda", dtype=dtype)
     cache_t = torch.zeros(n_pages + 4, C, page, device="cuda", dtype=dtype)
     cd, rd = dev(c, dtype), dev(r, dtype)
-    for p in range(length):
-        cache[order[p // page], p % page, :C] = cd[p]
-        cache[order[p // page], p % page, C:C + R] = rd[p]
+    at = torch.tensor([order[p // page] * page + p % page for p in range(length)], device="cuda")
+    cache.view(-1, width)[at, :C] = cd
+    cache.view(-1, width)[at, C:C + R] = rd
     cache_t.copy_(cache[:, :, :C].transpose(1, 2))
     qld, qrd = dev(ql, dtype), dev(qr, dtype)
     scale = 0.4 / (C + R) ** 0.5 * 3
@@ -273,10 +273,10 @@ def test_one_key_on_both_sides_of_every_edge(dtype, decoded):
     """The row's queries fit one key: the first and last of the window and their neighbours outside and inside, page and segment
     borders, the row itself; windows that end on, before and behind such borders."""
     length = 300
-    for window in (1, 2, 63, 64, 65, 87, 112, 200):
+    for window in (1, 64, 65, 87, 200):
         row = 281
         lo = row - window + 1
-        for key in sorted({max(0, lo - 2), max(0, lo - 1), lo, lo + 1, row - 1, row, 255, 256, 271, 272, 192}):
+        for key in sorted({max(0, lo - 2), max(0, lo - 1), lo, lo + 1, row - 1, row, 255, 256, 192}):
             if key > row:
                 continue
             for C, R, page in ((32, 32, 16), (48, 8, 16), (10, 6, 4)):
@@ -435,6 +435,15 @@ def test_routing_by_groups_picks_and_weights(case):
     ids1, w1 = torch.empty(n, k, device="cuda", dtype=torch.int32), torch.empty(n, k, device="cuda")
     o.route_topk_align(dev(z[:n]), None, ids1, w1, k, o.SCORE_SOFTMAX, "always", 1.0, *arrays(), groups=(G, keep))
     assert torch.equal(ids1, ids[:n]) and torch.equal(w1, w[:n])
+    # one slot more: expert number X with weight 1, grouped with the others
+    more, w_more = torch.empty(rows, k + 1, device="cuda", dtype=torch.int32), torch.empty(rows, k + 1, device="cuda")
+    for r in (n, rows):
+        counts, offsets, pairs, active, n_active = (torch.empty(s, device="cuda", dtype=torch.int32) for s in (X + 1, X + 2, r * (k + 1), X + 1, 1))
+        if X < 1024:
+            o.route_topk_align(dev(z[:r]), None, more[:r], w_more[:r], k, o.SCORE_SOFTMAX, "always", 1.0, counts, offsets, pairs, active, n_active, groups=(G, keep))
+            assert torch.equal(more[:r, :k], ids[:r]) and bool((more[:r, k] == X).all()) and bool((w_more[:r, k] == 1).all())
+            assert int(counts[X]) == r and pairs[int(offsets[X]):].tolist() == [t * (k + 1) + k for t in range(r)]
+            assert all(more[:r].flatten()[pairs[int(offsets[e]):int(offsets[e + 1])].long()].eq(e).all() for e in range(X + 1))
     one, none = torch.empty_like(ids), torch.empty_like(ids)
     o.route_topk(dev(z), None, one, w, k, o.SCORE_SOFTMAX, "always", 1.0, groups=(1, 1))
     o.route_topk(dev(z), None, none, w, k, o.SCORE_SOFTMAX, "always", 1.0)
@@ -664,6 +673,9 @@ def test_which_kernels_a_serving_step_takes():
         for s in seen:
             assert s["embed_bigram"] == 1 and s["rmsnorm_shift"] == 4 and s["latent_prep"] == 4 and s["head_norm_gate"] == 2 and s["moe_combine"] == 3
             assert s["rmsnorm"] == 1 and "scale_add" not in s and "combine_rows" not in s and "token_shift" not in s and "head_gate" not in s
+        # the shared expert of layer 3 is as wide as the routed ones and goes through their launches, layer 0's has its own
+        if dtype == "bfloat16":
+            assert seen[2]["gemm_skinny.grouped"] == 3 * 2 + 2 * 2
         assert seen[0]["decayed_state.chunks"] == 2 and "state_scan" not in seen[0]
         assert seen[1]["state_scan"] == 2 and seen[2]["state_step"] == 2
         assert seen[0]["route_topk"] == 3 and seen[2]["route_topk_align"] == 3
