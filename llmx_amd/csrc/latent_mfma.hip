@@ -292,12 +292,15 @@ __global__ void __launch_bounds__(256) latent_attention_merge_kernel(const int* 
 // the first product, and the item stores its sums, maximum and sum of weights for the join.
 #define LW_LDW 68     // floats a column's 64 weights take in LDS (padded)
 
-template <int DPW, int LW_TILES, int KS>    // dim tiles of 16 a wave owns; column tiles; k-steps whose key loads are in flight together
+// PIPE (prompt portions whose keys have KS k-steps and latents 64 DPW values): all of a segment's keys are asked for while the segment before
+// is worked on, its values while its scores are formed, the page ids a segment ahead of both; one wave a SIMD has the
+// registers for it and nothing else to hide a load behind.
+template <int DPW, int LW_TILES, int KS, bool PIPE>    // dim tiles of 16 a wave owns; column tiles; k-steps whose key loads are in flight together
 __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaArgs a) {
     constexpr int COLS = 16 * LW_TILES;
-    constexpr bool EARLY_VALUES = LW_TILES == 1;
+    constexpr bool EARLY_VALUES = LW_TILES == 1 && !PIPE;
     extern __shared__ __align__(16) bf16_t qs[];   // [64][ldc + 8], then the weights and the waves' maxima
-    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, col = lane & 15, g = lane >> 4;
+    const int tid = threadIdx.x, wave = __builtin_amdgcn_readfirstlane(tid >> 6), lane = tid & 63, col = lane & 15, g = lane >> 4;
     const int* item = a.items + LM_ITEM_INTS * (size_t)blockIdx.x;
     const int row0 = item[0], rows = item[1], head0 = item[2], heads = item[3], slot = item[6];
     const int C = a.C, R = a.R, CR = a.ldc, ldq = CR + 8, pt = a.page_tokens;
@@ -359,14 +362,30 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
         for (int dt = 0; dt < DPW; ++dt) o[ct][dt] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
     }
 
+    // where a segment's key of this lane and its two groups of eight values begin, in cache rows and in values
+    auto key_row = [&](int seg) {
+        const int key = min(max(seg + 16 * wave + col, range.lo_min), p_max);
+        return (size_t)table[key / pt] * pt + key % pt;
+    };
+    auto value_at = [&](int seg, int c) {
+        const int key0 = min(max(seg + 32 * c + 8 * g, first_group), last_group);
+        return ((size_t)table[key0 / pt] * C + col) * pt + key0 % pt;
+    };
+    bf16x8_t kn[PIPE ? KS : 1];
+    size_t k_next = 0, v_now[2] = {0, 0}, v_next[2] = {0, 0};
+    if (PIPE) {
+        const bf16_t* kp = a.cache + key_row(key_begin) * CR + 8 * g;
+        v_next[0] = value_at(key_begin, 0);
+        v_next[1] = value_at(key_begin, 1);
+#pragma unroll
+        for (int j = 0; j < (PIPE ? KS : 0); ++j) kn[j] = *reinterpret_cast<const bf16x8_t*>(kp + 32 * j);
+    }
     for (int seg0 = key_begin; seg0 <= key_last; seg0 += LM_SEG) {
         const int buf = (seg0 / LM_SEG) & 1;
         float* wbuf = ws + buf * COLS * LW_LDW;
         float* mbuf = pmax + buf * 4 * COLS;
         // scores of this wave's 16 keys (key 16 wave + lane % 16 in the tile's row lane % 16) against the four tiles
-        int key = seg0 + 16 * wave + col;
-        key = min(max(key, range.lo_min), p_max);
-        const bf16_t* kp = a.cache + ((size_t)table[key / pt] * pt + key % pt) * CR + 8 * g;
+        const bf16_t* kp = PIPE ? nullptr : a.cache + key_row(seg0) * CR + 8 * g;
         f32x4_t s[LW_TILES];
 #pragma unroll
         for (int ct = 0; ct < LW_TILES; ++ct) s[ct] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
@@ -374,20 +393,43 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
         // with the keys, and wait for nothing but the page ids
         bf16x8_t vf[2][DPW];
         auto value_loads = [&](int c) {
-            int key0 = seg0 + 32 * c + 8 * g;
-            key0 = min(max(key0, first_group), last_group);
-            const bf16_t* vp = a.cache_t + ((size_t)table[key0 / pt] * C + col) * pt + key0 % pt;
+            const bf16_t* vp = a.cache_t + (PIPE ? v_now[c] : value_at(seg0, c));
 #pragma unroll
             for (int dt = 0; dt < DPW; ++dt) {
-                const int tile = 16 * (wave * DPW + dt) < C ? wave * DPW + dt : 0;
+                const int tile = PIPE || 16 * (wave * DPW + dt) < C ? wave * DPW + dt : 0;
                 vf[c][dt] = *reinterpret_cast<const bf16x8_t*>(vp + (size_t)16 * tile * pt);
             }
         };
-        if (EARLY_VALUES) {
-            value_loads(0);
-            value_loads(1);
+        if (PIPE) {
+            v_now[0] = v_next[0];
+            v_now[1] = v_next[1];
+            const int after = seg0 + LM_SEG <= key_last ? seg0 + LM_SEG : seg0;     // past the end: the last segment's again, never used
+            k_next = key_row(after);
+            v_next[0] = value_at(after, 0);
+            v_next[1] = value_at(after, 1);
         }
-        for (int st0 = 0; st0 < steps; st0 += KS) {
+        if (PIPE) __builtin_amdgcn_sched_barrier(0);     // the phases' loads stay in this order, and no phase's operands are brought before it
+        if (EARLY_VALUES || PIPE) value_loads(0);
+        if (PIPE) __builtin_amdgcn_sched_barrier(0);
+        if (EARLY_VALUES) value_loads(1);
+        if (PIPE) {
+#pragma unroll
+            for (int j = 0; j < (PIPE ? KS : 0); ++j) {
+#pragma unroll
+                for (int ct = 0; ct < LW_TILES; ++ct) {
+                    const uint4 q = *reinterpret_cast<const uint4*>(qs + (16 * ct + col) * ldq + 32 * j + 8 * g);
+                    s[ct] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kn[j], __builtin_bit_cast(bf16x8_t, q), s[ct], 0, 0, 0);
+                }
+                if (j % 2 == 1) __builtin_amdgcn_sched_barrier(0);
+            }
+            value_loads(1);
+            __builtin_amdgcn_sched_barrier(0);
+            const bf16_t* np = a.cache + k_next * CR + 8 * g;
+#pragma unroll
+            for (int j = 0; j < (PIPE ? KS : 0); ++j) kn[j] = *reinterpret_cast<const bf16x8_t*>(np + 32 * j);
+            __builtin_amdgcn_sched_barrier(0);
+        }
+        for (int st0 = PIPE ? steps : 0; st0 < steps; st0 += KS) {
             bf16x8_t kf[KS];
 #pragma unroll
             for (int j = 0; j < KS; ++j) kf[j] = *reinterpret_cast<const bf16x8_t*>(kp + 32 * (st0 + j < steps ? st0 + j : steps - 1));
@@ -452,10 +494,10 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
         }
 #pragma unroll
         for (int c = 0; c < 2; ++c) {
-            if (!EARLY_VALUES) value_loads(c);
+            if (!EARLY_VALUES && !PIPE) value_loads(c);
 #pragma unroll
             for (int dt = 0; dt < DPW; ++dt)
-                if (16 * (wave * DPW + dt) < C) {
+                if (PIPE || 16 * (wave * DPW + dt) < C) {
 #pragma unroll
                     for (int ct = 0; ct < LW_TILES; ++ct) o[ct][dt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[c][dt], pf[ct][c], o[ct][dt], 0, 0, 0);
                 }
@@ -506,30 +548,33 @@ extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, 
     if (n_merges > 0 && (!merges || !part_o || !part_ml)) return -2;
     LatentMfmaArgs a{(const bf16_t*)q_lat, (const bf16_t*)q_rot, (const bf16_t*)cache, (const bf16_t*)cache_t, pos, row_entry, tables, items,
                      (bf16_t*)out, part_o, part_ml, scale, T, H, C, R, ldc, page_tokens, max_blocks, window, row_major};
-#define LLMX_LT(DPW, TILES, KS, count, first)                                                                                        \
+#define LLMX_LT(DPW, TILES, KS, PIPE, count, first)                                                                                        \
     {                                                                                                                                 \
         static bool raised = false;                                                                                                   \
         if (!raised) {                                                                                                                \
-            if (hipFuncSetAttribute((const void*)latent_attention_tiles_kernel<DPW, TILES, KS>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) return -1; \
+            if (hipFuncSetAttribute((const void*)latent_attention_tiles_kernel<DPW, TILES, KS, PIPE>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) return -1; \
             raised = true;                                                                                                            \
         }                                                                                                                             \
         a.items = items + LM_ITEM_INTS * (size_t)(first);                                                                             \
         const size_t lds = sizeof(bf16_t) * 16 * TILES * (size_t)(ldc + 8) + sizeof(float) * (2 * 16 * TILES * LW_LDW + 2 * 4 * 16 * TILES); \
-        hipLaunchKernelGGL((latent_attention_tiles_kernel<DPW, TILES, KS>), dim3(count), dim3(256), lds, stream, a);                 \
+        hipLaunchKernelGGL((latent_attention_tiles_kernel<DPW, TILES, KS, PIPE>), dim3(count), dim3(256), lds, stream, a);                 \
     }
     if (n_tile_items > 0) {      // the list's first items: four column tiles each, a workgroup of four waves
         llmx_note_launch(LK_LATENT_ATTENTION_TILES);
-        if (C <= 64) LLMX_LT(1, 4, 6, n_tile_items, 0)
-        else if (C <= 128) LLMX_LT(2, 4, 6, n_tile_items, 0)
-        else if (C <= 256) LLMX_LT(4, 4, 6, n_tile_items, 0)
-        else LLMX_LT(8, 4, 6, n_tile_items, 0)
+        const int steps = ldc / 32;
+        if (C == 512 && steps == 18) LLMX_LT(8, 4, 18, true, n_tile_items, 0)
+        else if (C == 256 && steps == 10) LLMX_LT(4, 4, 10, true, n_tile_items, 0)
+        else if (C <= 64) LLMX_LT(1, 4, 6, false, n_tile_items, 0)
+        else if (C <= 128) LLMX_LT(2, 4, 6, false, n_tile_items, 0)
+        else if (C <= 256) LLMX_LT(4, 4, 6, false, n_tile_items, 0)
+        else LLMX_LT(8, 4, 6, false, n_tile_items, 0)
     }
     if (n_row_items > 0) {       // then the decoded rows' items: one column tile, a workgroup of four waves
         llmx_note_launch(LK_LATENT_ATTENTION_ROWS);
-        if (C <= 64) LLMX_LT(1, 1, 18, n_row_items, n_tile_items)
-        else if (C <= 128) LLMX_LT(2, 1, 18, n_row_items, n_tile_items)
-        else if (C <= 256) LLMX_LT(4, 1, 18, n_row_items, n_tile_items)
-        else LLMX_LT(8, 1, 18, n_row_items, n_tile_items)
+        if (C <= 64) LLMX_LT(1, 1, 18, false, n_row_items, n_tile_items)
+        else if (C <= 128) LLMX_LT(2, 1, 18, false, n_row_items, n_tile_items)
+        else if (C <= 256) LLMX_LT(4, 1, 18, false, n_row_items, n_tile_items)
+        else LLMX_LT(8, 1, 18, false, n_row_items, n_tile_items)
     }
 #undef LLMX_LT
     if (n_items > 0) {

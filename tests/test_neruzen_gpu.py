@@ -248,7 +248,8 @@ ATT_TOL = {torch.float32: 2e-5, torch.bfloat16: 2e-2}
 
 @pytest.mark.parametrize("dtype", DTYPES, ids=DTYPE_IDS)
 @pytest.mark.parametrize("case", [(4, 48, 8, 16, 150, 40), (3, 10, 6, 4, 60, 5), (16, 32, 32, 16, 300, 101), (20, 96, 32, 16, 200, 64), (2, 64, 16, 16, 140, 65),
-                                  (5, 128, 64, 32, 400, 129), (16, 512, 64, 16, 700, 300), (8, 16, 8, 8, 90, 1), (1, 16, 0, 48, 500, 2), (6, 64, 8, 16, 200, 1000)],
+                                  (5, 128, 64, 32, 400, 129), (16, 512, 64, 16, 700, 300), (8, 16, 8, 8, 90, 1), (1, 16, 0, 48, 500, 2), (6, 64, 8, 16, 200, 1000),
+                                  (7, 256, 64, 16, 330, 170)],
                          ids=lambda c: "x".join(map(str, c)))
 def test_windowed_attention_over_shuffled_pages(dtype, case):
     H, C, R, page, length, window = case
