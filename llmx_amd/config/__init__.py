@@ -7,5 +7,7 @@ from .bonerax import BoneraxConfig
 from .givozen import GivozenConfig
 from .salipel import SalipelConfig
 from .neruzen import NeruzenConfig
+from .vivulorn import VivulornConfig
 
-__all__ = ["ConfigError", "KeyReader", "read_json", "MiniMaxM3Config", "NenotarConfig", "BoneraxConfig", "GivozenConfig", "SalipelConfig", "NeruzenConfig"]
+__all__ = ["ConfigError", "KeyReader", "read_json", "MiniMaxM3Config", "NenotarConfig", "BoneraxConfig", "GivozenConfig", "SalipelConfig", "NeruzenConfig",
+           "VivulornConfig"]

@@ -12,7 +12,7 @@ enum : int { QKNORM_NONE = 0, QKNORM_PROJECTION = 1, QKNORM_HEAD = 2 };
 #define ATT_PREP_MAX_D 256
 
 struct QkvArgs {
-    const float* qkv;  // [T, q_width + 2 kv_width] f32: q | k | v
+    const float* qkv;  // [T, ld] f32: q | k | v at a row's start
     const float* q_weight;
     const float* k_weight;
     const float* cos_sin;  // [positions, rotary_dim] f32: cos of the rotary_dim/2 pairs, then sin
@@ -26,6 +26,7 @@ struct QkvArgs {
     int n_heads, n_kv_heads, head_dim, rotary_dim, norm_mode;
     int page_tokens, max_blocks, write_kv;
     int q_slices, k_slices;  // blocks that share a row's q (k) projection: each norms with the whole sum and writes its slice
+    int ld, v_dim;           // row stride of qkv; a value head's width
     int pairing;             // which dims of a head rotate together: ROPE_HALVES (i, i + R/2) or ROPE_INTERLEAVED (2i, 2i + 1)
 };
 
@@ -59,7 +60,7 @@ __global__ void __launch_bounds__(256) qknorm_rope_kvwrite_kernel(QkvArgs a) {
     const int t = blockIdx.x;
     const int D = a.head_dim;
     const int qw = a.n_heads * D, kw = a.n_kv_heads * D;
-    const float* row = a.qkv + (size_t)t * (qw + 2 * kw);
+    const float* row = a.qkv + (size_t)t * a.ld;
     const int p = a.pos[t];
     const float* cs = a.cos_sin + (size_t)p * a.rotary_dim;
     const bool normed = a.norm_mode != QKNORM_NONE;
@@ -94,8 +95,13 @@ __global__ void __launch_bounds__(256) qknorm_rope_kvwrite_kernel(QkvArgs a) {
         const int h = i / D, d = i % D;
         const size_t head_at = (size_t)page * a.n_kv_heads + h;
         st(kc + (head_at * a.page_tokens + slot) * D + d, normed_rotated(krow, a.k_weight, cs, i, D, a.rotary_dim, normed, r, a.pairing));
-        st(vc + (head_at * D + d) * a.page_tokens + slot, krow[kw + i]);
+        if (a.v_dim == D) st(vc + (head_at * D + d) * a.page_tokens + slot, krow[kw + i]);
     }
+    if (a.v_dim == D) return;
+    const int vw = a.n_kv_heads * a.v_dim, v_per = (vw + a.k_slices - 1) / a.k_slices;      // values of a width of their own
+    const int v_begin = ((int)blockIdx.y - a.q_slices) * v_per, v_end = min(vw, v_begin + v_per);
+    for (int i = v_begin + threadIdx.x; i < v_end; i += 256)
+        st(vc + (((size_t)page * a.n_kv_heads + i / a.v_dim) * a.v_dim + i % a.v_dim) * a.page_tokens + slot, krow[kw + i]);
 }
 
 // The form for many rows (prompt portions): one block norms and rotates a row's q, another its k and writes k and v.
@@ -175,7 +181,7 @@ __global__ void __launch_bounds__(256) qknorm_rope_kvwrite_rows_kernel(QkvArgs a
     const int t = blockIdx.x, tid = threadIdx.x;
     const int D = a.head_dim;
     const int qw = a.n_heads * D, kw = a.n_kv_heads * D;
-    const float* row = a.qkv + (size_t)t * (qw + 2 * kw);
+    const float* row = a.qkv + (size_t)t * a.ld;
     const int p = a.pos[t];
     const float* cs = a.cos_sin + (size_t)p * a.rotary_dim;
     if (blockIdx.y == 0) {
@@ -223,8 +229,9 @@ static void launch_qkv_rows(const QkvArgs& a, int rows, int qw, int kw, hipStrea
 extern "C" int llmx_qknorm_rope_kvwrite(const float* qkv, const float* q_weight, const float* k_weight, const float* cos_sin, const int* pos,
                                         const int* row_entry, const int* tables, void* q_out, void* k_cache, void* v_cache, int dtype,
                                         float eps, int rows, int n_heads, int n_kv_heads, int head_dim, int rotary_dim, int norm_mode,
-                                        int page_tokens, int max_blocks, int write_kv, int pairing, hipStream_t stream) {
+                                        int page_tokens, int max_blocks, int write_kv, int pairing, int ld, int v_dim, hipStream_t stream) {
     if (rows <= 0) return 0;
+    if (v_dim < 1 || ld < (n_heads + n_kv_heads) * head_dim + n_kv_heads * v_dim) return -2;
     if (norm_mode != QKNORM_NONE && norm_mode != QKNORM_PROJECTION) return -2;
     if (pairing != ROPE_HALVES && pairing != ROPE_INTERLEAVED) return -2;
     // few rows: many blocks a row, so the chip is used; many rows: two blocks a row, so the sum is not formed over and over
@@ -237,8 +244,8 @@ extern "C" int llmx_qknorm_rope_kvwrite(const float* qkv, const float* q_weight,
         if (k_slices > 4) k_slices = 4;
     }
     QkvArgs a{qkv, q_weight, k_weight, cos_sin, pos, row_entry, tables, q_out, k_cache, v_cache, eps,
-              n_heads, n_kv_heads, head_dim, rotary_dim, norm_mode, page_tokens, max_blocks, write_kv, q_slices, k_slices, pairing};
-    if (rows > 256 && qw <= 32 * 256 && kw <= 32 * 256 && head_dim <= 256) {   // rows kept in registers
+              n_heads, n_kv_heads, head_dim, rotary_dim, norm_mode, page_tokens, max_blocks, write_kv, q_slices, k_slices, ld, v_dim, pairing};
+    if (rows > 256 && v_dim == head_dim && qw <= 32 * 256 && kw <= 32 * 256 && head_dim <= 256) {   // rows kept in registers
         llmx_note_launch(LK_QKNORM_ROPE_KVWRITE_ROWS);
         if (dtype == LLMX_F32) launch_qkv_rows<float, float>(a, rows, qw, kw, stream);
         else launch_qkv_rows<bf16_t, bf16_t>(a, rows, qw, kw, stream);

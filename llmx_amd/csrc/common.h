@@ -241,8 +241,17 @@ __device__ __forceinline__ void rms_rows_as_1024(const float* __restrict__ X, si
 // (e^z - 1 - z) + z/2.  Both go through these two functions, so a product with the activation gives the bits of the product
 // followed by the activation's kernel.
 // RELU2: max(z, 0)^2, no numbers.
-enum : int { LLMX_ACT_NONE = 0, LLMX_ACT_XIELU = 1, LLMX_ACT_RELU2 = 2 };
+// BIAS: z + b_n; GELU_BIAS: gelu(z + b_n), the exact gelu x Phi(x); b one number a feature of the product.  BIAS also goes with
+// the adding epilogue: C + (z + b_n).
+enum : int { LLMX_ACT_NONE = 0, LLMX_ACT_XIELU = 1, LLMX_ACT_RELU2 = 2, LLMX_ACT_BIAS = 3, LLMX_ACT_GELU_BIAS = 4 };
 __host__ __device__ __forceinline__ bool llmx_act_reads_params(int kind) { return kind == LLMX_ACT_XIELU; }
+__host__ __device__ __forceinline__ bool llmx_act_reads_vector(int kind) { return kind == LLMX_ACT_BIAS || kind == LLMX_ACT_GELU_BIAS; }
+// Whether a product with this epilogue (adding or not) can apply the activation, its numbers given.
+__host__ __forceinline__ bool llmx_act_fits(int kind, const float* params, bool stores, bool adds) {
+    if (kind == LLMX_ACT_NONE) return true;
+    if (kind < 0 || kind > LLMX_ACT_GELU_BIAS || !(stores || (adds && kind == LLMX_ACT_BIAS))) return false;
+    return params || !(llmx_act_reads_params(kind) || llmx_act_reads_vector(kind));
+}
 __device__ __forceinline__ float softplus_f(float v) { return log1pf(expf(-fabsf(v))) + fmaxf(v, 0.0f); }
 // The activation's numbers as a kernel reads them at its start (uniform loads, long before the epilogue needs them).
 struct ActParams {
@@ -272,7 +281,17 @@ struct ActFn {
         }
         return v;
     }
+    // with the feature's own number (BIAS, GELU_BIAS; 0 for the others)
+    __device__ __forceinline__ float operator()(float v, float bias) const {
+        if (!llmx_act_reads_vector(kind)) return (*this)(v);
+        const float z = v + bias;
+        return kind == LLMX_ACT_GELU_BIAS ? 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)) : z;
+    }
 };
+// The number of feature n (of N) that an activation reads, 0 where it reads none.
+__device__ __forceinline__ float act_feature(int kind, const float* __restrict__ params, int n, int N) {
+    return llmx_act_reads_vector(kind) ? params[n < N ? n : N - 1] : 0.0f;
+}
 
 // A gated unit of two pre-activations (gate, up), as the products' gated epilogue and the kernel of its own compute it.
 // SILU: silu(gate) * up.  CLAMPED: g = min(gate, limit), u = clamp(up, -limit, limit); g sigmoid(1.702 g) (u + 1).

@@ -26,7 +26,7 @@ struct GemmArgs {
     int a_div;
     long w_group_stride;
     int up_offset;  // EPI_SWIGLU: W row n is the gate row, W row n + up_offset the up row
-    int act;        // EPI_STORE: an activation applied to what is stored (LLMX_ACT_*), with its parameters on the device
+    int act;        // EPI_STORE, EPI_ADD: an activation applied to the product (LLMX_ACT_*), with its parameters on the device
     const float* act_params;
     GluArgs glu;    // EPI_SWIGLU: the gated unit and its per-row values
 };
@@ -53,7 +53,7 @@ __global__ void __launch_bounds__(256) gemm_generic_kernel(GemmArgs g) {
     const int tile_step = g.group_offsets ? GT_BM : GT_BM * gridDim.y;
     const int first = g.group_offsets ? row_begin : row_begin + blockIdx.y * GT_BM;
     const int tx = tid % 16, ty = tid / 16;
-    const ActFn act(EPI == EPI_STORE ? g.act : LLMX_ACT_NONE, g.act_params);
+    const ActFn act(EPI != EPI_SWIGLU ? g.act : LLMX_ACT_NONE, g.act_params);
 
     for (int m0 = first; m0 < row_end; m0 += tile_step) {
         if (tid < GT_BM) {
@@ -133,10 +133,9 @@ __global__ void __launch_bounds__(256) gemm_generic_kernel(GemmArgs g) {
                 if (EPI == EPI_SWIGLU) {
                     // the gated unit; by default silu(g) * u with silu(x) = x / (1 + exp(-x))
                     v = glu(v, accu[i][j]);
-                } else if (EPI == EPI_ADD) {
-                    v = ld(c) + v;
                 } else {
-                    v = act(v);
+                    v = act(v, act_feature(act.kind, g.act_params, n, g.N));
+                    if (EPI == EPI_ADD) v = ld(c) + v;
                 }
                 st(c, v);
             }
@@ -171,10 +170,10 @@ extern "C" int llmx_gemm_generic(const void* A, int a_dtype, const void* W, int 
     if (n_groups == 0 && M <= 0) return 0;
     llmx_note_launch(n_groups ? LK_GEMM_GENERIC_GROUPED : LK_GEMM_GENERIC);
     GemmArgs g{A, W, C, M, N, K, lda, ldw, ldc, n_groups ? group_offsets : nullptr, list, a_div > 0 ? a_div : 1, w_group_stride, up_offset,
-               epi == EPI_STORE ? act : LLMX_ACT_NONE, act_params,
+               epi != EPI_SWIGLU ? act : LLMX_ACT_NONE, act_params,
                GluArgs{epi == EPI_SWIGLU ? glu_kind : LLMX_GLU_SILU, glu_limit, epi == EPI_SWIGLU ? glu_row_scale : nullptr,
                        epi == EPI_SWIGLU ? glu_row_gate : nullptr, glu_row_gate_ld}};
-    if (act != LLMX_ACT_NONE && (epi != EPI_STORE || (llmx_act_reads_params(act) && !act_params))) return -2;
+    if (!llmx_act_fits(act, act_params, epi == EPI_STORE, epi == EPI_ADD)) return -2;
     dim3 grid;
     grid.x = (N + GT_BN - 1) / GT_BN;
     if (n_groups) {

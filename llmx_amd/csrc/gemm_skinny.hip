@@ -41,7 +41,7 @@ struct SkinnyArgs {
     const float* norm_w;
     float norm_eps;
     int x_rows;
-    // SK_STORE: an activation applied to what is stored (LLMX_ACT_*), with its parameters on the device
+    // SK_STORE, SK_ADD: an activation applied to the product (LLMX_ACT_*), with its parameters on the device
     int act;
     const float* act_params;
     GluArgs glu;    // SK_SWIGLU: the gated unit and its per-row values
@@ -66,6 +66,7 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
     const int r = lane & 15, kg = lane >> 4;
     const int n0 = blockIdx.x * 16;
     const ActParams act_params(EPI == SK_STORE ? g.act : LLMX_ACT_NONE, g.act_params);
+    const bool act_vector = EPI != SK_SWIGLU && llmx_act_reads_vector(g.act);      // numbers a feature, asked for long before the epilogue
     const bf16_t* W = g.W;
     int row_begin = 0, row_end = g.M;
     if (GROUPED) {
@@ -142,7 +143,11 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
 #pragma unroll
             for (int a = 0; a < NACC; ++a) acc[t][a] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
         // what an adding epilogue joins: asked for now, used after the loop
-        float c_old[MT][4];
+        float c_old[MT][4], act_n[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+        if (act_vector && wave == 0) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) act_n[i] = act_feature(g.act, g.act_params, n0 + 4 * kg + i, g.N);
+        }
         if (EPI == SK_ADD && wave == 0) {
 #pragma unroll
             for (int t = 0; t < MT; ++t) {
@@ -231,8 +236,9 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
                     if (n0 + 4 * kg + i >= g.N) continue;
                     float x = v[0][i];
                     if (EPI == SK_SWIGLU) x = glu(x, v[1][i]);
+                    if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x, act_n[i]);
+                    if (EPI == SK_ADD && act_vector) x = x + act_n[i];
                     if (EPI == SK_ADD) x = c_old[t][i] + x;
-                    if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x);
                     st(c + i, x);
                 }
             }
@@ -253,6 +259,7 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_two_strips_kernel(SkinnyA
     const int r = lane & 15, kg = lane >> 4;
     const int n0 = blockIdx.x * 32;
     const ActParams act_params(EPI == SK_STORE ? g.act : LLMX_ACT_NONE, g.act_params);
+    const bool act_vector = EPI != SK_SWIGLU && llmx_act_reads_vector(g.act);      // numbers a feature, asked for long before the epilogue
     const int K = g.K;
     const int steps_total = (K + 31) >> 5;
     const int per = (steps_total + KS - 1) / KS;
@@ -270,6 +277,13 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_two_strips_kernel(SkinnyA
         ap[t] = g.A + (size_t)(a_in[t] ? m : 0) * g.lda + kg * 8;
     }
     f32x4_t acc[MT][2];
+    float act_n[2][4] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
+    if (act_vector && wave == 0) {
+#pragma unroll
+        for (int q = 0; q < 2; ++q)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) act_n[q][i] = act_feature(g.act, g.act_params, n0 + 16 * q + 4 * kg + i, g.N);
+    }
 #pragma unroll
     for (int t = 0; t < MT; ++t)
 #pragma unroll
@@ -320,8 +334,9 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_two_strips_kernel(SkinnyA
             for (int i = 0; i < 4; ++i) {
                 if (n0 + 16 * q + 4 * kg + i >= g.N) continue;
                 float x = v[i];
+                if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x, act_n[q][i]);
+                if (EPI == SK_ADD && act_vector) x = x + act_n[q][i];
                 if (EPI == SK_ADD) x = ld(c + i) + x;
-                if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x);
                 st(c + i, x);
             }
         }
@@ -421,10 +436,10 @@ extern "C" int llmx_gemm_skinny(const void* A, const void* W, void* C, int c_dty
     if (grouped && max_active <= 0) return 0;
     if (X && (!norm_w || epi == SK_ADD || !llmx_gemm_skinny_normed_ok(x_rows, K) || (!grouped && x_rows != M))) return -2;
     SkinnyArgs g{(const bf16_t*)A, (const bf16_t*)W, C, M, N, K, lda, ldc, active, n_active, group_offsets, list, a_div > 0 ? a_div : 1,
-                 w_group_stride, up_offset, X, norm_w, norm_eps, x_rows, epi == SK_STORE ? act : LLMX_ACT_NONE, act_params,
+                 w_group_stride, up_offset, X, norm_w, norm_eps, x_rows, epi != SK_SWIGLU ? act : LLMX_ACT_NONE, act_params,
                  GluArgs{epi == SK_SWIGLU ? glu_kind : LLMX_GLU_SILU, glu_limit, epi == SK_SWIGLU ? glu_row_scale : nullptr,
                          epi == SK_SWIGLU ? glu_row_gate : nullptr, glu_row_gate_ld}};
-    if (act != LLMX_ACT_NONE && (epi != SK_STORE || (llmx_act_reads_params(act) && !act_params))) return -2;
+    if (!llmx_act_fits(act, act_params, epi == SK_STORE, epi == SK_ADD)) return -2;
     dim3 grid((N + 15) / 16, grouped ? max_active : 1, 1);
     int mt = 1;
     if (!grouped && epi != SK_SWIGLU) mt = M <= 16 ? 1 : (M <= 32 ? 2 : 4);

@@ -85,7 +85,7 @@ struct TileArgs {
     const int* tile_stats;  // grouped, optional: [0] = sum over groups of ceil(rows / 128)
     int run_if_big;         // with tile_stats: 1: this launch works only if the groups fill 128-row tiles, 0: only if not
     int run_tiles;          // dense lean form, > 0: workgroup z multiplies only K's run z (this many 64-wide tiles) and stores its sums at C + z * M * ldc
-    int act;                // TL_STORE: an activation applied to what is stored (LLMX_ACT_*; a launch of runs' sums leaves it to the kernel that adds them)
+    int act;                // TL_STORE, TL_ADD: an activation applied to the product (LLMX_ACT_*; a launch of runs' sums leaves it to the kernel that adds them)
     const float* act_params;
     GluArgs glu;            // TL_SWIGLU: the gated unit and its per-row values
 };
@@ -449,10 +449,10 @@ __global__ void __launch_bounds__(256) gemm_tile_kernel(TileArgs g) {
 #pragma unroll
             for (int f = 0; f < 4; ++f) {
                 float v[4] = {acc[f][t][0], acc[f][t][1], acc[f][t][2], acc[f][t][3]};
-                if (EPI == TL_STORE && g.act != LLMX_ACT_NONE) {
+                if (g.act != LLMX_ACT_NONE) {
                     const ActFn act(g.act, g.act_params);
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) v[i] = act(v[i]);
+                    for (int i = 0; i < 4; ++i) v[i] = act(v[i], act_feature(g.act, g.act_params, n0 + 64 * wn + 16 * f + fq + i, g.N));
                 }
                 store_quad<EPI == TL_ADD>(crow, n0 + 64 * wn + 16 * f + fq, g.N, rows_aligned, v);
             }
@@ -719,10 +719,10 @@ __global__ void __launch_bounds__(512) gemm_wide_kernel(TileArgs g) {
 #pragma unroll
             for (int f = 0; f < 4; ++f) {
                 float v[4] = {acc[f][q][0], acc[f][q][1], acc[f][q][2], acc[f][q][3]};
-                if (EPI == TL_STORE && g.act != LLMX_ACT_NONE) {
+                if (g.act != LLMX_ACT_NONE) {
                     const ActFn act(g.act, g.act_params);
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) v[i] = act(v[i]);
+                    for (int i = 0; i < 4; ++i) v[i] = act(v[i], act_feature(g.act, g.act_params, n0 + 64 * wn + 16 * f + fq + i, g.N));
                 }
                 store_quad<EPI == TL_ADD>(crow, n0 + 64 * wn + 16 * f + fq, g.N, rows_aligned, v);
             }
@@ -804,10 +804,10 @@ __global__ void __launch_bounds__(256) gemm_runs_sum_kernel(const float* __restr
 #pragma unroll
         for (int i = 0; i < 4; ++i) v[i] = r == 0 ? x[i] : v[i] + x[i];
     }
-    if (!ADD && act_kind != LLMX_ACT_NONE) {
+    if (act_kind != LLMX_ACT_NONE) {
         const ActFn act(act_kind, act_params);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = act(v[i]);
+        for (int i = 0; i < 4; ++i) v[i] = act(v[i], act_feature(act_kind, act_params, n + i, N));
     }
     store_quad<ADD>(C + (size_t)m * ldc, n, N, ldc % 4 == 0 && ((uintptr_t)C & 15) == 0, v);
 }
@@ -850,10 +850,10 @@ extern "C" int llmx_gemm_tile(const void* A, const void* W, void* C, int c_dtype
     const int steps = (K + 31) / 32, per = (steps + ks - 1) / ks;
     const bool lean = K % TL_BK == 0 && (ks == 1 || per % 2 == 0) && llmx_gemm_tile_offsets_fit(M, N, K, lda, epi, n_groups, a_div, up_offset);
     TileArgs g{(const bf16_t*)A, (const bf16_t*)W, C, M, N, K, lda, ldc, group_offsets, list, n_groups, a_div > 0 ? a_div : 1,
-               w_group_stride, up_offset, 0, ks, 64, nullptr, 0, 0, epi == TL_STORE ? act : LLMX_ACT_NONE, act_params,
+               w_group_stride, up_offset, 0, ks, 64, nullptr, 0, 0, epi != TL_SWIGLU ? act : LLMX_ACT_NONE, act_params,
                GluArgs{epi == TL_SWIGLU ? glu_kind : LLMX_GLU_SILU, glu_limit, epi == TL_SWIGLU ? glu_row_scale : nullptr,
                        epi == TL_SWIGLU ? glu_row_gate : nullptr, glu_row_gate_ld}};
-    if (act != LLMX_ACT_NONE && (epi != TL_STORE || (llmx_act_reads_params(act) && !act_params))) return -2;
+    if (!llmx_act_fits(act, act_params, epi == TL_STORE, epi == TL_ADD)) return -2;
     auto launch = [&](int form, int tiles_y) -> int {
         g.bm = form_rows(form);
         g.m_tiles = (M + g.bm - 1) / g.bm;
@@ -887,7 +887,7 @@ extern "C" int llmx_gemm_tile(const void* A, const void* W, void* C, int c_dtype
         const dim3 sum_grid((unsigned)((quads + 255) / 256));
         if (epi == TL_ADD) {
             if (c_dtype != LLMX_F32) return -2;
-            hipLaunchKernelGGL((gemm_runs_sum_kernel<true, float>), sum_grid, dim3(256), 0, stream, (const float*)runs_scratch, (float*)C, M, N, ldc, runs, 0, nullptr);
+            hipLaunchKernelGGL((gemm_runs_sum_kernel<true, float>), sum_grid, dim3(256), 0, stream, (const float*)runs_scratch, (float*)C, M, N, ldc, runs, g.act, g.act_params);
         } else if (c_dtype == LLMX_BF16) {
             hipLaunchKernelGGL((gemm_runs_sum_kernel<false, bf16_t>), sum_grid, dim3(256), 0, stream, (const float*)runs_scratch, (bf16_t*)C, M, N, ldc, runs, g.act, g.act_params);
         } else {

@@ -162,6 +162,7 @@ struct LatentAttnArgs {
     void* out;           // [H, T, C]
     float scale;
     int T, H, C, R, ldc, page_tokens, max_blocks, window, row_major;
+    const float* sink;   // [H] or null: one more logit a head in the denominator, with no key and no value
 };
 
 #define LAT_MAX_C 2048
@@ -224,21 +225,27 @@ __global__ void __launch_bounds__(64) latent_attention_generic_kernel(LatentAttn
         m = m_new;
         __syncthreads();
     }
+    float shrink = 1.0f;
+    if (a.sink) {
+        const float top = fmaxf(m, a.sink[h]);
+        shrink = expf(m - top);
+        l = l * shrink + expf(a.sink[h] - top);
+    }
     T* out = (T*)a.out + q_at * C;
 #pragma unroll
     for (int i = 0; i < LAT_MAX_C / 64; ++i) {
         const int d = lane + 64 * i;
-        if (d < C) st(out + d, acc[i] / l);
+        if (d < C) st(out + d, a.sink ? acc[i] * shrink / l : acc[i] / l);
     }
 }
 
 extern "C" int llmx_latent_attention_generic(const void* q_lat, const void* q_rot, const void* cache, const int* pos, const int* row_entry,
                                              const int* tables, void* out, int dtype, float scale, int T, int H, int C, int R, int ldc, int page_tokens,
-                                             int max_blocks, int window, int row_major, hipStream_t stream) {
+                                             int max_blocks, int window, int row_major, const float* sink, hipStream_t stream) {
     if (T <= 0 || H <= 0) return 0;
     if (C <= 0 || C > LAT_MAX_C || R < 0 || C + R > LAT_MAX_CR || ldc < C + R) return -2;
     llmx_note_launch(LK_LATENT_ATTENTION_GENERIC);
-    LatentAttnArgs a{q_lat, q_rot, cache, pos, row_entry, tables, out, scale, T, H, C, R, ldc, page_tokens, max_blocks, window, row_major};
+    LatentAttnArgs a{q_lat, q_rot, cache, pos, row_entry, tables, out, scale, T, H, C, R, ldc, page_tokens, max_blocks, window, row_major, sink};
     if (dtype == LLMX_F32) hipLaunchKernelGGL(latent_attention_generic_kernel<float>, dim3(T, H), dim3(64), 0, stream, a);
     else hipLaunchKernelGGL(latent_attention_generic_kernel<bf16_t>, dim3(T, H), dim3(64), 0, stream, a);
     return LLMX_CHECK_LAUNCH();

@@ -38,7 +38,15 @@ struct LatentMfmaArgs {
     float* part_ml;         // [slots, 16, 2]: its maximum and its sum of weights
     float scale;
     int T, H, C, R, ldc, page_tokens, max_blocks, window, row_major;
+    const float* sink;      // [H] or null: one more logit a head in the softmax's denominator, with no key and no value
 };
+
+// The factor on a finished column's sums: 1 / l, the head's sink, where there is one, joining l.
+__device__ __forceinline__ float latent_finish(const float* sink, int h, float m, float l) {
+    if (!sink) return 1.0f / l;
+    const float s = sink[h], top = fmaxf(m, s), shrink = __expf(m - top);
+    return shrink / (l * shrink + __expf(s - top));
+}
 
 // Where a (head, row)'s queries and result lie, in rows of C (or R) values.
 __device__ __forceinline__ size_t latent_row(const LatentMfmaArgs& a, int h, int r) {
@@ -219,7 +227,7 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
     }
     if (!live) return;
     bf16_t* out = a.out + latent_row(a, c_head, c_row) * C;
-    const float inv = 1.0f / l;
+    const float inv = latent_finish(a.sink, c_head, m, l);
 #pragma unroll
     for (int dt = 0; dt < CT; ++dt) {
         if (16 * dt < C) {
@@ -235,7 +243,8 @@ __global__ void __launch_bounds__(64) latent_attention_mfma_kernel(LatentMfmaArg
 // the slots in order, eight slots' loads in flight.
 #define LM_MERGE_MAX 1024    // slots of one column whose weights fit the workgroup's LDS; longer columns take rounds
 __global__ void __launch_bounds__(256) latent_attention_merge_kernel(const int* __restrict__ merges, const float* __restrict__ part_o,
-                                                                   const float* __restrict__ part_ml, bf16_t* __restrict__ out, int T, int C, int H, int row_major) {
+                                                                   const float* __restrict__ part_ml, bf16_t* __restrict__ out, int T, int C, int H, int row_major,
+                                                                   const float* __restrict__ sink) {
     __shared__ float weight[LM_MERGE_MAX];
     __shared__ float scratch[4];
     const int* mg = merges + LM_ITEM_INTS * (size_t)blockIdx.x;
@@ -274,7 +283,7 @@ __global__ void __launch_bounds__(256) latent_attention_merge_kernel(const int* 
                 }
         }
     }
-    const float inv = 1.0f / L;
+    const float inv = latent_finish(sink, head0 + c, M, L);
 #pragma unroll
     for (int e = 0; e < 2; ++e)
         if (threadIdx.x + 256 * e < C) out[(row_major ? (size_t)row * H + head0 + c : (size_t)(head0 + c) * T + row) * C + threadIdx.x + 256 * e] = f32_to_bf16(acc[e] * inv);
@@ -520,7 +529,7 @@ __global__ void __launch_bounds__(256) latent_attention_tiles_kernel(LatentMfmaA
     for (int ct = 0; ct < LW_TILES; ++ct) {
         if (!live[ct]) continue;
         bf16_t* out = a.out + latent_row(a, c_head, c_row[ct]) * C;
-        const float inv = 1.0f / l[ct];
+        const float inv = latent_finish(a.sink, c_head, m[ct], l[ct]);
 #pragma unroll
         for (int dt = 0; dt < DPW; ++dt) {
             const int d0 = 16 * (wave * DPW + dt);
@@ -542,12 +551,12 @@ extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, 
                                           const int* row_entry, const int* tables, const int* items, int n_items, int n_tile_items, int n_row_items,
                                           const int* merges, int n_merges,
                                           void* out, float* part_o, float* part_ml, float scale, int T, int H, int C, int R, int ldc, int page_tokens,
-                                          int max_blocks, int window, int row_major, hipStream_t stream) {
+                                          int max_blocks, int window, int row_major, const float* sink, hipStream_t stream) {
     if (n_items <= 0 && n_tile_items <= 0 && n_row_items <= 0) return 0;
     if (!llmx_latent_attention_mfma_ok(C, R, ldc, page_tokens) || window < 0) return -2;
     if (n_merges > 0 && (!merges || !part_o || !part_ml)) return -2;
     LatentMfmaArgs a{(const bf16_t*)q_lat, (const bf16_t*)q_rot, (const bf16_t*)cache, (const bf16_t*)cache_t, pos, row_entry, tables, items,
-                     (bf16_t*)out, part_o, part_ml, scale, T, H, C, R, ldc, page_tokens, max_blocks, window, row_major};
+                     (bf16_t*)out, part_o, part_ml, scale, T, H, C, R, ldc, page_tokens, max_blocks, window, row_major, sink};
 #define LLMX_LT(DPW, TILES, KS, PIPE, count, first)                                                                                        \
     {                                                                                                                                 \
         static bool raised = false;                                                                                                   \
@@ -589,7 +598,7 @@ extern "C" int llmx_latent_attention_mfma(const void* q_lat, const void* q_rot, 
     }
     if (n_merges > 0) {
         llmx_note_launch(LK_LATENT_ATTENTION_MERGE);
-        hipLaunchKernelGGL(latent_attention_merge_kernel, dim3(n_merges, 16), dim3(256), 0, stream, merges, part_o, part_ml, (bf16_t*)out, T, C, H, row_major);
+        hipLaunchKernelGGL(latent_attention_merge_kernel, dim3(n_merges, 16), dim3(256), 0, stream, merges, part_o, part_ml, (bf16_t*)out, T, C, H, row_major, sink);
     }
     return LLMX_CHECK_LAUNCH();
 }

@@ -1,5 +1,5 @@
-// Layer norm with a weight and no bias, and the element-wise steps of layers that norm a sublayer's result before it
-// joins the residual: y = (x - mean) / sqrt(var + eps) * w, var the mean of the squared deviations.  Everything is float32
+// Layer norm with a weight and an optional bias, and the element-wise steps of layers that norm a sublayer's result before it
+// joins the residual: y = (x - mean) / sqrt(var + eps) * w (+ b), var the mean of the squared deviations.  Everything is float32
 // arithmetic on float32 rows; only what a product reads next is stored in the activation type.
 // A row's sums are formed by 256 threads: thread v adds elements v, v + 256, ... in this order, a wave adds its threads'
 // sums with wave_sum, and the four waves' sums are added in wave order: a function of the row's length only.
@@ -42,7 +42,7 @@ __device__ __forceinline__ void row_moments(const float* __restrict__ row, int n
 // out[r] = LN(x[pick ? pick[r] : r]) in the activation type and/or float32
 template <typename TO, bool KEPT>
 __global__ void __launch_bounds__(LN_THREADS) layernorm_kernel(const float* __restrict__ x, const int* __restrict__ pick, const float* __restrict__ w,
-                                                             float eps, TO* __restrict__ out, float* __restrict__ out32, int n) {
+                                                             const float* __restrict__ bias, float eps, TO* __restrict__ out, float* __restrict__ out32, int n) {
     __shared__ float scratch[LN_THREADS / 64];
     const int r = blockIdx.x, tid = threadIdx.x;
     const float* row = x + (size_t)(pick ? pick[r] : r) * n;
@@ -53,27 +53,29 @@ __global__ void __launch_bounds__(LN_THREADS) layernorm_kernel(const float* __re
         for (int j = 0; j < LN_KEPT; ++j) {
             const int i = tid + LN_THREADS * j;
             if (i < n) {
-                const float y = (v[j] - mean) * rstd * w[i];
+                float y = (v[j] - mean) * rstd * w[i];
+                if (bias) y = y + bias[i];
                 if (out) st(out + (size_t)r * n + i, y);
                 if (out32) out32[(size_t)r * n + i] = y;
             }
         }
     } else {
         for (int i = tid; i < n; i += LN_THREADS) {
-            const float y = (row[i] - mean) * rstd * w[i];
+            float y = (row[i] - mean) * rstd * w[i];
+            if (bias) y = y + bias[i];
             if (out) st(out + (size_t)r * n + i, y);
             if (out32) out32[(size_t)r * n + i] = y;
         }
     }
 }
 
-extern "C" int llmx_layernorm(const float* x, const int* pick, const float* w, float eps, void* out, int out_dtype, float* out32, int rows, int n,
+extern "C" int llmx_layernorm(const float* x, const int* pick, const float* w, const float* bias, float eps, void* out, int out_dtype, float* out32, int rows, int n,
                               hipStream_t stream) {
     if (rows <= 0) return 0;
     if (n <= 0 || !w || (!out && !out32)) return -2;
     llmx_note_launch(LK_LAYERNORM);
     const bool kept = n <= LN_THREADS * LN_KEPT;
-#define LLMX_LN(TO, K) hipLaunchKernelGGL((layernorm_kernel<TO, K>), dim3(rows), dim3(LN_THREADS), 0, stream, x, pick, w, eps, (TO*)out, out32, n)
+#define LLMX_LN(TO, K) hipLaunchKernelGGL((layernorm_kernel<TO, K>), dim3(rows), dim3(LN_THREADS), 0, stream, x, pick, w, bias, eps, (TO*)out, out32, n)
     if (out_dtype == LLMX_F32) {
         if (kept) LLMX_LN(float, true);
         else LLMX_LN(float, false);
@@ -159,6 +161,28 @@ extern "C" int llmx_cast_rows(const float* x, void* out, int out_dtype, long tot
     const dim3 grid((unsigned)((total + 1023) / 1024));
     if (out_dtype == LLMX_F32) hipLaunchKernelGGL(cast_rows_kernel<float>, grid, dim3(256), 0, stream, x, (float*)out, (size_t)total);
     else hipLaunchKernelGGL(cast_rows_kernel<bf16_t>, grid, dim3(256), 0, stream, x, (bf16_t*)out, (size_t)total);
+    return LLMX_CHECK_LAUNCH();
+}
+
+// out[t] = [x[t] | y[t]] in the activation type, x and y float32 rows of n values: what a product of two joined streams reads.
+// y null: only the first half is written (the second is there from before).
+template <typename TO>
+__global__ void __launch_bounds__(256) join_rows_kernel(const float* __restrict__ x, const float* __restrict__ y, TO* __restrict__ out, int n, size_t total) {
+    const size_t at = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (at >= total) return;
+    const size_t t = at / (size_t)n, i = at % (size_t)n;
+    TO* row = out + t * 2 * (size_t)n;
+    st(row + i, x[at]);
+    if (y) st(row + n + i, y[at]);
+}
+
+extern "C" int llmx_join_rows(const float* x, const float* y, void* out, int out_dtype, int rows, int n, hipStream_t stream) {
+    if (rows <= 0 || n <= 0) return 0;
+    llmx_note_launch(LK_JOIN_ROWS);
+    const size_t total = (size_t)rows * n;
+    const dim3 grid((unsigned)((total + 255) / 256));
+    if (out_dtype == LLMX_F32) hipLaunchKernelGGL(join_rows_kernel<float>, grid, dim3(256), 0, stream, x, y, (float*)out, n, total);
+    else hipLaunchKernelGGL(join_rows_kernel<bf16_t>, grid, dim3(256), 0, stream, x, y, (bf16_t*)out, n, total);
     return LLMX_CHECK_LAUNCH();
 }
 

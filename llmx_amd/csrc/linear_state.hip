@@ -1,7 +1,7 @@
 // Mixers that carry a matrix state from token to token: for every head a float32 matrix S [D key channels, V value
 // channels] in the request's state slot (stored in tiles of 8 value channels, [head][tile][D][8], the last tile padded, so
 // that the block that owns a tile reads and writes one run of memory), updated once a token:
-//     S <- diag(g_t) S                         (a decay a key channel, acting on S's rows)
+//     S <- diag(g_t) S                         (a decay a key channel, acting on S's rows, or one for the head)
 //     u  = beta_t (v_t - S^T k_t)              (delta rule; without it u = v_t: gated linear attention)
 //     S <- S + k_t u^T,   o_t = S^T q_t        (the read-out sees the token's own write)
 // A column of S (one value channel) never meets another, so the scan gives every column to 32 lanes that hold a
@@ -24,9 +24,9 @@ struct DeltaPrepArgs {
     const float* pre;
     int ld;
     const float* conv_w;
-    const float* step_pre;   // [T, H*D] (rows step_ld apart): the decay's projection before its bias
+    const float* step_pre;   // [T, H*D] (rows step_ld apart): the decay's projection before its bias; head_decay: [T, H]
     int step_ld;
-    const float* dt_bias;    // [H*D]
+    const float* dt_bias;    // [H*D]; head_decay: [H]
     const float* a_log;      // [H]
     const float* state;
     long state_stride;
@@ -37,13 +37,13 @@ struct DeltaPrepArgs {
     float* q;       // [T, G*D]
     float* k;       // [T, G*D]
     float* v;       // [T, H*V]
-    float* decay;   // [T, H*D]
+    float* decay;   // [T, H*D]; head_decay: [T, H]
     float* beta;    // [T, H]
-    int G, H, D, V, taps, beta_col;
+    int G, H, D, V, taps, beta_col, head_decay;
 };
 
 // One wave a (row, unit): the units of a row are its 2 G heads of q and k (convolution, silu, unit norm), its H heads of
-// v (convolution, silu), its H heads of decays, and beta; a unit's values stay in the wave's registers.
+// v (convolution, silu), its H heads of decays (where every key channel has its own), and beta (with the decays a head); a unit's values stay in the wave's registers.
 #define PREP_MAX 256     // values of a head a wave keeps (4 a lane): the scan's limit on a head's key channels
 __device__ __forceinline__ float conv_silu_at(const DeltaPrepArgs& a, const float* __restrict__ tail, int C, int row0, int i, int c) {
     float acc = 0.0f;
@@ -81,7 +81,7 @@ __global__ void __launch_bounds__(64) delta_prep_kernel(DeltaPrepArgs a) {
     } else if (unit < 2 * a.G + a.H) {                  // a head of v
         const int h = unit - 2 * a.G;
         for (int d = lane; d < a.V; d += 64) a.v[(size_t)t * HV + h * a.V + d] = conv_silu_at(a, tail, C, row0, i, 2 * GD + h * a.V + d);
-    } else if (unit < 2 * a.G + 2 * a.H) {              // a head's decays
+    } else if (!a.head_decay && unit < 2 * a.G + 2 * a.H) {   // a head's decays
         const int h = unit - 2 * a.G - a.H;
         const float rate = expf(a.a_log[h]);
         for (int d = lane; d < a.D; d += 64) {
@@ -89,21 +89,24 @@ __global__ void __launch_bounds__(64) delta_prep_kernel(DeltaPrepArgs a) {
             a.decay[(size_t)t * HD + c] = expf(-rate * softplus_f(a.step_pre[(size_t)t * a.step_ld + c] + a.dt_bias[c]));
         }
     } else {
-        for (int c = lane; c < a.H; c += 64) a.beta[(size_t)t * a.H + c] = sigmoid_ls(a.pre[(size_t)t * a.ld + a.beta_col + c]);
+        for (int c = lane; c < a.H; c += 64) {
+            a.beta[(size_t)t * a.H + c] = sigmoid_ls(a.pre[(size_t)t * a.ld + a.beta_col + c]);
+            if (a.head_decay) a.decay[(size_t)t * a.H + c] = expf(-expf(a.a_log[c]) * softplus_f(a.step_pre[(size_t)t * a.step_ld + c] + a.dt_bias[c]));
+        }
     }
 }
 
 extern "C" int llmx_delta_prep(const float* pre, int ld, const float* conv_w, const float* step_pre, int step_ld, const float* dt_bias,
                                const float* a_log, const float* state, long state_stride, int tail_off, const int* slot_read,
                                const int* row_entry, const int* entry_rows, float* q, float* k, float* v, float* decay, float* beta, int rows, int G,
-                               int H, int D, int V, int taps, int beta_col, hipStream_t stream) {
+                               int H, int D, int V, int taps, int beta_col, int head_decay, hipStream_t stream) {
     if (rows <= 0) return 0;
     const long C = 2L * G * D + (long)H * V;
-    if (taps < 1 || G < 1 || H % G || D > PREP_MAX || beta_col + H > ld || C > ld || step_ld < H * D) return -2;
+    if (taps < 1 || G < 1 || H % G || D > PREP_MAX || beta_col + H > ld || C > ld || step_ld < (head_decay ? H : H * D)) return -2;
     DeltaPrepArgs a{pre, ld, conv_w, step_pre, step_ld, dt_bias, a_log, state, state_stride, tail_off, slot_read, row_entry, entry_rows,
-                    q, k, v, decay, beta, G, H, D, V, taps, beta_col};
+                    q, k, v, decay, beta, G, H, D, V, taps, beta_col, head_decay};
     llmx_note_launch(LK_DELTA_PREP);
-    hipLaunchKernelGGL(delta_prep_kernel, dim3(rows, 2 * G + 2 * H + 1), dim3(64), 0, stream, a);
+    hipLaunchKernelGGL(delta_prep_kernel, dim3(rows, 2 * G + (head_decay ? H : 2 * H) + 1), dim3(64), 0, stream, a);
     return LLMX_CHECK_LAUNCH();
 }
 
@@ -151,6 +154,7 @@ struct StateScanArgs {
     const float* tail_src;
     int tail_ld, tail_C, taps, tail_off;
     int max_rows_here;   // > 0: entries of more rows are left to another kernel
+    int head_decay;      // decay [T, H]: one for all of a head's key channels
     StateOperands operands;
 };
 
@@ -200,7 +204,7 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
     const int hq = h / a.share;
     const float* kp = a.k + (size_t)hq * a.D;
     const float* qp = a.q + (size_t)hq * a.D;
-    const float* gp = a.decay + (size_t)h * a.D;
+    const float* gp = a.decay + (size_t)h * (a.head_decay ? 1 : a.D);
     const float* vp = a.v + (size_t)h * a.V + tile * SCAN_COLS;
     float stage[STAGE], vstage = 0.0f, bstage = 0.0f;
     auto fetch = [&](int t0) {
@@ -211,7 +215,8 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
             const size_t row = (size_t)(row0 + min(t0 + tt, n - 1));
             const int dd = d < a.D ? d : 0;
             const float* src = which == 0 ? kp + row * a.ldk : which == 1 ? qp + row * a.ldq : gp + row * a.ldg;
-            const float x = KIND == STATE_OPERANDS_PLAIN || which == 2 ? src[dd] : state_key<KIND>(a.operands, src, row, dd);
+            const int at = which == 2 && a.head_decay ? 0 : dd;
+            const float x = KIND == STATE_OPERANDS_PLAIN || which == 2 ? src[at] : state_key<KIND>(a.operands, src, row, dd);
             stage[u] = d < a.D ? x : 0.0f;
         }
         if (tid < CH * SCAN_COLS) {
@@ -357,7 +362,7 @@ __global__ void __launch_bounds__(64 * CN) state_step_kernel(StateScanArgs a) {
     const int hq = h / a.share;
     const float k = state_key<KIND>(a.operands, a.k + row * a.ldk + (size_t)hq * a.D, row, dd);
     const float q = state_key<KIND>(a.operands, a.q + row * a.ldq + (size_t)hq * a.D, row, dd);
-    const float g = a.decay[row * a.ldg + (size_t)h * a.D + dd];
+    const float g = a.decay[row * a.ldg + (a.head_decay ? h : (size_t)h * a.D + dd)];
     const float* vp = a.v + row * a.ldv + (size_t)h * a.V;
     float v[STEP_TILES][4];
 #pragma unroll
@@ -427,12 +432,12 @@ extern "C" int llmx_state_scan(const float* q, int ldq, const float* k, int ldk,
                                const float* beta, float* state, long state_stride, const int* slot_read, const int* slot_write,
                                const int* entry_rows, float* out, float out_scale, int n_entries, int H, int share, int D, int V,
                                const float* tail_src, int tail_ld, int tail_C, int taps, int tail_off, int max_rows, int max_rows_here, int operands,
-                               const float* cos_sin, const int* pos, int rot_dims, hipStream_t stream) {
+                               const float* cos_sin, const int* pos, int rot_dims, int head_decay, hipStream_t stream) {
     if (n_entries <= 0) return 0;
     if (operands < 0 || operands > 2 || (operands == STATE_OPERANDS_ROTATED && (!cos_sin || !pos || rot_dims < 2 || rot_dims % 2 || rot_dims > D))) return -2;
     if (H < 1 || share < 1 || H % share || D < 1 || D > 256 || V < 1 || (taps > 1 && !tail_src)) return -2;
     StateScanArgs a{q, k, v, decay, beta, ldq, ldk, ldv, ldg, state, state_stride, slot_read, slot_write, entry_rows, out, out_scale,
-                    H, share, D, V, tail_src, tail_ld, tail_C, taps, tail_off, max_rows_here, StateOperands{cos_sin, pos, rot_dims}};
+                    H, share, D, V, tail_src, tail_ld, tail_C, taps, tail_off, max_rows_here, head_decay, StateOperands{cos_sin, pos, rot_dims}};
     const dim3 grid((unsigned)(H * ((V + SCAN_COLS - 1) / SCAN_COLS)), (unsigned)n_entries);
     if (max_rows == 1 && !beta && taps <= 1 && state_stride % 4 == 0 && ((uintptr_t)state & 15) == 0) {
         llmx_note_launch(LK_STATE_STEP);

@@ -87,7 +87,8 @@
     X(EMBED_BIGRAM, "embed_bigram")                                                                                       \
     X(TOKEN_SHIFT, "token_shift")                                                                                         \
     X(RMSNORM_SHIFT, "rmsnorm_shift")                                                                                     \
-    X(DECAYED_STATE_CHUNKS, "decayed_state.chunks")
+    X(DECAYED_STATE_CHUNKS, "decayed_state.chunks")                                                                       \
+    X(JOIN_ROWS, "join_rows")
 
 enum LlmxLaunchKind : int {
 #define LLMX_X(id, name) LK_##id,

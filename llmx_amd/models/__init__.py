@@ -8,6 +8,7 @@ from . import bonerax  # noqa: F401  (registers Bonerax)
 from . import givozen  # noqa: F401  (registers Givozen)
 from . import salipel  # noqa: F401  (registers Salipel)
 from . import neruzen  # noqa: F401  (registers Neruzen)
+from . import vivulorn  # noqa: F401  (registers Vivulorn)
 
 __all__ = ["ArchitectureEntry", "architecture_of", "architectures", "assemble", "read_config", "read_model_dir",
            "register_architecture", "unregister_architecture"]

@@ -64,9 +64,9 @@ def _declare(h) -> None:
         "llmx_latent_prep": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, I, I, I, P],
         "llmx_latent_down": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, I, P],
         "llmx_latent_queries": [P, P, P, P, P, I, I, I, I, I, I, I, I, I, P],
-        "llmx_latent_attention_mfma": [P, P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, I, I, P],
+        "llmx_latent_attention_mfma": [P, P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, I, I, P, P],
         "llmx_latent_attention_mfma_ok": [I, I, I, I],
-        "llmx_latent_attention_generic": [P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, P],
+        "llmx_latent_attention_generic": [P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, P, P],
         "llmx_head_gate": [P, P, I, P, I, I, I, I, P],
         "llmx_embed_bigram": [P, P, I, P, P, P, P, P, P, P, I, I, F, I, L, L, P],
         "llmx_token_shift": [P, P, F, P, P, L, P, P, P, P, P, P, P, I, I, I, P],
@@ -77,7 +77,7 @@ def _declare(h) -> None:
         "llmx_read_probe": [P, L, P, P],
         "llmx_attention_partial_pad": [],
         "llmx_gemm_generic": [P, I, P, I, P, I, I, I, I, I, I, I, I, I, P, P, I, L, I, I, P, I, F, P, P, I, P],
-        "llmx_qknorm_rope_kvwrite": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, P],
+        "llmx_qknorm_rope_kvwrite": [P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, I, I, P],
         "llmx_paged_attention_generic": [P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, P, I, I, I, I, I, F, P, P, I, P],
         "llmx_head_norm_rope_kvwrite": [P, P, P, P, P, P, P, P, P, P, P, I, F, I, I, I, I, I, I, I, I, I, I, I, P, I, I, I, I, P],
         "llmx_gate_heads": [P, I, P, I, I, I, I, P],
@@ -85,15 +85,16 @@ def _declare(h) -> None:
         "llmx_add_rows_vector": [P, P, P, I, I, P],
         "llmx_act_polynorm": [P, P, F, P, I, I, I, P],
         "llmx_act_glu": [P, I, P, P, I, I, F, P, I, I, I, P],
-        "llmx_layernorm": [P, P, P, F, P, I, P, I, I, P],
+        "llmx_layernorm": [P, P, P, P, F, P, I, P, I, I, P],
+        "llmx_join_rows": [P, P, P, I, I, I, P],
         "llmx_layernorm_add": [P, P, P, F, P, I, I, I, P],
         "llmx_cast_rows": [P, P, I, L, P],
         "llmx_combine_rows": [P, P, F, P, P, F, I, I, I, P],
         "llmx_scale_softcap": [P, F, F, L, P],
-        "llmx_delta_prep": [P, I, P, P, I, P, P, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, P],
+        "llmx_delta_prep": [P, I, P, P, I, P, P, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
         "llmx_cast_cols": [P, I, P, I, I, I, P],
         "llmx_sigmoid_root": [P, P, F, P, I, I, P],
-        "llmx_state_scan": [P, I, P, I, P, I, P, I, P, P, L, P, P, P, P, F, I, I, I, I, I, P, I, I, I, I, I, I, I, P, P, I, P],
+        "llmx_state_scan": [P, I, P, I, P, I, P, I, P, P, L, P, P, P, P, F, I, I, I, I, I, P, I, I, I, I, I, I, I, P, P, I, I, P],
         "llmx_decayed_state_chunks": [P, I, P, I, P, I, P, P, L, P, P, P, I, P, I, P, P, F, I, I, I, I, P, P, I, P],
         "llmx_decayed_state_rows": [],
         "llmx_head_norm_gate": [P, P, P, I, P, I, F, I, I, I, I, I, I, I, F, F, P, P],
@@ -102,7 +103,7 @@ def _declare(h) -> None:
         "llmx_attention_rules_ok": [I, I, I, I],
         "llmx_attention_rules_segment": [],
         "llmx_memory_prep": [P, I, I, I, I, I, P, P, F, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, P],
-        "llmx_paged_attention_mfma": [P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, P, I, P],
+        "llmx_paged_attention_mfma": [P, P, P, P, P, P, P, I, I, I, P, I, P, P, P, F, I, I, I, I, I, I, I, P, I, I, P],
         "llmx_route_topk": [P, P, I, L, P, P, P, I, I, I, I, I, F, P, I, I, I, P],
         "llmx_moe_align": [P, I, I, P, P, P, P, P, P, P, P],
         "llmx_route_topk_align": [P, P, I, L, P, P, P, I, I, I, I, I, F, I, I, I, P, P, P, P, P, P],
@@ -499,13 +500,15 @@ def latent_queries(q: torch.Tensor, cos_sin: torch.Tensor, pos: torch.Tensor, q_
 
 def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tensor, pos: torch.Tensor, row_entry: torch.Tensor,
                      tables: torch.Tensor, out: torch.Tensor, scale: float, window: int = 0, scratch=None,
-                     cache_t: Optional[torch.Tensor] = None, plan: Optional["LatentPlan"] = None, row_major: bool = False) -> None:
+                     cache_t: Optional[torch.Tensor] = None, plan: Optional["LatentPlan"] = None, row_major: bool = False,
+                     sink: Optional[torch.Tensor] = None) -> None:
     """Causal softmax attention of every (head, row) over its request's paged latents, the last `window` keys (0: all): score =
     (q_lat . c + q_rot . k_rot) * scale, result = sum of weights * c.  q_lat and out [H, T, C], q_rot [H, T, R] (with
     `row_major` [T, H, ...]), cache [pages, page_tokens, at least C + R].  `scratch(name, shape, dtype)`: storage that lives as
     long as the caller's step.  With `cache_t` (the latents once more, [pages, C, page_tokens]) and a `plan` (latent_plan, made
     for the same window) the matrix-core kernel runs, where latent_attention_mfma_ok says it can and the cache's rows are
-    latent_cache_width wide with zeros behind the key part; otherwise the universal kernel."""
+    latent_cache_width wide with zeros behind the key part; otherwise the universal kernel.  `sink` [H] float32: one more logit
+    a head in the softmax's denominator, unscaled, without a key or a value."""
     if row_major:
         T, H, C = q_lat.shape
     else:
@@ -529,13 +532,13 @@ def latent_attention(q_lat: torch.Tensor, q_rot: torch.Tensor, cache: torch.Tens
                                                 _dev(tables, "tables", torch.int32), _dev(plan.items, "items", torch.int32), plan.n_items,
                                                 plan.n_tile_items, plan.n_row_items, _dev(plan.merges, "merges", torch.int32), plan.n_merges, _dev(out, "out"),
                                                 _dev(part_o, "part_o"), _dev(part_ml, "part_ml"), float(scale), T, H, C, R, width, page_tokens,
-                                                tables.shape[1], int(window), 1 if row_major else 0, _stream()),
+                                                tables.shape[1], int(window), 1 if row_major else 0, _dev(sink, "sink", torch.float32, (H,)), _stream()),
                "latent_attention_mfma")
         return
     _check(lib().llmx_latent_attention_generic(_dev(q_lat, "q_lat"), _dev(q_rot, "q_rot"), _dev(cache, "cache"), _dev(pos, "pos", torch.int32, (T,)),
                                                _dev(row_entry, "row_entry", torch.int32, (T,)), _dev(tables, "tables", torch.int32),
                                                _dev(out, "out"), _code(q_lat.dtype), float(scale), T, H, C, R, width, page_tokens, tables.shape[1],
-                                               int(window), 1 if row_major else 0, _stream()), "latent_attention")
+                                               int(window), 1 if row_major else 0, _dev(sink, "sink", torch.float32, (H,)), _stream()), "latent_attention")
 
 
 def latent_cache_width(rank: int, rot_dim: int) -> int:
@@ -668,16 +671,16 @@ def rmsnorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: Optional[tor
 
 
 def layernorm(x: torch.Tensor, weight: torch.Tensor, eps: float, out: Optional[torch.Tensor], out32: Optional[torch.Tensor] = None,
-              pick: Optional[torch.Tensor] = None) -> None:
-    """out[r] = (x - mean) / sqrt(var + eps) * weight of row x[pick[r]] (or x[r]), var the mean of the squared deviations;
+              pick: Optional[torch.Tensor] = None, bias: Optional[torch.Tensor] = None) -> None:
+    """out[r] = (x - mean) / sqrt(var + eps) * weight (+ bias) of row x[pick[r]] (or x[r]), var the mean of the squared deviations;
     out in its own dtype, out32 an optional float32 copy."""
     n = x.shape[-1]
     rows = pick.shape[0] if pick is not None else x.shape[0]
     if out is None and out32 is None:
         raise KernelError("layernorm needs an output")
     _check(lib().llmx_layernorm(_dev(x, "x", torch.float32), _dev(pick, "pick", torch.int32), _dev(weight, "weight", torch.float32, (n,)),
-                                float(eps), _dev(out, "out", shape=(rows, n)), _code(out.dtype) if out is not None else F32,
-                                _dev(out32, "out32", torch.float32, (rows, n)), rows, n, _stream()), "layernorm")
+                                _dev(bias, "bias", torch.float32, (n,)), float(eps), _dev(out, "out", shape=(rows, n)),
+                                _code(out.dtype) if out is not None else F32, _dev(out32, "out32", torch.float32, (rows, n)), rows, n, _stream()), "layernorm")
 
 
 def layernorm_add(x: torch.Tensor, y: torch.Tensor, weight: torch.Tensor, eps: float, copy: Optional[torch.Tensor] = None) -> None:
@@ -693,6 +696,13 @@ def cast_rows(x: torch.Tensor, out: torch.Tensor) -> None:
     if out.shape != x.shape:
         raise KernelError("cast_rows: shapes do not agree")
     _check(lib().llmx_cast_rows(_dev(x, "x", torch.float32), _dev(out, "out"), _code(out.dtype), x.numel(), _stream()), "cast_rows")
+
+
+def join_rows(x: torch.Tensor, y: Optional[torch.Tensor], out: torch.Tensor) -> None:
+    """out[t] = [x[t] | y[t]] in out's type, x and y float32 [T, n], out [T, 2n]; y None: the second half is left as it is."""
+    rows, n = x.shape
+    _check(lib().llmx_join_rows(_dev(x, "x", torch.float32), _dev(y, "y", torch.float32, (rows, n)), _dev(out, "out", shape=(rows, 2 * n)),
+                                _code(out.dtype), rows, n, _stream()), "join_rows")
 
 
 def cast_cols(x: torch.Tensor, out: torch.Tensor) -> None:
@@ -726,26 +736,28 @@ def _rows_view(t: torch.Tensor, name: str, rows: int, cols: int):
 def delta_prep(pre: torch.Tensor, conv_w: torch.Tensor, step_pre: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor,
                state: torch.Tensor, tail_off: int, slot_read: torch.Tensor, row_entry: torch.Tensor, entry_rows: torch.Tensor,
                q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, beta: torch.Tensor, G: int, H: int, D: int, V: int,
-               beta_col: int) -> None:
+               beta_col: int, head_decay: bool = False) -> None:
     """A delta-rule mixer's rows made ready for the scan (see csrc/linear_state.hip): from the fused in-projection `pre`
     [T, ld] = q (G*D) | k (G*D) | v (H*V) | ... | beta (H) at beta_col: the short causal convolution (conv_w [C, taps], the
     inputs of earlier steps from the state's tail at `tail_off`) with silu, unit-norm q and k heads, v, the decay
-    exp(-exp(a_log) softplus(step_pre + dt_bias)) [T, H*D] and beta = sigmoid [T, H]."""
+    exp(-exp(a_log) softplus(step_pre + dt_bias)) [T, H*D] and beta = sigmoid [T, H].  `head_decay`: one decay a head, step_pre
+    and decay [T, H], dt_bias [H]."""
     T, ld = pre.shape
+    DW = H if head_decay else H * D
     C = 2 * G * D + H * V
     taps = conv_w.shape[1]
     n_e = entry_rows.shape[0]
     if state.dim() != 2 or tail_off + (taps - 1) * C > state.shape[1]:
         raise KernelError("delta_prep: the state does not hold the convolution's tail")
-    step_at, step_ld = _rows_view(step_pre, "step_pre", T, H * D)
+    step_at, step_ld = _rows_view(step_pre, "step_pre", T, DW)
     _check(lib().llmx_delta_prep(_dev(pre, "pre", torch.float32), ld, _dev(conv_w, "conv_w", torch.float32, (C, taps)),
-                                 step_at, step_ld, _dev(dt_bias, "dt_bias", torch.float32, (H * D,)),
+                                 step_at, step_ld, _dev(dt_bias, "dt_bias", torch.float32, (DW,)),
                                  _dev(a_log, "a_log", torch.float32, (H,)), _dev(state, "state", torch.float32), state.shape[1], int(tail_off),
                                  _dev(slot_read, "slot_read", torch.int32, (n_e,)), _dev(row_entry, "row_entry", torch.int32, (T,)),
                                  _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)), _dev(q, "q", torch.float32, (T, G * D)),
                                  _dev(k, "k", torch.float32, (T, G * D)), _dev(v, "v", torch.float32, (T, H * V)),
-                                 _dev(decay, "decay", torch.float32, (T, H * D)), _dev(beta, "beta", torch.float32, (T, H)),
-                                 T, G, H, D, V, taps, int(beta_col), _stream()), "delta_prep")
+                                 _dev(decay, "decay", torch.float32, (T, DW)), _dev(beta, "beta", torch.float32, (T, H)),
+                                 T, G, H, D, V, taps, int(beta_col), 1 if head_decay else 0, _stream()), "delta_prep")
 
 
 def sigmoid_root(z: torch.Tensor, bias: Optional[torch.Tensor], tau: float, out: torch.Tensor) -> None:
@@ -782,7 +794,7 @@ def state_matrix_plain(flat: torch.Tensor, H: int, D: int, V: int) -> torch.Tens
 def state_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, beta: Optional[torch.Tensor], state: torch.Tensor,
                slot_read: torch.Tensor, slot_write: torch.Tensor, entry_rows: torch.Tensor, out: torch.Tensor, out_scale: float,
                H: int, qk_heads: int, D: int, V: int, tail=None, max_rows: int = 0, operands: Optional["StateOperands"] = None,
-               max_rows_here: int = 0) -> None:
+               max_rows_here: int = 0, head_decay: bool = False) -> None:
     """The matrix-state recurrence over each entry's rows (csrc/linear_state.hip): per head S <- diag(decay) S;
     u = beta (v - S^T k) (u = v without beta); S <- S + k u^T; out = out_scale * S^T q.  q, k [T, qk_heads*D], v [T, H*V],
     decay [T, H*D] are float32 views whose rows may be columns of wider tensors; state [slots, width] float32 holds S at
@@ -791,7 +803,7 @@ def state_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     single tokens stage smaller chunks; the results are the same).  `tail` = (source [T, C] view, taps, offset):
     the convolution tail [taps - 1, C] at `offset` of the state is handed on from the step's rows of `source`.  `operands`: what
     is made of q, k and v as they are read (None: nothing).  `max_rows_here` > 0: entries of more rows are left alone (another
-    kernel takes them: decayed_state_chunks)."""
+    kernel takes them: decayed_state_chunks).  `head_decay`: decay [T, H], one for all of a head's key channels."""
     T = out.shape[0]
     n_e = entry_rows.shape[0]
     if H % qk_heads or state.dim() != 2 or state.shape[1] < state_matrix_size(H, D, V) or D > 256:
@@ -799,7 +811,7 @@ def state_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
     qa, ldq = _rows_view(q, "q", T, qk_heads * D)
     ka, ldk = _rows_view(k, "k", T, qk_heads * D)
     va, ldv = _rows_view(v, "v", T, H * V)
-    ga, ldg = _rows_view(decay, "decay", T, H * D)
+    ga, ldg = _rows_view(decay, "decay", T, H if head_decay else H * D)
     ta, tld, tC, taps, toff = 0, 0, 0, 0, 0
     if tail is not None:
         src, taps, toff = tail
@@ -811,7 +823,7 @@ def state_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.T
                                  state.shape[1], _dev(slot_read, "slot_read", torch.int32, (n_e,)), _dev(slot_write, "slot_write", torch.int32, (n_e,)),
                                  _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)), _dev(out, "out", torch.float32, (T, H * V)), float(out_scale),
                                  n_e, H, H // qk_heads, D, V, ta, tld, tC, int(taps), int(toff), int(max_rows), int(max_rows_here),
-                                 *_operand_args(operands, T, D), _stream()), "state_scan")
+                                 *_operand_args(operands, T, D), 1 if head_decay else 0, _stream()), "state_scan")
 
 
 OPERANDS_PLAIN, OPERANDS_SILU, OPERANDS_ROTATED = 0, 1, 2
@@ -1021,15 +1033,20 @@ def gemm_f32_takes_normed_rows(rows: int, w: torch.Tensor) -> bool:
     return rows <= NORMED_ROWS_PAY and gemm_f32_can_norm_rows(rows, w)
 
 
-ACT_NONE, ACT_XIELU, ACT_RELU2 = 0, 1, 2      # activations a storing product can apply to what it stores (RELU2: max(z, 0)^2, no numbers)
+# activations a storing product can apply to what it stores: xIELU (two numbers), RELU2: max(z, 0)^2; BIAS: z + b_n and GELU_BIAS: the
+# exact gelu of z + b_n, b one number a feature.  BIAS goes with the adding epilogue too: c + (z + b_n)
+ACT_NONE, ACT_XIELU, ACT_RELU2, ACT_BIAS, ACT_GELU_BIAS = 0, 1, 2, 3, 4
 
 
-def _act_args(act, epilogue: int, what: str):
-    """The two values the product kernels take for `act` = (kind, params or None)."""
+def _act_args(act, epilogue: int, what: str, features: int = 0):
+    """The two values the product kernels take for `act` = (kind, params or None); `features`: the product's."""
     if act is None:
         return 0, 0
+    if act[0] in (ACT_BIAS, ACT_GELU_BIAS) and epilogue in ((EPI_STORE, EPI_ADD) if act[0] == ACT_BIAS else (EPI_STORE,)):
+        return act[0], _dev(act[1], "activation parameters", torch.float32, (features,))
     if epilogue != EPI_STORE or act[0] not in (ACT_XIELU, ACT_RELU2):
-        raise KernelError(f"{what}: an activation goes with the store epilogue, and xIELU and the squared relu are the ones built")
+        raise KernelError(f"{what}: an activation goes with the store epilogue (a bias with the adding one too), and xIELU, the squared relu, "
+                          f"a bias and the gelu of a biased value are the ones built")
     if act[0] == ACT_XIELU:
         return ACT_XIELU, _dev(act[1], "activation parameters", torch.float32, (2,))
     return ACT_RELU2, 0
@@ -1055,8 +1072,8 @@ def gemm(a, w: torch.Tensor, c: torch.Tensor, epilogue: int = EPI_STORE, force_g
     `a` may be NormedRows where gemm_takes_normed_rows says so: the product reads bfloat16(norm(x)).
     `scratch(name, shape, dtype)` gives storage that lives as long as the caller's step (a step's workspace): with it,
     products of some tens of rows multiply K's runs in workgroups of their own; the bits are the same either way.
-    `act` = (ACT_XIELU, params) | (ACT_RELU2, None): with EPI_STORE, c = activation(a @ w^T), params the activation's
-    numbers on the device (xIELU: float32 (p, q)); the bits of the product followed by the activation's own kernel (act_xielu).
+    `act` = (ACT_XIELU, params) | (ACT_RELU2, None) | (ACT_BIAS, b) | (ACT_GELU_BIAS, b): with EPI_STORE, c = activation(a @ w^T),
+    params the activation's numbers on the device (xIELU: float32 (p, q); b: float32 [N], ACT_BIAS with EPI_ADD too); the bits of the product followed by the activation's own kernel (act_xielu).
     `glu`: the gated epilogue's unit (see Glu); None: silu(gate) * up."""
     M, K = a.shape
     if _glu_apart(glu, epilogue):
@@ -1067,8 +1084,8 @@ def gemm(a, w: torch.Tensor, c: torch.Tensor, epilogue: int = EPI_STORE, force_g
         act_glu(pre, glu, c)
         return
     glu_args = glu.args(M) if glu is not None and not glu.plain else _NO_GLU
-    act_args = _act_args(act, epilogue, "gemm")
     N = w.shape[0] // 2 if epilogue == EPI_SWIGLU else w.shape[0]   # swiglu: w holds gate rows, then up rows
+    act_args = _act_args(act, epilogue, "gemm", N)
     if w.shape[1] != K or tuple(c.shape) != (M, N):
         raise KernelError(f"gemm shapes do not agree: a {tuple(a.shape)}, w {tuple(w.shape)}, c {tuple(c.shape)}")
     if isinstance(a, NormedRows):
@@ -1167,10 +1184,16 @@ def qknorm_rope_kvwrite(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_w
                         pos: torch.Tensor, row_entry: torch.Tensor, tables: torch.Tensor, q_out: torch.Tensor,
                         k_cache: torch.Tensor, v_cache: torch.Tensor, eps: float, n_heads: int, n_kv_heads: int, head_dim: int,
                         rotary_dim: int, norm_mode: int, write_kv: bool = True, pairing: int = ROPE_HALVES) -> None:
+    """From float32 rows qkv = q (H*D) | k (G*D) | v (G*VD) | ...: an RMS norm over all of q and over all of k (norm_mode
+    QKNORM_PROJECTION; QKNORM_NONE: none), the rotation a head, q to q_out, k and v to the row's page.  The value width VD is
+    the value cache's; what follows v in a row is left alone."""
     rows = qkv.shape[0]
     qw, kw = n_heads * head_dim, n_kv_heads * head_dim
     n_pages, hk, page_tokens, d = k_cache.shape
-    if ((hk, d) != (n_kv_heads, head_dim) or tuple(v_cache.shape) != (n_pages, hk, d, page_tokens) or k_cache.dtype != q_out.dtype
+    v_dim = v_cache.shape[2]
+    if qkv.dim() != 2 or qkv.shape[1] < qw + kw + n_kv_heads * v_dim:
+        raise KernelError(f"qknorm_rope_kvwrite: rows of {tuple(qkv.shape)} do not hold q | k | v")
+    if ((hk, d) != (n_kv_heads, head_dim) or tuple(v_cache.shape) != (n_pages, hk, v_dim, page_tokens) or k_cache.dtype != q_out.dtype
             or v_cache.dtype != q_out.dtype):
         raise KernelError("qknorm_rope_kvwrite: cache shape or dtype does not fit the heads")
     if rotary_dim % 2 or rotary_dim > head_dim or cos_sin.shape[1] != rotary_dim:
@@ -1181,11 +1204,11 @@ def qknorm_rope_kvwrite(qkv: torch.Tensor, q_weight: Optional[torch.Tensor], k_w
     elif norm_mode != QKNORM_NONE:
         raise KernelError("qknorm_rope_kvwrite: only a norm over the whole projection, or none, is built")
     _check(lib().llmx_qknorm_rope_kvwrite(
-        _dev(qkv, "qkv", torch.float32, (rows, qw + 2 * kw)), _dev(q_weight, "q_weight"), _dev(k_weight, "k_weight"),
+        _dev(qkv, "qkv", torch.float32), _dev(q_weight, "q_weight"), _dev(k_weight, "k_weight"),
         _dev(cos_sin, "cos_sin", torch.float32), _dev(pos, "pos", torch.int32, (rows,)), _dev(row_entry, "row_entry", torch.int32, (rows,)),
         _dev(tables, "tables", torch.int32), _dev(q_out, "q_out", shape=(rows, qw)), _dev(k_cache, "k_cache"), _dev(v_cache, "v_cache"),
         _code(q_out.dtype), float(eps), rows, n_heads, n_kv_heads, head_dim, rotary_dim, norm_mode, page_tokens, tables.shape[1],
-        1 if write_kv else 0, int(pairing), _stream()), "qknorm_rope_kvwrite")
+        1 if write_kv else 0, int(pairing), qkv.shape[1], v_dim, _stream()), "qknorm_rope_kvwrite")
 
 
 def head_norm_rope_kvwrite(qkv: torch.Tensor, bias: Optional[torch.Tensor], q_weight: Optional[torch.Tensor], k_weight: Optional[torch.Tensor],
@@ -1453,7 +1476,7 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     a width of their own (v_cache [pages, kv_heads, v_dim, page_tokens], out [rows, heads * v_dim]).  `head_gate`: a float32
     view [rows, heads] (its rows may be columns of a wider projection): the result of (row, head) is multiplied by the
     sigmoid of its entry before it is stored, by whichever kernel stores it.  `output_gate`: such a view [rows, heads * v_dim],
-    a logit a value of the result (the universal kernel).  `rules` (ScoreRules): the universal kernel's further score and
+    a logit a value of the result, whichever kernel stores it.  `rules` (ScoreRules): the universal kernel's further score and
     visibility rules; with several maps `out` may be float32 whatever the cache's type (a later kernel joins the maps).
     `rules_plan` (from `rules_plan`, for this step's rows and these rules): where the sizes allow (`attention_rules_ok`) the
     matrix-core kernel for rules runs instead of the universal one."""
@@ -1470,7 +1493,12 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     common = (_dev(q, "q"), _dev(k_cache, "k_cache"), _dev(v_cache, "v_cache", shape=(n_pages, n_kv_heads, v_dim, page_tokens)),
               _dev(pos, "pos", torch.int32, (rows,)), _dev(row_entry, "row_entry", torch.int32, (rows,)), _dev(tables, "tables", torch.int32))
     gate_at, gate_ld = _rows_view(head_gate, "head_gate", rows, n_heads) if head_gate is not None else (None, 0)
-    special = (rules is not None and not rules.plain) or output_gate is not None
+    if output_gate is not None and (head_gate is not None or maps != 1):
+        raise KernelError("paged_attention: one gate, and on one map a head")
+    gate_wide = 1 if output_gate is not None else 0
+    if gate_wide:
+        gate_at, gate_ld = _rows_view(output_gate, "output_gate", rows, n_heads * v_dim)
+    special = rules is not None and not rules.plain
     if plan is not None and plan.n_items and v_dim == head_dim and attention_mfma_ok(q.dtype, head_dim, page_tokens) and not special:
         part_o = part_ml = None
         if plan.n_slots:
@@ -1484,15 +1512,9 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
                                                _dev(plan.merges, "merges", torch.int32), plan.n_merges, _dev(out, "out"),
                                                _dev(part_o, "part_o"), _dev(part_ml, "part_ml"), float(scale), n_heads, n_kv_heads,
                                                head_dim, page_tokens, tables.shape[1], int(window), (1 if plan.wide_items else 0) | (2 if plan.short_merge else 0), gate_at, gate_ld,
-                                               _stream()),
+                                               gate_wide, _stream()),
                "paged_attention_mfma")
         return
-    gate_wide = 0
-    if output_gate is not None:
-        if head_gate is not None or maps != 1:
-            raise KernelError("paged_attention: one gate, and on one map a head")
-        gate_at, gate_ld = _rows_view(output_gate, "output_gate", rows, n_heads * v_dim)
-        gate_wide = 1
     r = rules if rules is not None else ScoreRules()
     if rules_plan is not None and (rules_plan.n_items or rules_plan.n_group_items) and attention_rules_ok(q.dtype, head_dim, v_dim, page_tokens):
         part_o = part_ml = None

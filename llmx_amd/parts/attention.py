@@ -107,9 +107,9 @@ class Attention(Mixer):
             raise ValueError("attention: a gate a head or a gate a value, not both")
         if self.difference and (self.head_gate or self.head_temperature):
             raise ValueError("attention: two score maps a head go without a gate or temperature a head")
-        # what only the universal kernel carries out
+        # what the plain kernels do not carry out (a gate a value they do)
         self.special = bool(self.keep_first or self.chunk or self.softcap or self.distance_slopes or self.sink or self.values_from_keys
-                            or self.value_norm or self.output_gate or self.difference)
+                            or self.value_norm or self.difference)
         self.names = dict(_NAMES)
         unknown = set(p.get("names") or {}) - set(_NAMES)
         if unknown:
@@ -119,12 +119,12 @@ class Attention(Mixer):
         self.kv_width = self.kv_heads * self.maps * self.head_dim
         self.v_width = 0 if self.values_from_keys else self.kv_heads * self.v_dim
         self.o_width = self.heads * self.v_dim
-        # the plain case (one width, no biases, no norm a head) keeps the kernel that norms whole projections
-        self.by_head = (self.norm_mode == ops.QKNORM_HEAD or self.bias or self.v_dim != self.head_dim or self.head_temperature
-                        or self.head_gate or self.special)
+        # the plain case (no biases, no norm a head) keeps the kernel that norms whole projections
+        self.by_head = (self.norm_mode == ops.QKNORM_HEAD or self.bias or self.head_temperature or self.special
+                        or (self.norm_mode == ops.QKNORM_NONE and (self.head_gate or self.v_dim != self.head_dim)))
         self.gate_width = self.heads if self.head_gate else self.o_width if self.output_gate else 0
         if self.by_head and self.norm_mode == ops.QKNORM_PROJECTION:
-            raise ValueError("attention: a norm over the whole projection goes with values as wide as keys and no biases")
+            raise ValueError("attention: a norm over the whole projection goes with no biases, temperature or further rules")
         self.wqkv = self.wo = self.q_norm = self.k_norm = self.b_qkv = self.b_o = self.temperature = None
         self.sink_logits = self.slopes = self.rules = None
         self.lam = 0.0
@@ -193,7 +193,7 @@ class Attention(Mixer):
             # one number for the layer, formed once from the four vectors
             lq1, lk1, lq2, lk2 = (tensors[self.tensor(r)].to(torch.float64) for r in ("lambda_q1", "lambda_k1", "lambda_q2", "lambda_k2"))
             self.lam = float(torch.exp((lq1 * lk1).sum()) - torch.exp((lq2 * lk2).sum())) + self.diff
-        if self.special:
+        if self.special or self.v_dim != self.head_dim:
             self.rules = ops.ScoreRules(self.keep_first, self.chunk, self.softcap, self.slopes, self.sink_logits, self.maps)
 
     def output_bias(self):
@@ -222,7 +222,8 @@ class Attention(Mixer):
                                                   self.maps, step.device, window, self.keep_first, self.chunk, shared=shared))
 
     def _rules_mfma(self, act, page_tokens):
-        return self.special and ops.attention_rules_ok(act, self.head_dim, self.v_dim, page_tokens)
+        # also where values have a width of their own, which the plain matrix-core kernel does not take
+        return (self.special or self.v_dim != self.head_dim) and ops.attention_rules_ok(act, self.head_dim, self.v_dim, page_tokens)
 
     def graph_key(self, step):
         # a recorded step holds the plan's addresses and launch sizes; the universal kernel has no plan

@@ -170,12 +170,12 @@ class Embedding(Part):
 
 
 class ResidualInput(Part):
-    """Something added to the residual between two run-order entries (before the entry that names it)."""
+    """Something done to the residual between two run-order entries (before the entry that names it): added, or put in its place."""
     #: True when forward wants the embedding's rows as the step's first layer saw them; the engine then keeps a copy
     wants_embedding = False
 
     def forward(self, step, x: torch.Tensor, embedding_rows: Optional[torch.Tensor]) -> None:
-        """x (float32 [T, hidden]) += the part's addition; embedding_rows: float32 [T, hidden] when wanted, else None."""
+        """x (float32 [T, hidden]) += the part's addition, or what the part makes of x; embedding_rows: float32 [T, hidden] when wanted, else None."""
         raise NotImplementedError
 
 

@@ -1,6 +1,6 @@
 """The arrangements of a layer's parts.
 
-"prenorm": x += mixer(norm(x)); x += ffn(norm(x)) with the residual x in float32: the arrangement of
+"prenorm": x += mixer(norm(x)); x += ffn(norm(x)) with the residual x in float32 (the second optional): the arrangement of
 /root/reference/src/model/arch/minimax_m3.hpp:247-287 (norm, mixer joined into the residual, norm, feed-forward joined).
 "parallel": x += s1 * mixer(norm1(x)) + s2 * ffn(norm2(x)) with both norms of the same x, learned factors s1, s2 a
 coordinate (or constants), and an optional per-layer token input after the sum; without a second norm both sublayers read
@@ -26,11 +26,13 @@ class PreNormBlock:
     def __init__(self, spec: BlockSpec, ctx: BuildContext):
         self.mixer_norm = build_part("norm", spec.mixer_norm, ctx)
         self.mixer = build_part("mixer", spec.mixer, ctx)
-        self.ffn_norm = build_part("norm", spec.ffn_norm, ctx)
-        self.ffn = build_part("feed_forward", spec.ffn, ctx)
+        if (spec.ffn is None) != (spec.ffn_norm is None):
+            raise ValueError("prenorm block: a feed-forward comes with its norm, and a norm with its feed-forward")
+        self.ffn_norm = build_part("norm", spec.ffn_norm, ctx) if spec.ffn_norm is not None else None
+        self.ffn = build_part("feed_forward", spec.ffn, ctx) if spec.ffn is not None else None
 
     def parts(self):
-        return [self.mixer_norm, self.mixer, self.ffn_norm, self.ffn]
+        return [p for p in (self.mixer_norm, self.mixer, self.ffn_norm, self.ffn) if p is not None]
 
     @staticmethod
     def normed(step, norm, part, x):
@@ -49,6 +51,8 @@ class PreNormBlock:
     def forward(self, step, x: torch.Tensor, cache: LayerCache) -> None:
         h, h32 = self.normed(step, self.mixer_norm, self.mixer, x)
         self.mixer.forward(step, h, x, True, cache, h32)
+        if self.ffn is None:
+            return
         h, h32 = self.normed(step, self.ffn_norm, self.ffn, x)
         self.ffn.forward(step, h, x, True, h32)
 

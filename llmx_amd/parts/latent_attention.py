@@ -4,7 +4,7 @@ Per row, from the input h:  q = W_q h, or through a latent of its own q = W_uq r
 rot_dim rotated];  W_dkv h = [latent of kv_rank | one key part of rot_dim]: the latent is RMS-normed (weight `dkv.norm`) and
 is, with the rotated key part that all heads share, all that is cached.  Head n's key for a token is [W_uk,n c | k_rot], its
 value W_uv,n c; score = (q_plain . W_uk,n c + q_rot . k_rot) * scale, softmax over the request's keys up to the row (the last
-`window` of them), and the head's result is multiplied by sigmoid(W_g h)_n, where there is a gate, before the output
+`window` of them; with a sink the denominator also holds exp(sink_n), a learned number a head), and the head's result is multiplied by sigmoid(W_g h)_n, where there is a gate, before the output
 projection.
 
 Neither keys nor values are ever expanded: q_lat = W_uk,n^T q_plain (a grouped product, one group a head) turns the
@@ -28,8 +28,9 @@ MAX_LATENT_KEY = 4096      # latent + rotated key part: a query row in a workgro
 class LatentAttention(Mixer):
     """params: hidden, heads, dim (unrotated query/key dims a head), rot_dim (rotated dims a head), vdim, kv_rank, scale (the
     factor on the scores), eps (of the latents' norms), gate ("head_sigmoid" | None), position (PartSpec of a rotary encoding
-    whose dims are at most rot_dim), window (None: every earlier key), q_rank (None: one query projection).
-    Tensors <prefix>q (or dq, dq.norm, uq), dkv, dkv.norm, uk, uv, g, o."""
+    whose dims are at most rot_dim), window (None: every earlier key), q_rank (None: one query projection), sink (True: a logit
+    a head in the softmax's denominator).
+    Tensors <prefix>q (or dq, dq.norm, uq), dkv, dkv.norm, uk, uv, g, sink, o."""
     graph_safe = True
 
     def __init__(self, params, prefix, ctx: BuildContext):
@@ -45,6 +46,7 @@ class LatentAttention(Mixer):
         self.scale = float(p["scale"])
         self.window = int(p["window"]) if p.get("window") else None
         self.q_rank = int(p["q_rank"]) if p.get("q_rank") else 0
+        self.sink = bool(p.get("sink", False))
         self.gate = p.get("gate", "head_sigmoid")
         if self.gate not in ("head_sigmoid", None):
             raise ValueError(f"latent attention: gate {self.gate!r} is not 'head_sigmoid' or None")
@@ -66,6 +68,7 @@ class LatentAttention(Mixer):
         self.first_width = self.q_rank or self.q_width
         # without a gate the heads' rows lie row by row, so that the last grouped product stores what the output projection reads
         self.row_major = self.gate is None
+        self.sink_logits = None
         self.w_in = self.w_o = self.latent_norm = self.q_norm = self.w_uq = self.w_uk_t = self.w_uv = None
 
     def _matrix_cores(self) -> bool:
@@ -94,6 +97,8 @@ class LatentAttention(Mixer):
                  TensorSpec(self.name("o"), (E, self.heads * self.vdim))]
         if self.q_rank:
             specs += [TensorSpec(self.name("dq.norm"), (self.q_rank,), "norm"), TensorSpec(self.name("uq"), (self.q_width, self.q_rank))]
+        if self.sink:
+            specs.append(TensorSpec(self.name("sink"), (self.heads,), "bias", dtype="float32", init=("uniform", -1.0, 1.0)))
         if g:
             specs.append(TensorSpec(self.name("g"), (g, E), into=(fused, shape, (slice(q + d, q + d + g),))))
         return specs
@@ -102,6 +107,8 @@ class LatentAttention(Mixer):
         self.w_in = tensors[self.name("in")]
         self.w_o = tensors[self.name("o")]
         self.latent_norm = tensors[self.name("dkv.norm")]
+        if self.sink:
+            self.sink_logits = tensors[self.name("sink")]
         if self.q_rank:
             self.q_norm, self.w_uq = tensors[self.name("dq.norm")], tensors[self.name("uq")]
         # q_lat = W_uk,n^T q_plain: the grouped product wants each head's matrix as [out = kv_rank, in = dim]
@@ -150,7 +157,7 @@ class LatentAttention(Mixer):
                          active, n_active, token_rows=T)
         mixed = step.buf("latent.mixed", (*lead, self.rank), act)
         ops.latent_attention(q_lat, q_rot, latents, step.positions, step.row_entry, tables, mixed, self.scale, window=self.window or 0,
-                             scratch=step.buf, cache_t=cache_t, plan=self._plan(step), row_major=self.row_major)
+                             scratch=step.buf, cache_t=cache_t, plan=self._plan(step), row_major=self.row_major, sink=self.sink_logits)
         joined = step.buf("latent.joined", (T, H * self.vdim), act)
         values = joined.view(H * T, self.vdim) if self.row_major else step.buf("latent.values", (H * T, self.vdim), torch.float32)
         ops.grouped_gemm(mixed.view(H * T, self.rank), self.w_uv, values, offsets, pairs, 1, ops.EPI_STORE, active, n_active, token_rows=T)

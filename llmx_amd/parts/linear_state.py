@@ -5,6 +5,7 @@ All decay S's rows (channel by channel, or a head's all alike) and add an outer 
     gated linear attention:  u_t = v_t,                               g_t = sigmoid(z_t)^(1/tau)
     constant decay a head:   u_t = v_t,                               g_t = a number of the model
     gated delta rule:        u_t = beta_t (v_t - (diag(g_t) S_(t-1))^T k_t),   g_t = exp(-exp(A) softplus(step_t + dt_bias))
+    the same a head:         g_t one number for all of a head's key channels, from a projection of the input to one number a head
 with z_t and step_t low-rank projections of the input.  The delta rule's q, k and v first pass a short causal convolution
 over time and silu, and q and k are made unit vectors a head.  The read-out is RMS-normed a head, gated, and projected.
 Products may read rounded rows; decays, gates, unit norms, the recurrence and the state are float32 in both paths.
@@ -75,6 +76,74 @@ class GatedLinearAttention(Mixer):
         ops.state_scan(view("q"), view("k"), view("v"), decay, None, cache.state, step.entry_held_slots, step.entry_slots, step.entry_rows, o,
                        float(D) ** -0.5, H, H, D, V, max_rows=step.max_rows_per_entry)
         gated = step.buf("gla.gated", (T, H * V), step.act_dtype)
+        ops.head_norm_gate(o, self.norm, view("g"), gated, self.eps, H, V, ops.GATE_SILU)
+        ops.gemm(gated, self.w_o, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)
+
+
+class HeadDeltaRule(Mixer):
+    """The gated delta rule with one decay a head: g = exp(-exp(A_log_h) softplus(W_a h + dt_bias)).
+    params: hidden, heads, kv_heads (q and k heads; head h reads q/k head h / (heads / kv_heads)), dim, vdim, conv (taps), eps.
+    Tensors <prefix>q, k, v (+ .conv [channels, taps]), b, a, A_log, dt_bias, g, norm, o; every projection of the input is part of
+    one product.  result = W_o (rmsnorm_head(o) * w * silu(W_g h)).  Convolutions, unit norms, decays, the recurrence and its
+    state are float32 in both paths."""
+    graph_safe = True
+    steps_between_slots = True
+
+    def __init__(self, params, prefix, ctx):
+        super().__init__(params, prefix, ctx)
+        p = params
+        self.hidden, self.heads, self.kv_heads = int(p["hidden"]), int(p["heads"]), int(p["kv_heads"])
+        self.dim, self.vdim, self.taps = int(p["dim"]), int(p["vdim"]), int(p["conv"])
+        self.eps = float(p["eps"])
+        if min(self.heads, self.kv_heads, self.dim, self.vdim, self.taps) < 1 or self.dim > 256:
+            raise ValueError("delta rule: heads, kv_heads, dim (at most 256), vdim and conv are at least 1")
+        if self.heads % self.kv_heads:
+            raise ValueError("delta rule: the head count must be divisible by the q/k head count")
+        GD, HV, H = self.kv_heads * self.dim, self.heads * self.vdim, self.heads
+        self.channels = 2 * GD + HV
+        # the fused in-projection's columns: q | k | v (the convolved channels, in this order) | g | b | a
+        C = self.channels
+        self.cols = {"q": (0, GD), "k": (GD, GD), "v": (2 * GD, HV), "g": (C, HV), "b": (C + HV, H), "a": (C + HV + H, H)}
+        self.in_width = C + HV + 2 * H
+        self.state_matrix = ops.state_matrix_size(H, self.dim, self.vdim)
+        self.w_in = self.conv = self.a_log = self.dt_bias = self.norm = self.w_o = None
+
+    def cache_need(self):
+        return StateNeed((self.state_matrix + (self.taps - 1) * self.channels,), "float32")
+
+    def tensor_specs(self, available):
+        E, H, V = self.hidden, self.heads, self.vdim
+        fused, shape = self.name("in"), (self.in_width, E)
+        specs = [TensorSpec(self.name(n), (w, E), into=(fused, shape, (slice(at, at + w),))) for n, (at, w) in self.cols.items()]
+        taps_of, taps_shape = self.name("conv"), (self.channels, self.taps)
+        specs += [TensorSpec(self.name(f"{n}.conv"), (self.cols[n][1], self.taps), "bias",
+                             into=(taps_of, taps_shape, (slice(self.cols[n][0], self.cols[n][0] + self.cols[n][1]),)), init=("uniform", -0.5, 0.5))
+                  for n in ("q", "k", "v")]
+        return specs + [TensorSpec(self.name("A_log"), (H,), "bias", init=("uniform", -1.0, 1.0)),
+                        TensorSpec(self.name("dt_bias"), (H,), "bias"),
+                        TensorSpec(self.name("norm"), (V,), "norm"),
+                        TensorSpec(self.name("o"), (E, H * V))]
+
+    def load(self, tensors):
+        self.w_in, self.conv = tensors[self.name("in")], tensors[self.name("conv")]
+        self.a_log, self.dt_bias = tensors[self.name("A_log")], tensors[self.name("dt_bias")]
+        self.norm, self.w_o = tensors[self.name("norm")], tensors[self.name("o")]
+
+    def forward(self, step, h, out, accumulate, cache: LayerCache, h32=None):
+        T, H, G, D, V = step.rows, self.heads, self.kv_heads, self.dim, self.vdim
+        f32 = torch.float32
+        pre = step.buf("delta.pre", (T, self.in_width), f32)
+        ops.gemm(h, self.w_in, pre, scratch=step.buf)
+        view = lambda n: pre[:, self.cols[n][0]:self.cols[n][0] + self.cols[n][1]]
+        q, k = step.buf("delta.q", (T, G * D), f32), step.buf("delta.k", (T, G * D), f32)
+        v, decay, beta = step.buf("delta.v", (T, H * V), f32), step.buf("delta.head_decay", (T, H), f32), step.buf("delta.beta", (T, H), f32)
+        ops.delta_prep(pre, self.conv, view("a"), self.dt_bias, self.a_log, cache.state, self.state_matrix, step.entry_held_slots,
+                       step.row_entry, step.entry_rows, q, k, v, decay, beta, G, H, D, V, self.cols["b"][0], head_decay=True)
+        o = step.buf("delta.o", (T, H * V), f32)
+        tail = (pre[:, :self.channels], self.taps, self.state_matrix) if self.taps > 1 else None
+        ops.state_scan(q, k, v, decay, beta, cache.state, step.entry_held_slots, step.entry_slots, step.entry_rows, o, float(D) ** -0.5,
+                       H, G, D, V, tail=tail, max_rows=step.max_rows_per_entry, head_decay=True)
+        gated = step.buf("delta.gated", (T, H * V), step.act_dtype)
         ops.head_norm_gate(o, self.norm, view("g"), gated, self.eps, H, V, ops.GATE_SILU)
         ops.gemm(gated, self.w_o, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)
 
@@ -311,3 +380,4 @@ register("mixer", "decayed_linear_attention", DecayedLinearAttention)
 register("mixer", "gated_matrix_memory", GatedMatrixMemory)
 register("mixer", "gated_linear_attention", GatedLinearAttention)
 register("mixer", "channel_delta_rule", ChannelDeltaRule)
+register("mixer", "head_delta_rule", HeadDeltaRule)

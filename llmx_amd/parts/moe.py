@@ -271,8 +271,9 @@ class DenseGLU(FeedForward):
 
 
 class DenseAct(FeedForward):
-    """params: hidden, intermediate, activation ("xielu" | "polynorm"), eps (polynorm).  y = W_down act(W_up h); tensors
-    <prefix>up, down, and <prefix>act: for xIELU (p, q): act(z) = softplus(p) z^2 + z/2 for z > 0, (1/2 + softplus(q))
+    """params: hidden, intermediate, activation ("xielu" | "polynorm" | "gelu"), eps (polynorm).  y = W_down act(W_up h); tensors
+    <prefix>up, down; for gelu (the exact one) also the biases up.b and down.b: y = W_down gelu(W_up h + b) + b'; for the others
+    <prefix>act: for xIELU (p, q): act(z) = softplus(p) z^2 + z/2 for z > 0, (1/2 + softplus(q))
     (e^z - 1 - z) + z/2 otherwise; for polynorm (a, b, c, e): act(z) = a U(z) + b U(z^2) + c U(z^3) + e with powers element by
     element and U dividing a row of inner values by its root mean square (eps inside the root): it needs the whole row, so
     it is a kernel of its own between the two products, in float32."""
@@ -283,13 +284,17 @@ class DenseAct(FeedForward):
         self.hidden = int(params["hidden"])
         self.intermediate = int(params["intermediate"])
         self.activation = str(params.get("activation", "xielu"))
-        if self.activation not in ("xielu", "polynorm"):
-            raise ValueError(f"dense feed-forward: activation {self.activation!r} is not one of ['polynorm', 'xielu']")
+        if self.activation not in ("xielu", "polynorm", "gelu"):
+            raise ValueError(f"dense feed-forward: activation {self.activation!r} is not one of ['gelu', 'polynorm', 'xielu']")
         self.eps = float(params.get("eps", 0.0))
-        self.w_up = self.w_down = self.act = None
+        self.biased = self.activation == "gelu"
+        self.w_up = self.w_down = self.act = self.b_up = self.b_down = None
 
     def tensor_specs(self, available):
         F, E = self.intermediate, self.hidden
+        if self.biased:
+            return [TensorSpec(self.name("up"), (F, E)), TensorSpec(self.name("up.b"), (F,), "bias"),
+                    TensorSpec(self.name("down"), (E, F)), TensorSpec(self.name("down.b"), (E,), "bias")]
         numbers = 2 if self.activation == "xielu" else 4
         return [TensorSpec(self.name("up"), (F, E)), TensorSpec(self.name("down"), (E, F)),
                 TensorSpec(self.name("act"), (numbers,), "bias", dtype="float32", init=("uniform", -1.0, 1.0))]
@@ -297,7 +302,10 @@ class DenseAct(FeedForward):
     def load(self, tensors):
         self.w_up = tensors[self.name("up")]
         self.w_down = tensors[self.name("down")]
-        self.act = tensors[self.name("act")]
+        if self.biased:
+            self.b_up, self.b_down = tensors[self.name("up.b")], tensors[self.name("down.b")]
+        else:
+            self.act = tensors[self.name("act")]
 
     def forward(self, step, h, out, accumulate, h32=None):
         a = step.buf("dense.act", (step.rows, self.intermediate), step.act_dtype)
@@ -305,6 +313,10 @@ class DenseAct(FeedForward):
             z = step.buf("dense.pre", (step.rows, self.intermediate), torch.float32)
             ops.gemm(h, self.w_up, z, scratch=step.buf)
             ops.act_polynorm(z, self.act, self.eps, a)
+        elif self.biased:       # both biases and the activation in the products' epilogues
+            ops.gemm(h, self.w_up, a, scratch=step.buf, act=(ops.ACT_GELU_BIAS, self.b_up))
+            ops.gemm(a, self.w_down, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf, act=(ops.ACT_BIAS, self.b_down))
+            return
         else:
             ops.gemm(h, self.w_up, a, scratch=step.buf, act=(ops.ACT_XIELU, self.act))      # the activation in the product's epilogue
         ops.gemm(a, self.w_down, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)

@@ -1,5 +1,5 @@
-"""Norms of float32 rows.  RMSNorm: y = x * (r * w), r = 1/sqrt(mean(x^2) + eps); LayerNorm (a weight, no bias):
-y = (x - mean) / sqrt(var + eps) * w, var the mean of the squared deviations.  All in float32.
+"""Norms of float32 rows.  RMSNorm: y = x * (r * w), r = 1/sqrt(mean(x^2) + eps); LayerNorm (a weight, a bias if there is one):
+y = (x - mean) / sqrt(var + eps) * w (+ b), var the mean of the squared deviations.  All in float32.
 
 Order of operations as the reference computes it (/root/reference/src/backends/cpu/cpu_backend.hpp:1437-1459): the
 reciprocal root times the weight is formed first, then multiplied into x.
@@ -72,8 +72,8 @@ class RMSNorm(Norm):
 
 class LayerNorm(Norm):
     """params: width, eps; tensor (the name's last part, "weight" by default; "" when the prefix is the whole name).
-    Tensor: <prefix><tensor>, (width,).  `add_into` is the form an arrangement uses that norms a sublayer's result on its
-    way into the residual."""
+    bias (None: none; else the name of the bias tensor below the prefix).  Tensors: <prefix><tensor> and <prefix><bias>, (width,).
+    `add_into` is the form an arrangement uses that norms a sublayer's result on its way into the residual (without a bias)."""
     graph_safe = True
 
     def __init__(self, params, prefix, ctx):
@@ -81,19 +81,28 @@ class LayerNorm(Norm):
         self.width = int(params["width"])
         self.eps = float(params["eps"])
         self.tensor = str(params.get("tensor", "weight"))
+        self.bias_tensor = str(params["bias"]) if params.get("bias") else None
         self.weight: Optional[torch.Tensor] = None
+        self.bias: Optional[torch.Tensor] = None
 
     def tensor_specs(self, available):
-        return [TensorSpec(self.name(self.tensor), (self.width,), "norm")]
+        specs = [TensorSpec(self.name(self.tensor), (self.width,), "norm")]
+        if self.bias_tensor:
+            specs.append(TensorSpec(self.name(self.bias_tensor), (self.width,), "bias"))
+        return specs
 
     def load(self, tensors):
         self.weight = tensors[self.name(self.tensor)]
+        if self.bias_tensor:
+            self.bias = tensors[self.name(self.bias_tensor)]
 
     def forward(self, step, x, out, out32=None, pick=None):
-        ops.layernorm(x, self.weight, self.eps, out, out32, pick)
+        ops.layernorm(x, self.weight, self.eps, out, out32, pick, bias=self.bias)
 
     def add_into(self, step, x, y, copy=None):
         """x += norm(y); `copy` (optional) receives the new rows in its own type."""
+        if self.bias is not None:
+            raise ValueError("layer norm: a norm that joins the residual has no bias")
         ops.layernorm_add(x, y, self.weight, self.eps, copy)
 
 

@@ -102,9 +102,7 @@ def wavelength_scaled_frequencies(dims: int, base: float, scaling) -> np.ndarray
 def scaled_table(positions: int, dims: int, base: float, scaling, exact_angles: bool = False) -> np.ndarray:
     """[positions, dims] float32: magnitude * cos of the dims/2 pairs' angles, then magnitude * sin.  The angle is the
     float32 product of the position and the float32 frequency; cos and sin are evaluated in float64 on it and rounded
-    once, as `neox_table` does.  `exact_angles`: the angle too is a float64 product (unscaled frequencies only)."""
-    if exact_angles and scaling:
-        raise ValueError("rotary table: exact angles go with unscaled frequencies")
+    once, as `neox_table` does.  `exact_angles`: the angle too is a float64 product (the wavelength form's always is)."""
     if dims == 0:
         return np.zeros((positions, 0), dtype=np.float32)
     if scaling and "low" in scaling:           # {factor, low, high, original}: rescaled by wavelength
@@ -115,7 +113,7 @@ def scaled_table(positions: int, dims: int, base: float, scaling, exact_angles: 
     f, magnitude = blended_frequencies(dims, base, scaling)      # None, or {factor, original, fast, slow}
     if exact_angles:
         angle = np.arange(positions, dtype=np.float64)[:, None] * f[None, :]
-        return np.concatenate([np.cos(angle), np.sin(angle)], axis=1).astype(np.float32)
+        return (np.concatenate([np.cos(angle), np.sin(angle)], axis=1) * magnitude).astype(np.float32)
     pos = np.arange(positions, dtype=np.float32)[:, None]
     angle = (pos * f.astype(np.float32)[None, :]).astype(np.float32).astype(np.float64)
     return (np.concatenate([np.cos(angle), np.sin(angle)], axis=1) * magnitude).astype(np.float32)
