@@ -19,6 +19,12 @@ with routed SwiGLU experts beside a shared one) and the two models nearest to it
 experts, picks and expert width (matrix states of the same size a head, windowed attention, routed experts), and a Nenotar
 of the same width, layers, heads and latent (no window) with the same active feed-forward weights.
 
+`python bench.py --design vivulorn` does the same for a Vivulorn (softmax attention, then twice the pair of softmax attention and a
+delta rule without feed-forward, latent attention, a delta rule; dense gelu feed-forwards) and the two models nearest to it: a
+Bonerax with a layer for every layer run, of the same width, heads and head widths, in turn attention (over every key) beside a
+small delta rule and a delta rule alone, with dense SwiGLU feed-forwards of the same weights; and a Nenotar of the same width,
+heads, latent and feed-forward.  A repeated layer's weights count each time they run.
+
 `python bench.py --design nenotar` measures, at sizes that resemble a real model's layers, a Nenotar (latent attention
 and minGRU layers in turn, each with a dense xIELU feed-forward and a per-layer token input) and a MiniMax-M3 of the
 same width, layers, heads and vocabulary whose routed experts hold the same active weights a token: one 2,048-token
@@ -291,6 +297,74 @@ def neruzen_mixing_flops(cfg, T: int) -> float:
     return total
 
 
+# name -> (width, heads, kv heads, delta heads (of 128 x 128), delta q/k heads, ff, vocab); attention heads of 128, latent heads of
+# 128 unrotated + 64 rotated dims over a latent of 512 (values 128); seven layer runs
+VIVULORN_SIZES = {
+    "w2048": (2048, 16, 4, 16, 8, 8192, 32768),
+    "w4096": (4096, 32, 8, 32, 16, 16384, 32768),
+    "w256": (256, 2, 1, 2, 1, 768, 1024),
+}
+
+
+def vivulorn_config(width, heads, kv_heads, rec_heads, rec_kv, ff, vocab):
+    from llmx_amd.config.nenotar import RotaryScaling
+    from llmx_amd.config.vivulorn import AttentionConfig, DeltaConfig, LatentAttentionConfig, LayerConfig, LoopConfig, VivulornConfig
+    a = AttentionConfig(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, rot_base=1e6, rot_dims=128,
+                        rot_scaling=RotaryScaling(4.0, 4096.0, 32.0, 1.0))
+    d = DeltaConfig(heads=rec_heads, kv_heads=rec_kv, dim=128, vdim=128, conv=4)
+    m = LatentAttentionConfig(heads=heads, dim=128, rot_dim=64, vdim=128, kv_rank=512, scale=192 ** -0.5, rot_base=10000.0)
+    layers = (LayerConfig("attention", a, ff), LayerConfig("attention", a, ff), LayerConfig("delta", d), LayerConfig("latent_attention", m, ff),
+              LayerConfig("delta", d, ff))
+    return VivulornConfig(vocab=vocab, width=width, norm_eps=1e-6, embedding_scale=1.0, layers=layers, loop=LoopConfig(1, 3, 2), logit_softcap=30.0)
+
+
+def vivulorn_bonerax(width, heads, kv_heads, rec_heads, rec_kv, ff, vocab):
+    from llmx_amd.config.bonerax import BoneraxConfig, DeltaConfig, LayerConfig, MLPConfig, ParallelConfig, RotaryScaling, WindowAttentionConfig
+    left = WindowAttentionConfig(heads=heads, kv_heads=kv_heads, dim=128, vdim=128, scale=128 ** -0.5, window=1 << 20, rot_base=1e6,
+                                 rot_dims=128, rot_scaling=RotaryScaling(4.0, 4096.0, 32.0, 1.0))
+    small = max(1, rec_heads // 4)
+    kinds = [("parallel", ParallelConfig(left, DeltaConfig(heads=small, kv_heads=small, dim=128, vdim=128, conv=4), 0.8, 0.9)),
+             ("channel_delta", DeltaConfig(heads=rec_heads, kv_heads=rec_kv, dim=128, vdim=128, conv=4))]
+    mlp, rank = MLPConfig("dense", max(64, 2 * ff // 3 // 64 * 64)), max(16, width // 32)
+    return BoneraxConfig(vocab=vocab, width=width, norm_eps=1e-6, logit_scale=1.0, logit_softcap=30.0,
+                         layers=tuple(LayerConfig(*kinds[i % 2], mlp) for i in range(7)), ranks={i: {"decay": rank, "gate": rank} for i in range(7)})
+
+
+def vivulorn_nenotar(width, heads, kv_heads, rec_heads, rec_kv, ff, vocab):
+    return nenotar_config(width, 7, heads, ff, 3 * width // 2, 128, vocab)
+
+
+def vivulorn_weights(cfg) -> float:
+    """Elements of the weight matrices a step multiplies by, summed over the layer runs (a repeated layer counts each time it runs)."""
+    E, total = cfg.width, 0.0
+    for i, opens in cfg.passes():
+        layer = cfg.layers[i]
+        m = layer.mixer
+        if layer.type == "attention":
+            total += E * (m.heads * m.dim + m.kv_heads * (m.dim + m.vdim) + 2 * m.heads * m.vdim)
+        elif layer.type == "latent_attention":
+            total += E * (m.heads * (m.dim + m.rot_dim) + m.kv_rank + m.rot_dim) + m.heads * m.kv_rank * (m.dim + m.vdim) + m.heads * m.vdim * E
+        else:
+            total += E * (2 * m.kv_heads * m.dim + 3 * m.heads * m.vdim + 2 * m.heads)
+        total += 2 * E * (layer.ff or 0) + (2 * E * E if opens else 0)
+    return total
+
+
+def vivulorn_mixing_flops(cfg, T: int) -> float:
+    """Multiply-adds x 2 of the mixers' own work over a T-token prompt: scores and value products over the causal half (the
+    latent's over the latents themselves); the states' decay, correction, outer product and read-out a token."""
+    total = 0.0
+    for i, _ in cfg.passes():
+        m = cfg.layers[i].mixer
+        if cfg.layers[i].type == "attention":
+            total += 2.0 * m.heads * (m.dim + m.vdim) * T * (T + 1) / 2
+        elif cfg.layers[i].type == "latent_attention":
+            total += 2.0 * m.heads * (2 * m.kv_rank + m.rot_dim) * T * (T + 1) / 2
+        else:
+            total += T * m.heads * m.dim * m.vdim * 7.0
+    return total
+
+
 def _layer_mixers(layer):
     """(windowed attention or None, [recurrences as (heads, dim, vdim, delta?)]) of a Bonerax layer."""
     m = layer.mixer
@@ -346,6 +420,9 @@ def prompt_flops(engine, T) -> float:
     elif cfg.architecture == "Neruzen":
         dense = 2.0 * T * neruzen_work(cfg, T)[0] + 2.0 * vocab * engine.spec.hidden_size
         attn = neruzen_mixing_flops(cfg, T)
+    elif cfg.architecture == "Vivulorn":
+        dense = 2.0 * T * vivulorn_weights(cfg) + 2.0 * vocab * engine.spec.hidden_size
+        attn = vivulorn_mixing_flops(cfg, T)
     elif cfg.architecture == "Bonerax":
         attn = 0.0
         for layer in cfg.layers:
@@ -434,6 +511,8 @@ def measure(engine, torch, steps, warmup):
             need = 2 * (salipel_work(cfg, batch)[1] + vocab * engine.spec.hidden_size) + batch * cache_bytes_read(engine, CONTEXT - steps / 2)
         if cfg.architecture == "Neruzen":
             need = 2 * (neruzen_work(cfg, batch)[1] + vocab * engine.spec.hidden_size) + batch * cache_bytes_read(engine, CONTEXT - steps / 2)
+        if cfg.architecture == "Vivulorn":
+            need = 2 * (vivulorn_weights(cfg) + vocab * engine.spec.hidden_size) + batch * cache_bytes_read(engine, CONTEXT - steps / 2)
         if cfg.architecture == "Givozen":       # weights by layer run; the head is the embedding's table, read whole
             need = 2 * (givozen_work(cfg, batch)[1] + vocab * engine.spec.hidden_size) + batch * cache_bytes_read(engine, CONTEXT - steps / 2)
         rec.update({f"decode_b{batch}_tok_s": round(batch / dt, 2), f"decode_b{batch}_ms": round(dt * 1e3, 4),
@@ -448,6 +527,8 @@ DESIGNS = {
     "salipel": ("Salipel", "MiniMax-M3 (GQA attention, routed SwiGLU experts)", SALIPEL_SIZES, salipel_config, salipel_closest),
     "neruzen": ("Neruzen", "Bonerax (gated matrix states, windowed attention, routed SwiGLU experts)", NERUZEN_SIZES, neruzen_config, neruzen_bonerax,
                 ("closest_latent", "Nenotar (latent attention, minGRU, dense xIELU)", neruzen_nenotar)),
+    "vivulorn": ("Vivulorn", "Bonerax (channel-wise delta rule, attention, dense SwiGLU)", VIVULORN_SIZES, vivulorn_config, vivulorn_bonerax,
+                 ("closest_latent", "Nenotar (latent attention, minGRU, dense xIELU)", vivulorn_nenotar)),
 }
 
 
