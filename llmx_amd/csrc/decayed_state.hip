@@ -8,15 +8,9 @@
 //   starts  a thread 4 key channels of a (head, value channel): walks the request's chunks in order from its state slot, leaves in
 //           `starts` the state before each chunk and writes the last state to the request's slot;
 //   rows    a workgroup a (chunk, head): scores, the decayed causal weights, the read-out of the state and the value product.
-// Everything is float32; 16x16x4 instructions (A: row lane % 16, k lane / 16; B: column lane % 16, k lane / 16; the result:
-// rows 4 (lane / 16) + 0..3 of column lane % 16).  The 4 k-slots of an instruction are dealt so that a lane's operands of four
-// instructions are 16 neighbouring bytes.
+// Everything is float32.
 // starts: [chunk][head][value channel, padded to 16][key channel, padded to 16].
-#include "state_operands.h"
-
-typedef float f32x4_t __attribute__((ext_vector_type(4)));
-
-#define DS_ROWS 64       // rows of a chunk
+#include "state_chunks.h"
 
 struct DecayedArgs {
     const float* q;
@@ -37,71 +31,14 @@ struct DecayedArgs {
     StateOperands operands;
 };
 
-__device__ __forceinline__ f32x4_t mfma4(float a, float b, f32x4_t c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
-
-// A chunk's keys into LDS rows of LDK floats (channels from D on and rows from n on hold zeros).  VEC: 16-byte loads, as many in
-// flight as a thread has to bring (see state_keys4_load for what they ask for); otherwise value by value.
-template <int NU, int KIND, bool VEC, int LDK>
-__device__ __forceinline__ void stage_keys(const DecayedArgs& a, int row0, int n, int h, float* ks) {
-    constexpr int DP = 16 * NU;
-    const int tid = threadIdx.x;
-    if (VEC) {
-        constexpr int PER_ROW = DP / 4, PER_THREAD = DS_ROWS * PER_ROW / 256, TURN = PER_THREAD < 8 ? PER_THREAD : 8;
-#pragma unroll
-        for (int b = 0; b < PER_THREAD; b += TURN) {
-            StateKeys4 raw[TURN];
-#pragma unroll
-            for (int u = 0; u < TURN; ++u) {
-                const int i = tid + 256 * (b + u), j = i / PER_ROW, d = 4 * (i % PER_ROW);
-                const size_t row = (size_t)(row0 + min(j, n - 1));
-                raw[u] = state_keys4_load<KIND>(a.operands, a.k + row * a.ldk + (size_t)h * a.D, row, d < a.D ? d : 0);
-            }
-#pragma unroll
-            for (int u = 0; u < TURN; ++u) {
-                const int i = tid + 256 * (b + u), j = i / PER_ROW, d = 4 * (i % PER_ROW);
-                const state4_t x = state_keys4<KIND>(raw[u]);
-                *reinterpret_cast<state4_t*>(ks + j * LDK + d) = d < a.D && j < n ? x : state4_t{0.0f, 0.0f, 0.0f, 0.0f};
-            }
-        }
-        return;
-    }
-    for (int i = tid; i < DS_ROWS * DP; i += 256) {
-        const int j = i / DP, d = i % DP;
-        const size_t row = (size_t)(row0 + min(j, n - 1));
-        const float x = state_key<KIND>(a.operands, a.k + row * a.ldk + (size_t)h * a.D, row, min(d, a.D - 1));
-        ks[j * LDK + d] = d < a.D && j < n ? x : 0.0f;
-    }
-}
-
-// 64 value channels from v0 on of a chunk's rows, row j times weight(j).
-template <int KIND, bool VEC, int LDV, typename Weight>
-__device__ __forceinline__ void stage_values(const DecayedArgs& a, int row0, int n, int h, int v0, float* vs, Weight weight) {
-    const int tid = threadIdx.x;
-    if (VEC) {
-        state4_t raw[4];
-#pragma unroll
-        for (int u = 0; u < 4; ++u) {
-            const int i = tid + 256 * u, j = i / 16, v = v0 + 4 * (i % 16);
-            const size_t row = (size_t)(row0 + min(j, n - 1));
-            raw[u] = *reinterpret_cast<const state4_t*>(a.v + row * a.ldv + (size_t)h * a.V + (v < a.V ? v : 0));
-        }
-#pragma unroll
-        for (int u = 0; u < 4; ++u) {
-            const int i = tid + 256 * u, j = i / 16, v = v0 + 4 * (i % 16);
-            const float w = j < n ? weight(j) : 0.0f;
-            state4_t x;
-#pragma unroll
-            for (int e = 0; e < 4; ++e) x[e] = v < a.V && j < n ? state_value<KIND>(raw[u][e]) * w : 0.0f;
-            *reinterpret_cast<state4_t*>(vs + j * LDV + 4 * (i % 16)) = x;
-        }
-        return;
-    }
-    for (int i = tid; i < DS_ROWS * 64; i += 256) {
-        const int j = i / 64, v = v0 + i % 64;
-        const size_t row = (size_t)(row0 + min(j, n - 1));
-        const float x = state_value<KIND>(a.v[row * a.ldv + (size_t)h * a.V + min(v, a.V - 1)]);
-        vs[j * LDV + i % 64] = v < a.V && j < n ? x * weight(j) : 0.0f;
-    }
+// The rows of chunk blockIdx.x and head blockIdx.y.
+__device__ __forceinline__ ChunkRows chunk_rows(const DecayedArgs& a) {
+    const int* chunk = a.chunks + 4 * (size_t)blockIdx.x;
+    const int row0 = chunk[1], n = chunk[2], h = blockIdx.y;
+    return ChunkRows{a.q + (size_t)row0 * a.ldq + (size_t)h * a.D, a.k + (size_t)row0 * a.ldk + (size_t)h * a.D,
+                     a.v + (size_t)row0 * a.ldv + (size_t)h * a.V, a.ldq, a.ldk, a.ldv, row0, n, a.D, a.V, a.DR, a.VR,
+                     a.starts + ((size_t)blockIdx.x * a.H + h) * a.VR * a.DR, a.out + (size_t)row0 * a.H * a.V + (size_t)h * a.V, a.H * a.V,
+                     a.out_scale, a.operands};
 }
 
 // NU: a head's key channels in tiles of 16, padded
@@ -112,12 +49,12 @@ __global__ void __launch_bounds__(256) decayed_sums_kernel(DecayedArgs a) {
     float* ks = lds;                       // [64][LDK]
     float* vs = lds + DS_ROWS * LDK;       // [64][LDV]: values times g^(n-1-j)
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, c = lane & 15, g = lane >> 4;
-    const int* chunk = a.chunks + 4 * (size_t)blockIdx.x;
-    const int row0 = chunk[1], n = chunk[2], h = blockIdx.y, v0 = 64 * blockIdx.z;
+    const ChunkRows rows = chunk_rows(a);
+    const int n = rows.n, h = blockIdx.y, v0 = 64 * blockIdx.z;
     const float* pw = a.powers + (size_t)h * (DS_ROWS + 1);
     const int steps = (n + 3) / 4;
-    stage_values<KIND, VEC, LDV>(a, row0, n, h, v0, vs, [&](int j) { return pw[n - 1 - j]; });
-    stage_keys<NU, KIND, VEC, LDK>(a, row0, n, h, ks);
+    stage_values<KIND, VEC, LDV>(rows, v0, vs, [&](int j) { return pw[n - 1 - j]; });
+    stage_keys<NU, KIND, VEC, LDK>(rows, ks);
     __syncthreads();
     if (v0 + 16 * wave >= a.VR) return;
     f32x4_t acc[NU];
@@ -176,145 +113,26 @@ __global__ void __launch_bounds__(256) decayed_starts_kernel(DecayedArgs a) {
         if (v < a.V && d + i < a.D) to[8 * i] = S[i];
 }
 
+// The decays of one head from the table of its decay's powers.
+struct PowerDecay {
+    const float* pw;           // [65] in LDS: g^0 .. g^64
+    __device__ __forceinline__ float between(int i, int j) const { return pw[i - j]; }
+    __device__ __forceinline__ float upto(int i) const { return pw[i + 1]; }
+};
+
 template <int NU, int KIND, bool VEC>
 __global__ void __launch_bounds__(256) decayed_rows_kernel(DecayedArgs a) {
-    constexpr int DP = 16 * NU, LDK = DP + 4, LDV = 64 + 4;
     extern __shared__ __align__(16) float lds[];
-    float* ks = lds;                       // [64][LDK]: keys, then the state's value channels (64 at a time)
-    float* vs = lds + DS_ROWS * LDK;       // [64][LDV]
-    float* pw = vs + DS_ROWS * LDV;        // [65]
-    const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63, c = lane & 15, g = lane >> 4;
-    const int* chunk = a.chunks + 4 * (size_t)blockIdx.x;
-    const int row0 = chunk[1], n = chunk[2], h = blockIdx.y;
-    for (int i = tid; i <= DS_ROWS; i += 256) pw[i] = a.powers[(size_t)h * (DS_ROWS + 1) + i];
-
-    // the wave's 16 query rows, in registers: lane (c, g) holds row 16 wave + c, channels 16 u + 4 g + 0..3
-    f32x4_t q[NU];
-    {
-        const size_t row = (size_t)(row0 + min(16 * wave + c, n - 1));
-        const float* head = a.q + row * a.ldq + (size_t)h * a.D;
-        if (VEC) {
-            constexpr int TURN = NU < 8 ? NU : 8;
-#pragma unroll
-            for (int b = 0; b < NU; b += TURN) {
-                StateKeys4 raw[TURN];
-#pragma unroll
-                for (int u = 0; u < TURN; ++u) {
-                    const int d = 16 * (b + u) + 4 * g;
-                    raw[u] = state_keys4_load<KIND>(a.operands, head, row, d < a.D ? d : 0);
-                }
-#pragma unroll
-                for (int u = 0; u < TURN; ++u) {
-                    const state4_t x = state_keys4<KIND>(raw[u]);
-                    q[b + u] = 16 * (b + u) + 4 * g < a.D ? x : state4_t{0.0f, 0.0f, 0.0f, 0.0f};
-                }
-            }
-        } else {
-#pragma unroll
-            for (int u = 0; u < NU; ++u)
-#pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const int d = 16 * u + 4 * g + e;
-                    const float x = state_key<KIND>(a.operands, head, row, min(d, a.D - 1));
-                    q[u][e] = d < a.D ? x : 0.0f;
-                }
-        }
-    }
-    stage_keys<NU, KIND, VEC, LDK>(a, row0, n, h, ks);
-    __syncthreads();
-    // scores transposed: s[t][e] of key row 16 t + 4 g + e against query row 16 wave + c, t up to the wave's own tile
-    f32x4_t s[4];
-#pragma unroll
-    for (int t = 0; t < 4; ++t) s[t] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll
-    for (int u = 0; u < NU; ++u) {
-#pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            if (t <= wave) {
-                const f32x4_t kf = *reinterpret_cast<const f32x4_t*>(ks + (16 * t + c) * LDK + 16 * u + 4 * g);
-#pragma unroll
-                for (int e = 0; e < 4; ++e) s[t] = mfma4(kf[e], q[u][e], s[t]);
-            }
-        }
-    }
-    const int i_row = 16 * wave + c;
-#pragma unroll
-    for (int t = 0; t < 4; ++t)
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int back = i_row - (16 * t + 4 * g + e);
-            s[t][e] = back >= 0 ? s[t][e] * pw[back] : 0.0f;      // pw holds g^0 .. g^64
-        }
-    const float* start = a.starts + ((size_t)blockIdx.x * a.H + h) * a.VR * a.DR;
-    for (int v0 = 0; v0 < a.VR; v0 += 64) {
-        __syncthreads();       // the keys, or the slice before, have been read by every wave
-        {
-            constexpr int PER_ROW = DP / 4, PER_THREAD = 64 * PER_ROW / 256, TURN = PER_THREAD < 8 ? PER_THREAD : 8;
-#pragma unroll
-            for (int b = 0; b < PER_THREAD; b += TURN) {
-                f32x4_t x[TURN];
-#pragma unroll
-                for (int u = 0; u < TURN; ++u) {
-                    const int i = tid + 256 * (b + u), v = i / PER_ROW, d = 4 * (i % PER_ROW);
-                    const bool in = v0 + v < a.VR && d < a.DR;
-                    x[u] = *reinterpret_cast<const f32x4_t*>(start + (size_t)(in ? v0 + v : 0) * a.DR + (in ? d : 0));
-                    if (!in) x[u] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
-                }
-#pragma unroll
-                for (int u = 0; u < TURN; ++u) {
-                    const int i = tid + 256 * (b + u);
-                    *reinterpret_cast<f32x4_t*>(ks + (i / PER_ROW) * LDK + 4 * (i % PER_ROW)) = x[u];
-                }
-            }
-        }
-        stage_values<KIND, VEC, LDV>(a, row0, n, h, v0, vs, [](int) { return 1.0f; });
-        __syncthreads();
-        f32x4_t o[4];
-#pragma unroll
-        for (int t = 0; t < 4; ++t) o[t] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll
-        for (int u = 0; u < NU; ++u)
-#pragma unroll
-            for (int vt = 0; vt < 4; ++vt) {
-                const f32x4_t sf = *reinterpret_cast<const f32x4_t*>(ks + (16 * vt + c) * LDK + 16 * u + 4 * g);
-#pragma unroll
-                for (int e = 0; e < 4; ++e) o[vt] = mfma4(q[u][e], sf[e], o[vt]);
-            }
-        // o[vt][e]: row 16 wave + 4 g + e, value channel v0 + 16 vt + c
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const float keep = pw[16 * wave + 4 * g + e + 1];
-#pragma unroll
-            for (int vt = 0; vt < 4; ++vt) o[vt][e] *= keep;
-        }
-#pragma unroll
-        for (int t = 0; t < 4; ++t) {
-            if (t <= wave) {
-#pragma unroll
-                for (int e = 0; e < 4; ++e)
-#pragma unroll
-                    for (int vt = 0; vt < 4; ++vt) o[vt] = mfma4(s[t][e], vs[(16 * t + 4 * g + e) * LDV + 16 * vt + c], o[vt]);
-            }
-        }
-#pragma unroll
-        for (int e = 0; e < 4; ++e) {
-            const int i = 16 * wave + 4 * g + e;
-            if (i < n) {
-                float* to = a.out + (size_t)(row0 + i) * a.H * a.V + (size_t)h * a.V;
-#pragma unroll
-                for (int vt = 0; vt < 4; ++vt) {
-                    const int v = v0 + 16 * vt + c;
-                    if (v < a.V) to[v] = o[vt][e] * a.out_scale;
-                }
-            }
-        }
-    }
+    float* pw = lds + state_rows_lds(NU);
+    const ChunkRows rows = chunk_rows(a);
+    for (int i = threadIdx.x; i <= DS_ROWS; i += 256) pw[i] = a.powers[(size_t)blockIdx.y * (DS_ROWS + 1) + i];
+    state_rows_read<NU, KIND, VEC>(rows, PowerDecay{pw}, lds);
 }
 
 template <int NU, int KIND, bool VEC>
 static int launch_decayed(const DecayedArgs& a, int n_chunks, int n_long, hipStream_t stream) {
     constexpr size_t lds_sums = sizeof(float) * DS_ROWS * (16 * NU + 16 + 64 + 16);
-    constexpr size_t lds_rows = sizeof(float) * (DS_ROWS * (16 * NU + 4 + 64 + 4) + DS_ROWS + 1);
+    constexpr size_t lds_rows = sizeof(float) * (state_rows_lds(NU) + DS_ROWS + 1);
     static bool raised = false;
     if (!raised) {
         if (hipFuncSetAttribute((const void*)decayed_sums_kernel<NU, KIND, VEC>, hipFuncAttributeMaxDynamicSharedMemorySize, 160 * 1024) != hipSuccess) return -1;

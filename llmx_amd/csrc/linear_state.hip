@@ -39,6 +39,7 @@ struct DeltaPrepArgs {
     float* v;       // [T, H*V]
     float* decay;   // [T, H*D]; head_decay: [T, H]
     float* beta;    // [T, H]
+    float* log_decay;   // [T, H] or null: with head_decay, the decays' logarithms too
     int G, H, D, V, taps, beta_col, head_decay;
 };
 
@@ -91,7 +92,11 @@ __global__ void __launch_bounds__(64) delta_prep_kernel(DeltaPrepArgs a) {
     } else {
         for (int c = lane; c < a.H; c += 64) {
             a.beta[(size_t)t * a.H + c] = sigmoid_ls(a.pre[(size_t)t * a.ld + a.beta_col + c]);
-            if (a.head_decay) a.decay[(size_t)t * a.H + c] = expf(-expf(a.a_log[c]) * softplus_f(a.step_pre[(size_t)t * a.step_ld + c] + a.dt_bias[c]));
+            if (a.head_decay) {
+                const float l = -expf(a.a_log[c]) * softplus_f(a.step_pre[(size_t)t * a.step_ld + c] + a.dt_bias[c]);
+                a.decay[(size_t)t * a.H + c] = expf(l);
+                if (a.log_decay) a.log_decay[(size_t)t * a.H + c] = l;
+            }
         }
     }
 }
@@ -99,12 +104,12 @@ __global__ void __launch_bounds__(64) delta_prep_kernel(DeltaPrepArgs a) {
 extern "C" int llmx_delta_prep(const float* pre, int ld, const float* conv_w, const float* step_pre, int step_ld, const float* dt_bias,
                                const float* a_log, const float* state, long state_stride, int tail_off, const int* slot_read,
                                const int* row_entry, const int* entry_rows, float* q, float* k, float* v, float* decay, float* beta, int rows, int G,
-                               int H, int D, int V, int taps, int beta_col, int head_decay, hipStream_t stream) {
+                               int H, int D, int V, int taps, int beta_col, int head_decay, float* log_decay, hipStream_t stream) {
     if (rows <= 0) return 0;
     const long C = 2L * G * D + (long)H * V;
     if (taps < 1 || G < 1 || H % G || D > PREP_MAX || beta_col + H > ld || C > ld || step_ld < (head_decay ? H : H * D)) return -2;
     DeltaPrepArgs a{pre, ld, conv_w, step_pre, step_ld, dt_bias, a_log, state, state_stride, tail_off, slot_read, row_entry, entry_rows,
-                    q, k, v, decay, beta, G, H, D, V, taps, beta_col, head_decay};
+                    q, k, v, decay, beta, log_decay, G, H, D, V, taps, beta_col, head_decay};
     llmx_note_launch(LK_DELTA_PREP);
     hipLaunchKernelGGL(delta_prep_kernel, dim3(rows, 2 * G + (head_decay ? H : 2 * H) + 1), dim3(64), 0, stream, a);
     return LLMX_CHECK_LAUNCH();
@@ -182,7 +187,7 @@ __global__ void __launch_bounds__(SCAN_THREADS) state_scan_kernel(StateScanArgs 
     const int h = blockIdx.x / tiles, tile = blockIdx.x % tiles;
     const int e = blockIdx.y;
     const int row0 = a.entry_rows[2 * e], n = a.entry_rows[2 * e + 1];
-    if (a.max_rows_here > 0 && n > a.max_rows_here) return;
+    if (a.max_rows_here > 0 && n > a.max_rows_here) return;     // its tail is the other kernel's too
     const int j = tile * SCAN_COLS + c;
     const bool col = j < a.V;
     const int d0 = s * R;           // where the lane's operands lie in a staged row; its i-th key channel is 32 i + s

@@ -88,7 +88,8 @@
     X(TOKEN_SHIFT, "token_shift")                                                                                         \
     X(RMSNORM_SHIFT, "rmsnorm_shift")                                                                                     \
     X(DECAYED_STATE_CHUNKS, "decayed_state.chunks")                                                                       \
-    X(JOIN_ROWS, "join_rows")
+    X(JOIN_ROWS, "join_rows")                                                                                             \
+    X(DELTA_CHUNKS, "delta_chunks")
 
 enum LlmxLaunchKind : int {
 #define LLMX_X(id, name) LK_##id,

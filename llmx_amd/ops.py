@@ -91,7 +91,8 @@ def _declare(h) -> None:
         "llmx_cast_rows": [P, P, I, L, P],
         "llmx_combine_rows": [P, P, F, P, P, F, I, I, I, P],
         "llmx_scale_softcap": [P, F, F, L, P],
-        "llmx_delta_prep": [P, I, P, P, I, P, P, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P],
+        "llmx_delta_prep": [P, I, P, P, I, P, P, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P],
+        "llmx_delta_chunks": [P, I, P, I, P, I, P, P, P, L, P, P, P, P, I, P, I, P, P, P, P, P, P, F, I, I, I, I, P, I, I, I, I, P],
         "llmx_cast_cols": [P, I, P, I, I, I, P],
         "llmx_sigmoid_root": [P, P, F, P, I, I, P],
         "llmx_state_scan": [P, I, P, I, P, I, P, I, P, P, L, P, P, P, P, F, I, I, I, I, I, P, I, I, I, I, I, I, I, P, P, I, I, P],
@@ -736,12 +737,12 @@ def _rows_view(t: torch.Tensor, name: str, rows: int, cols: int):
 def delta_prep(pre: torch.Tensor, conv_w: torch.Tensor, step_pre: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor,
                state: torch.Tensor, tail_off: int, slot_read: torch.Tensor, row_entry: torch.Tensor, entry_rows: torch.Tensor,
                q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, beta: torch.Tensor, G: int, H: int, D: int, V: int,
-               beta_col: int, head_decay: bool = False) -> None:
+               beta_col: int, head_decay: bool = False, log_decay: Optional[torch.Tensor] = None) -> None:
     """A delta-rule mixer's rows made ready for the scan (see csrc/linear_state.hip): from the fused in-projection `pre`
     [T, ld] = q (G*D) | k (G*D) | v (H*V) | ... | beta (H) at beta_col: the short causal convolution (conv_w [C, taps], the
     inputs of earlier steps from the state's tail at `tail_off`) with silu, unit-norm q and k heads, v, the decay
     exp(-exp(a_log) softplus(step_pre + dt_bias)) [T, H*D] and beta = sigmoid [T, H].  `head_decay`: one decay a head, step_pre
-    and decay [T, H], dt_bias [H]."""
+    and decay [T, H], dt_bias [H]; `log_decay` [T, H] then receives the decays' logarithms."""
     T, ld = pre.shape
     DW = H if head_decay else H * D
     C = 2 * G * D + H * V
@@ -757,7 +758,8 @@ def delta_prep(pre: torch.Tensor, conv_w: torch.Tensor, step_pre: torch.Tensor, 
                                  _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)), _dev(q, "q", torch.float32, (T, G * D)),
                                  _dev(k, "k", torch.float32, (T, G * D)), _dev(v, "v", torch.float32, (T, H * V)),
                                  _dev(decay, "decay", torch.float32, (T, DW)), _dev(beta, "beta", torch.float32, (T, H)),
-                                 T, G, H, D, V, taps, int(beta_col), 1 if head_decay else 0, _stream()), "delta_prep")
+                                 T, G, H, D, V, taps, int(beta_col), 1 if head_decay else 0, _dev(log_decay, "log_decay", torch.float32, (T, H)), _stream()),
+           "delta_prep")
 
 
 def sigmoid_root(z: torch.Tensor, bias: Optional[torch.Tensor], tau: float, out: torch.Tensor) -> None:
@@ -855,7 +857,7 @@ DECAYED_CHUNKS_MIN_ROWS = 128   # an entry of at least this many rows in the ste
 
 
 class DecayedPlan:
-    """The chunks of a step's long entries for decayed_state_chunks, and the most rows an entry may have that is not one."""
+    """The chunks of a step's long entries for decayed_state_chunks and delta_chunks, and the most rows an entry may have that is not one."""
 
     def __init__(self, row_counts, rows_a_chunk, device):
         import numpy as np
@@ -916,6 +918,42 @@ def decayed_state_chunks(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, powe
                                            _dev(plan.entry_chunks, "entry_chunks", torch.int32), plan.n_long, _dev(starts, "starts"),
                                            _dev(out, "out", torch.float32, (T, H * V)), float(out_scale), H, D, V, *_operand_args(operands, T, D),
                                            _stream()), "decayed_state_chunks")
+
+
+def delta_chunks(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, log_decay: torch.Tensor, beta: torch.Tensor, state: torch.Tensor,
+                 slot_read: torch.Tensor, slot_write: torch.Tensor, entry_rows: torch.Tensor, out: torch.Tensor, out_scale: float, H: int, qk_heads: int,
+                 D: int, V: int, plan: DecayedPlan, tail=None, scratch=None) -> None:
+    """state_scan's delta rule with one decay a head, given by its logarithm (log_decay, beta [T, H]), over the rows of the plan's
+    long entries only, chunk by chunk (csrc/delta_chunks.hip): q, k [T, qk_heads*D], v [T, H*V] float32 views, out [T, H*V], the
+    state and the convolution's `tail` as state_scan keeps them.  `scratch(name, shape, dtype)`: storage that lives as long as the
+    caller's step."""
+    T = out.shape[0]
+    n_e = entry_rows.shape[0]
+    if H % qk_heads or state.dim() != 2 or state.shape[1] < state_matrix_size(H, D, V) or D > 256 or plan.rows != T:
+        raise KernelError("delta_chunks: heads, widths, plan or state do not fit")
+    rows = lib().llmx_decayed_state_rows()
+    qa, ldq = _rows_view(q, "q", T, qk_heads * D)
+    ka, ldk = _rows_view(k, "k", T, qk_heads * D)
+    va, ldv = _rows_view(v, "v", T, H * V)
+    ta, tld, tC, taps, toff = 0, 0, 0, 0, 0
+    if tail is not None:
+        src, taps, toff = tail
+        tC = src.shape[1]
+        ta, tld = _rows_view(src, "tail source", T, tC)
+        if toff < state_matrix_size(H, D, V) or toff + (taps - 1) * tC > state.shape[1]:
+            raise KernelError("delta_chunks: the state does not hold the convolution's tail")
+    get, n = scratch or _scratch_now(out.device), plan.n_chunks
+    DR, VR = -(-D // 16) * 16, -(-V // 16) * 16
+    W, U = get("delta.chunk_w", (n, H, rows, DR), torch.float32), get("delta.chunk_u", (n, H, rows, VR), torch.float32)
+    decays, keep = get("delta.chunk_decays", (n, H, rows), torch.float32), get("delta.chunk_keep", (n, H), torch.float32)
+    starts = get("delta.chunk_starts", (n, H, VR, DR), torch.float32)
+    _check(lib().llmx_delta_chunks(qa, ldq, ka, ldk, va, ldv, _dev(beta, "beta", torch.float32, (T, H)), _dev(log_decay, "log_decay", torch.float32, (T, H)),
+                                   _dev(state, "state", torch.float32), state.shape[1], _dev(slot_read, "slot_read", torch.int32, (n_e,)),
+                                   _dev(slot_write, "slot_write", torch.int32, (n_e,)), _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)),
+                                   _dev(plan.chunks, "chunks", torch.int32), n, _dev(plan.entry_chunks, "entry_chunks", torch.int32), plan.n_long,
+                                   _dev(W, "W"), _dev(U, "U"), _dev(decays, "decays"), _dev(keep, "keep"), _dev(starts, "starts"),
+                                   _dev(out, "out", torch.float32, (T, H * V)), float(out_scale), H, H // qk_heads, D, V, ta, tld, tC, int(taps), int(toff),
+                                   _stream()), "delta_chunks")
 
 
 GATE_SIGMOID, GATE_SILU = 0, 1

@@ -84,7 +84,8 @@ class HeadDeltaRule(Mixer):
     """The gated delta rule with one decay a head: g = exp(-exp(A_log_h) softplus(W_a h + dt_bias)).
     params: hidden, heads, kv_heads (q and k heads; head h reads q/k head h / (heads / kv_heads)), dim, vdim, conv (taps), eps.
     Tensors <prefix>q, k, v (+ .conv [channels, taps]), b, a, A_log, dt_bias, g, norm, o; every projection of the input is part of
-    one product.  result = W_o (rmsnorm_head(o) * w * silu(W_g h)).  Convolutions, unit norms, decays, the recurrence and its
+    one product.  result = W_o (rmsnorm_head(o) * w * silu(W_g h)).  Runs of many rows go chunk by chunk over the matrix cores, short
+    ones row by row.  Convolutions, unit norms, decays, the recurrence and its
     state are float32 in both paths."""
     graph_safe = True
     steps_between_slots = True
@@ -137,12 +138,20 @@ class HeadDeltaRule(Mixer):
         view = lambda n: pre[:, self.cols[n][0]:self.cols[n][0] + self.cols[n][1]]
         q, k = step.buf("delta.q", (T, G * D), f32), step.buf("delta.k", (T, G * D), f32)
         v, decay, beta = step.buf("delta.v", (T, H * V), f32), step.buf("delta.head_decay", (T, H), f32), step.buf("delta.beta", (T, H), f32)
+        # a decode step's entries are never long (nothing for a graph to hold)
+        plan = step.shared("decayed.plan", lambda: ops.decayed_plan([e.n for e in step.entries], step.device))
+        log_decay = step.buf("delta.log_decay", (T, H), f32) if plan is not None else None
         ops.delta_prep(pre, self.conv, view("a"), self.dt_bias, self.a_log, cache.state, self.state_matrix, step.entry_held_slots,
-                       step.row_entry, step.entry_rows, q, k, v, decay, beta, G, H, D, V, self.cols["b"][0], head_decay=True)
+                       step.row_entry, step.entry_rows, q, k, v, decay, beta, G, H, D, V, self.cols["b"][0], head_decay=True, log_decay=log_decay)
         o = step.buf("delta.o", (T, H * V), f32)
         tail = (pre[:, :self.channels], self.taps, self.state_matrix) if self.taps > 1 else None
-        ops.state_scan(q, k, v, decay, beta, cache.state, step.entry_held_slots, step.entry_slots, step.entry_rows, o, float(D) ** -0.5,
-                       H, G, D, V, tail=tail, max_rows=step.max_rows_per_entry, head_decay=True)
+        if plan is not None:
+            ops.delta_chunks(q, k, v, log_decay, beta, cache.state, step.entry_held_slots, step.entry_slots, step.entry_rows, o, float(D) ** -0.5,
+                             H, G, D, V, plan, tail=tail, scratch=step.buf)
+        if plan is None or plan.short_entries:
+            ops.state_scan(q, k, v, decay, beta, cache.state, step.entry_held_slots, step.entry_slots, step.entry_rows, o, float(D) ** -0.5,
+                           H, G, D, V, tail=tail, max_rows=step.max_rows_per_entry, head_decay=True,
+                           max_rows_here=ops.DECAYED_CHUNKS_MIN_ROWS - 1 if plan is not None else 0)
         gated = step.buf("delta.gated", (T, H * V), step.act_dtype)
         ops.head_norm_gate(o, self.norm, view("g"), gated, self.eps, H, V, ops.GATE_SILU)
         ops.gemm(gated, self.w_o, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)
