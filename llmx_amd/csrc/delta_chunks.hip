@@ -253,17 +253,17 @@ __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkA
     const int* ec = a.entry_chunks + 4 * (size_t)blockIdx.y;
     const int entry = ec[0], c0 = ec[1], nc = ec[2];
     const int h = blockIdx.x % a.H, vt = blockIdx.x / a.H;
+    const int row0 = a.entry_rows[2 * entry], rows = a.entry_rows[2 * entry + 1];      // its chunks' rows follow each other
     const size_t slot_r = (size_t)a.slot_read[entry] * a.state_stride, slot_w = (size_t)a.slot_write[entry] * a.state_stride;
 
     if (a.taps > 1) {       // the request's workgroups share the tail's channels out among themselves
         const float* old = a.state + slot_r + a.tail_off;
         float* fresh = a.state + slot_w + a.tail_off;
-        const int row0 = a.entry_rows[2 * entry], n = a.entry_rows[2 * entry + 1];
         const int per = (a.tail_C + (int)gridDim.x - 1) / (int)gridDim.x, end = min(a.tail_C, ((int)blockIdx.x + 1) * per);
         for (int ch = (int)blockIdx.x * per + tid; ch < end; ch += NT)
             for (int p = 0; p < a.taps - 1; ++p) {          // ascending: in place, a value is read before its place is written
-                const int idx = n - (a.taps - 1) + p;
-                fresh[(size_t)p * a.tail_C + ch] = idx >= 0 ? a.tail_src[(size_t)(row0 + idx) * a.tail_ld + ch] : old[(size_t)(n + p) * a.tail_C + ch];
+                const int idx = rows - (a.taps - 1) + p;
+                fresh[(size_t)p * a.tail_C + ch] = idx >= 0 ? a.tail_src[(size_t)(row0 + idx) * a.tail_ld + ch] : old[(size_t)(rows + p) * a.tail_C + ch];
             }
     }
 
@@ -292,8 +292,8 @@ __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkA
         const float* W = a.W + at * DS_ROWS * a.DR;
 #pragma unroll
         for (int i = 0; i < 4; ++i) x.w[i] = *reinterpret_cast<const f32x4_t*>(W + (size_t)(16 * i + c) * a.DR + wd);
-        const int row0 = a.chunks[4 * (size_t)ch + 1], n = a.chunks[4 * (size_t)ch + 2];
-        const float* kp = a.k + (size_t)row0 * a.ldk + (size_t)(h / a.share) * a.D + kd;
+        const int ahead = (ch - c0) * DS_ROWS, n = min(DS_ROWS, rows - ahead);
+        const float* kp = a.k + (size_t)(row0 + ahead) * a.ldk + (size_t)(h / a.share) * a.D + kd;
 #pragma unroll
         for (int s = 0; s < 4; ++s)
 #pragma unroll

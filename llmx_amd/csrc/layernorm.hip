@@ -1,124 +1,168 @@
 // Layer norm with a weight and an optional bias, and the element-wise steps of layers that norm a sublayer's result before it
 // joins the residual: y = (x - mean) / sqrt(var + eps) * w (+ b), var the mean of the squared deviations.  Everything is float32
 // arithmetic on float32 rows; only what a product reads next is stored in the activation type.
-// A row's sums are formed by 256 threads: thread v adds elements v, v + 256, ... in this order, a wave adds its threads'
-// sums with wave_sum, and the four waves' sums are added in wave order: a function of the row's length only.
+// A row's sums are formed by 256 threads: thread v adds elements 4v .. 4v + 3, then those 1,024 further on, ... in this order (rows
+// whose length is no multiple of 4: elements v, v + 256, ...), a wave adds its threads' sums with wave_sum, and the four waves' sums
+// are added in wave order: a function of the row's length only.
 #include "common.h"
 
 #define LN_THREADS 256
-#define LN_KEPT 16      // values a thread keeps in registers: rows of at most 4,096 values are read once
+#define LN_QUADS 4      // groups of four values a thread keeps in registers: rows of at most 4,096 values are read once
 
-// mean and 1 / sqrt(var + eps) of a row; v[] receives the thread's values when the row fits the registers
-template <bool KEPT>
-__device__ __forceinline__ void row_moments(const float* __restrict__ row, int n, float eps, float* scratch, float (&v)[LN_KEPT], float& mean,
-                                            float& rstd) {
-    const int tid = threadIdx.x;
+typedef float ln4_t __attribute__((ext_vector_type(4)));
+
+// Up to four neighbouring values of a row: element 4 at (VEC: one 16-byte access; else elements at, at + 256, ... one by one), zeros
+// past the row's end.
+template <bool VEC>
+struct LnPlace {
+    static __device__ __forceinline__ int element(int group, int i) {
+        return VEC ? 4 * ((int)threadIdx.x + LN_THREADS * group) + i : (int)threadIdx.x + LN_THREADS * (4 * group + i);
+    }
+    static __device__ __forceinline__ ln4_t load(const float* __restrict__ row, int group, int n) {
+        if (VEC) {
+            const int at = element(group, 0);
+            return at < n ? *reinterpret_cast<const ln4_t*>(row + at) : ln4_t{0.0f, 0.0f, 0.0f, 0.0f};
+        }
+        ln4_t v;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = element(group, i) < n ? row[element(group, i)] : 0.0f;
+        return v;
+    }
+    template <typename TO>
+    static __device__ __forceinline__ void store(TO* __restrict__ row, int group, int n, const ln4_t& y) {
+        if (VEC) {
+            const int at = element(group, 0);
+            if (at >= n) return;
+            if constexpr (sizeof(TO) == 4) *reinterpret_cast<ln4_t*>(row + at) = y;
+            else {
+                typedef uint32_t u32x2_ln __attribute__((ext_vector_type(2)));
+                *reinterpret_cast<u32x2_ln*>(row + at) = u32x2_ln{(uint32_t)f32_to_bf16(y[0]) | ((uint32_t)f32_to_bf16(y[1]) << 16),
+                                                                  (uint32_t)f32_to_bf16(y[2]) | ((uint32_t)f32_to_bf16(y[3]) << 16)};
+            }
+            return;
+        }
+#pragma unroll
+        for (int i = 0; i < 4; ++i)
+            if (element(group, i) < n) st(row + element(group, i), y[i]);
+    }
+};
+
+// mean and 1 / sqrt(var + eps) of a row whose groups get(0), get(1), ... gives
+template <bool VEC, typename Get>
+__device__ __forceinline__ void row_moments(Get get, int groups, int n, float eps, float* scratch, float& mean, float& rstd) {
     float s = 0.0f;
-    if (KEPT) {
-#pragma unroll
-        for (int j = 0; j < LN_KEPT; ++j) v[j] = tid + LN_THREADS * j < n ? row[tid + LN_THREADS * j] : 0.0f;
-#pragma unroll
-        for (int j = 0; j < LN_KEPT; ++j) s += v[j];
-    } else {
-        for (int i = tid; i < n; i += LN_THREADS) s += row[i];
+    for (int j = 0; j < groups; ++j) {
+        const ln4_t v = get(j);
+        s += (v[0] + v[1]) + (v[2] + v[3]);
     }
     mean = block_sum<LN_THREADS / 64>(s, scratch) / (float)n;
     float q = 0.0f;
-    if (KEPT) {
+    for (int j = 0; j < groups; ++j) {
+        const ln4_t v = get(j);
 #pragma unroll
-        for (int j = 0; j < LN_KEPT; ++j) {
-            const float d = tid + LN_THREADS * j < n ? v[j] - mean : 0.0f;
-            q = fmaf(d, d, q);
-        }
-    } else {
-        for (int i = tid; i < n; i += LN_THREADS) {
-            const float d = row[i] - mean;
+        for (int i = 0; i < 4; ++i) {
+            const float d = LnPlace<VEC>::element(j, i) < n ? v[i] - mean : 0.0f;
             q = fmaf(d, d, q);
         }
     }
     rstd = 1.0f / sqrtf(block_sum<LN_THREADS / 64>(q, scratch) / (float)n + eps);
 }
 
+__device__ __forceinline__ ln4_t ln_apply(const ln4_t& v, float mean, float rstd, const ln4_t& w) {
+    return ln4_t{(v[0] - mean) * rstd * w[0], (v[1] - mean) * rstd * w[1], (v[2] - mean) * rstd * w[2], (v[3] - mean) * rstd * w[3]};
+}
+
+// The row in registers (KEPT groups, with the weights and what else the end needs asked for together at the start), or read again.
 // out[r] = LN(x[pick ? pick[r] : r]) in the activation type and/or float32
-template <typename TO, bool KEPT>
+template <typename TO, int KEPT, bool VEC>
 __global__ void __launch_bounds__(LN_THREADS) layernorm_kernel(const float* __restrict__ x, const int* __restrict__ pick, const float* __restrict__ w,
                                                              const float* __restrict__ bias, float eps, TO* __restrict__ out, float* __restrict__ out32, int n) {
+    typedef LnPlace<VEC> P;
     __shared__ float scratch[LN_THREADS / 64];
-    const int r = blockIdx.x, tid = threadIdx.x;
+    const int r = blockIdx.x;
     const float* row = x + (size_t)(pick ? pick[r] : r) * n;
-    float v[LN_KEPT], mean, rstd;
-    row_moments<KEPT>(row, n, eps, scratch, v, mean, rstd);
-    if (KEPT) {
+    float mean, rstd;
+    auto finish = [&](int j, const ln4_t& v, const ln4_t& wj, const ln4_t& bj) {
+        ln4_t y = ln_apply(v, mean, rstd, wj);
+        if (bias) y = ln4_t{y[0] + bj[0], y[1] + bj[1], y[2] + bj[2], y[3] + bj[3]};
+        if (out) P::store(out + (size_t)r * n, j, n, y);
+        if (out32) P::store(out32 + (size_t)r * n, j, n, y);
+    };
+    if (KEPT > 0) {
+        ln4_t v[KEPT > 0 ? KEPT : 1], wk[KEPT > 0 ? KEPT : 1], bk[KEPT > 0 ? KEPT : 1];
 #pragma unroll
-        for (int j = 0; j < LN_KEPT; ++j) {
-            const int i = tid + LN_THREADS * j;
-            if (i < n) {
-                float y = (v[j] - mean) * rstd * w[i];
-                if (bias) y = y + bias[i];
-                if (out) st(out + (size_t)r * n + i, y);
-                if (out32) out32[(size_t)r * n + i] = y;
-            }
+        for (int j = 0; j < KEPT; ++j) {
+            v[j] = P::load(row, j, n);
+            wk[j] = P::load(w, j, n);
+            bk[j] = bias ? P::load(bias, j, n) : ln4_t{0.0f, 0.0f, 0.0f, 0.0f};
         }
+        row_moments<VEC>([&](int j) { return v[j]; }, KEPT, n, eps, scratch, mean, rstd);
+#pragma unroll
+        for (int j = 0; j < KEPT; ++j) finish(j, v[j], wk[j], bk[j]);
     } else {
-        for (int i = tid; i < n; i += LN_THREADS) {
-            float y = (row[i] - mean) * rstd * w[i];
-            if (bias) y = y + bias[i];
-            if (out) st(out + (size_t)r * n + i, y);
-            if (out32) out32[(size_t)r * n + i] = y;
-        }
+        const int groups = (n + 4 * LN_THREADS - 1) / (4 * LN_THREADS);
+        row_moments<VEC>([&](int j) { return P::load(row, j, n); }, groups, n, eps, scratch, mean, rstd);
+        for (int j = 0; j < groups; ++j) finish(j, P::load(row, j, n), P::load(w, j, n), bias ? P::load(bias, j, n) : ln4_t{0.0f, 0.0f, 0.0f, 0.0f});
     }
 }
+
+static bool ln_vec(int n, const void* a, const void* b, const void* c, const void* d, const void* e) {
+    return n % 4 == 0 && (((uintptr_t)a | (uintptr_t)b | (uintptr_t)c | (uintptr_t)d | (uintptr_t)e) & 15) == 0;
+}
+// groups of four values a thread keeps: 1, 2 or 4; 0: the row is too long
+static int ln_kept(int n) { return n <= 4 * LN_THREADS ? 1 : n <= 8 * LN_THREADS ? 2 : n <= 4 * LN_THREADS * LN_QUADS ? LN_QUADS : 0; }
+#define LN_FORMS(TO)                                                            \
+    do {                                                                        \
+        if (vec) { if (kept == 1) LLMX_LN(TO, 1, true); else if (kept == 2) LLMX_LN(TO, 2, true); else if (kept) LLMX_LN(TO, LN_QUADS, true); else LLMX_LN(TO, 0, true); } \
+        else { if (kept == 1) LLMX_LN(TO, 1, false); else if (kept == 2) LLMX_LN(TO, 2, false); else if (kept) LLMX_LN(TO, LN_QUADS, false); else LLMX_LN(TO, 0, false); } \
+    } while (0)
 
 extern "C" int llmx_layernorm(const float* x, const int* pick, const float* w, const float* bias, float eps, void* out, int out_dtype, float* out32, int rows, int n,
                               hipStream_t stream) {
     if (rows <= 0) return 0;
     if (n <= 0 || !w || (!out && !out32)) return -2;
     llmx_note_launch(LK_LAYERNORM);
-    const bool kept = n <= LN_THREADS * LN_KEPT;
-#define LLMX_LN(TO, K) hipLaunchKernelGGL((layernorm_kernel<TO, K>), dim3(rows), dim3(LN_THREADS), 0, stream, x, pick, w, bias, eps, (TO*)out, out32, n)
-    if (out_dtype == LLMX_F32) {
-        if (kept) LLMX_LN(float, true);
-        else LLMX_LN(float, false);
-    } else {
-        if (kept) LLMX_LN(bf16_t, true);
-        else LLMX_LN(bf16_t, false);
-    }
+    const int kept = ln_kept(n);
+    const bool vec = ln_vec(n, x, w, bias, out, out32);
+#define LLMX_LN(TO, K, V) hipLaunchKernelGGL((layernorm_kernel<TO, K, V>), dim3(rows), dim3(LN_THREADS), 0, stream, x, pick, w, bias, eps, (TO*)out, out32, n)
+    if (out_dtype == LLMX_F32) LN_FORMS(float);
+    else LN_FORMS(bf16_t);
 #undef LLMX_LN
     return LLMX_CHECK_LAUNCH();
 }
 
 // x[r] += LN(y[r]) * w: a sublayer's result joins the residual after its own norm; `copy` (optional) receives the new row
 // in the activation type for the product that reads it next.
-template <typename TO, bool KEPT>
+template <typename TO, int KEPT, bool VEC>
 __global__ void __launch_bounds__(LN_THREADS) layernorm_add_kernel(float* __restrict__ x, const float* __restrict__ y, const float* __restrict__ w,
                                                                  float eps, TO* __restrict__ copy, int n) {
+    typedef LnPlace<VEC> P;
     __shared__ float scratch[LN_THREADS / 64];
-    const int r = blockIdx.x, tid = threadIdx.x;
+    const int r = blockIdx.x;
     const float* row = y + (size_t)r * n;
     float* xr = x + (size_t)r * n;
-    float v[LN_KEPT], mean, rstd;
-    float old[LN_KEPT];
-    if (KEPT) {
+    float mean, rstd;
+    auto finish = [&](int j, const ln4_t& v, const ln4_t& wj, const ln4_t& old) {
+        const ln4_t z = ln_apply(v, mean, rstd, wj);
+        const ln4_t s = ln4_t{old[0] + z[0], old[1] + z[1], old[2] + z[2], old[3] + z[3]};
+        P::store(xr, j, n, s);
+        if (copy) P::store(copy + (size_t)r * n, j, n, s);
+    };
+    if (KEPT > 0) {
+        ln4_t v[KEPT > 0 ? KEPT : 1], wk[KEPT > 0 ? KEPT : 1], old[KEPT > 0 ? KEPT : 1];
 #pragma unroll
-        for (int j = 0; j < LN_KEPT; ++j) old[j] = tid + LN_THREADS * j < n ? xr[tid + LN_THREADS * j] : 0.0f;
-    }
-    row_moments<KEPT>(row, n, eps, scratch, v, mean, rstd);
-    if (KEPT) {
-#pragma unroll
-        for (int j = 0; j < LN_KEPT; ++j) {
-            const int i = tid + LN_THREADS * j;
-            if (i < n) {
-                const float s = old[j] + (v[j] - mean) * rstd * w[i];
-                xr[i] = s;
-                if (copy) st(copy + (size_t)r * n + i, s);
-            }
+        for (int j = 0; j < KEPT; ++j) {
+            v[j] = P::load(row, j, n);
+            old[j] = P::load(xr, j, n);
+            wk[j] = P::load(w, j, n);
         }
+        row_moments<VEC>([&](int j) { return v[j]; }, KEPT, n, eps, scratch, mean, rstd);
+#pragma unroll
+        for (int j = 0; j < KEPT; ++j) finish(j, v[j], wk[j], old[j]);
     } else {
-        for (int i = tid; i < n; i += LN_THREADS) {
-            const float s = xr[i] + (row[i] - mean) * rstd * w[i];
-            xr[i] = s;
-            if (copy) st(copy + (size_t)r * n + i, s);
-        }
+        const int groups = (n + 4 * LN_THREADS - 1) / (4 * LN_THREADS);
+        row_moments<VEC>([&](int j) { return P::load(row, j, n); }, groups, n, eps, scratch, mean, rstd);
+        for (int j = 0; j < groups; ++j) finish(j, P::load(row, j, n), P::load(w, j, n), P::load(xr, j, n));
     }
 }
 
@@ -127,15 +171,11 @@ extern "C" int llmx_layernorm_add(float* x, const float* y, const float* w, floa
     if (rows <= 0) return 0;
     if (n <= 0 || !w) return -2;
     llmx_note_launch(LK_LAYERNORM_ADD);
-    const bool kept = n <= LN_THREADS * LN_KEPT;
-#define LLMX_LN(TO, K) hipLaunchKernelGGL((layernorm_add_kernel<TO, K>), dim3(rows), dim3(LN_THREADS), 0, stream, x, y, w, eps, (TO*)copy, n)
-    if (copy_dtype == LLMX_F32) {
-        if (kept) LLMX_LN(float, true);
-        else LLMX_LN(float, false);
-    } else {
-        if (kept) LLMX_LN(bf16_t, true);
-        else LLMX_LN(bf16_t, false);
-    }
+    const int kept = ln_kept(n);
+    const bool vec = ln_vec(n, x, y, w, copy, nullptr);
+#define LLMX_LN(TO, K, V) hipLaunchKernelGGL((layernorm_add_kernel<TO, K, V>), dim3(rows), dim3(LN_THREADS), 0, stream, x, y, w, eps, (TO*)copy, n)
+    if (copy_dtype == LLMX_F32) LN_FORMS(float);
+    else LN_FORMS(bf16_t);
 #undef LLMX_LN
     return LLMX_CHECK_LAUNCH();
 }
@@ -166,23 +206,40 @@ extern "C" int llmx_cast_rows(const float* x, void* out, int out_dtype, long tot
 
 // out[t] = [x[t] | y[t]] in the activation type, x and y float32 rows of n values: what a product of two joined streams reads.
 // y null: only the first half is written (the second is there from before).
-template <typename TO>
+template <typename TO, int PER>
 __global__ void __launch_bounds__(256) join_rows_kernel(const float* __restrict__ x, const float* __restrict__ y, TO* __restrict__ out, int n, size_t total) {
-    const size_t at = (size_t)blockIdx.x * 256 + threadIdx.x;
+    const size_t at = PER * ((size_t)blockIdx.x * 256 + threadIdx.x);
     if (at >= total) return;
-    const size_t t = at / (size_t)n, i = at % (size_t)n;
+    const size_t t = at / (size_t)n, i = at % (size_t)n;       // PER divides n: a thread's values lie in one row
     TO* row = out + t * 2 * (size_t)n;
-    st(row + i, x[at]);
-    if (y) st(row + n + i, y[at]);
+    float a[PER], b[PER];
+#pragma unroll
+    for (int u = 0; u < PER; ++u) a[u] = x[at + u];
+    if (y) {
+#pragma unroll
+        for (int u = 0; u < PER; ++u) b[u] = y[at + u];
+    }
+#pragma unroll
+    for (int u = 0; u < PER; ++u) st(row + i + u, a[u]);
+    if (y) {
+#pragma unroll
+        for (int u = 0; u < PER; ++u) st(row + n + i + u, b[u]);
+    }
 }
 
 extern "C" int llmx_join_rows(const float* x, const float* y, void* out, int out_dtype, int rows, int n, hipStream_t stream) {
     if (rows <= 0 || n <= 0) return 0;
     llmx_note_launch(LK_JOIN_ROWS);
     const size_t total = (size_t)rows * n;
-    const dim3 grid((unsigned)((total + 255) / 256));
-    if (out_dtype == LLMX_F32) hipLaunchKernelGGL(join_rows_kernel<float>, grid, dim3(256), 0, stream, x, y, (float*)out, n, total);
-    else hipLaunchKernelGGL(join_rows_kernel<bf16_t>, grid, dim3(256), 0, stream, x, y, (bf16_t*)out, n, total);
+    const int per = n % 4 == 0 ? 4 : 1;
+    const dim3 grid((unsigned)((total / per + 255) / 256));
+    if (out_dtype == LLMX_F32) {
+        if (per == 4) hipLaunchKernelGGL((join_rows_kernel<float, 4>), grid, dim3(256), 0, stream, x, y, (float*)out, n, total);
+        else hipLaunchKernelGGL((join_rows_kernel<float, 1>), grid, dim3(256), 0, stream, x, y, (float*)out, n, total);
+    } else {
+        if (per == 4) hipLaunchKernelGGL((join_rows_kernel<bf16_t, 4>), grid, dim3(256), 0, stream, x, y, (bf16_t*)out, n, total);
+        else hipLaunchKernelGGL((join_rows_kernel<bf16_t, 1>), grid, dim3(256), 0, stream, x, y, (bf16_t*)out, n, total);
+    }
     return LLMX_CHECK_LAUNCH();
 }
 

@@ -101,6 +101,88 @@ __global__ void __launch_bounds__(64) delta_prep_kernel(DeltaPrepArgs a) {
     }
 }
 
+// The same for many rows: a wave takes DP_ROWS consecutive rows of a q or k head (or of 64 NC channels of v), its channels' weights
+// and last TAPS - 1 inputs in registers, so that an input is read once; a block of rows may cross from one request to the next.
+// Every value is formed by the operations of the kernel above: the same bits.
+#define DP_ROWS 16
+template <int TAPS, int NC>
+__global__ void __launch_bounds__(64) delta_prep_rows_kernel(DeltaPrepArgs a, int rows) {
+    const int unit = blockIdx.y, lane = threadIdx.x;
+    const int t0 = blockIdx.x * DP_ROWS, t1 = min(rows, t0 + DP_ROWS);
+    const int GD = a.G * a.D, HV = a.H * a.V;
+    const int C = 2 * GD + HV;
+    const int v_units = (HV + 64 * NC - 1) / (64 * NC);
+    if (unit >= 2 * a.G + v_units) {                    // beta and the decays a head
+        for (int i = lane; i < (t1 - t0) * a.H; i += 64) {
+            const int t = t0 + i / a.H, c = i % a.H;
+            a.beta[(size_t)t * a.H + c] = sigmoid_ls(a.pre[(size_t)t * a.ld + a.beta_col + c]);
+            const float l = -expf(a.a_log[c]) * softplus_f(a.step_pre[(size_t)t * a.step_ld + c] + a.dt_bias[c]);
+            a.decay[(size_t)t * a.H + c] = expf(l);
+            if (a.log_decay) a.log_decay[(size_t)t * a.H + c] = l;
+        }
+        return;
+    }
+    const bool keyed = unit < 2 * a.G;
+    const int c0 = keyed ? unit * a.D : 2 * GD + (unit - 2 * a.G) * 64 * NC;
+    const int width = keyed ? a.D : min(64 * NC, C - c0);
+    float* out = unit < a.G ? a.q + c0 : keyed ? a.k + (c0 - GD) : a.v + (c0 - 2 * GD);
+    const size_t out_ld = keyed ? GD : HV;
+    bool in[NC];
+    int ch[NC];
+    float w[NC][TAPS], x[NC][TAPS];                     // x[.][j]: the input that tap j weighs
+#pragma unroll
+    for (int u = 0; u < NC; ++u) {
+        in[u] = lane + 64 * u < width;
+        ch[u] = c0 + (in[u] ? lane + 64 * u : 0);
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) {
+            w[u][j] = a.conv_w[(size_t)ch[u] * TAPS + j];
+            x[u][j] = 0.0f;
+        }
+    }
+    bool fresh = true;
+    for (int b = t0; b < t1; b += 4) {                  // four rows' inputs in flight together
+        float ahead[4][NC];
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+            for (int u = 0; u < NC; ++u) ahead[r][u] = a.pre[(size_t)min(b + r, t1 - 1) * a.ld + ch[u]];
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int t = b + r;
+            if (t >= t1) break;
+            const int e = a.row_entry[t], row0 = a.entry_rows[2 * e], i = t - row0;
+            if (fresh || i == 0) {                      // the inputs before this row: of this step, or from the request's tail
+                const float* tail = a.state + (size_t)a.slot_read[e] * a.state_stride + a.tail_off;
+#pragma unroll
+                for (int j = 0; j + 1 < TAPS; ++j) {
+                    const int idx = i - (TAPS - 1) + j;
+#pragma unroll
+                    for (int u = 0; u < NC; ++u)
+                        x[u][j + 1] = idx >= 0 ? a.pre[(size_t)(row0 + idx) * a.ld + ch[u]] : tail[(size_t)(TAPS - 1 + idx) * C + ch[u]];
+                }
+                fresh = false;
+            }
+            float y[NC], ss = 0.0f;
+#pragma unroll
+            for (int u = 0; u < NC; ++u) {
+#pragma unroll
+                for (int j = 0; j + 1 < TAPS; ++j) x[u][j] = x[u][j + 1];
+                x[u][TAPS - 1] = ahead[r][u];
+                float acc = 0.0f;
+#pragma unroll
+                for (int j = 0; j < TAPS; ++j) acc = fmaf(w[u][j], x[u][j], acc);
+                y[u] = in[u] ? acc * sigmoid_ls(acc) : 0.0f;
+                ss = fmaf(y[u], y[u], ss);
+            }
+            const float scale = keyed ? 1.0f / sqrtf(wave_sum(ss) + 1e-6f) : 1.0f;
+#pragma unroll
+            for (int u = 0; u < NC; ++u)
+                if (in[u]) out[(size_t)t * out_ld + lane + 64 * u] = keyed ? y[u] * scale : y[u];
+        }
+    }
+}
+
 extern "C" int llmx_delta_prep(const float* pre, int ld, const float* conv_w, const float* step_pre, int step_ld, const float* dt_bias,
                                const float* a_log, const float* state, long state_stride, int tail_off, const int* slot_read,
                                const int* row_entry, const int* entry_rows, float* q, float* k, float* v, float* decay, float* beta, int rows, int G,
@@ -111,6 +193,18 @@ extern "C" int llmx_delta_prep(const float* pre, int ld, const float* conv_w, co
     DeltaPrepArgs a{pre, ld, conv_w, step_pre, step_ld, dt_bias, a_log, state, state_stride, tail_off, slot_read, row_entry, entry_rows,
                     q, k, v, decay, beta, log_decay, G, H, D, V, taps, beta_col, head_decay};
     llmx_note_launch(LK_DELTA_PREP);
+    if (rows >= 256 && head_decay && taps >= 2 && taps <= 4) {
+        const int nc = D <= 64 ? 1 : D <= 128 ? 2 : 4;
+        const dim3 grid((rows + DP_ROWS - 1) / DP_ROWS, 2 * G + (H * V + 64 * nc - 1) / (64 * nc) + 1);
+#define LLMX_DP(T_, N_) hipLaunchKernelGGL((delta_prep_rows_kernel<T_, N_>), grid, dim3(64), 0, stream, a, rows)
+#define LLMX_DPT(T_) do { if (nc == 1) LLMX_DP(T_, 1); else if (nc == 2) LLMX_DP(T_, 2); else LLMX_DP(T_, 4); } while (0)
+        if (taps == 2) LLMX_DPT(2);
+        else if (taps == 3) LLMX_DPT(3);
+        else LLMX_DPT(4);
+#undef LLMX_DPT
+#undef LLMX_DP
+        return LLMX_CHECK_LAUNCH();
+    }
     hipLaunchKernelGGL(delta_prep_kernel, dim3(rows, 2 * G + (head_decay ? H : 2 * H) + 1), dim3(64), 0, stream, a);
     return LLMX_CHECK_LAUNCH();
 }
@@ -433,6 +527,188 @@ static void launch_state_step(const StateScanArgs& a, int operands, int n_entrie
     else hipLaunchKernelGGL((state_step_kernel<CN, STATE_OPERANDS_PLAIN>), grid, block, 0, stream, a);
 }
 
+// Steps of single tokens of the delta rule, preparation and recurrence in one launch: the layout of state_step_kernel, the rows'
+// operands formed by every workgroup for its own head (q and k by a wave each, its value channels by one) from the projection and
+// the convolution's tail while the state is on its way, and the correction's sum over the key channels added in the scan's order:
+// a row gets the bits of delta_prep and the scan.  The new tail and state go to the entry's other slot (slot_write differs from
+// slot_read), so every workgroup may read the old ones whenever it likes.
+// Grid (H * ceil(tiles / STEP_TILES), entries); every entry has one row.
+struct DeltaStepArgs {
+    DeltaPrepArgs prep;      // q, k, v, decay and beta are not written
+    float* state;
+    const int* slot_write;
+    float* out;              // [T, H*V]
+    float out_scale;
+};
+
+// Channel ch of a single-row entry: the taps' inputs asked for four at a time.
+__device__ __forceinline__ float conv_silu_step(const DeltaPrepArgs& a, const float* __restrict__ tail, int C, size_t row, int ch) {
+    float acc = 0.0f;
+    for (int j0 = 0; j0 < a.taps; j0 += 4) {
+        float x[4], w[4];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int j = min(j0 + u, a.taps - 1);
+            x[u] = j < a.taps - 1 ? tail[(size_t)j * C + ch] : a.pre[row * a.ld + ch];
+            w[u] = a.conv_w[(size_t)ch * a.taps + j];
+        }
+#pragma unroll
+        for (int u = 0; u < 4; ++u)
+            if (j0 + u < a.taps) acc = fmaf(w[u], x[u], acc);
+    }
+    return acc * sigmoid_ls(acc);
+}
+
+template <int CN>
+__global__ void __launch_bounds__(64 * CN) delta_step_kernel(DeltaStepArgs s) {
+    typedef float f32x4_t __attribute__((ext_vector_type(4)));
+    __shared__ __attribute__((aligned(16))) f32x4_t part[STEP_TILES][CN][64];
+    __shared__ float qs[PREP_MAX], ks[PREP_MAX], vs[STEP_TILES * SCAN_COLS], dots[STEP_TILES * SCAN_COLS], head_beta, head_decay;
+    const DeltaPrepArgs& a = s.prep;
+    const int tid = threadIdx.x, chunk = tid >> 6, lane = tid & 63;
+    const int tiles = (a.V + SCAN_COLS - 1) / SCAN_COLS, blocks = (tiles + STEP_TILES - 1) / STEP_TILES;
+    const int h = blockIdx.x / blocks, tile0 = (blockIdx.x % blocks) * STEP_TILES, e = blockIdx.y;
+    const int d = 32 * chunk + (lane >> 1), half = lane & 1;
+    const bool live = d < a.D;
+    const int dd = live ? d : 0;
+    const size_t slot_r = (size_t)a.slot_read[e] * a.state_stride, slot_w = (size_t)s.slot_write[e] * a.state_stride;
+    const size_t at = ((size_t)h * tiles + tile0) * a.D * SCAN_COLS + (size_t)dd * SCAN_COLS + 4 * half;
+    const size_t tile_floats = (size_t)a.D * SCAN_COLS;
+    f32x4_t S[STEP_TILES];
+#pragma unroll
+    for (int u = 0; u < STEP_TILES; ++u)
+        S[u] = *reinterpret_cast<const f32x4_t*>(a.state + slot_r + at + (tile0 + u < tiles ? u : 0) * tile_floats);
+    const size_t row = (size_t)a.entry_rows[2 * e];
+    const int GD = a.G * a.D, HV = a.H * a.V, C = 2 * GD + HV;
+    const float* tail = a.state + slot_r + a.tail_off;
+    const int c0 = (h / (a.H / a.G)) * a.D;
+    for (int unit = chunk; unit < 3; unit += CN) {
+        if (unit < 2) {                                 // q, k
+            float y[PREP_MAX / 64], ss = 0.0f;
+#pragma unroll
+            for (int u = 0; u < (CN + 1) / 2; ++u) {    // CN chunks of 32 channels
+                y[u] = lane + 64 * u < a.D ? conv_silu_step(a, tail, C, row, unit * GD + c0 + lane + 64 * u) : 0.0f;
+                ss = fmaf(y[u], y[u], ss);
+            }
+            const float r = 1.0f / sqrtf(wave_sum(ss) + 1e-6f);
+#pragma unroll
+            for (int u = 0; u < (CN + 1) / 2; ++u) (unit == 0 ? qs : ks)[lane + 64 * u] = y[u] * r;
+        } else if (lane < STEP_TILES * SCAN_COLS) {     // the workgroup's value channels
+            const int j = tile0 * SCAN_COLS + lane;
+            vs[lane] = j < a.V ? conv_silu_step(a, tail, C, row, 2 * GD + h * a.V + j) : 0.0f;
+        } else if (lane == STEP_TILES * SCAN_COLS) {
+            head_beta = sigmoid_ls(a.pre[row * a.ld + a.beta_col + h]);
+            if (a.head_decay) head_decay = expf(-expf(a.a_log[h]) * softplus_f(a.step_pre[row * a.step_ld + h] + a.dt_bias[h]));
+        }
+    }
+    {       // the tail moves on by one row, the entry's workgroups sharing its channels out
+        float* fresh = s.state + slot_w + a.tail_off;
+        const int per = (C + (int)gridDim.x - 1) / (int)gridDim.x, end = min(C, ((int)blockIdx.x + 1) * per);
+        for (int ch = (int)blockIdx.x * per + tid; ch < end; ch += 64 * CN)
+            for (int p = 0; p < a.taps - 1; ++p) fresh[(size_t)p * C + ch] = p + 1 < a.taps - 1 ? tail[(size_t)(p + 1) * C + ch] : a.pre[row * a.ld + ch];
+    }
+    __syncthreads();
+    const float k = ks[dd], q = qs[dd], beta = head_beta;
+    const float g = a.head_decay ? head_decay
+                                 : expf(-expf(a.a_log[h]) * softplus_f(a.step_pre[row * a.step_ld + (size_t)h * a.D + dd] + a.dt_bias[(size_t)h * a.D + dd]));
+    // the sum of a tile's parts over the key channels, in the scan's order; lanes of one parity end with the same four columns
+    auto tile_sum = [&](int u) {
+        f32x4_t o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            float x;
+            if (CN == 2) x = part[u][0][lane][i] + part[u][1 % CN][lane][i];
+            else if (CN == 4) x = (part[u][0][lane][i] + part[u][2 % CN][lane][i]) + (part[u][1 % CN][lane][i] + part[u][3 % CN][lane][i]);
+            else
+                x = ((part[u][0][lane][i] + part[u][2 % CN][lane][i]) + (part[u][4 % CN][lane][i] + part[u][6 % CN][lane][i])) +
+                    ((part[u][1 % CN][lane][i] + part[u][3 % CN][lane][i]) + (part[u][5 % CN][lane][i] + part[u][7 % CN][lane][i]));
+            uint32_t p0, p1;
+            halves_pair32(__float_as_uint(x), p0, p1);       // channels 16 apart
+            x = __uint_as_float(p0) + __uint_as_float(p1);
+            rows_pair16(__float_as_uint(x), p0, p1);         // 8 apart
+            x = __uint_as_float(p0) + __uint_as_float(p1);
+            x += row_rotate<8>(x);
+            x += row_rotate<4>(x);
+            x += row_rotate<2>(x);
+            o[i] = x;
+        }
+        return o;
+    };
+#pragma unroll
+    for (int u = 0; u < STEP_TILES; ++u) {
+        f32x4_t o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            S[u][i] = S[u][i] * g;
+            o[i] = live ? k * S[u][i] : 0.0f;
+        }
+        part[u][chunk][lane] = o;
+    }
+    __syncthreads();
+    for (int u = chunk; u < STEP_TILES; u += CN) {
+        const f32x4_t o = tile_sum(u);
+        if (lane < 2) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) dots[u * SCAN_COLS + 4 * lane + i] = o[i];
+        }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < STEP_TILES; ++u) {
+        f32x4_t o;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            const int j = u * SCAN_COLS + 4 * half + i;
+            S[u][i] = fmaf(k, beta * (vs[j] - dots[j]), S[u][i]);
+            o[i] = live ? q * S[u][i] : 0.0f;
+        }
+        part[u][chunk][lane] = o;
+        if (tile0 + u < tiles && live) {
+            // columns past V keep what they held
+            float* to = s.state + slot_w + at + u * tile_floats;
+            const int left = a.V - ((tile0 + u) * SCAN_COLS + 4 * half);
+            if (left >= 4) *reinterpret_cast<f32x4_t*>(to) = S[u];
+            else
+                for (int i = 0; i < left; ++i) to[i] = S[u][i];
+        }
+    }
+    __syncthreads();
+    for (int u = chunk; u < STEP_TILES; u += CN) {
+        const int tile = tile0 + u;
+        if (tile >= tiles) break;
+        const f32x4_t o = tile_sum(u);
+        if (lane < 2) {
+            float* to = s.out + row * (size_t)HV + (size_t)h * a.V + tile * SCAN_COLS + 4 * lane;
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+                if (tile * SCAN_COLS + 4 * lane + i < a.V) to[i] = o[i] * s.out_scale;
+        }
+    }
+}
+
+// Whether llmx_delta_step takes a state whose slots are `stride` floats apart.
+extern "C" int llmx_delta_step_ok(int D, long stride) { return D >= 1 && D <= PREP_MAX && stride % 4 == 0 ? 1 : 0; }
+
+extern "C" int llmx_delta_step(const float* pre, int ld, const float* conv_w, const float* step_pre, int step_ld, const float* dt_bias,
+                               const float* a_log, float* state, long state_stride, int tail_off, const int* slot_read, const int* slot_write,
+                               const int* entry_rows, float* out, float out_scale, int n_entries, int G, int H, int D, int V, int taps, int beta_col,
+                               int head_decay, hipStream_t stream) {
+    if (n_entries <= 0) return 0;
+    const long C = 2L * G * D + (long)H * V;
+    if (!llmx_delta_step_ok(D, state_stride) || ((uintptr_t)state & 15) || taps < 1 || G < 1 || H < 1 || H % G || V < 1 || beta_col + H > ld || C > ld ||
+        step_ld < (head_decay ? H : H * D)) return -2;
+    DeltaStepArgs s{DeltaPrepArgs{pre, ld, conv_w, step_pre, step_ld, dt_bias, a_log, state, state_stride, tail_off, slot_read, nullptr, entry_rows,
+                                  nullptr, nullptr, nullptr, nullptr, nullptr, nullptr, G, H, D, V, taps, beta_col, head_decay},
+                    state, slot_write, out, out_scale};
+    llmx_note_launch(LK_DELTA_STEP);
+    const int tiles = (V + SCAN_COLS - 1) / SCAN_COLS;
+    const dim3 grid((unsigned)(H * ((tiles + STEP_TILES - 1) / STEP_TILES)), (unsigned)n_entries);
+    if (D <= 64) hipLaunchKernelGGL(delta_step_kernel<2>, grid, dim3(128), 0, stream, s);
+    else if (D <= 128) hipLaunchKernelGGL(delta_step_kernel<4>, grid, dim3(256), 0, stream, s);
+    else hipLaunchKernelGGL(delta_step_kernel<8>, grid, dim3(512), 0, stream, s);
+    return LLMX_CHECK_LAUNCH();
+}
+
 extern "C" int llmx_state_scan(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, const float* decay, int ldg,
                                const float* beta, float* state, long state_stride, const int* slot_read, const int* slot_write,
                                const int* entry_rows, float* out, float out_scale, int n_entries, int H, int share, int D, int V,
@@ -500,14 +776,16 @@ struct HeadNormArgs {
     const float* den_floor;
 };
 
-// WAVES 1: a wave a head, as above.  More: a workgroup of that many waves a head, for norms over long rows (all heads of a row
+// WAVES 1: a wave a head, as above, four heads a workgroup; up to 8 values a lane stay in registers.  More: a workgroup of that many waves a head, for norms over long rows (all heads of a row
 // normed together); the waves' sums are added in wave order.
 template <typename TO, int WAVES>
-__global__ void __launch_bounds__(64 * WAVES) head_norm_gate_kernel(HeadNormArgs a, TO* __restrict__ out) {
+__global__ void __launch_bounds__(WAVES == 1 ? 256 : 64 * WAVES) head_norm_gate_kernel(HeadNormArgs a, TO* __restrict__ out) {
     __shared__ float scratch[WAVES];
     constexpr int NT = 64 * WAVES;
-    const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
+    const int t = blockIdx.x, h = WAVES == 1 ? 4 * (int)blockIdx.y + ((int)threadIdx.x >> 6) : (int)blockIdx.y;
+    const int lane = WAVES == 1 ? threadIdx.x & 63 : threadIdx.x;
     const int H = a.H, V = a.V;
+    if (WAVES == 1 && h >= H) return;
     const float* row = a.o + ((size_t)t * H + h) * a.o_head;
     float den = 1.0f;
     if (a.den_floor) den = fmaxf(fabsf(row[V]), a.den_floor[(size_t)t * H + h]) + 1e-6f;
@@ -520,7 +798,7 @@ __global__ void __launch_bounds__(64 * WAVES) head_norm_gate_kernel(HeadNormArgs
     float ss = 0.0f;
     // a workgroup's row of at most KEPT values a thread stays in registers, everything asked for before the sum is formed
     constexpr int KEPT = 8;
-    if (WAVES > 1 && V <= NT * KEPT) {
+    if (V <= NT * KEPT) {
         const float* zr = a.z ? a.z + (size_t)t * a.ldz + (size_t)h * V : nullptr;
         const float* w = a.w ? (a.w_wide ? a.w + (size_t)h * V : a.w) : nullptr;
         float x[KEPT], z[KEPT], wk[KEPT];
@@ -533,7 +811,7 @@ __global__ void __launch_bounds__(64 * WAVES) head_norm_gate_kernel(HeadNormArgs
         }
 #pragma unroll
         for (int u = 0; u < KEPT; ++u) ss = fmaf(x[u], x[u], ss);
-        const float r = 1.0f / sqrtf(block_sum<WAVES>(ss, scratch) / (float)V + a.eps);
+        const float r = 1.0f / sqrtf((WAVES == 1 ? wave_sum(ss) : block_sum<WAVES>(ss, scratch)) / (float)V + a.eps);
         TO* dst = out + ((size_t)t * H + h) * V;
 #pragma unroll
         for (int u = 0; u < KEPT; ++u) {
@@ -581,8 +859,8 @@ extern "C" int llmx_head_norm_gate(const float* o, const float* w, const float* 
         else hipLaunchKernelGGL((head_norm_gate_kernel<bf16_t, 8>), dim3(rows, H), dim3(512), 0, stream, a, (bf16_t*)out);
         return LLMX_CHECK_LAUNCH();
     }
-    if (out_dtype == LLMX_F32) hipLaunchKernelGGL((head_norm_gate_kernel<float, 1>), dim3(rows, H), dim3(64), 0, stream, a, (float*)out);
-    else hipLaunchKernelGGL((head_norm_gate_kernel<bf16_t, 1>), dim3(rows, H), dim3(64), 0, stream, a, (bf16_t*)out);
+    if (out_dtype == LLMX_F32) hipLaunchKernelGGL((head_norm_gate_kernel<float, 1>), dim3(rows, (H + 3) / 4), dim3(256), 0, stream, a, (float*)out);
+    else hipLaunchKernelGGL((head_norm_gate_kernel<bf16_t, 1>), dim3(rows, (H + 3) / 4), dim3(256), 0, stream, a, (bf16_t*)out);
     return LLMX_CHECK_LAUNCH();
 }
 

@@ -89,7 +89,8 @@
     X(RMSNORM_SHIFT, "rmsnorm_shift")                                                                                     \
     X(DECAYED_STATE_CHUNKS, "decayed_state.chunks")                                                                       \
     X(JOIN_ROWS, "join_rows")                                                                                             \
-    X(DELTA_CHUNKS, "delta_chunks")
+    X(DELTA_CHUNKS, "delta_chunks")                                                                                       \
+    X(DELTA_STEP, "delta_step")
 
 enum LlmxLaunchKind : int {
 #define LLMX_X(id, name) LK_##id,

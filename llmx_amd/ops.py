@@ -92,6 +92,8 @@ def _declare(h) -> None:
         "llmx_combine_rows": [P, P, F, P, P, F, I, I, I, P],
         "llmx_scale_softcap": [P, F, F, L, P],
         "llmx_delta_prep": [P, I, P, P, I, P, P, P, L, I, P, P, P, P, P, P, P, P, I, I, I, I, I, I, I, I, P, P],
+        "llmx_delta_step": [P, I, P, P, I, P, P, P, L, I, P, P, P, P, F, I, I, I, I, I, I, I, I, P],
+        "llmx_delta_step_ok": [I, L],
         "llmx_delta_chunks": [P, I, P, I, P, I, P, P, P, L, P, P, P, P, I, P, I, P, P, P, P, P, P, F, I, I, I, I, P, I, I, I, I, P],
         "llmx_cast_cols": [P, I, P, I, I, I, P],
         "llmx_sigmoid_root": [P, P, F, P, I, I, P],
@@ -760,6 +762,32 @@ def delta_prep(pre: torch.Tensor, conv_w: torch.Tensor, step_pre: torch.Tensor, 
                                  _dev(decay, "decay", torch.float32, (T, DW)), _dev(beta, "beta", torch.float32, (T, H)),
                                  T, G, H, D, V, taps, int(beta_col), 1 if head_decay else 0, _dev(log_decay, "log_decay", torch.float32, (T, H)), _stream()),
            "delta_prep")
+
+
+def delta_step_ok(D: int, state: torch.Tensor) -> bool:
+    """Whether delta_step takes heads of D key channels and this state tensor."""
+    return bool(lib().llmx_delta_step_ok(int(D), state.shape[1]))
+
+
+def delta_step(pre: torch.Tensor, conv_w: torch.Tensor, step_pre: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, state: torch.Tensor,
+               tail_off: int, slot_read: torch.Tensor, slot_write: torch.Tensor, entry_rows: torch.Tensor, out: torch.Tensor, out_scale: float, G: int,
+               H: int, D: int, V: int, beta_col: int, head_decay: bool = False) -> None:
+    """delta_prep and state_scan (with the tail) of a step in which every entry has one row, in one launch and with their bits:
+    out [T, H*V].  slot_write[e] must differ from slot_read[e]."""
+    T, ld = pre.shape
+    C = 2 * G * D + H * V
+    DW = H if head_decay else H * D
+    taps = conv_w.shape[1]
+    n_e = entry_rows.shape[0]
+    if state.dim() != 2 or tail_off < state_matrix_size(H, D, V) or tail_off + (taps - 1) * C > state.shape[1] or n_e != T:
+        raise KernelError("delta_step: the state does not hold the matrices and the convolution's tail, or an entry has not one row")
+    step_at, step_ld = _rows_view(step_pre, "step_pre", T, DW)
+    _check(lib().llmx_delta_step(_dev(pre, "pre", torch.float32), ld, _dev(conv_w, "conv_w", torch.float32, (C, taps)), step_at, step_ld,
+                                 _dev(dt_bias, "dt_bias", torch.float32, (DW,)), _dev(a_log, "a_log", torch.float32, (H,)),
+                                 _dev(state, "state", torch.float32), state.shape[1], int(tail_off), _dev(slot_read, "slot_read", torch.int32, (n_e,)),
+                                 _dev(slot_write, "slot_write", torch.int32, (n_e,)), _dev(entry_rows, "entry_rows", torch.int32, (n_e, 2)),
+                                 _dev(out, "out", torch.float32, (T, H * V)), float(out_scale), n_e, G, H, D, V, taps, int(beta_col),
+                                 1 if head_decay else 0, _stream()), "delta_step")
 
 
 def sigmoid_root(z: torch.Tensor, bias: Optional[torch.Tensor], tau: float, out: torch.Tensor) -> None:

@@ -110,7 +110,8 @@ class HeadDeltaRule(Mixer):
         self.w_in = self.conv = self.a_log = self.dt_bias = self.norm = self.w_o = None
 
     def cache_need(self):
-        return StateNeed((self.state_matrix + (self.taps - 1) * self.channels,), "float32")
+        # slots a multiple of four floats apart, so that the step of single tokens reads them 16 bytes at a time
+        return StateNeed((-(-(self.state_matrix + (self.taps - 1) * self.channels) // 4) * 4,), "float32")
 
     def tensor_specs(self, available):
         E, H, V = self.hidden, self.heads, self.vdim
@@ -136,6 +137,19 @@ class HeadDeltaRule(Mixer):
         pre = step.buf("delta.pre", (T, self.in_width), f32)
         ops.gemm(h, self.w_in, pre, scratch=step.buf)
         view = lambda n: pre[:, self.cols[n][0]:self.cols[n][0] + self.cols[n][1]]
+        o = step.buf("delta.o", (T, H * V), f32)
+        if step.max_rows_per_entry == 1 and ops.delta_step_ok(D, cache.state):      # single tokens: one launch, the scan's bits
+            ops.delta_step(pre, self.conv, view("a"), self.dt_bias, self.a_log, cache.state, self.state_matrix, step.entry_held_slots,
+                           step.entry_slots, step.entry_rows, o, float(D) ** -0.5, G, H, D, V, self.cols["b"][0], head_decay=True)
+        else:
+            self._rows(step, pre, view, o, cache)
+        gated = step.buf("delta.gated", (T, H * V), step.act_dtype)
+        ops.head_norm_gate(o, self.norm, view("g"), gated, self.eps, H, V, ops.GATE_SILU)
+        ops.gemm(gated, self.w_o, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)
+
+    def _rows(self, step, pre, view, o, cache):
+        T, H, G, D, V = step.rows, self.heads, self.kv_heads, self.dim, self.vdim
+        f32 = torch.float32
         q, k = step.buf("delta.q", (T, G * D), f32), step.buf("delta.k", (T, G * D), f32)
         v, decay, beta = step.buf("delta.v", (T, H * V), f32), step.buf("delta.head_decay", (T, H), f32), step.buf("delta.beta", (T, H), f32)
         # a decode step's entries are never long (nothing for a graph to hold)
@@ -143,7 +157,6 @@ class HeadDeltaRule(Mixer):
         log_decay = step.buf("delta.log_decay", (T, H), f32) if plan is not None else None
         ops.delta_prep(pre, self.conv, view("a"), self.dt_bias, self.a_log, cache.state, self.state_matrix, step.entry_held_slots,
                        step.row_entry, step.entry_rows, q, k, v, decay, beta, G, H, D, V, self.cols["b"][0], head_decay=True, log_decay=log_decay)
-        o = step.buf("delta.o", (T, H * V), f32)
         tail = (pre[:, :self.channels], self.taps, self.state_matrix) if self.taps > 1 else None
         if plan is not None:
             ops.delta_chunks(q, k, v, log_decay, beta, cache.state, step.entry_held_slots, step.entry_slots, step.entry_rows, o, float(D) ** -0.5,
@@ -152,9 +165,6 @@ class HeadDeltaRule(Mixer):
             ops.state_scan(q, k, v, decay, beta, cache.state, step.entry_held_slots, step.entry_slots, step.entry_rows, o, float(D) ** -0.5,
                            H, G, D, V, tail=tail, max_rows=step.max_rows_per_entry, head_decay=True,
                            max_rows_here=ops.DECAYED_CHUNKS_MIN_ROWS - 1 if plan is not None else 0)
-        gated = step.buf("delta.gated", (T, H * V), step.act_dtype)
-        ops.head_norm_gate(o, self.norm, view("g"), gated, self.eps, H, V, ops.GATE_SILU)
-        ops.gemm(gated, self.w_o, out, ops.EPI_ADD if accumulate else ops.EPI_STORE, scratch=step.buf)
 
 
 class ChannelDeltaRule(Mixer):
