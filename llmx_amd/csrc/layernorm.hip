@@ -1,9 +1,10 @@
 // Layer norm with a weight and an optional bias, and the element-wise steps of layers that norm a sublayer's result before it
 // joins the residual: y = (x - mean) / sqrt(var + eps) * w (+ b), var the mean of the squared deviations.  Everything is float32
 // arithmetic on float32 rows; only what a product reads next is stored in the activation type.
-// A row's sums are formed by 256 threads: thread v adds elements 4v .. 4v + 3, then those 1,024 further on, ... in this order (rows
-// whose length is no multiple of 4: elements v, v + 256, ...), a wave adds its threads' sums with wave_sum, and the four waves' sums
-// are added in wave order: a function of the row's length only.
+// A row's sums are formed by 256 threads: thread v adds elements v, v + 256, ... in this order, a wave adds its threads' sums with
+// wave_sum, and the four waves' sums are added in wave order.  Norms with a bias whose rows are a multiple of 4 long deal the elements
+// out by fours instead (4v .. 4v + 3, then those 1,024 further on, ...), so that a thread reads and writes 16 bytes at a time.  Either
+// way a row's bits depend on its length and its norm only.
 #include "common.h"
 
 #define LN_THREADS 256
@@ -53,7 +54,8 @@ __device__ __forceinline__ void row_moments(Get get, int groups, int n, float ep
     float s = 0.0f;
     for (int j = 0; j < groups; ++j) {
         const ln4_t v = get(j);
-        s += (v[0] + v[1]) + (v[2] + v[3]);
+        if (VEC) s += (v[0] + v[1]) + (v[2] + v[3]);
+        else s = (((s + v[0]) + v[1]) + v[2]) + v[3];
     }
     mean = block_sum<LN_THREADS / 64>(s, scratch) / (float)n;
     float q = 0.0f;
@@ -123,7 +125,7 @@ extern "C" int llmx_layernorm(const float* x, const int* pick, const float* w, c
     if (n <= 0 || !w || (!out && !out32)) return -2;
     llmx_note_launch(LK_LAYERNORM);
     const int kept = ln_kept(n);
-    const bool vec = ln_vec(n, x, w, bias, out, out32);
+    const bool vec = bias && ln_vec(n, x, w, bias, out, out32);
 #define LLMX_LN(TO, K, V) hipLaunchKernelGGL((layernorm_kernel<TO, K, V>), dim3(rows), dim3(LN_THREADS), 0, stream, x, pick, w, bias, eps, (TO*)out, out32, n)
     if (out_dtype == LLMX_F32) LN_FORMS(float);
     else LN_FORMS(bf16_t);
@@ -172,7 +174,7 @@ extern "C" int llmx_layernorm_add(float* x, const float* y, const float* w, floa
     if (n <= 0 || !w) return -2;
     llmx_note_launch(LK_LAYERNORM_ADD);
     const int kept = ln_kept(n);
-    const bool vec = ln_vec(n, x, y, w, copy, nullptr);
+    const bool vec = false;      // no bias: see above
 #define LLMX_LN(TO, K, V) hipLaunchKernelGGL((layernorm_add_kernel<TO, K, V>), dim3(rows), dim3(LN_THREADS), 0, stream, x, y, w, eps, (TO*)copy, n)
     if (copy_dtype == LLMX_F32) LN_FORMS(float);
     else LN_FORMS(bf16_t);
