@@ -81,7 +81,7 @@ def test_the_record_of_one_real_layer():
     assert "long" not in rec        # the long-context configuration belongs to the default run only
 
 
-@pytest.mark.parametrize("design,title", [("nenotar", "Nenotar"), ("salipel", "Salipel"), ("neruzen", "Neruzen")])
+@pytest.mark.parametrize("design,title", [("nenotar", "Nenotar"), ("salipel", "Salipel"), ("neruzen", "Neruzen"), ("vivulorn", "Vivulorn")])
 def test_the_record_of_a_design_beside_its_closest_model(design, title):
     """`--design NAME` at a small size: one JSON line, both models with prompt and decode rates that follow from their
     times and fractions that follow from the work."""
