@@ -236,6 +236,70 @@ __device__ __forceinline__ void rms_rows_as_1024(const float* __restrict__ X, si
     }
 }
 
+// A layer norm (weight and bias) of a few rows inside another kernel, with the bits of the layer norm kernel's form for norms with a
+// bias: 256 threads, thread v adds elements 4v .. 4v + 3 of every 1,024 as (v0 + v1) + (v2 + v3), each wave its threads' sums with
+// wave_sum, the four waves' sums in wave order; then the squared deviations likewise, each with fmaf.  A workgroup of NW waves does the
+// same: wave w stands for the waves w, w + NW, ... of those four (with 8 waves the last four only wait).  Rows of n values, n a multiple
+// of 4, at most 4,096; 16-byte aligned.  scratch32: 32 floats of LDS.  The caller puts a barrier between the stores and their first read.
+template <int NW, typename Store>
+__device__ __forceinline__ void layer_norm_rows_as_256(const float* __restrict__ X, size_t ldx, int rows, int n, const float* __restrict__ w,
+                                                       const float* __restrict__ bias, float eps, float* scratch32, Store store) {
+    typedef float quad_t __attribute__((ext_vector_type(4)));
+    constexpr int VW = NW >= 4 ? 1 : 4 / NW;      // waves of the 256-thread block that one wave stands for
+    const int wave = threadIdx.x / LLMX_WAVE, lane = threadIdx.x & (LLMX_WAVE - 1);
+    const bool works = wave < 4;
+    for (int row = 0; row < rows; ++row) {
+        const float* x = X + (size_t)row * ldx;
+        quad_t v[VW][4], wk[VW][4], bk[VW][4];
+#pragma unroll
+        for (int u = 0; u < VW; ++u)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int at = 4 * ((wave + u * NW) * LLMX_WAVE + lane + 256 * j);
+                const bool in = works && at < n;
+                v[u][j] = in ? *reinterpret_cast<const quad_t*>(x + at) : quad_t{0.0f, 0.0f, 0.0f, 0.0f};
+                wk[u][j] = in ? *reinterpret_cast<const quad_t*>(w + at) : quad_t{0.0f, 0.0f, 0.0f, 0.0f};
+                bk[u][j] = in ? *reinterpret_cast<const quad_t*>(bias + at) : quad_t{0.0f, 0.0f, 0.0f, 0.0f};
+            }
+        float* scratch = scratch32 + 8 * (row & 1);       // rows take turns in two sets
+#pragma unroll
+        for (int u = 0; u < VW; ++u) {
+            float s = 0.0f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j) s += (v[u][j][0] + v[u][j][1]) + (v[u][j][2] + v[u][j][3]);
+            s = wave_sum(s);
+            if (works && lane == 0) scratch[wave + u * NW] = s;
+        }
+        __syncthreads();
+        const float mean = (((scratch[0] + scratch[1]) + scratch[2]) + scratch[3]) / (float)n;
+#pragma unroll
+        for (int u = 0; u < VW; ++u) {
+            float q = 0.0f;
+#pragma unroll
+            for (int j = 0; j < 4; ++j)
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    const float d = 4 * ((wave + u * NW) * LLMX_WAVE + lane + 256 * j) < n ? v[u][j][i] - mean : 0.0f;
+                    q = fmaf(d, d, q);
+                }
+            q = wave_sum(q);
+            if (works && lane == 0) scratch[4 + wave + u * NW] = q;
+        }
+        __syncthreads();
+        const float rstd = 1.0f / sqrtf((((scratch[4] + scratch[5]) + scratch[6]) + scratch[7]) / (float)n + eps);
+#pragma unroll
+        for (int u = 0; u < VW; ++u)
+#pragma unroll
+            for (int j = 0; j < 4; ++j) {
+                const int at = 4 * ((wave + u * NW) * LLMX_WAVE + lane + 256 * j);
+                if (works && at < n) {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) store(row, at + i, (v[u][j][i] - mean) * rstd * wk[u][j][i] + bk[u][j][i]);
+                }
+            }
+    }
+}
+
 // A one-argument activation that a product applies to what it stores (the store epilogue only), or a kernel of its own.
 // xIELU with two learned numbers (p, q) read from the device: z > 0: softplus(p) z^2 + z/2; z <= 0: (1/2 + softplus(q))
 // (e^z - 1 - z) + z/2.  Both go through these two functions, so a product with the activation gives the bits of the product

@@ -287,22 +287,33 @@ __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkA
     const int first = EL * tid;                             // the thread's values: row and column from its place in a tile's lanes
     const int u_row0 = 16 * (first >> 8) + 4 * ((first & 255) >> 6), u_col = ((first & 255) >> 2) & 15, u_e0 = first & 3;
     const int kd = min(16 * wave + c, a.D - 1), wd = real ? 16 * wave + 4 * g : 0;
+    // a thread's places within a chunk's operands; what moves from chunk to chunk (and from row to row) is the same for every thread
+    const uint32_t w_at = (uint32_t)(c * a.DR + wd), k_at = (uint32_t)(4 * g * a.ldk + kd), u_at = (uint32_t)((u_row0 + u_e0) * a.VR + 16 * vt + u_col);
+    const uint32_t d_at = (uint32_t)(u_row0 + u_e0);
     auto fetch = [&](Operands& x, int ch) {
         const size_t at = (size_t)ch * a.H + h;
         const float* W = a.W + at * DS_ROWS * a.DR;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) x.w[i] = *reinterpret_cast<const f32x4_t*>(W + (size_t)(16 * i + c) * a.DR + wd);
+        for (int i = 0; i < 4; ++i) x.w[i] = *reinterpret_cast<const f32x4_t*>(W + (size_t)(16 * i) * a.DR + w_at);
         const int ahead = (ch - c0) * DS_ROWS, n = min(DS_ROWS, rows - ahead);
-        const float* kp = a.k + (size_t)(row0 + ahead) * a.ldk + (size_t)(h / a.share) * a.D + kd;
+        const float* kp = a.k + (size_t)(row0 + ahead) * a.ldk + (size_t)(h / a.share) * a.D;
+        if (n == DS_ROWS) {
 #pragma unroll
-        for (int s = 0; s < 4; ++s)
+            for (int s = 0; s < 4; ++s)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) x.k[4 * s + e] = kp[(size_t)min(16 * s + 4 * g + e, n - 1) * a.ldk];
+                for (int e = 0; e < 4; ++e) x.k[4 * s + e] = (kp + (size_t)(16 * s + e) * a.ldk)[k_at];
+        } else {
+#pragma unroll
+            for (int s = 0; s < 4; ++s)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) x.k[4 * s + e] = kp[(size_t)min(16 * s + 4 * g + e, n - 1) * a.ldk + kd];
+        }
+        const float* U = a.U + at * DS_ROWS * a.VR;
+        const float* decays = a.decays + at * DS_ROWS;
 #pragma unroll
         for (int y = 0; y < EL; ++y) {
-            const int row = u_row0 + u_e0 + y;
-            x.u0[y] = a.U[(at * DS_ROWS + row) * a.VR + 16 * vt + u_col];
-            x.decay[y] = a.decays[at * DS_ROWS + row];
+            x.u0[y] = (U + (size_t)y * a.VR)[u_at];
+            x.decay[y] = (decays + y)[d_at];
         }
         x.keep = a.keep[at];
     };
@@ -326,7 +337,7 @@ __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkA
             for (int w = 1; w < NU; ++w) sum += part[w][first + y];
             const float u = x.u0[y] - sum;
             const int row = u_row0 + u_e0 + y;
-            a.U[(at * DS_ROWS + row) * a.VR + 16 * vt + u_col] = u;
+            (a.U + (at * DS_ROWS + y) * a.VR)[u_at] = u;
             us[row * LDU + u_col] = u * x.decay[y];
         }
         __syncthreads();

@@ -13,7 +13,7 @@
 //
 // Normed rows: for steps of very few rows the product can take the float32 residual rows and an RMSNorm's weights
 // instead of A; every workgroup forms the normed, rounded rows itself (in LDS) while its first weights travel, and no
-// norm kernel is launched.  The rows' values are the norm kernel's, bit for bit.
+// norm kernel is launched.  The rows' values are the norm kernel's, bit for bit.  With a bias the norm is a layer norm.
 #include "common.h"
 
 typedef __bf16 bf16x8_t __attribute__((ext_vector_type(8)));
@@ -41,6 +41,7 @@ struct SkinnyArgs {
     const float* norm_w;
     float norm_eps;
     int x_rows;
+    const float* norm_bias;    // not null: a layer norm with this bias
     // SK_STORE, SK_ADD: an activation applied to the product (LLMX_ACT_*), with its parameters on the device
     int act;
     const float* act_params;
@@ -109,8 +110,9 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
         if (PIPELINED) fetch_weights(s_begin, r0);
         if (NORMED && !rows_normed) {
             // the step's rows, normed and rounded as the norm kernel stores them, while the first weights travel
-            rms_rows_as_1024<KS>(g.X, (size_t)K, g.x_rows, K, g.norm_w, g.norm_eps, norm_scratch,
-                                 [&](int row, int i, float y) { normed_rows[(size_t)row * K + i] = f32_to_bf16(y); });
+            auto keep = [&](int row, int i, float y) { normed_rows[(size_t)row * K + i] = f32_to_bf16(y); };
+            if (g.norm_bias) layer_norm_rows_as_256<KS>(g.X, (size_t)K, g.x_rows, K, g.norm_w, g.norm_bias, g.norm_eps, norm_scratch, keep);
+            else rms_rows_as_1024<KS>(g.X, (size_t)K, g.x_rows, K, g.norm_w, g.norm_eps, norm_scratch, keep);
             rows_normed = true;   // the barrier below stands between these stores and the first read
         }
         if (tid < MT * 16) {
@@ -427,7 +429,7 @@ extern "C" int llmx_gemm_skinny_normed_ok(int x_rows, int K) {
 extern "C" int llmx_gemm_skinny(const void* A, const void* W, void* C, int c_dtype, int M, int N, int K, int lda, int ldc, int epi, int ks,
                                 int n_groups, int max_active, const int* active, const int* n_active, const int* group_offsets,
                                 const int* list, int a_div, long w_group_stride, int up_offset, const float* X, const float* norm_w,
-                                float norm_eps, int x_rows, int act, const float* act_params, int glu_kind, float glu_limit,
+                                float norm_eps, int x_rows, const float* norm_bias, int act, const float* act_params, int glu_kind, float glu_limit,
                                 const float* glu_row_scale, const float* glu_row_gate, int glu_row_gate_ld, hipStream_t stream) {
     if (N <= 0 || K <= 0) return 0;
     if (K % 8) return -2;
@@ -435,8 +437,9 @@ extern "C" int llmx_gemm_skinny(const void* A, const void* W, void* C, int c_dty
     if (!grouped && M <= 0) return 0;
     if (grouped && max_active <= 0) return 0;
     if (X && (!norm_w || epi == SK_ADD || !llmx_gemm_skinny_normed_ok(x_rows, K) || (!grouped && x_rows != M))) return -2;
+    if (X && norm_bias && (K % 4 || K > 4096 || (((uintptr_t)X | (uintptr_t)norm_w | (uintptr_t)norm_bias) & 15))) return -2;
     SkinnyArgs g{(const bf16_t*)A, (const bf16_t*)W, C, M, N, K, lda, ldc, active, n_active, group_offsets, list, a_div > 0 ? a_div : 1,
-                 w_group_stride, up_offset, X, norm_w, norm_eps, x_rows, epi != SK_SWIGLU ? act : LLMX_ACT_NONE, act_params,
+                 w_group_stride, up_offset, X, norm_w, norm_eps, x_rows, norm_bias, epi != SK_SWIGLU ? act : LLMX_ACT_NONE, act_params,
                  GluArgs{epi == SK_SWIGLU ? glu_kind : LLMX_GLU_SILU, glu_limit, epi == SK_SWIGLU ? glu_row_scale : nullptr,
                          epi == SK_SWIGLU ? glu_row_gate : nullptr, glu_row_gate_ld}};
     if (!llmx_act_fits(act, act_params, epi == SK_STORE, epi == SK_ADD)) return -2;

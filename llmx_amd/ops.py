@@ -110,7 +110,7 @@ def _declare(h) -> None:
         "llmx_route_topk": [P, P, I, L, P, P, P, I, I, I, I, I, F, P, I, I, I, P],
         "llmx_moe_align": [P, I, I, P, P, P, P, P, P, P, P],
         "llmx_route_topk_align": [P, P, I, L, P, P, P, I, I, I, I, I, F, I, I, I, P, P, P, P, P, P],
-        "llmx_gemm_skinny": [P, P, P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, I, L, I, P, P, F, I, I, P, I, F, P, P, I, P],
+        "llmx_gemm_skinny": [P, P, P, I, I, I, I, I, I, I, I, I, I, P, P, P, P, I, L, I, P, P, F, I, P, I, P, I, F, P, P, I, P],
         "llmx_gemm_skinny_normed_ok": [I, I],
         "llmx_gemm_skinny_f32_normed_ok": [I, I],
         "llmx_argmax_rows": [P, P, P, P, I, I, P],
@@ -1059,18 +1059,22 @@ def _skinny_ok(a: torch.Tensor, w: torch.Tensor, c: torch.Tensor, epilogue: int)
 
 
 class NormedRows:
-    """The float32 rows x seen through an RMSNorm (weight, eps), not yet computed: a product that reads its rows this way
+    """The float32 rows x seen through an RMSNorm (weight, eps), or with a `bias` a layer norm, not yet computed: a product that reads its rows this way
     forms norm(x) itself while its weights travel (steps of very few rows only), and no norm kernel runs."""
 
-    def __init__(self, x: torch.Tensor, weight: torch.Tensor, eps: float):
-        self.x, self.weight, self.eps = x, weight, float(eps)
+    def __init__(self, x: torch.Tensor, weight: torch.Tensor, eps: float, bias: Optional[torch.Tensor] = None):
+        self.x, self.weight, self.eps, self.bias = x, weight, float(eps), bias
         self.shape = x.shape
+        if bias is not None and (x.shape[1] % 4 or x.shape[1] > LAYER_NORMED_MAX):
+            raise KernelError(f"normed rows: a layer norm of {x.shape[1]} values is not one a product forms itself")
 
     def args(self):
-        return _dev(self.x, "x", torch.float32), _dev(self.weight, "norm weight", torch.float32, (self.x.shape[1],)), self.eps, self.x.shape[0]
+        return _dev(self.x, "x", torch.float32), _dev(self.weight, "norm weight", torch.float32, (self.x.shape[1],)), self.eps, self.x.shape[0], \
+            _dev(self.bias, "norm bias", torch.float32, (self.x.shape[1],))
 
 
-_NO_NORM = (0, 0, 0.0, 0)
+_NO_NORM = (0, 0, 0.0, 0, 0)
+LAYER_NORMED_MAX = 4096      # values of a row that a product forms a layer norm of (with a bias) itself
 
 
 NORMED_ROWS_PAY = 1   # rows up to which a product that norms its own rows beats the norm kernel (measured: 1 row 3.07 -> 2.98 ms a step,
@@ -1757,7 +1761,7 @@ def gemm_f32(a, w: torch.Tensor, c: torch.Tensor, add: bool = False, parts: Opti
     if w.shape[1] != K or tuple(c.shape) != (M, N):
         raise KernelError(f"gemm_f32 shapes do not agree: a {tuple(a.shape)}, w {tuple(w.shape)}, c {tuple(c.shape)}")
     normed = isinstance(a, NormedRows)    # the product reads norm(x), unrounded, formed by its own workgroups
-    if normed and not gemm_f32_can_norm_rows(M, w):
+    if normed and (a.bias is not None or not gemm_f32_can_norm_rows(M, w)):
         raise KernelError("gemm_f32: normed rows are not taken for this product")
     if K % 4:
         if parts is not None:

@@ -129,6 +129,9 @@ class LatentAttention(Mixer):
         # a recorded step reads the groups' lists and the plan's items; the key keeps them alive
         return self._groups(step), self._plan(step)
 
+    def takes_deferred_norm(self, step):
+        return ops.gemm_takes_normed_rows(step.rows, self.w_in, torch.float32)
+
     def forward(self, step, h, out, accumulate, cache: LayerCache, h32=None):
         T, H, act = step.rows, self.heads, step.act_dtype
         lead = (T, H) if self.row_major else (H, T)

@@ -131,6 +131,9 @@ class HeadDeltaRule(Mixer):
         self.a_log, self.dt_bias = tensors[self.name("A_log")], tensors[self.name("dt_bias")]
         self.norm, self.w_o = tensors[self.name("norm")], tensors[self.name("o")]
 
+    def takes_deferred_norm(self, step):
+        return ops.gemm_takes_normed_rows(step.rows, self.w_in, torch.float32)
+
     def forward(self, step, h, out, accumulate, cache: LayerCache, h32=None):
         T, H, G, D, V = step.rows, self.heads, self.kv_heads, self.dim, self.vdim
         f32 = torch.float32

@@ -307,6 +307,9 @@ class DenseAct(FeedForward):
         else:
             self.act = tensors[self.name("act")]
 
+    def takes_deferred_norm(self, step):
+        return self.biased and ops.gemm_takes_normed_rows(step.rows, self.w_up, step.act_dtype)
+
     def forward(self, step, h, out, accumulate, h32=None):
         a = step.buf("dense.act", (step.rows, self.intermediate), step.act_dtype)
         if self.activation == "polynorm":

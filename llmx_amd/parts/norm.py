@@ -99,6 +99,12 @@ class LayerNorm(Norm):
     def forward(self, step, x, out, out32=None, pick=None):
         ops.layernorm(x, self.weight, self.eps, out, out32, pick, bias=self.bias)
 
+    def deferred(self, x):
+        # the products form the norm with a bias, of rows that fit a workgroup's registers
+        if self.bias is None or self.width % 4 or self.width > ops.LAYER_NORMED_MAX:
+            return None
+        return ops.NormedRows(x, self.weight, self.eps, self.bias)
+
     def add_into(self, step, x, y, copy=None):
         """x += norm(y); `copy` (optional) receives the new rows in its own type."""
         if self.bias is not None:
