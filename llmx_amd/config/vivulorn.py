@@ -162,6 +162,7 @@ def _read_layer(entry, i: int) -> LayerConfig:
                                       kv_rank=m.integer("kv_rank"), scale=m.real("scale", positive=True), rot_base=rot.real("base", positive=True))
         if rot.integer("dims") != mixer.rot_dim:
             raise rot.unsupported("dims", f"the rotated part of {mixer.rot_dim} turns whole")
+        rot.held("scaling", None)
         rot.finish((), ARCHITECTURE)
     m.finish((), ARCHITECTURE)
     mlp = r.child("mlp", required=False)

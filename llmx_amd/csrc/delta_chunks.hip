@@ -242,8 +242,8 @@ __global__ void __launch_bounds__(256) delta_chunk_solve_kernel(DeltaChunkArgs a
     }
 }
 
-// Grid (H * value tiles, long requests), a wave for every 16 key channels.  A chunk's operands are asked for while the chunk before
-// is worked on.
+// Grid (H * value tiles, long requests), a wave for every 16 key channels.  The operands of the chunks to
+// come are asked for while one is worked on.
 template <int NU>
 __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkArgs a) {
     constexpr int NT = 64 * NU, EL = 1024 / NT, LDU = 20;      // EL: values of the chunk's U (64 x 16) a thread adds up
@@ -287,21 +287,22 @@ __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkA
     const int first = EL * tid;                             // the thread's values: row and column from its place in a tile's lanes
     const int u_row0 = 16 * (first >> 8) + 4 * ((first & 255) >> 6), u_col = ((first & 255) >> 2) & 15, u_e0 = first & 3;
     const int kd = min(16 * wave + c, a.D - 1), wd = real ? 16 * wave + 4 * g : 0;
-    // a thread's places within a chunk's operands; what moves from chunk to chunk (and from row to row) is the same for every thread
-    const uint32_t w_at = (uint32_t)(c * a.DR + wd), k_at = (uint32_t)(4 * g * a.ldk + kd), u_at = (uint32_t)((u_row0 + u_e0) * a.VR + 16 * vt + u_col);
-    const uint32_t d_at = (uint32_t)(u_row0 + u_e0);
+    // a thread's places within a chunk's operands, in bytes from a base that is the same for every thread
+    const uint32_t w_at = 4u * (uint32_t)(c * a.DR + wd), k_at = 4u * (uint32_t)(4 * g * a.ldk + kd);
+    const uint32_t u_at = 4u * (uint32_t)((u_row0 + u_e0) * a.VR + 16 * vt + u_col), d_at = 4u * (uint32_t)(u_row0 + u_e0);
+    const uint32_t start_at = 4u * (uint32_t)((16 * vt + c) * a.DR + 16 * wave + 4 * g);
     auto fetch = [&](Operands& x, int ch) {
         const size_t at = (size_t)ch * a.H + h;
         const float* W = a.W + at * DS_ROWS * a.DR;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) x.w[i] = *reinterpret_cast<const f32x4_t*>(W + (size_t)(16 * i) * a.DR + w_at);
+        for (int i = 0; i < 4; ++i) x.w[i] = *reinterpret_cast<const f32x4_t*>(reinterpret_cast<const char*>(W + (size_t)(16 * i) * a.DR) + w_at);
         const int ahead = (ch - c0) * DS_ROWS, n = min(DS_ROWS, rows - ahead);
         const float* kp = a.k + (size_t)(row0 + ahead) * a.ldk + (size_t)(h / a.share) * a.D;
         if (n == DS_ROWS) {
 #pragma unroll
             for (int s = 0; s < 4; ++s)
 #pragma unroll
-                for (int e = 0; e < 4; ++e) x.k[4 * s + e] = (kp + (size_t)(16 * s + e) * a.ldk)[k_at];
+                for (int e = 0; e < 4; ++e) x.k[4 * s + e] = *reinterpret_cast<const float*>(reinterpret_cast<const char*>(kp + (size_t)(16 * s + e) * a.ldk) + k_at);
         } else {
 #pragma unroll
             for (int s = 0; s < 4; ++s)
@@ -312,14 +313,14 @@ __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkA
         const float* decays = a.decays + at * DS_ROWS;
 #pragma unroll
         for (int y = 0; y < EL; ++y) {
-            x.u0[y] = (U + (size_t)y * a.VR)[u_at];
-            x.decay[y] = (decays + y)[d_at];
+            x.u0[y] = *reinterpret_cast<const float*>(reinterpret_cast<const char*>(U + (size_t)y * a.VR) + u_at);
+            x.decay[y] = *reinterpret_cast<const float*>(reinterpret_cast<const char*>(decays + y) + d_at);
         }
         x.keep = a.keep[at];
     };
     auto work = [&](const Operands& x, int ch) {
         const size_t at = (size_t)ch * a.H + h;
-        if (real) *reinterpret_cast<f32x4_t*>(a.starts + (at * a.VR + 16 * vt + c) * a.DR + 16 * wave + 4 * g) = S;
+        if (real) *reinterpret_cast<f32x4_t*>(reinterpret_cast<char*>(a.starts + at * a.VR * a.DR) + start_at) = S;
         f32x4_t p[4];
 #pragma unroll
         for (int i = 0; i < 4; ++i) p[i] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
@@ -337,28 +338,39 @@ __global__ void __launch_bounds__(64 * NU) delta_chunk_states_kernel(DeltaChunkA
             for (int w = 1; w < NU; ++w) sum += part[w][first + y];
             const float u = x.u0[y] - sum;
             const int row = u_row0 + u_e0 + y;
-            (a.U + (at * DS_ROWS + y) * a.VR)[u_at] = u;
+            *reinterpret_cast<float*>(reinterpret_cast<char*>(a.U + (at * DS_ROWS + y) * a.VR) + u_at) = u;
             us[row * LDU + u_col] = u * x.decay[y];
         }
         __syncthreads();
+        float b[16];
+#pragma unroll
+        for (int s = 0; s < 4; ++s)
+#pragma unroll
+            for (int e = 0; e < 4; ++e) b[4 * s + e] = us[(16 * s + 4 * g + e) * LDU + c];
+        __builtin_amdgcn_sched_barrier(0);      // all of them asked for before the first product waits for one
         f32x4_t add[2];
         add[0] = f32x4_t{S[0] * x.keep, S[1] * x.keep, S[2] * x.keep, S[3] * x.keep};
         add[1] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
         for (int s = 0; s < 4; ++s)
 #pragma unroll
-            for (int e = 0; e < 4; ++e) add[e & 1] = mfma4(x.k[4 * s + e], us[(16 * s + 4 * g + e) * LDU + c], add[e & 1]);
+            for (int e = 0; e < 4; ++e) add[e & 1] = mfma4(x.k[4 * s + e], b[4 * s + e], add[e & 1]);
 #pragma unroll
         for (int e = 0; e < 4; ++e) S[e] = 16 * wave + 4 * g + e < a.D ? add[0][e] + add[1][e] : 0.0f;
     };
-    Operands even, odd;
-    fetch(even, c0);
-    for (int i = 0; i < nc; i += 2) {
-        fetch(odd, c0 + min(i + 1, nc - 1));
-        work(even, c0 + i);
-        if (i + 1 >= nc) break;
-        fetch(even, c0 + min(i + 2, nc - 1));
-        work(odd, c0 + i + 1);
+    // sets of operands that take turns: the next AHEAD chunks' are on their way while one is worked on (past the end the last again)
+    constexpr int AHEAD = NU > 8 ? 1 : 2;
+    Operands ring[AHEAD + 1];
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) fetch(ring[u], c0 + min(u, nc - 1));
+    for (int i = 0; i < nc; i += AHEAD + 1) {
+#pragma unroll
+        for (int u = 0; u <= AHEAD; ++u) {
+            if (i + u < nc) {
+                fetch(ring[(u + AHEAD) % (AHEAD + 1)], c0 + min(i + u + AHEAD, nc - 1));
+                work(ring[u], c0 + i + u);
+            }
+        }
     }
 #pragma unroll
     for (int e = 0; e < 4; ++e) {
@@ -407,7 +419,7 @@ extern "C" int llmx_delta_chunks(const float* q, int ldq, const float* k, int ld
     if (n_chunks <= 0 || n_long <= 0) return 0;
     if (H < 1 || H > 65535 || share < 1 || H % share || D < 1 || D > 256 || V < 1 || n_long > 65535 || (taps > 1 && !tail_src)) return -2;
     const int DR = (D + 15) / 16 * 16, VR = (V + 15) / 16 * 16;
-    if ((size_t)H * VR * DR > (size_t)1 << 30) return -2;
+    if ((size_t)H * VR * DR > (size_t)1 << 30 || (size_t)VR * DR > (size_t)1 << 28 || (size_t)ldk > (size_t)1 << 24) return -2;
     DeltaChunkArgs a{q, k, v, ldq, ldk, ldv, beta, log_decay, state, state_stride, slot_read, slot_write, chunks, entry_chunks, W, U, decays, keep,
                      starts, out, out_scale, H, share, D, V, DR, VR, tail_src, tail_ld, tail_C, taps, tail_off, entry_rows};
     llmx_note_launch(LK_DELTA_CHUNKS);

@@ -26,12 +26,12 @@ from vivulorn_cases import CONFIGS, PAGES, greedy, load_plain, model_folder, pla
 
 pytestmark = pytest.mark.gpu
 
-F32_TOL = 5e-5      # |engine - plain| over all logits relative to the largest |logit|: float32 sums in another order
-CUT_TOL = 3e-5      # two cuttings of the same tokens where one runs the recurrence by chunks, float32
+F32_TOL = 1e-5      # |engine - plain| over all logits relative to the largest |logit|: float32 sums in another order
+CUT_TOL = 1e-5      # two cuttings of the same tokens where one runs the recurrence by chunks, float32
 # the serving path against the plain implementation (float64, nothing rounded): the largest difference and the root mean square of
-# all, relative to the logits'
-BF16_TOL = {"A": 6e-2, "B": 6e-2, "C": 6e-2, "D": 6e-2}
-BF16_RMS = {"A": 2e-2, "B": 2e-2, "C": 2e-2, "D": 2e-2}
+# all, relative to the logits'.  Met: A 2.6e-2 and 9.2e-3, B 4.0e-3 and 4.1e-3, C 5.4e-3 and 4.9e-3, D 3.0e-2 and 7.3e-3
+BF16_TOL = {"A": 4e-2, "B": 8e-3, "C": 1e-2, "D": 4.5e-2}
+BF16_RMS = {"A": 1.3e-2, "B": 6e-3, "C": 7.5e-3, "D": 1.1e-2}
 ROOT = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
 DTYPES = [torch.float32, torch.bfloat16]
 DTYPE_IDS = ["float32", "bfloat16"]

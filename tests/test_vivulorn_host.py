@@ -205,7 +205,7 @@ def _broken(config, path, value):
     (("layers", 0, "mixer", "kv_heads"), 3, "kv_heads"), (("layers", 0, "mixer", "rot", "dims"), 34, "rot.dims"),
     (("layers", 0, "mixer", "rot", "scaling", "kind"), "yarn", "kind"), (("layers", 0, "mixer", "window"), 5, "window"),
     (("layers", 3, "mixer", "rot", "dims"), 8, "dims"), (("layers", 3, "mixer", "rot_dim"), 15, "dims"),
-    (("layers", 2, "mixer", "conv"), 0, "conv"), (("layers", 2, "mixer", "dim"), 300, "dim"), (("layers", 0, "mlp", "kind"), "moe", "kind"),
+    (("layers", 3, "mixer", "rot", "scaling"), {"factor": 2.0}, "scaling"), (("layers", 2, "mixer", "conv"), 0, "conv"), (("layers", 2, "mixer", "dim"), 300, "dim"), (("layers", 0, "mlp", "kind"), "moe", "kind"),
     (("loop", "stop"), 9, "loop"), (("loop", "times"), 0, "times"), (("logit_softcap",), -1.0, "logit_softcap"), (("embedding", "rows"), 1, "rows"),
     (("norm", "eps"), "x", "eps"), (("experts",), 4, "experts")], ids=lambda x: str(x) if not isinstance(x, (tuple, list)) else "-".join(map(str, x)))
 def test_configurations_that_are_refused(path, value, names):
@@ -220,5 +220,8 @@ def test_optional_keys():
     bare = copy.deepcopy(CONFIG_D)
     del bare["embedding"], bare["logit_softcap"]
     cfg = read_config(bare)
+    null = copy.deepcopy(CONFIG_A)
+    null["layers"][3]["mixer"]["rot"]["scaling"] = None
+    assert read_config(null) == read_config(copy.deepcopy(CONFIG_A))
     assert cfg.embedding_scale == 1.0 and cfg.logit_softcap is None and cfg.loop is None
     assert read_config(dict(CONFIG_C, name="x", seed=3)).vocab_size == CONFIG_C["vocab"]
