@@ -345,13 +345,12 @@ struct ActFn {
         }
         return v;
     }
-    // with the feature's own number (BIAS, GELU_BIAS; 0 for the others)
-    __device__ __forceinline__ float operator()(float v, float bias) const {
-        if (!llmx_act_reads_vector(kind)) return (*this)(v);
-        const float z = v + bias;
-        return kind == LLMX_ACT_GELU_BIAS ? 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)) : z;
-    }
 };
+// BIAS and GELU_BIAS of a value with its feature's number.
+__device__ __forceinline__ float biased_act(int kind, float v, float bias) {
+    const float z = v + bias;
+    return kind == LLMX_ACT_GELU_BIAS ? 0.5f * z * (1.0f + erff(z * 0.70710678118654752f)) : z;
+}
 // The number of feature n (of N) that an activation reads, 0 where it reads none.
 __device__ __forceinline__ float act_feature(int kind, const float* __restrict__ params, int n, int N) {
     return llmx_act_reads_vector(kind) ? params[n < N ? n : N - 1] : 0.0f;

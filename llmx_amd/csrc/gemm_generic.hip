@@ -134,7 +134,7 @@ __global__ void __launch_bounds__(256) gemm_generic_kernel(GemmArgs g) {
                     // the gated unit; by default silu(g) * u with silu(x) = x / (1 + exp(-x))
                     v = glu(v, accu[i][j]);
                 } else {
-                    v = act(v, act_feature(act.kind, g.act_params, n, g.N));
+                    v = llmx_act_reads_vector(act.kind) ? biased_act(act.kind, v, act_feature(act.kind, g.act_params, n, g.N)) : act(v);
                     if (EPI == EPI_ADD) v = ld(c) + v;
                 }
                 st(c, v);

@@ -54,9 +54,12 @@ __device__ __forceinline__ bf16x8_t load_frag(const bf16_t* p, bool in) {
     return __builtin_bit_cast(bf16x8_t, v);
 }
 
-template <int KS, int MT, int EPI, typename TC, bool GROUPED, int SK_UNROLL, bool NORMED>
+// NORM: what a product that norms its own rows forms (SK_RMS, SK_LAYER), or SK_ROWS: A is read.  BIASED: g.act reads a number a feature.
+enum : int { SK_ROWS = 0, SK_RMS = 1, SK_LAYER = 2 };
+template <int KS, int MT, int EPI, typename TC, bool GROUPED, int SK_UNROLL, int NORM, bool BIASED>
 __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
     constexpr int NACC = (EPI == SK_SWIGLU) ? 2 : 1;
+    constexpr bool NORMED = NORM != SK_ROWS;
     __shared__ float red[KS > 1 ? KS : 1][MT * NACC][256];
     __shared__ int rows_a[MT * 16];
     __shared__ int rows_c[MT * 16];
@@ -66,8 +69,7 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
     const int r = lane & 15, kg = lane >> 4;
     const int n0 = blockIdx.x * 16;
-    const ActParams act_params(EPI == SK_STORE ? g.act : LLMX_ACT_NONE, g.act_params);
-    const bool act_vector = EPI != SK_SWIGLU && llmx_act_reads_vector(g.act);      // numbers a feature, asked for long before the epilogue
+    const ActParams act_params(EPI == SK_STORE && !BIASED ? g.act : LLMX_ACT_NONE, g.act_params);
     const bf16_t* W = g.W;
     int row_begin = 0, row_end = g.M;
     if (GROUPED) {
@@ -111,7 +113,7 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
         if (NORMED && !rows_normed) {
             // the step's rows, normed and rounded as the norm kernel stores them, while the first weights travel
             auto keep = [&](int row, int i, float y) { normed_rows[(size_t)row * K + i] = f32_to_bf16(y); };
-            if (g.norm_bias) layer_norm_rows_as_256<KS>(g.X, (size_t)K, g.x_rows, K, g.norm_w, g.norm_bias, g.norm_eps, norm_scratch, keep);
+            if (NORM == SK_LAYER) layer_norm_rows_as_256<KS>(g.X, (size_t)K, g.x_rows, K, g.norm_w, g.norm_bias, g.norm_eps, norm_scratch, keep);
             else rms_rows_as_1024<KS>(g.X, (size_t)K, g.x_rows, K, g.norm_w, g.norm_eps, norm_scratch, keep);
             rows_normed = true;   // the barrier below stands between these stores and the first read
         }
@@ -146,7 +148,7 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
             for (int a = 0; a < NACC; ++a) acc[t][a] = f32x4_t{0.0f, 0.0f, 0.0f, 0.0f};
         // what an adding epilogue joins: asked for now, used after the loop
         float c_old[MT][4], act_n[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-        if (act_vector && wave == 0) {
+        if (BIASED && wave == 0) {      // asked for long before the epilogue
 #pragma unroll
             for (int i = 0; i < 4; ++i) act_n[i] = act_feature(g.act, g.act_params, n0 + 4 * kg + i, g.N);
         }
@@ -238,8 +240,8 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
                     if (n0 + 4 * kg + i >= g.N) continue;
                     float x = v[0][i];
                     if (EPI == SK_SWIGLU) x = glu(x, v[1][i]);
-                    if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x, act_n[i]);
-                    if (EPI == SK_ADD && act_vector) x = x + act_n[i];
+                    if (BIASED) x = EPI == SK_STORE ? biased_act(g.act, x, act_n[i]) : x + act_n[i];
+                    else if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x);
                     if (EPI == SK_ADD) x = c_old[t][i] + x;
                     st(c + i, x);
                 }
@@ -253,15 +255,14 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_kernel(SkinnyArgs g) {
 // more bytes of rows (from the caches, again for every strip) than of weights; a workgroup that multiplies the rows'
 // fragments into two strips fetches them half as often.  A wave's steps, their rounds of four and the order in which
 // the waves' sums are added are those of the kernel above: the same bits.
-template <int KS, int MT, int EPI, typename TC>
+template <int KS, int MT, int EPI, typename TC, bool BIASED>
 __global__ void __launch_bounds__(64 * KS) gemm_skinny_two_strips_kernel(SkinnyArgs g) {
     static_assert(EPI != SK_SWIGLU, "one weight strip a feature strip");
     __shared__ float red[KS > 1 ? KS : 1][MT * 2][256];
     const int tid = threadIdx.x, wave = tid >> 6, lane = tid & 63;
     const int r = lane & 15, kg = lane >> 4;
     const int n0 = blockIdx.x * 32;
-    const ActParams act_params(EPI == SK_STORE ? g.act : LLMX_ACT_NONE, g.act_params);
-    const bool act_vector = EPI != SK_SWIGLU && llmx_act_reads_vector(g.act);      // numbers a feature, asked for long before the epilogue
+    const ActParams act_params(EPI == SK_STORE && !BIASED ? g.act : LLMX_ACT_NONE, g.act_params);
     const int K = g.K;
     const int steps_total = (K + 31) >> 5;
     const int per = (steps_total + KS - 1) / KS;
@@ -280,7 +281,7 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_two_strips_kernel(SkinnyA
     }
     f32x4_t acc[MT][2];
     float act_n[2][4] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}};
-    if (act_vector && wave == 0) {
+    if (BIASED && wave == 0) {
 #pragma unroll
         for (int q = 0; q < 2; ++q)
 #pragma unroll
@@ -336,8 +337,8 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_two_strips_kernel(SkinnyA
             for (int i = 0; i < 4; ++i) {
                 if (n0 + 16 * q + 4 * kg + i >= g.N) continue;
                 float x = v[i];
-                if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x, act_n[q][i]);
-                if (EPI == SK_ADD && act_vector) x = x + act_n[q][i];
+                if (BIASED) x = EPI == SK_STORE ? biased_act(g.act, x, act_n[q][i]) : x + act_n[q][i];
+                else if (EPI == SK_STORE && g.act != LLMX_ACT_NONE) x = ActFn(g.act, act_params)(x);
                 if (EPI == SK_ADD) x = ld(c + i) + x;
                 st(c + i, x);
             }
@@ -351,36 +352,54 @@ __global__ void __launch_bounds__(64 * KS) gemm_skinny_two_strips_kernel(SkinnyA
 
 // Returns -2 (and launches nothing) for a combination that has no kernel: normed rows with several tiles of rows or
 // with an adding epilogue.
-template <int KS, int MT, int EPI, typename TC>
-static int launch_grouped(const SkinnyArgs& g, dim3 grid, bool grouped, hipStream_t stream) {
+template <int KS, int MT, int EPI, typename TC, bool BIASED>
+static int launch_dense(const SkinnyArgs& g, dim3 grid, hipStream_t stream) {
     if (g.X) {
         // normed rows: one tile of rows, the rows kept in LDS
         if constexpr (MT == 1 && EPI != SK_ADD) {
             const size_t lds = (size_t)g.x_rows * g.K * sizeof(bf16_t);
-            llmx_note_launch(grouped ? LK_GEMM_SKINNY_GROUPED_NORMED : LK_GEMM_SKINNY_NORMED);
-            if (grouped)
-                hipLaunchKernelGGL((gemm_skinny_kernel<KS, 1, EPI, TC, true, SKINNY_ROUND(MT, EPI), true>), grid, dim3(64 * KS), lds, stream, g);
+            llmx_note_launch(LK_GEMM_SKINNY_NORMED);
+            if (g.norm_bias)
+                hipLaunchKernelGGL((gemm_skinny_kernel<KS, 1, EPI, TC, false, SKINNY_ROUND(MT, EPI), SK_LAYER, BIASED>), grid, dim3(64 * KS), lds, stream, g);
             else
-                hipLaunchKernelGGL((gemm_skinny_kernel<KS, 1, EPI, TC, false, SKINNY_ROUND(MT, EPI), true>), grid, dim3(64 * KS), lds, stream, g);
+                hipLaunchKernelGGL((gemm_skinny_kernel<KS, 1, EPI, TC, false, SKINNY_ROUND(MT, EPI), SK_RMS, BIASED>), grid, dim3(64 * KS), lds, stream, g);
             return 0;
         }
         return -2;
-    }
-    if (grouped) {
-        llmx_note_launch(LK_GEMM_SKINNY_GROUPED);
-        hipLaunchKernelGGL((gemm_skinny_kernel<KS, MT, EPI, TC, true, SKINNY_ROUND(MT, EPI), false>), grid, dim3(64 * KS), 0, stream, g);
-        return 0;
     }
     if constexpr (MT > 1 && EPI != SK_SWIGLU) {
         // several tiles of rows: two strips a workgroup where that still gives the chip enough workgroups
         if ((g.N + 31) / 32 >= SKINNY_TWO_STRIPS_MIN_WORKGROUPS) {
             llmx_note_launch(LK_GEMM_SKINNY_TWO_STRIPS);
-            hipLaunchKernelGGL((gemm_skinny_two_strips_kernel<KS, MT, EPI, TC>), dim3((g.N + 31) / 32), dim3(64 * KS), 0, stream, g);
+            hipLaunchKernelGGL((gemm_skinny_two_strips_kernel<KS, MT, EPI, TC, BIASED>), dim3((g.N + 31) / 32), dim3(64 * KS), 0, stream, g);
             return 0;
         }
     }
     llmx_note_launch(LK_GEMM_SKINNY);
-    hipLaunchKernelGGL((gemm_skinny_kernel<KS, MT, EPI, TC, false, SKINNY_ROUND(MT, EPI), false>), grid, dim3(64 * KS), 0, stream, g);
+    hipLaunchKernelGGL((gemm_skinny_kernel<KS, MT, EPI, TC, false, SKINNY_ROUND(MT, EPI), SK_ROWS, BIASED>), grid, dim3(64 * KS), 0, stream, g);
+    return 0;
+}
+
+template <int KS, int MT, int EPI, typename TC>
+static int launch_grouped(const SkinnyArgs& g, dim3 grid, bool grouped, hipStream_t stream) {
+    const bool biased = llmx_act_reads_vector(g.act);
+    if (!grouped) {
+        if constexpr (EPI != SK_SWIGLU)
+            if (biased) return launch_dense<KS, MT, EPI, TC, true>(g, grid, stream);
+        return launch_dense<KS, MT, EPI, TC, false>(g, grid, stream);
+    }
+    if (biased || g.norm_bias) return -2;      // no grouped product has a number a feature or a layer norm
+    if (g.X) {
+        if constexpr (MT == 1 && EPI != SK_ADD) {
+            const size_t lds = (size_t)g.x_rows * g.K * sizeof(bf16_t);
+            llmx_note_launch(LK_GEMM_SKINNY_GROUPED_NORMED);
+            hipLaunchKernelGGL((gemm_skinny_kernel<KS, 1, EPI, TC, true, SKINNY_ROUND(MT, EPI), SK_RMS, false>), grid, dim3(64 * KS), lds, stream, g);
+            return 0;
+        }
+        return -2;
+    }
+    llmx_note_launch(LK_GEMM_SKINNY_GROUPED);
+    hipLaunchKernelGGL((gemm_skinny_kernel<KS, MT, EPI, TC, true, SKINNY_ROUND(MT, EPI), SK_ROWS, false>), grid, dim3(64 * KS), 0, stream, g);
     return 0;
 }
 

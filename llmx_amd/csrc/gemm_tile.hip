@@ -449,10 +449,13 @@ __global__ void __launch_bounds__(256) gemm_tile_kernel(TileArgs g) {
 #pragma unroll
             for (int f = 0; f < 4; ++f) {
                 float v[4] = {acc[f][t][0], acc[f][t][1], acc[f][t][2], acc[f][t][3]};
-                if (g.act != LLMX_ACT_NONE) {
+                if (llmx_act_reads_vector(g.act)) {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) v[i] = biased_act(g.act, v[i], act_feature(g.act, g.act_params, n0 + 64 * wn + 16 * f + fq + i, g.N));
+                } else if (EPI == TL_STORE && g.act != LLMX_ACT_NONE) {
                     const ActFn act(g.act, g.act_params);
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) v[i] = act(v[i], act_feature(g.act, g.act_params, n0 + 64 * wn + 16 * f + fq + i, g.N));
+                    for (int i = 0; i < 4; ++i) v[i] = act(v[i]);
                 }
                 store_quad<EPI == TL_ADD>(crow, n0 + 64 * wn + 16 * f + fq, g.N, rows_aligned, v);
             }
@@ -719,10 +722,13 @@ __global__ void __launch_bounds__(512) gemm_wide_kernel(TileArgs g) {
 #pragma unroll
             for (int f = 0; f < 4; ++f) {
                 float v[4] = {acc[f][q][0], acc[f][q][1], acc[f][q][2], acc[f][q][3]};
-                if (g.act != LLMX_ACT_NONE) {
+                if (llmx_act_reads_vector(g.act)) {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) v[i] = biased_act(g.act, v[i], act_feature(g.act, g.act_params, n0 + 64 * wn + 16 * f + fq + i, g.N));
+                } else if (EPI == TL_STORE && g.act != LLMX_ACT_NONE) {
                     const ActFn act(g.act, g.act_params);
 #pragma unroll
-                    for (int i = 0; i < 4; ++i) v[i] = act(v[i], act_feature(g.act, g.act_params, n0 + 64 * wn + 16 * f + fq + i, g.N));
+                    for (int i = 0; i < 4; ++i) v[i] = act(v[i]);
                 }
                 store_quad<EPI == TL_ADD>(crow, n0 + 64 * wn + 16 * f + fq, g.N, rows_aligned, v);
             }
@@ -804,10 +810,13 @@ __global__ void __launch_bounds__(256) gemm_runs_sum_kernel(const float* __restr
 #pragma unroll
         for (int i = 0; i < 4; ++i) v[i] = r == 0 ? x[i] : v[i] + x[i];
     }
-    if (act_kind != LLMX_ACT_NONE) {
+    if (llmx_act_reads_vector(act_kind)) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] = biased_act(act_kind, v[i], act_feature(act_kind, act_params, n + i, N));
+    } else if (!ADD && act_kind != LLMX_ACT_NONE) {
         const ActFn act(act_kind, act_params);
 #pragma unroll
-        for (int i = 0; i < 4; ++i) v[i] = act(v[i], act_feature(act_kind, act_params, n + i, N));
+        for (int i = 0; i < 4; ++i) v[i] = act(v[i]);
     }
     store_quad<ADD>(C + (size_t)m * ldc, n, N, ldc % 4 == 0 && ((uintptr_t)C & 15) == 0, v);
 }
